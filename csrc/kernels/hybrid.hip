@@ -9,7 +9,9 @@
 // norm, latent attention's cached row, matrix memories, per-head products, gated units (plain and
 // clamped), and attention whose values are its keys before they rotate in neighbouring pairs.
 // The two attention kernels take options that further designs combine: row strides of the planes (values that are a
-// column block of the key rows), a cap on the scores, a sink in the softmax, several value heads under one head's weights.
+// column block of the key rows), a cap on the scores, a bias per unit of distance, a sink in the softmax (of score zero or
+// a learned one per head), first keys that stay visible outside a window, several value heads under one head's weights, a
+// gate per head and a scale on the result. Linear attention comes with decays per channel or one constant per head.
 //
 // A step's sequences are described by cu_q [B+1] (row ranges), positions [T] and slots [B]
 // (state slot of the sequence; < 0: padding row of a recorded step, skipped). A sequence whose
@@ -189,7 +191,8 @@ __global__ __launch_bounds__(64) void gla_scan_kernel(const float* __restrict__ 
                                                       const int32_t* __restrict__ positions,
                                                       const int32_t* __restrict__ slots, float* __restrict__ out, int H,
                                                       int D, int Dv, int mode, int nseg, int seg_len,
-                                                      const float* __restrict__ cs, long long state_stride, int ones) {
+                                                      const float* __restrict__ cs, long long state_stride, int ones,
+                                                      int v_silu) {
   const int b = blockIdx.z / nseg, seg = blockIdx.z % nseg, h = blockIdx.y;
   const int dv = blockIdx.x * 64 + threadIdx.x;
   const int slot = slots[b];
@@ -227,7 +230,7 @@ __global__ __launch_bounds__(64) void gla_scan_kernel(const float* __restrict__ 
   for (int t = r0; t < r1; ++t) {
 #pragma unroll
     for (int i = 0; i < NCH; ++i) cur[i] = nxt[i];
-    vcur = vnxt;
+    vcur = v_silu ? siluf_(vnxt) : vnxt;
     if (t + 1 < r1) fetch(t + 1, nxt, vnxt);
     float o = 0.f;
 #pragma unroll
@@ -262,7 +265,7 @@ constexpr int kSegRows = 64, kSegD = 32, kSegV = 128;
 __global__ __launch_bounds__(256) void scan_segment_state_kernel(
     const float* __restrict__ proj, int ld, const float4* __restrict__ prep, const int32_t* __restrict__ cu_q,
     const int32_t* __restrict__ slots, int H, int D, int Dv, int nseg, int seg_len, float* __restrict__ cs,
-    float* __restrict__ ca, int ones) {
+    float* __restrict__ ca, int ones, int v_silu) {
   __shared__ float2 ka[kSegRows][kSegD];            // (k, a) of the tile's key channels
   __shared__ float vs[kSegRows][kSegV];
   const int b = blockIdx.z / nseg, seg = blockIdx.z % nseg, h = blockIdx.y;
@@ -287,6 +290,7 @@ __global__ __launch_bounds__(256) void scan_segment_state_kernel(
     const int t = i / kSegV, dv = v0 + i % kSegV;
     float v = 0.f;
     if (t < n && dv < Dv) v = dv < Dvr ? proj[static_cast<size_t>(r0 + t) * ld + 2 * H * D + h * Dvr + dv] : 1.f;
+    if (v_silu) v = siluf_(v);
     vs[t][i % kSegV] = v;
   }
   __syncthreads();
@@ -346,15 +350,19 @@ __global__ void gla_carry_kernel(float* __restrict__ cs, const float* __restrict
 // ``ld_head`` apart in o (>= Dv); head h reads the weights w[h * w_stride ...] (w_stride 0: one
 // weight vector for all heads); act is silu (gate_kind 0) or sigmoid (1). With ``m`` [T, H] the
 // read-out is first divided by max(|o[Dv]|, exp(-m)) + 1e-6, o[Dv] being the column behind the head's values
-// (a matrix memory's normaliser . q, m its running maximum).
-template <bool AF32>
-__global__ void headnorm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w,
-                                     const float* __restrict__ gate, int ld_gate, void* __restrict__ out, int T, int H,
-                                     int Dv, float eps, int ld_head, int w_stride, int gate_kind,
-                                     const float* __restrict__ m) {
-  const int idx = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
-  const int lane = threadIdx.x & 63;
-  if (idx >= T * H) return;
+// (a matrix memory's normaliser . q, m its running maximum). ``ld_out``: row stride of the output (>= H * Dv: it may
+// be a column block of a wider matrix). WAVES = 4: a block per (row, head), for heads that are a whole row wide.
+template <bool AF32, int WAVES>
+__global__ __launch_bounds__(256) void headnorm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w,
+                                                            const float* __restrict__ gate, int ld_gate,
+                                                            void* __restrict__ out, int T, int H, int Dv, float eps,
+                                                            int ld_head, int w_stride, int gate_kind,
+                                                            const float* __restrict__ m, int ld_out) {
+  __shared__ float red[16];
+  constexpr int LANES = 64 * WAVES;
+  const int idx = WAVES == 1 ? blockIdx.x * 4 + (threadIdx.x >> 6) : blockIdx.x;
+  const int lane = WAVES == 1 ? (threadIdx.x & 63) : threadIdx.x;
+  if (WAVES == 1 && idx >= T * H) return;
   const int row = idx / H, h = idx % H;
   const float* orow = o + (static_cast<size_t>(row) * H + h) * ld_head;
   const float* grow = gate + static_cast<size_t>(row) * ld_gate + h * Dv;
@@ -362,18 +370,30 @@ __global__ void headnorm_gate_kernel(const float* __restrict__ o, const float* _
   float inv = 1.f;
   if (m != nullptr) inv = 1.f / (fmaxf(fabsf(orow[Dv]), expf(-m[idx])) + 1e-6f);
   float ss = 0.f;
-  for (int c = lane; c < Dv; c += 64) {
+  for (int c = lane; c < Dv; c += LANES) {
     const float v = orow[c] * inv;
     ss += v * v;
   }
-  ss = wave_sum(ss);
+  ss = WAVES == 1 ? wave_sum(ss) : block_sum(ss, red);
   const float r = inv / sqrtf(ss / static_cast<float>(Dv) + eps);
   typename Act<AF32>::type* dst = static_cast<typename Act<AF32>::type*>(out);
-  for (int c = lane; c < Dv; c += 64) {
+  for (int c = lane; c < Dv; c += LANES) {
     const float g = grow[c];
-    Act<AF32>::store(dst, static_cast<size_t>(row) * H * Dv + h * Dv + c,
+    Act<AF32>::store(dst, static_cast<size_t>(row) * ld_out + h * Dv + c,
                      orow[c] * r * wh[c] * (gate_kind == 0 ? siluf_(g) : sigmoidf_(g)));
   }
+}
+
+// Linear attention with ONE constant decay per head: operands (silu(q), silu(k), decay[h], -) of the same scan.
+__global__ void lightning_prepare_kernel(const float* __restrict__ proj, int ld, const float* __restrict__ decay,
+                                         float4* __restrict__ prep, long long n, int H, int D) {
+  const long long i = static_cast<long long>(blockIdx.x) * blockDim.x + threadIdx.x;
+  if (i >= n) return;
+  const int HD = H * D;
+  const long long t = i / HD;
+  const int c = static_cast<int>(i - t * HD);
+  const float* row = proj + t * ld;
+  prep[i] = make_float4(siluf_(row[c]), siluf_(row[HD + c]), decay[c / D], 0.f);
 }
 
 // ---------------------------------------------------------------- mLSTM: gates and prepared operands
@@ -682,14 +702,29 @@ __global__ __launch_bounds__(256) void rope_pairs_write_kernel(
 // applied to the ``nvh`` value heads vh0 .. vh0 + nvh - 1 side by side instead of its own group's (designs that
 // mix the heads' weights afterwards need every head's weights on every value head). Output row (t, h) has ``o_ld``
 // columns, written from column ``o_col0`` on.
+// Further options (AttnOpts): a bias per unit of distance (slope of the head times p - j, taken off the scaled score
+// before the cap), a learned sink score per head, the first ``keep`` keys visible whatever the window or chunk, a gate
+// logit per (row, head) and a scale on the result, and the row stride of the output.
 constexpr int kMaxVCols = 8;   // value width up to 512
+
+struct AttnOpts {
+  float softcap;
+  int sink;                    // the softmax's denominator carries an extra entry: of score sinks[h], or 0 without them
+  const float* sinks;          // [H]
+  const float* slopes;         // [H]
+  int keep;
+  const float* gate;           // [T, ld_gate], column h
+  int ld_gate;
+  float out_scale;
+  int o_row;                   // elements between the output rows of two tokens
+};
 
 template <bool CF32, bool AF32>
 __global__ __launch_bounds__(256) void attn_masked_kernel(
     const float* __restrict__ q, const void* __restrict__ kc, const void* __restrict__ vc,
     const int32_t* __restrict__ block_tables, int MB, const int32_t* __restrict__ row_seq,
     const int32_t* __restrict__ positions, void* __restrict__ out, int H, int G, int D, int Dv, int BS, float scale,
-    int chunk, int window, int k_ld, int v_ld, float softcap, int sink, int vh0, int nvh, int o_ld, int o_col0) {
+    int chunk, int window, int k_ld, int v_ld, AttnOpts opt, int vh0, int nvh, int o_ld, int o_col0) {
   extern __shared__ float lds[];
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int t = blockIdx.x;
@@ -709,7 +744,12 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
   const int32_t* table = block_tables + static_cast<size_t>(seq) * MB;
   const typename Act<CF32>::type* kbase = static_cast<const typename Act<CF32>::type*>(kc);
   const typename Act<CF32>::type* vbase = static_cast<const typename Act<CF32>::type*>(vc);
-  float m = sink ? 0.f : -INFINITY, l = sink ? 1.f : 0.f;
+  const float sink0 = opt.sinks != nullptr ? opt.sinks[h] : 0.f;
+  const float slope = opt.slopes != nullptr ? opt.slopes[h] : 0.f;
+  const float softcap = opt.softcap;
+  float m = opt.sink ? sink0 : -INFINITY, l = opt.sink ? 1.f : 0.f;
+  // the row's keys in order: the first ``kept`` ones (those the window no longer reaches), then lo .. p
+  const int kept = min(opt.keep, lo), nkeys = kept + p - lo + 1;
   float acc[kMaxVCols];
   int vcol[kMaxVCols], voff[kMaxVCols];            // a lane's value columns: column inside the head, row offset of the head's plane
   const int ncols = nvh * Dv;
@@ -726,9 +766,10 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
     voff[i] = vh0 < 0 ? 0 : (vh0 + vh - g) * BS;
   }
   __syncthreads();
-  for (int j0 = lo; j0 <= p; j0 += 64) {
-    const int j = j0 + lane;
-    const bool valid = j <= p;
+  for (int j0 = 0; j0 < nkeys; j0 += 64) {
+    const int jx = j0 + lane;
+    const int j = jx < kept ? jx : lo + jx - kept;
+    const bool valid = jx < nkeys;
     float s = -INFINITY;
     int crow = 0;
     if (valid) {
@@ -748,6 +789,7 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
       } else {
         for (int d = 0; d < D; ++d) dot += qs[d] * Act<CF32>::load(kr, d);
       }
+      dot -= slope * static_cast<float>(p - j);
       s = softcap > 0.f ? softcap * tanhf(dot / softcap) : dot;
     }
     const float mt = fmaxf(m, wave_max(s));
@@ -758,7 +800,7 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
     ps[lane] = pj;
     rows[lane] = crow;
     __syncthreads();
-    const int n = min(64, p - j0 + 1);
+    const int n = min(64, nkeys - j0);
 #pragma unroll
     for (int i = 0; i < kMaxVCols; ++i) {
       const int c = lane + 64 * i;
@@ -773,10 +815,12 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
     __syncthreads();
   }
   typename Act<AF32>::type* o = static_cast<typename Act<AF32>::type*>(out);
+  const float fin = opt.out_scale * (opt.gate != nullptr ? sigmoidf_(opt.gate[static_cast<size_t>(t) * opt.ld_gate + h]) : 1.f);
 #pragma unroll
   for (int i = 0; i < kMaxVCols; ++i) {
     const int c = lane + 64 * i;
-    if (live && c < ncols) Act<AF32>::store(o, (static_cast<size_t>(t) * H + h) * o_ld + o_col0 + c, acc[i] / l);
+    if (live && c < ncols)
+      Act<AF32>::store(o, static_cast<size_t>(t) * opt.o_row + static_cast<size_t>(h) * o_ld + o_col0 + c, acc[i] / l * fin);
   }
 }
 
@@ -842,7 +886,7 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
     const float* __restrict__ q, const void* __restrict__ kc, const void* __restrict__ vc,
     const int32_t* __restrict__ block_tables, int MB, const int32_t* __restrict__ cu_q,
     const int32_t* __restrict__ positions, void* __restrict__ out, int H, int G, int D, int Dv, int BS, float scale,
-    int chunk, int window, int k_ld, int v_ld, float softcap, int sink, int vh0, int nvh, int o_ld, int o_col0) {
+    int chunk, int window, int k_ld, int v_ld, AttnOpts opt, int vh0, int nvh, int o_ld, int o_col0) {
   extern __shared__ float lds[];
   const int b = blockIdx.z, h = blockIdx.y;
   const int q0 = cu_q[b], q1 = cu_q[b + 1];
@@ -911,19 +955,28 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
       vr[i] = load_raw8<CF32>(vc, vrow * v_ld + vin[i], von);
     }
   };
+  const float sink0 = opt.sinks != nullptr ? opt.sinks[h] : 0.f;
+  const float slope = opt.slopes != nullptr ? opt.slopes[h] : 0.f;
+  const float softcap = opt.softcap;
+  const int keep = opt.keep;
   float m[4], l[4];
   f32x4 o[kTileMaxVT];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
-    m[r] = sink ? 0.f : -INFINITY;
-    l[r] = sink ? 1.f : 0.f;
+    m[r] = opt.sink ? sink0 : -INFINITY;
+    l[r] = opt.sink ? 1.f : 0.f;
   }
 #pragma unroll
   for (int t = 0; t < kTileMaxVT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
   const float* Qw = Qs + wave * 16 * DS;
-  int j0 = (first_key(p0) / 16) * 16;
+  // tiles of the kept first keys, then from the first row's first key on (the same for the whole block)
+  const int lo_tile = (first_key(p0) / 16) * 16;
+  auto next_tile = [&](int j) { return j + 16 >= keep && j + 16 < lo_tile ? lo_tile : j + 16; };
+  int jn = 0;
+  int j0 = keep > 0 ? 0 : lo_tile;
   fetch(j0);
-  for (; j0 <= hi; j0 += 16) {
+  for (; j0 <= hi; j0 = jn) {
+    jn = next_tile(j0);
     __syncthreads();                                        // the previous tile has been consumed
 #pragma unroll
     for (int i = 0; i < 2; ++i)
@@ -932,8 +985,8 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
     for (int i = 0; i < NVU; ++i)
       if (vkey[i] >= 0) store_raw8<CF32>(vr[i], Vs + vkey[i] * VS + vcol[i]);
     __syncthreads();
-    if (j0 + 16 <= hi) fetch(j0 + 16);                      // in flight while this tile is computed
-    const bool mine = wave_rows > 0 && j0 <= wave_hi && j0 + 15 >= wave_lo;     // wave-uniform
+    if (jn <= hi) fetch(jn);                                // in flight while this tile is computed
+    const bool mine = wave_rows > 0 && j0 <= wave_hi && (j0 + 15 >= wave_lo || j0 < keep);     // wave-uniform
     if (!mine) continue;
     f32x4 sacc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};      // two chains keep the matrix pipe busy
     for (int d = 0; d < D; d += 8) {
@@ -946,8 +999,8 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
     for (int r = 0; r < 4; ++r) {
       const int row = 4 * lk + r;
       const int prow = pw0 + row;
-      const bool valid = row < wave_rows && j <= prow && j >= first_key(prow);
-      const float sraw = sacc[0][r] + sacc[1][r];
+      const bool valid = row < wave_rows && j <= prow && (j >= first_key(prow) || j < keep);
+      const float sraw = sacc[0][r] + sacc[1][r] - slope * static_cast<float>(prow - j);
       const float sv = valid ? (softcap > 0.f ? softcap * tanhf(sraw / softcap) : sraw) : -INFINITY;
       float mt = sv;
 #pragma unroll
@@ -988,16 +1041,14 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
   }
   typename Act<AF32>::type* dst = static_cast<typename Act<AF32>::type*>(out);
 #pragma unroll
-  for (int t = 0; t < kTileMaxVT; ++t) {
-    if (t < nt) {
+  for (int r = 0; r < 4; ++r) {
+    const int row = 4 * lk + r;
+    if (row >= wave_rows) continue;
+    const size_t tok = static_cast<size_t>(row0) + 16 * wave + row;
+    const float fin = opt.out_scale * (opt.gate != nullptr ? sigmoidf_(opt.gate[tok * opt.ld_gate + h]) : 1.f) / l[r];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int row = 4 * lk + r;
-        if (row < wave_rows)
-          Act<AF32>::store(dst, (static_cast<size_t>(row0 + 16 * wave + row) * H + h) * o_ld + o_col0 + t * 16 + lr,
-                           o[t][r] / l[r]);
-      }
-    }
+    for (int t = 0; t < kTileMaxVT; ++t)
+      if (t < nt) Act<AF32>::store(dst, tok * opt.o_row + static_cast<size_t>(h) * o_ld + o_col0 + t * 16 + lr, o[t][r] * fin);
   }
 }
 
@@ -1235,10 +1286,10 @@ LC_EXPORT int lc_mingru_scan(const void* zxg, void* state, const void* cu_q, con
 }
 
 // The scan over prepared operands (``prep``: T * H * D float4, see the prepare kernels): per head
-// S <- a S + k v^T over Dv value columns, the last ``ones`` of which read v = 1.
+// S <- a S + k v^T over Dv value columns, the last ``ones`` of which read v = 1; ``v_silu``: v is silu of the projection.
 static int launch_linear_scan(const void* proj, int ld, const void* prep, void* state, long long state_stride,
                               const void* cu_q, const void* positions, const void* slots, void* out, int B, int H, int D,
-                              int Dv, int ones, int max_len, void* scratch, hipStream_t st) {
+                              int Dv, int ones, int max_len, void* scratch, hipStream_t st, int v_silu = 0) {
   const bool segmented = max_len > 2 * kScanSegment;
   if (segmented && scratch == nullptr) return -1;
   const int nseg = segmented ? (max_len + kScanSegment - 1) / kScanSegment : 1;
@@ -1250,7 +1301,7 @@ static int launch_linear_scan(const void* proj, int ld, const void* prep, void* 
                                                 static_cast<float*>(state), static_cast<const int32_t*>(cu_q),      \
                                                 static_cast<const int32_t*>(positions),                             \
                                                 static_cast<const int32_t*>(slots), static_cast<float*>(out), H, D, \
-                                                Dv, MODE, nseg, kScanSegment, cs, state_stride, ones)
+                                                Dv, MODE, nseg, kScanSegment, cs, state_stride, ones, v_silu)
 #define LC_GLA_D(MODE)          \
   if (D <= 32) LC_GLA(32, MODE);  \
   else if (D <= 64) LC_GLA(64, MODE); \
@@ -1261,7 +1312,7 @@ static int launch_linear_scan(const void* proj, int ld, const void* prep, void* 
     const dim3 sgrid(((D + kSegD - 1) / kSegD) * ((Dv + kSegV - 1) / kSegV), H, B * nseg);
     scan_segment_state_kernel<<<sgrid, dim3(256), 0, st>>>(
         static_cast<const float*>(proj), ld, static_cast<const float4*>(prep), static_cast<const int32_t*>(cu_q),
-        static_cast<const int32_t*>(slots), H, D, Dv, nseg, kScanSegment, cs, ca, ones);
+        static_cast<const int32_t*>(slots), H, D, Dv, nseg, kScanSegment, cs, ca, ones, v_silu);
     const size_t n = static_cast<size_t>(H) * D * Dv;
     gla_carry_kernel<<<dim3(static_cast<unsigned>((n + 255) / 256), B), dim3(256), 0, st>>>(
         cs, ca, static_cast<const float*>(state), static_cast<const int32_t*>(cu_q),
@@ -1289,6 +1340,20 @@ LC_EXPORT int lc_gla_scan(const void* proj, int ld, const void* decay, void* sta
       1.f / tau, 1.f / sqrtf(static_cast<float>(D)));
   return launch_linear_scan(proj, ld, prep, state, state_stride, cu_q, positions, slots, out, B, H, D, Dv, 0, max_len,
                             scratch, st);
+}
+
+// One constant decay per head (``decay`` [H]); q, k and v are silu of the projection; no scale on q.
+LC_EXPORT int lc_lightning_scan(const void* proj, int ld, const void* decay, void* state, long long state_stride,
+                                const void* cu_q, const void* positions, const void* slots, void* out, int T, int B, int H,
+                                int D, int Dv, int max_len, void* scratch, void* prep, hipStream_t st) {
+  if (B <= 0 || T <= 0) return 0;
+  if (H <= 0 || D <= 0 || Dv <= 0 || D > 256 || ld < 2 * H * D + H * Dv || decay == nullptr) return -1;
+  if (prep == nullptr || state_stride < static_cast<long long>(H) * D * Dv) return -1;
+  const long long n = static_cast<long long>(T) * H * D;
+  lightning_prepare_kernel<<<dim3(static_cast<unsigned>((n + 255) / 256)), dim3(256), 0, st>>>(
+      static_cast<const float*>(proj), ld, static_cast<const float*>(decay), static_cast<float4*>(prep), n, H, D);
+  return launch_linear_scan(proj, ld, prep, state, state_stride, cu_q, positions, slots, out, B, H, D, Dv, 0, max_len,
+                            scratch, st, 1);
 }
 
 // mLSTM: gates and running maxima, prepared operands, then the scan over Dv + 1 value columns (the
@@ -1445,18 +1510,20 @@ LC_EXPORT int lc_head_linear(const void* A, int a_f32, int lda, const void* W, i
 
 LC_EXPORT int lc_headnorm_gate(const void* o, const void* w, const void* gate, int ld_gate, void* out, int act_f32,
                                int T, int H, int Dv, float eps, int ld_head, int w_stride, int gate_kind, const void* m,
-                               hipStream_t st) {
+                               int ld_out, hipStream_t st) {
   if (T <= 0) return 0;
-  if (H <= 0 || Dv <= 0 || ld_gate < H * Dv || ld_head < Dv || (m != nullptr && ld_head < Dv + 1)) return -1;
-  const dim3 grid((T * H + 3) / 4), block(256);
-  if (act_f32)
-    headnorm_gate_kernel<true><<<grid, block, 0, st>>>(static_cast<const float*>(o), static_cast<const float*>(w),
-                                                       static_cast<const float*>(gate), ld_gate, out, T, H, Dv, eps,
-                                                       ld_head, w_stride, gate_kind, static_cast<const float*>(m));
-  else
-    headnorm_gate_kernel<false><<<grid, block, 0, st>>>(static_cast<const float*>(o), static_cast<const float*>(w),
-                                                        static_cast<const float*>(gate), ld_gate, out, T, H, Dv, eps,
-                                                        ld_head, w_stride, gate_kind, static_cast<const float*>(m));
+  if (H <= 0 || Dv <= 0 || ld_gate < H * Dv || ld_head < Dv || (m != nullptr && ld_head < Dv + 1) || ld_out < H * Dv) return -1;
+  const bool wide = Dv >= 512;
+  const dim3 grid(wide ? T * H : (T * H + 3) / 4), block(256);
+#define LC_HN(A32, WAVES)                                                                                              \
+  headnorm_gate_kernel<A32, WAVES><<<grid, block, 0, st>>>(static_cast<const float*>(o), static_cast<const float*>(w), \
+                                                           static_cast<const float*>(gate), ld_gate, out, T, H, Dv, eps, \
+                                                           ld_head, w_stride, gate_kind, static_cast<const float*>(m), ld_out)
+  if (act_f32 && wide) LC_HN(true, 4);
+  else if (act_f32) LC_HN(true, 1);
+  else if (wide) LC_HN(false, 4);
+  else LC_HN(false, 1);
+#undef LC_HN
   LC_RETURN_LAST_ERROR();
 }
 
@@ -1483,12 +1550,17 @@ LC_EXPORT int lc_qkv_prep(const void* qkv, int ld, const void* qn, const void* k
 LC_EXPORT int lc_attn_masked(const void* q, const void* kc, const void* vc, int cache_f32, const void* block_tables,
                              int MB, const void* row_seq, const void* positions, void* out, int act_f32, int T, int H,
                              int G, int D, int Dv, int BS, float scale, int chunk, int window, int k_ld, int v_ld,
-                             float softcap, int sink, int vh0, int nvh, int o_ld, int o_col0, int vz, hipStream_t st) {
+                             float softcap, int sink, const void* sinks, const void* slopes, int keep, const void* gate,
+                             int ld_gate, float out_scale, int o_row, int vh0, int nvh, int o_ld, int o_col0, int vz,
+                             hipStream_t st) {
   if (T <= 0) return 0;
   if (H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || BS <= 0 || MB <= 0 || vz <= 0 || vz > 65535) return -1;
   // ``vz`` groups of nvh value heads each, one per block along z (vz = 1 unless value heads are named)
   if (nvh <= 0 || nvh * Dv > 64 * kMaxVCols || (vh0 < 0 && (nvh != 1 || vz != 1)) || (vh0 >= 0 && vh0 + vz * nvh > G)) return -1;
   if (k_ld < D || v_ld < Dv || o_col0 < 0 || o_ld < o_col0 + vz * nvh * Dv || softcap < 0.f) return -1;
+  if (keep < 0 || (gate != nullptr && ld_gate < H) || o_row < H * o_ld || (sinks != nullptr && !sink)) return -1;
+  const AttnOpts opt{softcap, sink, static_cast<const float*>(sinks), static_cast<const float*>(slopes), keep,
+                     static_cast<const float*>(gate), ld_gate, out_scale, o_row};
   const size_t lds = 4 * static_cast<size_t>(D + 128) * sizeof(float);
   if (lds > 64 * 1024) return -1;
   const dim3 grid(T, (H + 3) / 4, vz), block(256);
@@ -1496,7 +1568,7 @@ LC_EXPORT int lc_attn_masked(const void* q, const void* kc, const void* vc, int 
   attn_masked_kernel<C32, A32><<<grid, block, lds, st>>>(                                                       \
       static_cast<const float*>(q), kc, vc, static_cast<const int32_t*>(block_tables), MB,                      \
       static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(positions), out, H, G, D, Dv, BS, scale, \
-      chunk, window, k_ld, v_ld, softcap, sink, vh0, nvh, o_ld, o_col0)
+      chunk, window, k_ld, v_ld, opt, vh0, nvh, o_ld, o_col0)
   if (cache_f32 && act_f32) LC_ATT(true, true);
   else if (cache_f32) LC_ATT(true, false);
   else if (act_f32) LC_ATT(false, true);
@@ -1510,12 +1582,16 @@ LC_EXPORT int lc_attn_masked(const void* q, const void* kc, const void* vc, int 
 LC_EXPORT int lc_attn_tile(const void* q, const void* kc, const void* vc, int cache_f32, const void* block_tables,
                            int MB, const void* cu_q, const void* positions, void* out, int act_f32, int n_seq,
                            int max_len, int H, int G, int D, int Dv, int BS, float scale, int chunk, int window,
-                           int k_ld, int v_ld, float softcap, int sink, int vh0, int nvh, int o_ld, int o_col0,
-                           hipStream_t st) {
+                           int k_ld, int v_ld, float softcap, int sink, const void* sinks, const void* slopes, int keep,
+                           const void* gate, int ld_gate, float out_scale, int o_row, int vh0, int nvh, int o_ld,
+                           int o_col0, hipStream_t st) {
   if (n_seq <= 0 || max_len <= 0) return 0;
   if (H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || BS <= 0 || MB <= 0) return -1;
   if (nvh <= 0 || (vh0 < 0 && nvh != 1) || (vh0 >= 0 && vh0 + nvh > G)) return -1;
   if (k_ld < D || v_ld < Dv || o_col0 < 0 || o_ld < o_col0 + nvh * Dv || softcap < 0.f) return -1;
+  if (keep < 0 || (gate != nullptr && ld_gate < H) || o_row < H * o_ld || (sinks != nullptr && !sink)) return -1;
+  const AttnOpts opt{softcap, sink, static_cast<const float*>(sinks), static_cast<const float*>(slopes), keep,
+                     static_cast<const float*>(gate), ld_gate, out_scale, o_row};
   const int NC = nvh * Dv;
   // (16-byte loads of the staged tiles: rows and column blocks start on 16-byte borders)
   if (D % 8 || Dv % 8 || NC % 16 || NC > 16 * kTileMaxVT || D > 256 || k_ld % 8 || v_ld % 8) return -2;
@@ -1535,7 +1611,7 @@ LC_EXPORT int lc_attn_tile(const void* q, const void* kc, const void* vc, int ca
   attn_tile_kernel<C32, A32><<<grid, block, lds, st>>>(                                                         \
       static_cast<const float*>(q), kc, vc, static_cast<const int32_t*>(block_tables), MB,                      \
       static_cast<const int32_t*>(cu_q), static_cast<const int32_t*>(positions), out, H, G, D, Dv, BS, scale,   \
-      chunk, window, k_ld, v_ld, softcap, sink, vh0, nvh, o_ld, o_col0)
+      chunk, window, k_ld, v_ld, opt, vh0, nvh, o_ld, o_col0)
   if (cache_f32 && act_f32) LC_TILE(true, true);
   else if (cache_f32) LC_TILE(true, false);
   else if (act_f32) LC_TILE(false, true);

@@ -1,0 +1,484 @@
+// Kernels of hybrid decoder designs whose sublayers sit between two norms, gate their result from their own input and
+// read the previous token's input beside the current one: the residual step with the gate and both norms in one
+// launch, the token shift over per-sequence state, the attention pre-processing with short causal convolutions
+// (their last inputs are per-sequence state too), norms over the whole projection or per head, a rotation, a query
+// temperature, mixed values and the paged cache write, and the soft cap of the logits.
+//
+// A step's sequences are described by row_seq [T] (sequence of a row, < 0: padding), cu_q [B + 1] (row ranges),
+// positions [T] and slots [B] (state slot of the sequence, < 0: none). A sequence whose first row is at position 0
+// starts from zeros, so slots are never cleared. Rows of one launch run in any order: state that a launch both
+// reads and replaces is touched only by the block of the sequence's FIRST row, every number by one thread.
+#include "hybrid_common.h"
+
+namespace {
+
+// Where a row's sequence starts and which state it owns.
+struct RowSeq {
+  int first, rows;               // row range of the step
+  int slot;                      // < 0: none
+  bool fresh;                    // starts at position 0 (or has no state): zeros before it
+};
+
+LC_DEVICE RowSeq row_sequence(int t, const int32_t* __restrict__ row_seq, const int32_t* __restrict__ cu_q,
+                              const int32_t* __restrict__ positions, const int32_t* __restrict__ slots) {
+  RowSeq r{t, 1, -1, true};
+  const int b = row_seq[t];
+  if (b < 0) return r;
+  r.first = cu_q[b];
+  r.rows = cu_q[b + 1] - r.first;
+  r.slot = slots[b];
+  r.fresh = r.slot < 0 || positions[r.first] == 0;
+  return r;
+}
+
+// ---------------------------------------------------------------- residual step with a gate and two norms
+// With y [T, d]: v = y * sigmoid(gate) (gate given: logits, row stride ld_gate), then rms-normed times w_out (w_out
+// given), x += v. With w_in: h = x / sqrt(mean(x^2) + eps) * w_in, written to ``ha`` in the activation type and, when
+// given, to ``h32``. With ``mu`` (steps whose sequences all have ONE row): ``hs`` = h + (h' - h) * mu in the
+// activation type, h' the sequence's stored row (zeros at position 0), and h becomes the stored row.
+// A block per row. Rows of up to 4 * 256 * kStepVec coordinates whose pieces are 16-byte aligned (VEC) stay in registers
+// between the sums; others are read again.
+constexpr int kStepVec = 4;
+
+template <bool AF32>
+LC_DEVICE void store_act4(void* p, size_t i, const float4& v) {
+  if (AF32) {
+    *reinterpret_cast<float4*>(static_cast<float*>(p) + i) = v;
+  } else {
+    *reinterpret_cast<uint2*>(static_cast<bf16_t*>(p) + i) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
+  }
+}
+
+LC_DEVICE float4 shift4(const float4& h, const float4& p, const float4& m) {
+  return make_float4(h.x + (p.x - h.x) * m.x, h.y + (p.y - h.y) * m.y, h.z + (p.z - h.z) * m.z, h.w + (p.w - h.w) * m.w);
+}
+
+struct StepArgs {
+  float* x;
+  const float* y;
+  const float* gate;
+  int ld_gate;
+  const float* w_out;
+  const float* w_in;
+  float eps;
+  void* ha;
+  float* h32;
+  // the shift of single-row sequences
+  const float* mu;
+  float* state;
+  long long state_stride;
+  const int32_t* row_seq;
+  const int32_t* positions;
+  const int32_t* slots;
+  void* hs;
+  int d;
+};
+
+template <bool AF32, bool VEC>
+__global__ __launch_bounds__(256) void gated_step_kernel(StepArgs a) {
+  __shared__ float red[16];
+  const int t = blockIdx.x, d = a.d;
+  const size_t row = static_cast<size_t>(t) * d;
+  const float* grow = a.gate != nullptr ? a.gate + static_cast<size_t>(t) * a.ld_gate : nullptr;
+  float* prev = nullptr;                              // the sequence's stored row (null: none)
+  bool fresh = true;
+  if (a.mu != nullptr) {
+    const int b = a.row_seq[t];
+    const int slot = b < 0 ? -1 : a.slots[b];
+    if (slot >= 0) {
+      prev = a.state + static_cast<size_t>(slot) * a.state_stride;
+      fresh = a.positions[t] == 0;
+    }
+  }
+  if constexpr (VEC) {
+    const int n4 = d / 4;
+    float4 xv[kStepVec], yv[kStepVec];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < kStepVec; ++i) {
+      const int c = threadIdx.x + 256 * i;
+      xv[i] = yv[i] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (c < n4) {
+        xv[i] = reinterpret_cast<const float4*>(a.x + row)[c];
+        if (a.y != nullptr) {
+          float4 v = reinterpret_cast<const float4*>(a.y + row)[c];
+          if (grow != nullptr) {
+            const float4 g = reinterpret_cast<const float4*>(grow)[c];
+            v = make_float4(v.x * sigmoidf_(g.x), v.y * sigmoidf_(g.y), v.z * sigmoidf_(g.z), v.w * sigmoidf_(g.w));
+          }
+          ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+          yv[i] = v;
+        }
+      }
+    }
+    if (a.y != nullptr) {
+      const float r = a.w_out != nullptr ? 1.f / sqrtf(block_sum(ss, red) / static_cast<float>(d) + a.eps) : 1.f;
+#pragma unroll
+      for (int i = 0; i < kStepVec; ++i) {
+        const int c = threadIdx.x + 256 * i;
+        if (c < n4) {
+          float4 w = make_float4(1.f, 1.f, 1.f, 1.f);
+          if (a.w_out != nullptr) w = reinterpret_cast<const float4*>(a.w_out)[c];
+          xv[i].x += yv[i].x * r * w.x;
+          xv[i].y += yv[i].y * r * w.y;
+          xv[i].z += yv[i].z * r * w.z;
+          xv[i].w += yv[i].w * r * w.w;
+          reinterpret_cast<float4*>(a.x + row)[c] = xv[i];
+        }
+      }
+    }
+    if (a.w_in == nullptr) return;                    // the same for every thread
+    float s2 = 0.f;
+#pragma unroll
+    for (int i = 0; i < kStepVec; ++i) s2 += xv[i].x * xv[i].x + xv[i].y * xv[i].y + xv[i].z * xv[i].z + xv[i].w * xv[i].w;
+    const float r2 = 1.f / sqrtf(block_sum(s2, red) / static_cast<float>(d) + a.eps);
+#pragma unroll
+    for (int i = 0; i < kStepVec; ++i) {
+      const int c = threadIdx.x + 256 * i;
+      if (c < n4) {
+        const float4 w = reinterpret_cast<const float4*>(a.w_in)[c];
+        const float4 h = make_float4(xv[i].x * r2 * w.x, xv[i].y * r2 * w.y, xv[i].z * r2 * w.z, xv[i].w * r2 * w.w);
+        store_act4<AF32>(a.ha, row + 4 * c, h);
+        if (a.h32 != nullptr) reinterpret_cast<float4*>(a.h32 + row)[c] = h;
+        if (a.mu != nullptr) {
+          float4 p = make_float4(0.f, 0.f, 0.f, 0.f);
+          if (!fresh) p = reinterpret_cast<const float4*>(prev)[c];
+          store_act4<AF32>(a.hs, row + 4 * c, shift4(h, p, reinterpret_cast<const float4*>(a.mu)[c]));
+          if (prev != nullptr) reinterpret_cast<float4*>(prev)[c] = h;
+        }
+      }
+    }
+  } else {
+    typedef typename Act<AF32>::type act_t;
+    float r = 1.f;
+    auto result = [&](int c) { return grow != nullptr ? a.y[row + c] * sigmoidf_(grow[c]) : a.y[row + c]; };
+    if (a.y != nullptr && a.w_out != nullptr) {
+      float ss = 0.f;
+      for (int c = threadIdx.x; c < d; c += 256) {
+        const float v = result(c);
+        ss += v * v;
+      }
+      r = 1.f / sqrtf(block_sum(ss, red) / static_cast<float>(d) + a.eps);
+    }
+    float s2 = 0.f;
+    for (int c = threadIdx.x; c < d; c += 256) {
+      float v = a.x[row + c];
+      if (a.y != nullptr) {
+        v += result(c) * r * (a.w_out != nullptr ? a.w_out[c] : 1.f);
+        a.x[row + c] = v;
+      }
+      s2 += v * v;
+    }
+    if (a.w_in == nullptr) return;
+    const float r2 = 1.f / sqrtf(block_sum(s2, red) / static_cast<float>(d) + a.eps);
+    for (int c = threadIdx.x; c < d; c += 256) {      // (a thread reads what it wrote itself)
+      const float h = a.x[row + c] * r2 * a.w_in[c];
+      Act<AF32>::store(static_cast<act_t*>(a.ha), row + c, h);
+      if (a.h32 != nullptr) a.h32[row + c] = h;
+      if (a.mu != nullptr) {
+        const float p = fresh ? 0.f : prev[c];
+        Act<AF32>::store(static_cast<act_t*>(a.hs), row + c, h + (p - h) * a.mu[c]);
+        if (prev != nullptr) prev[c] = h;
+      }
+    }
+  }
+}
+
+// ---------------------------------------------------------------- token shift
+// hs[t] = h[t] + (h' - h[t]) * mu with h' the row before it in the sequence: row t - 1 of the step, or, for the first
+// row of a portion, the sequence's stored row (zeros at position 0). The block of the first row then stores the
+// portion's last row. One block per row, V = 4 coordinates per thread when the width allows.
+template <bool AF32, int V>
+__global__ __launch_bounds__(256) void token_shift_kernel(const float* __restrict__ h, const float* __restrict__ mu,
+                                                          float* __restrict__ state, long long state_stride,
+                                                          const int32_t* __restrict__ row_seq,
+                                                          const int32_t* __restrict__ cu_q,
+                                                          const int32_t* __restrict__ positions,
+                                                          const int32_t* __restrict__ slots, void* __restrict__ hs, int d) {
+  const int t = blockIdx.x;
+  const RowSeq s = row_sequence(t, row_seq, cu_q, positions, slots);
+  const bool first = t == s.first;
+  float* st = s.slot >= 0 ? state + static_cast<size_t>(s.slot) * state_stride : nullptr;
+  const size_t row = static_cast<size_t>(t) * d;
+  const float* last = h + static_cast<size_t>(s.first + s.rows - 1) * d;
+  typedef typename Act<AF32>::type act_t;
+  for (int c = threadIdx.x * V; c < d; c += 256 * V) {
+    if constexpr (V == 4) {
+      const float4 v = *reinterpret_cast<const float4*>(h + row + c);
+      float4 p = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (!first) p = *reinterpret_cast<const float4*>(h + row - d + c);
+      else if (!s.fresh) p = *reinterpret_cast<const float4*>(st + c);
+      store_act4<AF32>(hs, row + c, shift4(v, p, *reinterpret_cast<const float4*>(mu + c)));
+      if (first && st != nullptr) *reinterpret_cast<float4*>(st + c) = *reinterpret_cast<const float4*>(last + c);
+    } else {
+      const float v = h[row + c];
+      const float p = !first ? h[row - d + c] : (s.fresh ? 0.f : st[c]);
+      Act<AF32>::store(static_cast<act_t*>(hs), row + c, v + (p - v) * mu[c]);
+      if (first && st != nullptr) st[c] = last[c];
+    }
+  }
+}
+
+// ---------------------------------------------------------------- attention pre-processing
+// One block per token. qkv [T, ld] fp32: q [H*D] | k [G*D] | v [G*Dv] (C channels in all). In this order, each optional:
+//   a causal convolution over time per channel, conv_w [taps, C]: y_t = sum_j w[j] u_(t - taps + 1 + j); inputs before the
+//     step come from the sequence's state [taps - 1, C] (oldest first), zeros before the sequence's start. The block
+//     of a portion's first row also serves the next taps - 2 rows (they reach into the state as well) and then
+//     replaces the state by the portion's last taps - 1 inputs;
+//   norm 1: RMS over the whole query (key) projection, weights [H*D] / [G*D]; norm 2: per head, weights [D] shared;
+//   rotation of the first rot_dims coordinates of each q and k head (pairs: neighbours, otherwise i with
+//     i + rot_dims / 2) by position * inv_freq[i] (angles fp64);
+//   temperature: q *= 1 + coef * ln(floor((p + 1) / every) + 1);
+//   value mix: v <- (1 - lambda) v + lambda v_first[t]; before it v is written to v_save when given.
+// q goes to q_out [T, H*D] fp32, k and v to the paged planes [blocks, G, BS, D] / [blocks, G, BS, Dv].
+struct PrepArgs {
+  const float* qkv;
+  int ld;
+  const float* conv_w;
+  int taps;                       // 0: no convolution
+  float* state;
+  long long state_stride;
+  int norm;
+  const float* qn;
+  const float* kn;
+  float eps;
+  const double* inv_freq;
+  int rot_dims, pairs;
+  float t_coef;                   // 0: no temperature
+  double t_every;
+  const float* v_first;
+  int ld_vf;
+  float lambda;
+  float* v_save;
+  const int32_t* row_seq;
+  const int32_t* cu_q;
+  const int32_t* positions;
+  const int32_t* slots;
+  const int32_t* slot_mapping;
+  void* kc;
+  void* vc;
+  float* q_out;
+  int H, G, D, Dv, BS;
+};
+
+template <bool CF32>
+__global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs a) {
+  extern __shared__ float lds[];
+  __shared__ float red[16];
+  const int H = a.H, G = a.G, D = a.D, Dv = a.Dv;
+  const int nq = H * D, nk = G * D, nv = G * Dv, C = nq + nk + nv;
+  float* u = lds;                                    // [C] the token's channels
+  float* cs = u + C;                                 // [rot_dims] cos | sin
+  float* hr = cs + a.rot_dims;                       // [H + G] reciprocal norms per head
+  const int t0 = blockIdx.x;
+  const int hist = a.taps > 1 ? a.taps - 1 : 0;
+  RowSeq s{t0, 1, -1, true};
+  int count = 1;
+  if (hist > 0) {
+    s = row_sequence(t0, a.row_seq, a.cu_q, a.positions, a.slots);
+    const int r = t0 - s.first;
+    if (r > 0 && r < hist) return;                   // served by the portion's first row
+    if (r == 0) count = min(s.rows, hist);
+  }
+  float* st = s.slot >= 0 ? a.state + static_cast<size_t>(s.slot) * a.state_stride : nullptr;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int half = a.rot_dims >> 1;
+  for (int rr = 0; rr < count; ++rr) {
+    const int t = t0 + rr;
+    const int r = t - s.first;                       // row inside the portion
+    const int pos = a.positions[t];
+    const float* row = a.qkv + static_cast<size_t>(t) * a.ld;
+    if (a.taps > 0) {
+      for (int c = threadIdx.x; c < C; c += 256) {
+        float y = 0.f;
+        for (int j = 0; j < a.taps; ++j) {
+          const int k = r - hist + j;                // input row inside the portion, < 0: before it
+          float in = 0.f;
+          if (k >= 0) in = a.qkv[static_cast<size_t>(s.first + k) * a.ld + c];
+          else if (!s.fresh) in = st[static_cast<size_t>(k + hist) * C + c];
+          y += a.conv_w[static_cast<size_t>(j) * C + c] * in;
+        }
+        u[c] = y;
+      }
+    } else {
+      for (int c = threadIdx.x; c < C; c += 256) u[c] = row[c];
+    }
+    for (int j = threadIdx.x; j < half; j += 256) {
+      constexpr double kTwoPi = 6.283185307179586476925286766559;
+      double ang = static_cast<double>(pos) * a.inv_freq[j];
+      ang -= kTwoPi * rint(ang / kTwoPi);
+      float sn, cn;
+      sincosf(static_cast<float>(ang), &sn, &cn);
+      cs[j] = cn;
+      cs[half + j] = sn;
+    }
+    __syncthreads();
+    float temp = 1.f;
+    if (a.t_coef != 0.f) temp += a.t_coef * logf(static_cast<float>(floor((pos + 1.0) / a.t_every) + 1.0));
+    if (a.norm == 1) {
+      float sq = 0.f, sk = 0.f;
+      for (int i = threadIdx.x; i < nq; i += 256) sq += u[i] * u[i];
+      for (int i = threadIdx.x; i < nk; i += 256) sk += u[nq + i] * u[nq + i];
+      const float rq = 1.f / sqrtf(block_sum(sq, red) / static_cast<float>(nq) + a.eps);
+      const float rk = 1.f / sqrtf(block_sum(sk, red) / static_cast<float>(nk) + a.eps);
+      for (int i = threadIdx.x; i < nq; i += 256) u[i] *= rq * a.qn[i];
+      for (int i = threadIdx.x; i < nk; i += 256) u[nq + i] *= rk * a.kn[i];
+      __syncthreads();
+    } else if (a.norm == 2) {
+      for (int g = wave; g < H + G; g += 4) {        // q heads, then key heads, side by side
+        float ss = 0.f;
+        for (int i = lane; i < D; i += 64) ss += u[g * D + i] * u[g * D + i];
+        ss = wave_sum(ss);
+        if (lane == 0) hr[g] = 1.f / sqrtf(ss / static_cast<float>(D) + a.eps);
+      }
+      __syncthreads();
+      for (int i = threadIdx.x; i < nq + nk; i += 256) u[i] *= hr[i / D] * (i < nq ? a.qn[i % D] : a.kn[i % D]);
+      __syncthreads();
+    }
+    auto turned = [&](int at, int i) {               // coordinate i of the head at u[at]
+      const float v = u[at + i];
+      if (i >= a.rot_dims) return v;
+      if (a.pairs) {
+        const float c = cs[i >> 1], sn = cs[half + (i >> 1)], o = u[at + (i ^ 1)];
+        return (i & 1) ? v * c + o * sn : v * c - o * sn;
+      }
+      const int j = i < half ? i : i - half;
+      const float c = cs[j], sn = cs[half + j];
+      return i < half ? v * c - u[at + i + half] * sn : v * c + u[at + i - half] * sn;
+    };
+    for (int i = threadIdx.x; i < nq; i += 256) {
+      const int c = i % D;
+      a.q_out[static_cast<size_t>(t) * nq + i] = turned(i - c, c) * temp;
+    }
+    const int slot = a.slot_mapping[t];
+    const size_t blk = slot >= 0 ? slot / a.BS : 0, off = slot >= 0 ? slot % a.BS : 0;
+    typedef typename Act<CF32>::type cache_t;
+    if (slot >= 0)
+      for (int i = threadIdx.x; i < nk; i += 256) {
+        const int g = i / D, c = i - g * D;
+        Act<CF32>::store(static_cast<cache_t*>(a.kc), ((blk * G + g) * a.BS + off) * D + c, turned(nq + g * D, c));
+      }
+    for (int i = threadIdx.x; i < nv; i += 256) {
+      float v = u[nq + nk + i];
+      if (a.v_save != nullptr) a.v_save[static_cast<size_t>(t) * nv + i] = v;
+      if (a.v_first != nullptr) v = (1.f - a.lambda) * v + a.lambda * a.v_first[static_cast<size_t>(t) * a.ld_vf + i];
+      const int g = i / Dv, c = i - g * Dv;
+      if (slot >= 0) Act<CF32>::store(static_cast<cache_t*>(a.vc), ((blk * G + g) * a.BS + off) * Dv + c, v);
+    }
+    if (rr + 1 < count) __syncthreads();             // the next row reuses the buffers
+  }
+  if (hist > 0 && st != nullptr && t0 == s.first) {
+    // a thread owns a channel: it has read the old inputs above, and row j + rows is read before row j + 1 is written
+    for (int c = threadIdx.x; c < C; c += 256)
+      for (int j = 0; j < hist; ++j) {
+        const int k = s.rows - hist + j;
+        float in = 0.f;
+        if (k >= 0) in = a.qkv[static_cast<size_t>(s.first + k) * a.ld + c];
+        else if (!s.fresh) in = st[static_cast<size_t>(k + hist) * C + c];
+        st[static_cast<size_t>(j) * C + c] = in;
+      }
+  }
+}
+
+// ---------------------------------------------------------------- soft cap
+// x <- cap * tanh(x / cap), in place.
+__global__ void softcap_kernel(float* __restrict__ x, long long n, float cap) {
+  const long long i = static_cast<long long>(blockIdx.x) * blockDim.x + threadIdx.x;
+  if (i < n) x[i] = cap * tanhf(x[i] / cap);
+}
+
+bool aligned16(const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; }
+
+}  // namespace
+
+// ================================================================= launchers
+LC_EXPORT int lc_gated_step(void* x, const void* y, const void* gate, int ld_gate, const void* w_out, const void* w_in,
+                            float eps, void* ha, void* h32, int act_f32, const void* mu, void* state,
+                            long long state_stride, const void* row_seq, const void* positions, const void* slots, void* hs,
+                            int T, int d, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (d <= 0 || (y == nullptr && w_in == nullptr) || (w_in != nullptr && ha == nullptr)) return -1;
+  if (gate != nullptr && (y == nullptr || ld_gate < d)) return -1;
+  if (mu != nullptr && (w_in == nullptr || hs == nullptr || state == nullptr || row_seq == nullptr || positions == nullptr ||
+                        slots == nullptr || state_stride < d))
+    return -1;
+  const StepArgs a{static_cast<float*>(x), static_cast<const float*>(y), static_cast<const float*>(gate), ld_gate,
+                   static_cast<const float*>(w_out), static_cast<const float*>(w_in), eps, ha, static_cast<float*>(h32),
+                   static_cast<const float*>(mu), static_cast<float*>(state), state_stride,
+                   static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(positions),
+                   static_cast<const int32_t*>(slots), hs, d};
+  const bool vec = d % 4 == 0 && d <= 4 * 256 * kStepVec && ld_gate % 4 == 0 && state_stride % 4 == 0 && aligned16(x) &&
+                   aligned16(y) && aligned16(gate) && aligned16(w_out) && aligned16(w_in) && aligned16(ha) &&
+                   aligned16(h32) && aligned16(mu) && aligned16(state) && aligned16(hs);
+#define LC_GS(A32, V) gated_step_kernel<A32, V><<<dim3(T), dim3(256), 0, st>>>(a)
+  if (act_f32 && vec) LC_GS(true, true);
+  else if (act_f32) LC_GS(true, false);
+  else if (vec) LC_GS(false, true);
+  else LC_GS(false, false);
+#undef LC_GS
+  LC_RETURN_LAST_ERROR();
+}
+
+LC_EXPORT int lc_token_shift(const void* h, const void* mu, void* state, long long state_stride, const void* row_seq,
+                             const void* cu_q, const void* positions, const void* slots, void* hs, int act_f32, int T, int d,
+                             hipStream_t st) {
+  if (T <= 0) return 0;
+  if (d <= 0 || state_stride < d || h == nullptr || mu == nullptr || state == nullptr || slots == nullptr) return -1;
+  const bool vec = d % 4 == 0 && state_stride % 4 == 0 && aligned16(h) && aligned16(mu) && aligned16(state) && aligned16(hs);
+#define LC_TS(A32, V)                                                                                              \
+  token_shift_kernel<A32, V><<<dim3(T), dim3(256), 0, st>>>(                                                       \
+      static_cast<const float*>(h), static_cast<const float*>(mu), static_cast<float*>(state), state_stride,       \
+      static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(cu_q), static_cast<const int32_t*>(positions), \
+      static_cast<const int32_t*>(slots), hs, d)
+  if (act_f32 && vec) LC_TS(true, 4);
+  else if (act_f32) LC_TS(true, 1);
+  else if (vec) LC_TS(false, 4);
+  else LC_TS(false, 1);
+#undef LC_TS
+  LC_RETURN_LAST_ERROR();
+}
+
+LC_EXPORT int lc_attn_prep(const void* qkv, int ld, const void* conv_w, int taps, void* state, long long state_stride,
+                           int norm, const void* qn, const void* kn, float eps, const void* inv_freq, int rot_dims, int pairs,
+                           float t_coef, float t_every, const void* v_first, int ld_vf, float lambda, void* v_save,
+                           const void* row_seq, const void* cu_q, const void* positions, const void* slots,
+                           const void* slot_mapping, void* kc, void* vc, int cache_f32, void* q_out, int T, int H, int G,
+                           int D, int Dv, int BS, hipStream_t st) {
+  if (T <= 0) return 0;
+  if (H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || BS <= 0 || kc == nullptr || vc == nullptr || q_out == nullptr) return -1;
+  const int C = (H + G) * D + G * Dv;
+  if (ld < C || taps < 0 || norm < 0 || norm > 2 || (norm != 0 && (qn == nullptr || kn == nullptr))) return -1;
+  if (taps > 0 && conv_w == nullptr) return -1;
+  if (taps > 1 && (state == nullptr || state_stride < static_cast<long long>(taps - 1) * C || row_seq == nullptr ||
+                   cu_q == nullptr || slots == nullptr))
+    return -1;
+  if (rot_dims < 0 || rot_dims > D || (rot_dims & 1) || (rot_dims > 0 && inv_freq == nullptr)) return -1;
+  if ((t_coef != 0.f && !(t_every > 0.f)) || (v_first != nullptr && ld_vf < G * Dv)) return -1;
+  constexpr size_t kMaxLds = 159 * 1024;             // (the block sums' scratch is static)
+  const size_t lds = static_cast<size_t>(C + rot_dims + H + G) * sizeof(float);
+  if (lds > kMaxLds) return -2;
+  static LcDeviceOnce attr_once;
+  attr_once.run([&] {
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_prep_kernel<true>),
+                              hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(kMaxLds));
+    (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_prep_kernel<false>),
+                              hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(kMaxLds));
+  });
+  const PrepArgs a{static_cast<const float*>(qkv), ld, static_cast<const float*>(conv_w), taps, static_cast<float*>(state),
+                   state_stride, norm, static_cast<const float*>(qn), static_cast<const float*>(kn), eps,
+                   static_cast<const double*>(inv_freq), rot_dims, pairs, t_coef, static_cast<double>(t_every),
+                   static_cast<const float*>(v_first), ld_vf, lambda, static_cast<float*>(v_save),
+                   static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(cu_q),
+                   static_cast<const int32_t*>(positions), static_cast<const int32_t*>(slots),
+                   static_cast<const int32_t*>(slot_mapping), kc, vc, static_cast<float*>(q_out), H, G, D, Dv, BS};
+  if (cache_f32) attn_prep_kernel<true><<<dim3(T), dim3(256), lds, st>>>(a);
+  else attn_prep_kernel<false><<<dim3(T), dim3(256), lds, st>>>(a);
+  LC_RETURN_LAST_ERROR();
+}
+
+LC_EXPORT int lc_softcap(void* x, long long n, float cap, hipStream_t st) {
+  if (n <= 0) return 0;
+  if (!(cap > 0.f)) return -1;
+  softcap_kernel<<<dim3(static_cast<unsigned>((n + 255) / 256)), dim3(256), 0, st>>>(static_cast<float*>(x), n, cap);
+  LC_RETURN_LAST_ERROR();
+}

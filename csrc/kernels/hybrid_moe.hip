@@ -1,4 +1,4 @@
-// Routed feed-forwards of hybrid decoder designs: a softmax or sigmoid router with a bias-corrected,
+// Routed feed-forwards of hybrid decoder designs: a softmax or sigmoid router (or a softmax over the chosen logits) with a bias-corrected,
 // group-limited top-k choice, a counting sort of the (token, choice) pairs by expert for any number
 // of experts, per-expert products of any shape and type over the sorted rows (fp32 accumulation on
 // the vector ALUs, like the shape-agnostic GEMM), and the fp32 mix of the chosen experts' outputs,
@@ -12,7 +12,8 @@ constexpr int kMaxGroups = 64;
 
 // ---------------------------------------------------------------- routing
 // One wave per token. z [T, n] fp32 router logits (row stride ld). s = softmax(z) (score_fn 0) or sigmoid(z), each
-// output on its own (score_fn 1); choice = s + correction (no correction given: s); the n
+// output on its own (score_fn 1); score_fn 2: the choice goes by the logits and the weights are the softmax over the
+// chosen logits only; choice = s + correction (no correction given: s); the n
 // outputs form ``groups`` runs of n / groups neighbours, a run's score is its largest choice, the
 // ``keep`` best runs stay eligible (ties: the lower index); the ``top`` largest eligible choices are
 // taken (ties: the lower index) with weights s * scale.
@@ -32,6 +33,8 @@ __global__ __launch_bounds__(256) void route_grouped_kernel(const float* __restr
   float inv = 1.f;
   if (score_fn == 1) {
     for (int e = lane; e < n; e += 64) sc[e] = sigmoidf_(zr[e]);
+  } else if (score_fn == 2) {
+    for (int e = lane; e < n; e += 64) sc[e] = zr[e];
   } else {
     float mx = -INFINITY;
     for (int e = lane; e < n; e += 64) mx = fmaxf(mx, zr[e]);
@@ -78,6 +81,7 @@ __global__ __launch_bounds__(256) void route_grouped_kernel(const float* __restr
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   }
+  float first = 0.f, sum_top = 0.f;                 // score_fn 2: the largest chosen logit, the sum of the exponentials
   for (int k = 0; k < top; ++k) {
     float best = -INFINITY;
     int at = 0x7fffffff;
@@ -100,13 +104,21 @@ __global__ __launch_bounds__(256) void route_grouped_kernel(const float* __restr
     if (at >= n) at = k < n ? k : 0;                // nothing eligible is left (NaN logits): still a valid expert
     if (lane == 0) {
       ids[static_cast<size_t>(t) * top + k] = at;
-      wts[static_cast<size_t>(t) * top + k] = sc[at] * scale;
+      float wv = sc[at] * scale;
+      if (score_fn == 2) {
+        if (k == 0) first = sc[at];
+        wv = expf(sc[at] - first);
+        sum_top += wv;
+      }
+      wts[static_cast<size_t>(t) * top + k] = wv;
       ch[at] = -INFINITY;
     }
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   }
+  if (score_fn == 2 && lane == 0)                   // (the lane that wrote them)
+    for (int k = 0; k < top; ++k) wts[static_cast<size_t>(t) * top + k] *= scale / sum_top;
 }
 
 // ---------------------------------------------------------------- sort of the pairs by expert
@@ -261,7 +273,7 @@ LC_EXPORT int lc_route_grouped(const void* z, int ld, const void* corr, int T, i
   if (T <= 0) return 0;
   if (ld < n) return -1;
   if (n <= 0 || top <= 0 || top > kMaxTop || top > n || groups <= 0 || groups > kMaxGroups || n % groups || keep < 1 ||
-      keep > groups || top > keep * (n / groups) || score_fn < 0 || score_fn > 1)
+      keep > groups || top > keep * (n / groups) || score_fn < 0 || score_fn > 2)
     return -1;
   const size_t lds = 4 * static_cast<size_t>(2 * n + 2 * kMaxGroups) * sizeof(float);
   if (lds > 64 * 1024) return -1;

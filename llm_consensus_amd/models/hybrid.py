@@ -1,10 +1,31 @@
 """Hybrid decoders: a stack whose layers each pick one mixer -- chunk-masked attention over the
-paged cache, latent attention over a cache of compressed rows, minGRU, gated linear attention or
-mLSTM -- around an fp32 residual stream.
+paged cache, latent attention over a cache of compressed rows, minGRU, gated linear attention,
+mLSTM, or attention beside linear attention -- around an fp32 residual stream.
 
-Four designs are served, told apart by ``architecture`` in ``config.json`` (``DESIGNS``); the file lists
+Five designs are served, told apart by ``architecture`` in ``config.json`` (``DESIGNS``); the file lists
 the layers (``layers[i].type``, ``.mixer`` sizes, ``.mlp``), and every size and constant comes from
 there or from a tensor's shape.
+
+Kulivik (every sublayer between two norms, gated, reading the previous token beside the current one):
+
+* ``x = embed[token]``; a layer computes ``h = n1(x)``, ``x += n1b(sigmoid(R1 h + b1) * mixer(h~))`` and, if it has a
+  feed-forward, ``h = n2(x)``, ``x += n2b(sigmoid(R2 h + b2) * ff(h))`` with ``n(x) = x / sqrt(mean(x^2) + eps) * (1 + w)``.
+  ``h~_t = h_t + (h_(t-1) - h_t) * mu`` coordinate by coordinate (zeros before the first token): the previous row is
+  per-sequence state of every layer. Logits: ``cap * tanh(logit_scale * embed . n_final(x) / cap)``;
+* ``attention``: a short causal convolution over time on every channel of q, k and v (its last inputs are state too), RMS
+  norms over the whole query and key projections, no positions, all earlier keys, a learned sink score per head in the
+  softmax's denominator, a gate ``sigmoid(W_g h~)_h`` per head on its result;
+* ``attention_2``: biased projections, RMS norms per head, neighbouring pairs of the first ``rot.dims`` coordinates turn,
+  scores capped, a window of ``mask.size`` positions beside which the first ``mask.keep_first`` keys stay visible;
+* either kind with ``v_mix``: the first such layer's values of the same token are mixed into the layer's own before they
+  are cached, ``v <- (1 - l) v + l v_first``;
+* ``parallel``: two mixers on the same input, ``left_scale * left + right_scale * right``. Left: attention whose queries
+  grow with the position, ``q * (1 + coef ln(floor((p + 1) / every) + 1))``, and whose scores lose
+  ``2^(-8 (h + 1) / H) * (i - j)``. Right: linear attention with one constant decay per head, ``S <- a_h S + k v^T``,
+  ``o = S^T q`` with q, k, v = silu of the projections, an RMS norm over all heads together, a gate ``sigmoid(W_g h~)``.
+  Both results share one output product ``[W_left | W_right]``;
+* feed-forwards: the clamped gated unit (``g * sigmoid(1.702 g) * (u + 1)``), or a routed mixture of silu-gated experts
+  whose ``top`` largest (biased) router logits are chosen and weighted by the softmax over the chosen ones.
 
 Gizilorn (pre-norm, a residual of several parallel streams):
 
@@ -86,6 +107,7 @@ the step, prompt portions and single decoded tokens alike).
 from __future__ import annotations
 
 import json
+import math
 import zlib
 from dataclasses import dataclass, field
 from pathlib import Path
@@ -116,13 +138,17 @@ class Design:
                                     # biases or norms, values = the un-rotated keys, neighbouring pairs, ``mask.size`` = window)
                                     # | "talking" (biased q / k / v, rotate-half pairs on q and k, values turned by their own
                                     # position, capped scores, ``mask.size`` = window, a sink in the softmax, the heads'
-                                    # weights mixed by a matrix)
+                                    # weights mixed by a matrix) | "convolved" (a convolution over time on q / k / v,
+                                    # whole-projection norms, no positions, a learned sink and a gate per head)
     latent: str = "plain"           # latent attention: "plain" (no positions, all earlier rows, a gate per head) | "rotary" (a
                                     # turned key part shared by all heads beside the compressed row, a window, a gate per
                                     # output coordinate, ``kv_from``)
     embed_norm: bool = False        # an RMS norm (tensor ``embed.norm``) on the embedding rows
     hyper: bool = False             # the residual is ``streams`` parallel streams (tensors ``<layer>.hc<q>.{in,out,mix}``)
-    routed_ff: str = "grouped_relu2"    # "sigmoid_clamped": sigmoid scores, weight on the expert's input, clamped gated experts | "": none
+    routed_ff: str = "grouped_relu2"    # "sigmoid_clamped": sigmoid scores, weight on the expert's input, clamped gated experts |
+                                    # "top_silu": biased logits, softmax over the chosen ones, silu-gated experts | "": none
+    sandwich: bool = False          # norms on the sublayers' inputs AND results, results gated from the input, the mixer's input
+                                    # shifted towards the previous token's (tensors norm<q>, norm<q>b, rg<q>, rg<q>.b, shift)
     # constants of the clamped gated unit g * sigmoid(slope g) * (u + shift)
     glu_slope: float = 1.702
     glu_shift: float = 1.0
@@ -134,6 +160,8 @@ DESIGNS: Dict[str, Design] = {
                       dense_ff="glu_relu"),
     "Surevik": Design("Surevik", ("attention",), pre_norm=True, dense_ff="", norm="dyt", tied_head=True,
                       attention="keys_as_values", routed_ff="sigmoid_clamped"),
+    "Kulivik": Design("Kulivik", ("parallel", "attention", "attention_2"), pre_norm=True, norm_offset=1.0, sandwich=True,
+                      dense_ff="clamped_glu", tied_head=True, attention="convolved", routed_ff="top_silu"),
     "Gizilorn": Design("Gizilorn", ("attention", "latent_attention"), pre_norm=True, dense_ff="xielu", attention="talking",
                        latent="rotary", embed_norm=True, hyper=True, routed_ff=""),
 }
@@ -149,7 +177,10 @@ class MoESpec:
 
     ``unit`` "clamped_glu" (with ``score`` "sigmoid"): experts are down(g * sigmoid(slope g) * (u + shift)) with
     g = min(gate x, limit), u = clamp(up x, -limit, limit); the weight multiplies the expert's input; the
-    shared expert has a limit of its own and a sigmoid gate, one number per token."""
+    shared expert has a limit of its own and a sigmoid gate, one number per token.
+
+    ``unit`` "silu_glu" (with ``score`` "softmax_top"): experts are down(silu(gate x) * up x); the router has a bias, and
+    the chosen experts are weighted by the softmax over their logits."""
 
     experts: int
     ff: int
@@ -167,6 +198,10 @@ class MoESpec:
     @property
     def clamped(self) -> bool:
         return self.unit == "clamped_glu"
+
+    @property
+    def gated(self) -> bool:
+        return self.unit in ("clamped_glu", "silu_glu")
 
     @property
     def outputs(self) -> int:
@@ -206,13 +241,45 @@ class LayerSpec:
     gate_full: bool = False
     # mlstm: soft cap of the gate logits (0: none)
     gate_cap: float = 0.0
-    # feed-forward (0: none); ``moe``: a routed one instead of the dense one
+    # attention whose q / k / v go through the general pre-processing (ops.attn_prep): convolution taps (0: none), norm kind
+    # ("" | "whole" projection | per "head"), neighbouring rotary pairs, biases, values mixed with the first mixing
+    # layer's, query temperature (coef, every), first keys visible outside the window, a learned sink and a gate per
+    # head, a bias per unit of distance, a scale on the result; ``right``: linear attention beside it
+    prepped: bool = False
+    conv: int = 0
+    qk_norm: str = ""
+    rot_pairs: bool = False
+    biases: bool = False
+    v_mix: bool = False
+    q_temp: Tuple[float, float] = (0.0, 1.0)
+    keep_first: int = 0
+    head_sink: bool = False
+    head_gate: bool = False
+    distance_bias: bool = False
+    out_scale: float = 1.0
+    right: Optional["LayerSpec"] = None
+    # linear attention with one constant decay per head
+    decay: Tuple[float, ...] = ()
+    # width of the previous input row kept per sequence (token shift; 0: none)
+    shift: int = 0
+    # feed-forward (0: none) with the limit of a clamped unit; ``moe``: a routed one instead of the dense one
     ff: int = 0
+    ff_limit: float = 0.0
     moe: Optional[MoESpec] = None
 
     @property
+    def attends(self) -> bool:
+        """Attention over keys / values of its own width (anything but latent attention)."""
+        return self.type in ("attention", "attention_2", "parallel")
+
+    @property
     def owns_kv(self) -> bool:
-        return self.type == "attention" and self.kv_from < 0
+        return self.attends and self.kv_from < 0
+
+    @property
+    def channels(self) -> int:
+        """Width of q | k | v."""
+        return (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
 
     @property
     def owns_latent(self) -> bool:
@@ -222,8 +289,25 @@ class LayerSpec:
     def has_ff(self) -> bool:
         return self.ff > 0 or self.moe is not None
 
+    def state_parts(self) -> Dict[str, Tuple[int, int]]:
+        """(first column, numbers) of what a layer with several kinds of state keeps: the previous input row, the
+        convolution's last inputs, the linear attention's memory. Every part starts on a 16-byte border."""
+        sizes = {"shift": self.shift, "conv": max(0, self.conv - 1) * self.channels,
+                 "memory": self.right.state_size() if self.right is not None else 0}
+        out, at = {}, 0
+        for name, n in sizes.items():
+            if n:
+                out[name] = (at, n)
+                at += (n + 3) // 4 * 4
+        return out
+
     def state_size(self) -> int:
         """fp32 numbers of recurrent state per sequence."""
+        if self.prepped:
+            parts = list(self.state_parts().values())
+            return (parts[-1][0] + parts[-1][1] + 3) // 4 * 4 if parts else 0
+        if self.type == "lightning":
+            return self.heads * self.dim * self.vdim
         if self.type == "mingru":
             return self.width
         if self.type == "gla":
@@ -256,6 +340,7 @@ class HybridConfig:
     residual_mult: float = 1.0      # every sublayer output is scaled by this before it joins the stream
     loop: Tuple[int, int, int] = (0, 0, 1)      # layers [start, stop) run ``times`` times in a row (times 1: no loop)
     streams: int = 0                # parallel residual streams (designs with hyper-connections)
+    logit_softcap: float = 0.0      # > 0: logits become cap * tanh(logits / cap)
 
     @property
     def design(self) -> Design:
@@ -287,11 +372,11 @@ class HybridConfig:
 
     @property
     def num_heads(self) -> int:
-        return max([l.heads for l in self.layers if l.type in ("attention", "latent_attention")] or [1])
+        return max([l.heads for l in self.layers if l.attends or l.type == "latent_attention"] or [1])
 
     @property
     def num_kv_heads(self) -> int:
-        return max([l.kv_heads for l in self.layers if l.type == "attention"] or [1])
+        return max([l.kv_heads for l in self.layers if l.attends] or [1])
 
     def kv_elems_per_token(self) -> int:
         return sum(self.layers[i].cache_elems() for i, _ in self.runs)
@@ -324,6 +409,11 @@ class HybridConfig:
             raise ValueError(f"{self.name}: a sinusoidal position vector needs an even width")
         if self.design.hyper and (not 1 <= self.streams <= ops.MAX_STREAMS or self.looped):
             raise ValueError(f"{self.name}: 1..{ops.MAX_STREAMS} residual streams are needed, and no loop")
+        if self.logit_softcap < 0:
+            raise ValueError(f"{self.name}: the logits' cap is positive, or 0 for none")
+        mixing = [l for l in self.layers if l.v_mix]
+        if any(l.kv_heads * l.vdim != mixing[0].kv_heads * mixing[0].vdim for l in mixing):
+            raise ValueError(f"{self.name}: layers that mix values have one value width (kv_heads * vdim)")
         for i, l in enumerate(self.layers):
             if l.type not in known:
                 raise ValueError(f"{self.name}: layer {i}: unknown mixer {l.type!r} (known: {', '.join(known)})")
@@ -344,6 +434,8 @@ class HybridConfig:
                 raise ValueError(f"{self.name}: layer {i}: mLSTM takes dim <= 256 and a gate cap >= 0")
             if l.moe is not None:
                 m = l.moe
+                if m.unit == "silu_glu" and (m.score != "softmax_top" or m.identity or m.groups != 1 or m.shared_ff):
+                    raise ValueError(f"{self.name}: layer {i}: silu-gated experts are weighted by the softmax over the chosen logits")
                 if m.clamped and (m.score != "sigmoid" or m.identity or not m.limit > 0 or (m.shared_ff and not m.shared_limit > 0)):
                     raise ValueError(f"{self.name}: layer {i}: clamped gated experts take sigmoid scores, positive limits "
                                      f"and no identity experts")
@@ -354,16 +446,25 @@ class HybridConfig:
                     raise ValueError(f"{self.name}: layer {i}: the kept groups must hold `top` (at most 32) router outputs")
             if l.type == "mingru" and l.width <= 0:
                 raise ValueError(f"{self.name}: layer {i}: minGRU needs a width")
-            if l.type in ("attention", "gla") and (l.heads <= 0 or l.dim <= 0 or l.vdim <= 0):
+            if l.right is not None:
+                g = l.right
+                if g.heads <= 0 or g.dim <= 0 or g.dim > 256 or g.vdim <= 0 or len(g.decay) != g.heads:
+                    raise ValueError(f"{self.name}: layer {i}: linear attention takes heads, dim <= 256, vdim and a decay per head")
+            if l.prepped and (l.keep_first < 0 or l.window < 0 or l.softcap < 0 or l.conv < 0 or not l.q_temp[1] > 0):
+                raise ValueError(f"{self.name}: layer {i}: window, kept keys, cap and taps are not negative, q_temp.every is positive")
+            if l.prepped and (l.vdim > 512 or l.channels + l.rot_dims + l.heads + l.kv_heads > ops.ATTN_PREP_MAX_FLOATS):
+                raise ValueError(f"{self.name}: layer {i}: the kernels take vdim <= 512 and q | k | v of at most "
+                                 f"{ops.ATTN_PREP_MAX_FLOATS} channels")
+            if (l.attends or l.type == "gla") and (l.heads <= 0 or l.dim <= 0 or l.vdim <= 0):
                 raise ValueError(f"{self.name}: layer {i}: heads, dim and vdim are needed")
             if l.type == "gla" and (l.dim > 256 or not l.tau > 0):
                 raise ValueError(f"{self.name}: layer {i}: gated linear attention takes dim <= 256 and tau > 0")
-            if l.type == "attention":
+            if l.attends:
                 if l.kv_heads <= 0 or l.heads % l.kv_heads:
                     raise ValueError(f"{self.name}: layer {i}: heads must be a multiple of kv_heads")
                 if l.rot_dims % 2 or l.rot_dims > l.dim:
                     raise ValueError(f"{self.name}: layer {i}: rot.dims must be even and at most dim")
-                if l.vdim > 256:
+                if l.vdim > 256 and not l.prepped:
                     raise ValueError(f"{self.name}: layer {i}: the attention kernel takes vdim <= 256")
                 if l.talk and (l.kv_from >= 0 or l.chunk or l.softcap < 0 or l.window < 0 or (l.rotate_values and l.vdim % 2)):
                     raise ValueError(f"{self.name}: layer {i}: mixed heads take keys of their own, a cap >= 0, and values "
@@ -386,6 +487,42 @@ def _numel(shape) -> int:
     return n
 
 
+def _prepped_of(name: str, i: int, t: str, m: dict, width: int, ff: int, limit: float, moe: Optional[MoESpec]) -> LayerSpec:
+    """A Kulivik layer: its attention (the left half of a ``parallel`` mixer) with what stands beside it."""
+    a = m["left"] if t == "parallel" else m
+    mask, rot, temp = a.get("mask") or {}, a.get("rot") or {}, a.get("q_temp") or {}
+    kw = dict(heads=int(a["heads"]), kv_heads=int(a.get("kv_heads", a["heads"])), dim=int(a["dim"]), vdim=int(a.get("vdim", a["dim"])),
+              scale=float(a.get("scale", int(a["dim"]) ** -0.5)), v_mix=bool(a.get("v_mix", False)), prepped=True, shift=width,
+              ff=ff, ff_limit=limit, moe=moe)
+    if t == "attention":
+        return LayerSpec(t, conv=int(a.get("conv", 0)), qk_norm="whole", head_sink=True, head_gate=True, **kw)
+    if t == "attention_2":
+        return LayerSpec(t, biases=True, qk_norm="head", rot_dims=int(rot.get("dims", 0)), rot_pairs=True,
+                         rot_base=float(rot.get("base", 10000.0)), softcap=float(a.get("softcap") or 0.0),
+                         window=int(mask.get("size", 0)), keep_first=int(mask.get("keep_first", 0)), **kw)
+    r = m["right"]
+    right = LayerSpec("lightning", heads=int(r["heads"]), dim=int(r["dim"]), vdim=int(r.get("vdim", r["dim"])),
+                      decay=tuple(float(x) for x in r["decay"]), out_scale=float(m.get("right_scale", 1.0)))
+    return LayerSpec(t, q_temp=(float(temp.get("coef", 0.0)), float(temp.get("every", 1.0))), distance_bias=True,
+                     out_scale=float(m.get("left_scale", 1.0)), right=right, **kw)
+
+
+def _prepped_to_dict(l: LayerSpec) -> dict:
+    a = {"heads": l.heads, "kv_heads": l.kv_heads, "dim": l.dim, "vdim": l.vdim, "scale": l.scale}
+    if l.type == "parallel":
+        g = l.right
+        if l.q_temp[0]:
+            a["q_temp"] = {"coef": l.q_temp[0], "every": l.q_temp[1]}
+        return {"left": a, "left_scale": l.out_scale, "right_scale": g.out_scale,
+                "right": {"heads": g.heads, "dim": g.dim, "vdim": g.vdim, "decay": list(g.decay)}}
+    if l.v_mix:
+        a["v_mix"] = True
+    if l.type == "attention":
+        return {**a, "conv": l.conv}
+    return {**a, "softcap": l.softcap, "mask": {"size": l.window, "keep_first": l.keep_first},
+            "rot": {"dims": l.rot_dims, "base": l.rot_base}}
+
+
 def _mlp_of(name: str, i: int, mlp: Optional[dict], design: Design):
     """(ff, MoESpec or None) of a layer's ``mlp`` entry."""
     if mlp is None:
@@ -399,6 +536,9 @@ def _mlp_of(name: str, i: int, mlp: Optional[dict], design: Design):
         raise ValueError(f"{name}: layer {i}: feed-forward kind {kind!r} is not supported")
     r, g = mlp["router"], mlp["router"].get("groups") or {}
     shared = mlp.get("shared") or {}
+    if design.routed_ff == "top_silu":
+        return 0, MoESpec(experts=int(r["experts"]), ff=int(mlp["expert"]["ff"]), top=int(r["top"]), score="softmax_top",
+                          unit="silu_glu")
     if design.routed_ff == "sigmoid_clamped":
         return 0, MoESpec(experts=int(r["experts"]), ff=int(mlp["expert"]["ff"]), top=int(r["top"]),
                           shared_ff=int(shared.get("ff", 0)), score="sigmoid", unit="clamped_glu",
@@ -427,7 +567,10 @@ def config_from_dict(c: dict, name: str = "hybrid", tensor_shapes: Optional[Dict
         if t not in design.mixers:
             raise ValueError(f"{name}: layer {i}: unknown mixer {t!r} (known: {', '.join(design.mixers)})")
         ff, moe = _mlp_of(name, i, L.get("mlp"), design)
-        if t == "attention" and design.attention == "keys_as_values":
+        if design.sandwich:
+            limit = float((L.get("mlp") or {}).get("limit", math.inf)) if ff else 0.0
+            layers.append(_prepped_of(name, i, t, m, int(c["width"]), ff, limit, moe))
+        elif t == "attention" and design.attention == "keys_as_values":
             mask, rot = m.get("mask") or {}, m.get("rot") or {}
             layers.append(LayerSpec(t, heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])),
                                     dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])), scale=float(m["scale"]),
@@ -478,7 +621,8 @@ def config_from_dict(c: dict, name: str = "hybrid", tensor_shapes: Optional[Dict
                        max_position=int(c.get("max_position", 1 << 20)), model_type=arch.lower(), architecture=arch,
                        embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)),
                        logit_scale=float(c.get("logit_scale", 1.0)), residual_mult=float(c.get("residual_mult", 1.0)),
-                       loop=_loop_of(c.get("loop")), streams=int(c.get("streams", 1)) if design.hyper else 0)
+                       loop=_loop_of(c.get("loop")), streams=int(c.get("streams", 1)) if design.hyper else 0,
+                       logit_softcap=float(c.get("logit_softcap") or 0.0))
     cfg.validate()
     return cfg
 
@@ -486,7 +630,9 @@ def config_from_dict(c: dict, name: str = "hybrid", tensor_shapes: Optional[Dict
 def config_to_dict(cfg: HybridConfig) -> dict:
     layers = []
     for l in cfg.layers:
-        if l.type == "attention" and l.values_are_keys:
+        if l.prepped:
+            m = _prepped_to_dict(l)
+        elif l.type == "attention" and l.values_are_keys:
             m = {"heads": l.heads, "kv_heads": l.kv_heads, "dim": l.dim, "vdim": l.vdim, "scale": l.scale,
                  "mask": {"size": l.window}, "rot": {"dims": l.rot_dims, "base": l.rot_base}}
         elif l.type == "attention" and l.talk:
@@ -512,10 +658,15 @@ def config_to_dict(cfg: HybridConfig) -> dict:
         else:
             m = {"heads": l.heads, "dim": l.dim, "vdim": l.vdim, "gate_cap": l.gate_cap}
         mlp = {"kind": "dense", "ff": l.ff} if l.ff else None
+        if l.ff and cfg.design.dense_ff == "clamped_glu":
+            mlp["limit"] = l.ff_limit
         if l.moe is not None and l.moe.clamped:
             e = l.moe
             mlp = {"kind": "moe", "expert": {"ff": e.ff, "limit": e.limit}, "router": {"experts": e.experts, "top": e.top},
                    "shared": {"ff": e.shared_ff, "limit": e.shared_limit} if e.shared_ff else None}
+        elif l.moe is not None and l.moe.gated:
+            e = l.moe
+            mlp = {"kind": "moe", "expert": {"ff": e.ff}, "router": {"experts": e.experts, "top": e.top}}
         elif l.moe is not None:
             e = l.moe
             mlp = {"kind": "moe", "expert": {"ff": e.ff},
@@ -527,6 +678,11 @@ def config_to_dict(cfg: HybridConfig) -> dict:
            "norm": {"eps": cfg.rms_eps}, "layers": layers}
     if cfg.design.hyper:
         out["streams"] = cfg.streams
+        return out
+    if cfg.design.sandwich:
+        out["logit_scale"] = cfg.logit_scale
+        if cfg.logit_softcap:
+            out["logit_softcap"] = cfg.logit_softcap
         return out
     if cfg.design.pre_norm:
         out["embedding"] = {"scale": cfg.embed_scale}
@@ -573,11 +729,41 @@ def param_shapes(cfg: HybridConfig) -> Dict[str, tuple]:
         norm_tensors(p + "norm1")
         if l.has_ff:
             norm_tensors(p + "norm2")
+        if cfg.design.sandwich:
+            out[p + "shift"] = (d,)
+            for q in ("1", "2") if l.has_ff else ("1",):
+                norm_tensors(p + f"norm{q}b")
+                out[p + "rg" + q], out[p + f"rg{q}.b"] = (d, d), (d,)
         if cfg.design.hyper:
             for q in ("hc1.", "hc2.") if l.has_ff else ("hc1.",):
                 out[p + q + "in"], out[p + q + "out"], out[p + q + "mix"] = (cfg.streams,), (cfg.streams,), (cfg.streams, cfg.streams)
         m = p + "mix."
-        if l.type == "attention" and l.talk:
+        if l.prepped:
+            x = m + "left." if l.right is not None else m
+            rows = {"q": l.heads * l.dim, "k": l.kv_heads * l.dim, "v": l.kv_heads * l.vdim}
+            for n, k in rows.items():
+                out[x + n] = (k, d)
+                if l.biases:
+                    out[x + n + ".b"] = (k,)
+                if l.conv:
+                    out[x + n + ".conv"] = (k, l.conv)
+                if l.qk_norm and n != "v":
+                    out[x + n + ".norm"] = (k if l.qk_norm == "whole" else l.dim,)
+            out[x + "o"] = (d, l.heads * l.vdim)
+            if l.biases:
+                out[x + "o.b"] = (d,)
+            if l.v_mix:
+                out[x + "vmix"] = ()
+            if l.head_sink:
+                out[x + "sink"] = (l.heads,)
+            if l.head_gate:
+                out[x + "g"] = (l.heads, d)
+            if l.right is not None:
+                g, x = l.right, m + "right."
+                for n, k in (("q", g.heads * g.dim), ("k", g.heads * g.dim), ("v", g.heads * g.vdim), ("g", g.heads * g.vdim)):
+                    out[x + n] = (k, d)
+                out[x + "o"], out[x + "norm"] = (d, g.heads * g.vdim), (g.heads * g.vdim,)
+        elif l.type == "attention" and l.talk:
             out[m + "q"], out[m + "q.b"] = (l.heads * l.dim, d), (l.heads * l.dim,)
             out[m + "k"], out[m + "k.b"] = (l.kv_heads * l.dim, d), (l.kv_heads * l.dim,)
             out[m + "v"], out[m + "v.b"] = (l.kv_heads * l.vdim, d), (l.kv_heads * l.vdim,)
@@ -625,18 +811,20 @@ def param_shapes(cfg: HybridConfig) -> Dict[str, tuple]:
         if l.moe is not None:
             e = l.moe
             for j in range(e.experts):
-                if e.clamped:
+                if e.gated:
                     out[f + f"e{j}.gate"] = (e.ff, d)
                 out[f + f"e{j}.up"], out[f + f"e{j}.down"] = (e.ff, d), (d, e.ff)
             out[f + "router"] = (e.outputs, d)
-            if not e.clamped:
+            if e.score == "softmax_top":
+                out[f + "router.b"] = (e.outputs,)
+            if not e.gated:
                 out[f + "correction"] = (e.outputs,)
             if e.shared_ff:
                 if e.clamped:
                     out[f + "shared.gate"], out[f + "shared.sg"] = (e.shared_ff, d), (1, d)
                 out[f + "shared.up"], out[f + "shared.down"] = (e.shared_ff, d), (d, e.shared_ff)
         elif l.ff:
-            if cfg.design.dense_ff == "glu_relu":
+            if cfg.design.dense_ff in ("glu_relu", "clamped_glu"):
                 out[f + "gate"] = (l.ff, d)
             out[f + "up"], out[f + "down"] = (l.ff, d), (d, l.ff)
             if cfg.design.dense_ff == "xielu":
@@ -660,7 +848,8 @@ class StepLayout:
 
 class HybridCache:
     """Paged keys / values of the attention layers that own any, the paged compressed rows of the
-    latent-attention layers that own any, and the fp32 state slots of the recurrent layers, in ONE pool. Key
+    latent-attention layers that own any, and the fp32 state slots of the layers that keep state (recurrences, the
+    previous input row of a token shift, a convolution's last inputs), in ONE pool. Key
     planes are [blocks, G, BS, dim], value planes [blocks, G, BS, vdim], latent planes
     [blocks, 1, BS, kv_rank + rot_dim] (keys; their first kv_rank columns are the values) in the model's activation type; a state
     plane is [slots, size] fp32. Planes belong to layer RUNS (``HybridConfig.runs``): a layer that a
@@ -685,7 +874,7 @@ class HybridCache:
                     plan.append(("v", i, take(num_blocks * l.kv_heads * block_size * l.vdim * es)))
             elif l.owns_latent:
                 plan.append(("c", i, take(num_blocks * block_size * (l.kv_rank + l.rot_dim) * es)))
-            elif l.state_size():
+            if l.state_size():
                 plan.append(("s", i, take(max(1, num_slots) * l.state_size() * 4)))
         total = max(off, 256)
         if alloc is None:
@@ -724,6 +913,11 @@ class HybridCache:
 
     def state(self, run: int) -> torch.Tensor:
         return self._s[run]
+
+    def state_part(self, run: int, name: str) -> torch.Tensor:
+        """Column block of a state plane: [slots, numbers] of one of ``LayerSpec.state_parts``."""
+        at, n = self.cfg.layers[self.cfg.runs[run][0]].state_parts()[name]
+        return self._s[run][:, at:at + n]
 
     def copy_blocks(self, src: torch.Tensor, dst: torch.Tensor) -> None:
         # sequences with a state slot are never forked (csrc/core/kv_manager.cpp), so no block is
@@ -773,6 +967,17 @@ class HybridLayer:
     act: Optional[Tuple[float, float]] = None       # xIELU: (softplus(p), 1/2 + softplus(q))
     hc1: Optional["StreamWeights"] = None           # parallel residual streams: the mixer's read / write weights
     hc2: Optional["StreamWeights"] = None           # the feed-forward's
+    # sublayers between two norms, gated, with a token shift
+    norm1b: Optional[torch.Tensor] = None           # fp32 [d]: norm weight of the gated mixer result
+    norm2b: Optional[torch.Tensor] = None
+    shift: Optional[torch.Tensor] = None            # fp32 [d]
+    gate1: Optional[ops.LinearWeight] = None        # [d, d]: gate logits of the mixer's result, from its input before the shift
+    ff_in: Optional[ops.LinearWeight] = None        # gate logits of the feed-forward's result | gate | up (or | router)
+    conv_w: Optional[torch.Tensor] = None           # fp32 [taps, channels of q | k | v]
+    sinks: Optional[torch.Tensor] = None            # fp32 [H]
+    slopes: Optional[torch.Tensor] = None           # fp32 [H]: score taken off per unit of distance
+    v_lambda: float = 0.0                           # share of the first mixing layer's values
+    decay: Optional[torch.Tensor] = None            # fp32 [heads]: linear attention's constant decays
 
 
 @dataclass
@@ -866,7 +1071,9 @@ class HybridModel:
             if c.design.hyper:
                 for q in ("hc1", "hc2") if l.has_ff else ("hc1",):
                     kw[q] = StreamWeights(f32(load(p + q + ".in")), f32(load(p + q + ".out")), f32(load(p + q + ".mix")))
-            if l.type == "attention" and l.talk:
+            if l.prepped:
+                proj, out = self._load_prepped(p, l, load, lin, f32, inv_freqs, kw)
+            elif l.type == "attention" and l.talk:
                 if l.rot_dims:
                     kw["inv_freq"] = inv_freqs(l.rot_base, l.rot_dims)
                 if l.rotate_values:
@@ -929,7 +1136,16 @@ class HybridModel:
                 kw["head_norm"] = f32(load(m + "norm"))
                 out = lin(load(m + "o"))
             f = p + "mlp."
-            if l.moe is not None and l.moe.clamped:
+            if c.design.sandwich:
+                kw.update(shift=f32(load(p + "shift")), norm1b=norm_w(p + "norm1b"), gate1=lin(load(p + "rg1"), load(p + "rg1.b")))
+                if l.has_ff:
+                    kw["norm2b"] = norm_w(p + "norm2b")
+                    # one product of the feed-forward's input: gate logits of its result | gate | up, or | router
+                    names = ("router",) if l.moe is not None else ("gate", "up")
+                    rows = [load(f + n) for n in names]
+                    bias = [load(f + "router.b")] if l.moe is not None else [torch.zeros(2 * l.ff, device=dev)]
+                    kw["ff_in"] = lin(torch.cat([load(p + "rg2")] + rows, 0), torch.cat([load(p + "rg2.b")] + bias, 0), pad=True)
+            if l.moe is not None and l.moe.gated:
                 e = l.moe
                 # one product for the router's logits (32-bit: fp32 accumulation of the operands) and, when there is a
                 # shared expert, its gate | up units and its gate logit: gate | up | router | sg
@@ -937,7 +1153,8 @@ class HybridModel:
                 if e.shared_ff:
                     rows = [load(f + "shared.gate"), load(f + "shared.up")] + rows + [load(f + "shared.sg")]
                     kw["shared_down"] = lin(load(f + "shared.down"))
-                kw["router"] = lin(torch.cat(rows, 0), pad=True)
+                if not c.design.sandwich:           # (there the router's rows stand in ``ff_in``)
+                    kw["router"] = lin(torch.cat(rows, 0), pad=True)
                 ups = torch.stack([torch.cat([load(f + f"e{j}.gate"), load(f + f"e{j}.up")], 0) for j in range(e.experts)])
                 downs = torch.stack([load(f + f"e{j}.down") for j in range(e.experts)])
                 if dt == torch.bfloat16 and c.hidden_size % 64 == 0 and e.ff % 64 == 0 and dev.type == "cuda":
@@ -966,6 +1183,8 @@ class HybridModel:
                     kw["experts_down"] = ops.ExpertWeights.from_dense(downs, dev)
                 else:
                     kw["experts_up"], kw["experts_down"] = ups.to(dt).contiguous(), downs.to(dt).contiguous()
+            elif l.ff and c.design.sandwich:
+                kw["down"] = lin(load(f + "down"))
             elif l.ff and c.design.dense_ff == "xielu":
                 a = load(f + "act").double().cpu()
                 sp = torch.nn.functional.softplus(a)
@@ -987,6 +1206,37 @@ class HybridModel:
                     kw["norm2"] = f32(load(p + "norm2"))
             self.layers.append(HybridLayer(l, n1, proj, out, **kw))
 
+    def _load_prepped(self, p: str, l: LayerSpec, load, lin, f32, inv_freqs, kw: dict):
+        """Mixer weights of a layer whose q / k / v go through the general pre-processing: (input product, output
+        product); everything else goes to ``kw``. The input product is q | k | v (| a gate logit per head), or, with linear
+        attention beside it, q | k | v | its q | k | v | gate; the output product of the two then reads both results
+        side by side (their scales ride on the attention's result and on the linear attention's norm weight)."""
+        dev = self.device
+        m = p + "mix."
+        x = m + "left." if l.right is not None else m
+        Ws = [load(x + n) for n in ("q", "k", "v")] + ([load(x + "g")] if l.head_gate else [])
+        bias = torch.cat([load(x + n + ".b") for n in ("q", "k", "v")], 0) if l.biases else None
+        Wo, bo = load(x + "o"), load(x + "o.b") if l.biases else None
+        if l.conv:
+            kw["conv_w"] = torch.cat([load(x + n + ".conv") for n in ("q", "k", "v")], 0).t().contiguous()
+        if l.qk_norm:
+            kw["q_norm"], kw["k_norm"] = f32(load(x + "q.norm")), f32(load(x + "k.norm"))
+        if l.rot_dims:
+            kw["inv_freq"] = inv_freqs(l.rot_base, l.rot_dims)
+        if l.head_sink:
+            kw["sinks"] = f32(load(x + "sink"))
+        if l.distance_bias:
+            kw["slopes"] = torch.tensor([2.0 ** (-8.0 * (h + 1) / l.heads) for h in range(l.heads)], dtype=torch.float32, device=dev)
+        if l.v_mix:
+            kw["v_lambda"] = float(load(x + "vmix").item())
+        if l.right is not None:
+            g, x = l.right, m + "right."
+            Ws += [load(x + n) for n in ("q", "k", "v", "g")]
+            Wo = torch.cat([Wo, load(x + "o")], 1)
+            kw["decay"] = torch.tensor(g.decay, dtype=torch.float32, device=dev)
+            kw["head_norm"] = (f32(load(x + "norm")) * g.out_scale).contiguous()
+        return lin(torch.cat(Ws, 0), bias, pad=True), lin(Wo, bo)
+
     @classmethod
     def random_init(cls, cfg: HybridConfig, device, seed: int = 0, dtype: torch.dtype = torch.bfloat16,
                     **_ignored) -> "HybridModel":
@@ -999,7 +1249,7 @@ class HybridModel:
         def get(name: str) -> torch.Tensor:
             shape = shapes[name]
             gen.manual_seed((seed * 1000003 + zlib.crc32(name.encode())) & 0x7FFFFFFFFFFFFFFF)
-            offset_norm = cfg.design.norm_offset != 0.0 and name.split(".")[-1] in ("norm1", "norm2") or \
+            offset_norm = cfg.design.norm_offset != 0.0 and name.split(".")[-1] in ("norm1", "norm2", "norm1b", "norm2b") or \
                 (cfg.design.norm_offset != 0.0 and name == "final.norm")
             if ".hc" in name:                                    # streams that neither die out nor blow up
                 n = cfg.streams
@@ -1007,6 +1257,8 @@ class HybridModel:
                 t = t + 0.05 * torch.randn(shape, generator=gen)
             elif name.endswith("mix.talk"):
                 t = torch.eye(shape[0]) + 0.1 * torch.randn(shape, generator=gen)
+            elif cfg.design.sandwich and name.endswith((".shift", "mix.vmix")):
+                t = 0.7 * torch.rand(shape, generator=gen)
             elif name.endswith(".alpha"):
                 t = 0.6 + 0.1 * torch.randn(shape, generator=gen)
             elif len(shape) == 2:
@@ -1030,7 +1282,7 @@ class HybridModel:
         n = self.embed.numel() * self.embed.element_size() + self.lm_head.nbytes()
         n += self.loop_in.nbytes() if self.loop_in is not None else 0
         for L in self.layers:
-            for w in (L.proj, L.out, L.up, L.down, L.decay_up, L.gate_up, L.router, L.shared_up, L.shared_down):
+            for w in (L.proj, L.out, L.up, L.down, L.decay_up, L.gate_up, L.router, L.shared_up, L.shared_down, L.gate1, L.ff_in):
                 n += w.nbytes() if w is not None else 0
             for t in (L.key_up_t, L.value_up, L.experts_up, L.experts_down, L.talk):
                 t = t.data if isinstance(t, ops.ExpertWeights) else t
@@ -1074,6 +1326,8 @@ class HybridModel:
         T = token_ids.numel()
         self._portions = (meta.block_tables.shape[0], meta.prefill_tokens if meta.riders is not None else T) \
             if meta.is_prefill else (0, 0)
+        if c.design.sandwich:
+            return self._forward_sandwich(token_ids, positions, slot_mapping, meta, lay, cache, taps)
         if c.design.hyper:
             return self._forward_streams(token_ids, positions, slot_mapping, meta, lay, cache, taps)
         if c.design.pre_norm:
@@ -1180,6 +1434,98 @@ class HybridModel:
             if taps is not None:
                 taps.append(x.clone() if x is not None else ops.hc_step(xs, None, None, None, self.stream_sum, None, eps, None))
         return x
+
+    def _forward_sandwich(self, token_ids, positions, slot_mapping, meta, lay: StepLayout, cache: HybridCache,
+                          taps: Optional[list]) -> torch.Tensor:
+        """Layers whose sublayers sit between two norms. One launch gates and norms a sublayer's result, adds it to the
+        stream and norms the stream for the next sublayer. A mixer reads that row shifted towards the sequence's
+        previous one: the same launch does it when every sequence of the step has one row (the previous row is then
+        the stored one), a second launch when there are portions."""
+        c, dt, eps = self.cfg, self.dtype, self.cfg.rms_eps
+        x, _ = ops.embed_rows(token_ids, self.embed, None, meta.token_feed, c.embed_scale)
+        single = self._max_len == 1
+        runs = c.runs
+
+        def step(y, gate, w_out, r: int):
+            """The sublayer result joins the stream; (input, shifted input) of the mixer of run r."""
+            if r == len(runs):
+                ops.gated_step(x, y, gate, w_out, None, eps, dt)
+                return None, None
+            L = self.layers[runs[r][0]]
+            sh = ops.ShiftState(L.shift, cache.state_part(r, "shift"))
+            if single:
+                ha, _, hs = ops.gated_step(x, y, gate, w_out, L.norm1, eps, dt, shift=sh, lay=lay, positions=positions)
+                return ha, hs
+            ha, h32, _ = ops.gated_step(x, y, gate, w_out, L.norm1, eps, dt, want_f32=True)
+            return ha, ops.token_shift(h32, sh, lay, positions, dt)
+        shared: dict = {}                   # the first mixing layer's values of this step
+        ha, hs = step(None, None, None, 0)
+        for r, (i, _) in enumerate(runs):
+            L = self.layers[i]
+            y = self._attention_prepped(r, L, hs, positions, slot_mapping, lay, cache, shared)
+            gate, w_out = ops.linear(ha, L.gate1, out_f32=True), L.norm1b
+            if L.spec.has_ff:
+                ha, _, _ = ops.gated_step(x, y, gate, w_out, L.norm2, eps, dt)
+                fi = ops.linear(ha, L.ff_in, out_f32=True)              # gate logits of the result | gate | up, or | router
+                y = self._gated_experts(L, ha, fi[:, c.hidden_size:]) if L.spec.moe is not None else self._clamped_dense(L, fi)
+                gate, w_out = fi[:, :c.hidden_size], L.norm2b
+            ha, hs = step(y, gate, w_out, r + 1)
+            if taps is not None:
+                taps.append(x.clone())
+        return x
+
+    def _clamped_dense(self, L: HybridLayer, fi: torch.Tensor) -> torch.Tensor:
+        d, n, des = self.cfg.hidden_size, L.spec.ff, self.cfg.design
+        act = ops.glu_clamped(fi, d, d + n, n, L.spec.ff_limit, self.dtype, slope=des.glu_slope, shift=des.glu_shift)
+        return ops.linear(act, L.down, out_f32=True)
+
+    def _gated_experts(self, L: HybridLayer, xa: torch.Tensor, z: torch.Tensor) -> torch.Tensor:
+        """Routed feed-forward of silu-gated experts; z: router logits in the first columns. silu(g) u is the clamped gated
+        unit without a limit, with slope 1 and shift 0."""
+        e = L.spec.moe
+        ids, wts = ops.route_grouped(z[:, :e.experts], None, e.top, 1, 1, 1.0, score="softmax_top")
+        offsets, sorted_src, slot_of = ops.moe_sort(ids, e.experts)
+        rows = ids.numel()
+        if isinstance(L.experts_up, ops.ExpertWeights):
+            act = ops.grouped_linear(xa, sorted_src, offsets, L.experts_up, self.dtype, rows, glu_clamp=(None, math.inf, 1.0, 0.0))
+        else:
+            gu = ops.grouped_linear(xa, sorted_src, offsets, L.experts_up, torch.float32, rows)
+            act = ops.glu_clamped(gu, 0, e.ff, e.ff, math.inf, self.dtype, slope=1.0, shift=0.0)
+        ye = ops.grouped_linear(act, None, offsets, L.experts_down, torch.float32, rows)
+        return ops.moe_mix(ye, slot_of, ids, wts, xa, e.experts)
+
+    def _attention_prepped(self, r: int, L: HybridLayer, hs, positions, slot_mapping, lay: StepLayout, cache: HybridCache,
+                           shared: dict) -> torch.Tensor:
+        """Attention behind the general pre-processing, with linear attention beside it when the layer has any (both
+        results then lie side by side in front of one output product)."""
+        l = L.spec
+        H, G, D, Dv, C = l.heads, l.kv_heads, l.dim, l.vdim, l.channels
+        kc, vc = cache.k(r), cache.v(r)
+        proj = ops.linear(hs, L.proj, out_f32=True)
+        first = l.v_mix and "v" not in shared
+        q, v = ops.attn_prep(proj, positions, slot_mapping, lay, kc, vc, H, G, D, Dv, conv_w=L.conv_w,
+                             conv_state=cache.state_part(r, "conv") if l.conv > 1 else None, norm=l.qk_norm, q_norm=L.q_norm,
+                             k_norm=L.k_norm, eps=self.cfg.rms_eps, inv_freq=L.inv_freq, rot_dims=l.rot_dims, pairs=l.rot_pairs,
+                             temperature=l.q_temp, v_first=shared.get("v") if l.v_mix else None, v_mix=L.v_lambda, save_v=first)
+        if first:
+            shared["v"] = v
+        both = None
+        if l.right is not None:
+            g = l.right
+            both = torch.empty(hs.shape[0], H * Dv + g.heads * g.vdim, dtype=self.dtype, device=hs.device)
+        a = ops.attn_masked(q, kc, vc, lay.block_tables, lay.cu_q, lay.row_seq, positions, H, G, D, Dv, l.scale, 0, l.window,
+                            self.dtype, n_portions=self._portions[0], portion_rows=self._portions[1], max_len=self._max_len,
+                            softcap=l.softcap, sinks=L.sinks, slopes=L.slopes, keep=l.keep_first,
+                            gate=proj[:, C:C + H] if l.head_gate else None, out_scale=l.out_scale,
+                            out=both[:, :H * Dv] if both is not None else None)
+        if both is None:
+            return ops.linear(a, L.out, out_f32=True)
+        hd, hv = g.heads * g.dim, g.heads * g.vdim
+        o = ops.lightning_scan(proj[:, C:], L.decay, cache.state_part(r, "memory"), lay.cu_q, positions, lay.state_slots,
+                               g.heads, g.dim, g.vdim, self._max_len)
+        g0 = C + 2 * hd + hv
+        ops.rownorm_gate(o, L.head_norm, proj[:, g0:g0 + hv], self.cfg.rms_eps, self.dtype, out=both[:, H * Dv:])
+        return ops.linear(both, L.out, out_f32=True)
 
     def _residual_norm(self, x: torch.Tensor, y: Optional[torch.Tensor], norm, out: Optional[torch.Tensor] = None):
         """x += m * y (when y is given) and the design's norm of the new x in the activation type (when a
@@ -1345,7 +1691,8 @@ class HybridModel:
             xa = self._residual_norm(hidden_rows.contiguous(), None, self.final_norm)
         else:
             xa = ops.scalar_norm_add(hidden_rows, None, self.final_norm, self.cfg.rms_eps, self.dtype)
-        return ops.linear(xa, self.lm_head, out_f32=True)
+        z = ops.linear(xa, self.lm_head, out_f32=True)
+        return ops.softcap_(z, self.cfg.logit_softcap) if self.cfg.logit_softcap else z
 
     def target_logprobs(self, hidden_rows: torch.Tensor, ids: torch.Tensor) -> torch.Tensor:
         return ops.logprob_gather(self.logits(hidden_rows), ids)

@@ -1026,7 +1026,7 @@ def headnorm_gate(o: torch.Tensor, w: torch.Tensor, gate: torch.Tensor, Dv: int,
     o = o.contiguous()
     out = torch.empty(T, n, dtype=act_dtype, device=o.device)
     _hip().call("lc_headnorm_gate", o.data_ptr(), w.data_ptr(), gate.data_ptr(), gate.stride(0), out.data_ptr(),
-                _f32flag(act_dtype), T, n // Dv, Dv, float(eps), Dv, 0, 0, None)
+                _f32flag(act_dtype), T, n // Dv, Dv, float(eps), Dv, 0, 0, None, n)
     return out
 
 
@@ -1082,7 +1082,9 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
                 cu_q: torch.Tensor, row_seq: torch.Tensor, positions: torch.Tensor, H: int, G: int, D: int, Dv: int,
                 scale: float, chunk: int, window: int, act_dtype: torch.dtype, n_portions: int = 0,
                 portion_rows: int = 0, max_len: int = 0, softcap: float = 0.0, sink: bool = False,
-                all_value_heads: bool = False) -> torch.Tensor:
+                all_value_heads: bool = False, sinks: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None,
+                keep: int = 0, gate: Optional[torch.Tensor] = None, out_scale: float = 1.0,
+                out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of fp32 queries [T, H*D] over paged keys / values of widths D / Dv. The row at
     position p sees keys j <= p with j >= floor(p / chunk) * chunk (``chunk`` > 0) and
     j > p - window (``window`` > 0), counted from the start of its sequence. ``row_seq`` [T]
@@ -1092,15 +1094,27 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
     softcap * tanh(s / softcap). ``sink``: the softmax has a silent extra entry of score 0, so the
     weights sum to less than one. ``all_value_heads``: every query head's weights are applied to
     the values of ALL G key/value heads; the result is [T, H * G * Dv] (head, value head, column).
+    ``sinks`` (fp32 [H]): the silent entry's score per head. ``slopes`` (fp32 [H]): slope * (p - j) is taken off
+    the scaled score (before the cap). ``keep``: the first ``keep`` keys of the sequence stay visible outside the
+    window / chunk. ``gate`` (fp32 logits [T, H], may be a column slice): head h's result is multiplied by its
+    sigmoid; ``out_scale`` multiplies every result. ``out``: write into this [T, H * Dv] block (of a wider matrix).
 
     Two kernels: the first ``n_portions`` sequences (rows [0, portion_rows), the longest of
     ``max_len`` rows) are prompt portions and go, 64 rows of a head per block, through fp32 MFMA
     tiles; the rows behind them (single decoded tokens) and shapes the tiles do not take go
     through the row kernel, one wave per (row, head)."""
-    if not q.is_cuda:
-        return ref.attn_masked(q, k_cache, v_cache, block_tables, cu_q, positions, H, G, D, Dv, scale, chunk, window,
-                               act_dtype, softcap, sink, all_value_heads)
     T = q.shape[0]
+    for c in (sinks, slopes):
+        if c is not None and (c.numel() != H or c.dtype != torch.float32 or not c.is_contiguous()):
+            raise ValueError("attn_masked: sinks and slopes are fp32, one per head")
+    if gate is not None and (gate.shape != (T, H) or gate.dtype != torch.float32 or gate.stride(1) != 1):
+        raise ValueError("attn_masked: the gate is an fp32 [T, H] matrix")
+    if out is not None and (out.shape != (T, H * Dv) or out.dtype != act_dtype or out.stride(1) != 1 or all_value_heads):
+        raise ValueError("attn_masked: the output block is [T, H * Dv] in the activation type")
+    if not q.is_cuda:
+        y = ref.attn_masked(q, k_cache, v_cache, block_tables, cu_q, positions, H, G, D, Dv, scale, chunk, window,
+                            act_dtype, softcap, sink, all_value_heads, sinks, slopes, keep, gate, out_scale)
+        return y if out is None else out.copy_(y)
     if q.dtype != torch.float32 or not q.is_contiguous() or k_cache.dtype != v_cache.dtype:
         raise ValueError("attn_masked: contiguous fp32 queries, caches of one type")
     k_ld, v_ld = _cache_ld(k_cache, G, D, "key"), _cache_ld(v_cache, G, Dv, "value")
@@ -1110,7 +1124,9 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
         raise ValueError("attn_masked: the portions exceed the step")
     nv = G if all_value_heads else 1
     o_ld = nv * Dv
-    out = torch.empty(T, H * o_ld, dtype=act_dtype, device=q.device)
+    if out is None:
+        out = torch.empty(T, H * o_ld, dtype=act_dtype, device=q.device)
+    o_row = max(out.stride(0), H * o_ld)
     BS, MB, cf, af = k_cache.shape[2], block_tables.shape[1], _f32flag(k_cache.dtype), _f32flag(act_dtype)
 
     def value_groups(cap: int):
@@ -1119,7 +1135,10 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
             return [(-1, 1, 0)] if Dv <= cap else []
         n = cap // Dv
         return [(v0, min(n, G - v0), v0 * Dv) for v0 in range(0, G, n)] if n else []
-    opts = (float(softcap), 1 if sink else 0)
+    def opts(first: int):
+        g = gate[first:] if gate is not None else None
+        return (float(softcap), 1 if (sink or sinks is not None) else 0, _hip().ptr(sinks), _hip().ptr(slopes), int(keep),
+                _hip().ptr(g), max(gate.stride(0), H) if gate is not None else 0, float(out_scale), o_row)
     first = 0
     # value heads side by side in one tile: equal groups whose width the tiles take (whole MFMA steps of 16 columns)
     tile_cols = max([n * Dv for n in range(1, nv + 1) if nv % n == 0 and Dv % 8 == 0 and attn_tile_ok(D, n * Dv)] or [0])
@@ -1128,7 +1147,7 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
         for vh0, nvh, col0 in value_groups(tile_cols):
             _hip().call("lc_attn_tile", q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), cf, block_tables.data_ptr(),
                         MB, cu_q.data_ptr(), positions.data_ptr(), out.data_ptr(), af, int(n_portions), int(max_len), H, G,
-                        D, Dv, BS, float(scale), int(chunk), int(window), k_ld, v_ld, *opts, vh0, nvh, o_ld, col0)
+                        D, Dv, BS, float(scale), int(chunk), int(window), k_ld, v_ld, *opts(0), vh0, nvh, o_ld, col0)
         first = portion_rows
     if first < T:
         if Dv > 512:
@@ -1137,7 +1156,7 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
         _hip().call("lc_attn_masked", q[first:].data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), cf,
                     block_tables.data_ptr(), MB, row_seq[first:].data_ptr(), positions[first:].data_ptr(),
                     out[first:].data_ptr(), af, T - first, H, G, D, Dv, BS, float(scale), int(chunk), int(window),
-                    k_ld, v_ld, *opts, 0 if all_value_heads else -1, 1, o_ld, 0, nv)
+                    k_ld, v_ld, *opts(first), 0 if all_value_heads else -1, 1, o_ld, 0, nv)
     return out
 
 
@@ -1245,7 +1264,7 @@ def mlstm_out(o: torch.Tensor, m: torch.Tensor, w: torch.Tensor, gate: torch.Ten
         raise ValueError("mlstm_out: shapes do not fit the head sizes")
     out = torch.empty(T, H * Dv, dtype=act_dtype, device=o.device)
     _hip().call("lc_headnorm_gate", o.data_ptr(), w.data_ptr(), gate.data_ptr(), gate.stride(0), out.data_ptr(),
-                _f32flag(act_dtype), T, H, Dv, float(eps), Dv + 1, Dv, 1, m.data_ptr())
+                _f32flag(act_dtype), T, H, Dv, float(eps), Dv + 1, Dv, 1, m.data_ptr(), H * Dv)
     return out
 
 
@@ -1260,13 +1279,17 @@ def glu(y: torch.Tensor, act_dtype: torch.dtype, kind: str = "relu") -> torch.Te
     return out
 
 
+ROUTE_SCORES = ("softmax", "sigmoid", "softmax_top")
+
+
 def route_grouped(z: torch.Tensor, correction: Optional[torch.Tensor], top: int, groups: int, keep: int, scale: float,
                   score: str = "softmax"):
     """Group-limited top-k routing over fp32 router logits z [T, n] (see ops.reference.route_grouped):
     (ids int32 [T, top], weights fp32 [T, top]). ``score``: softmax over the outputs, or sigmoid of each;
-    ``correction`` may be None."""
-    if score not in ("softmax", "sigmoid"):
-        raise ValueError(f"route_grouped: score function {score!r}: softmax or sigmoid")
+    ``correction`` may be None. "softmax_top": the choice goes by the logits, the weights are the softmax over the
+    chosen logits only."""
+    if score not in ROUTE_SCORES:
+        raise ValueError(f"route_grouped: score function {score!r}: {', '.join(ROUTE_SCORES)}")
     T, n = z.shape
     if groups < 1 or n % groups or not 1 <= keep <= groups or top > keep * (n // groups):
         raise ValueError("route_grouped: groups must divide the router's width and the kept groups hold `top` outputs")
@@ -1277,7 +1300,7 @@ def route_grouped(z: torch.Tensor, correction: Optional[torch.Tensor], top: int,
     ids = torch.empty(T, top, dtype=torch.int32, device=z.device)
     wts = torch.empty(T, top, dtype=torch.float32, device=z.device)
     _hip().call("lc_route_grouped", z.data_ptr(), max(z.stride(0), n), _hip().ptr(correction), T, n, top, groups, keep,
-                float(scale), 1 if score == "sigmoid" else 0, ids.data_ptr(), wts.data_ptr())
+                float(scale), ROUTE_SCORES.index(score), ids.data_ptr(), wts.data_ptr())
     return ids, wts
 
 
@@ -1587,3 +1610,178 @@ def xielu(y: torch.Tensor, ap: float, an: float, act_dtype: torch.dtype) -> torc
     out = torch.empty(T, n, dtype=act_dtype, device=y.device)
     _hip().call("lc_xielu", y.data_ptr(), max(y.stride(0), n), out.data_ptr(), _f32flag(act_dtype), T, n, float(ap), float(an))
     return out
+
+
+# ---- gated residual steps between two norms, token shift, convolved / normed / mixed attention inputs, linear attention
+# with one decay per head (hybrid_gated.hip, hybrid.hip) ----
+@dataclass
+class ShiftState:
+    """What a token shift reads besides the step's rows: ``mu`` (fp32 [d]) and the sequences' stored rows, fp32
+    [slots, d] (may be a column block of a wider state plane)."""
+
+    mu: torch.Tensor
+    state: torch.Tensor
+
+    def check(self, d: int, what: str) -> None:
+        st = self.state
+        if self.mu.numel() != d or st.shape[1] != d or st.dtype != torch.float32 or st.stride(1) != 1:
+            raise ValueError(f"{what}: fp32 stored rows [slots, d] and a shift weight per coordinate")
+
+
+def gated_step(x: torch.Tensor, y: Optional[torch.Tensor], gate: Optional[torch.Tensor], w_out: Optional[torch.Tensor],
+               w_in: Optional[torch.Tensor], eps: float, act_dtype: torch.dtype, want_f32: bool = False,
+               shift: Optional[ShiftState] = None, lay=None, positions: Optional[torch.Tensor] = None):
+    """The residual step of a layer whose sublayers sit between two norms, one launch. With ``y`` (fp32 [T, d]):
+    v = y * sigmoid(gate) (``gate``: fp32 logits [T, d], may be a column slice), RMS-normed times ``w_out``, joins the
+    stream x (fp32, in place). With ``w_in``: h = rms_norm(x) * w_in. Returns (h in ``act_dtype``, h in fp32 when
+    ``want_f32``, shifted h): with ``shift`` (a step whose sequences all have ONE row; ``lay``: the step's layout)
+    the third is h + (h' - h) * mu in ``act_dtype``, h' the sequence's stored row, which becomes h."""
+    T, d = x.shape
+    if x.dtype != torch.float32 or not x.is_contiguous():
+        raise ValueError("gated_step: the residual stream is a contiguous fp32 tensor")
+    if y is not None and (y.shape != x.shape or y.dtype != torch.float32):
+        raise ValueError("gated_step: the sublayer output must be fp32 of the stream's shape")
+    if gate is not None and (y is None or gate.shape != x.shape or gate.dtype != torch.float32 or gate.stride(1) != 1):
+        raise ValueError("gated_step: gate logits are fp32 [T, d] and need a sublayer output")
+    if shift is not None:
+        shift.check(d, "gated_step")
+        if w_in is None or lay is None or positions is None or lay.state_slots is None:
+            raise ValueError("gated_step: a shift needs the input norm and the step's layout")
+    if not x.is_cuda:
+        return ref.gated_step(x, y, gate, w_out, w_in, eps, act_dtype, shift, lay, positions)
+    if y is None and w_in is None:
+        return None, None, None
+    dev = x.device
+    f32 = act_dtype == torch.float32
+    ha = torch.empty(T, d, dtype=act_dtype, device=dev) if w_in is not None else None
+    h32 = torch.empty(T, d, dtype=torch.float32, device=dev) if (w_in is not None and want_f32 and not f32) else None
+    hs = torch.empty(T, d, dtype=act_dtype, device=dev) if shift is not None else None
+    p = _hip().ptr
+    _hip().call("lc_gated_step", x.data_ptr(), p(y.contiguous() if y is not None else None), p(gate),
+                max(gate.stride(0), d) if gate is not None else 0, p(w_out), p(w_in), float(eps), p(ha), p(h32),
+                _f32flag(act_dtype), p(shift.mu) if shift else None, p(shift.state) if shift else None,
+                max(shift.state.stride(0), d) if shift else 0, p(lay.row_seq) if shift else None,
+                p(positions) if shift else None, p(lay.state_slots) if shift else None, p(hs), T, d)
+    return ha, (ha if f32 else h32), hs
+
+
+def token_shift(h: torch.Tensor, shift: ShiftState, lay, positions: torch.Tensor, act_dtype: torch.dtype) -> torch.Tensor:
+    """h + (h' - h) * mu in ``act_dtype``, h' the sequence's previous row: the row before in the step, the stored row
+    for a portion's first row (zeros at position 0). The stored rows become the portions' last rows. h fp32 [T, d]."""
+    T, d = h.shape
+    shift.check(d, "token_shift")
+    if h.dtype != torch.float32 or not h.is_contiguous() or lay.state_slots is None:
+        raise ValueError("token_shift: contiguous fp32 rows and the step's state slots")
+    if not h.is_cuda:
+        return ref.token_shift(h, shift, lay, positions, act_dtype)
+    hs = torch.empty(T, d, dtype=act_dtype, device=h.device)
+    _hip().call("lc_token_shift", h.data_ptr(), shift.mu.data_ptr(), shift.state.data_ptr(), max(shift.state.stride(0), d),
+                lay.row_seq.data_ptr(), lay.cu_q.data_ptr(), positions.data_ptr(), lay.state_slots.data_ptr(), hs.data_ptr(),
+                _f32flag(act_dtype), T, d)
+    return hs
+
+
+ATTN_PREP_MAX_FLOATS = 159 * 1024 // 4      # a token's channels, angles and head norms in one block's LDS
+
+
+def attn_prep(qkv: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Tensor, lay, k_cache: torch.Tensor,
+              v_cache: torch.Tensor, H: int, G: int, D: int, Dv: int, conv_w: Optional[torch.Tensor] = None,
+              conv_state: Optional[torch.Tensor] = None, norm: str = "", q_norm: Optional[torch.Tensor] = None,
+              k_norm: Optional[torch.Tensor] = None, eps: float = 0.0, inv_freq: Optional[torch.Tensor] = None,
+              rot_dims: int = 0, pairs: bool = False, temperature: Tuple[float, float] = (0.0, 1.0),
+              v_first: Optional[torch.Tensor] = None, v_mix: float = 0.0, save_v: bool = False):
+    """Attention pre-processing and cache write in one launch. qkv fp32 [T, >= (H + G) D + G Dv] = q | k | v. In this
+    order, each optional: a causal convolution per channel (``conv_w`` fp32 [taps, C], the newest tap last;
+    ``conv_state`` fp32 [slots, (taps - 1) * C], the sequences' last inputs, oldest first, updated in place); RMS
+    norms over the ``"whole"`` projection (weights [H D] / [G D]) or per ``"head"`` ([D]); a turn of the first ``rot_dims``
+    coordinates of q and k heads (``inv_freq`` fp64; ``pairs``: neighbours); q times
+    1 + coef * ln(floor((p + 1) / every) + 1) for ``temperature`` = (coef, every); values mixed with ``v_first`` (fp32
+    [T, G Dv]) by ``v_mix``. Returns (q fp32 [T, H D], the values before the mix when ``save_v``)."""
+    T = qkv.shape[0]
+    C = (H + G) * D + G * Dv
+    taps = conv_w.shape[0] if conv_w is not None else 0
+    if qkv.dtype != torch.float32 or qkv.stride(1) != 1 or qkv.shape[1] < C:
+        raise ValueError("attn_prep: fp32 projections q | k | v")
+    if k_cache.shape[1:] != (G, k_cache.shape[2], D) or v_cache.shape[1:] != (G, k_cache.shape[2], Dv) or \
+            not k_cache.is_contiguous() or not v_cache.is_contiguous() or k_cache.dtype != v_cache.dtype:
+        raise ValueError("attn_prep: cache planes do not fit the head sizes")
+    if conv_w is not None and (conv_w.shape != (taps, C) or conv_w.dtype != torch.float32 or not conv_w.is_contiguous()):
+        raise ValueError("attn_prep: convolution weights are fp32 [taps, channels]")
+    if taps > 1 and (conv_state is None or conv_state.shape[1] != (taps - 1) * C or conv_state.dtype != torch.float32
+                     or conv_state.stride(1) != 1 or lay.state_slots is None):
+        raise ValueError("attn_prep: the convolution's inputs before the step are fp32 [slots, (taps - 1) * channels]")
+    if norm not in ("", "whole", "head") or (norm and (q_norm.numel() != (H * D if norm == "whole" else D)
+                                                       or k_norm.numel() != (G * D if norm == "whole" else D))):
+        raise ValueError("attn_prep: norms over the whole projection or per head, with weights of that size")
+    if rot_dims and (inv_freq is None or inv_freq.dtype != torch.float64 or inv_freq.numel() != rot_dims // 2):
+        raise ValueError("attn_prep: rot_dims / 2 fp64 frequencies are needed")
+    if v_first is not None and (v_first.shape != (T, G * Dv) or v_first.dtype != torch.float32 or v_first.stride(1) != 1):
+        raise ValueError("attn_prep: the values to mix in are fp32 [T, G * Dv]")
+    if C + rot_dims + H + G > ATTN_PREP_MAX_FLOATS:
+        raise ValueError("attn_prep: a token's channels exceed one block's LDS")
+    if not qkv.is_cuda:
+        return ref.attn_prep(qkv, positions, slot_mapping, lay, k_cache, v_cache, H, G, D, Dv, conv_w, conv_state, norm, q_norm,
+                             k_norm, eps, inv_freq, rot_dims, pairs, temperature, v_first, v_mix, save_v)
+    q = torch.empty(T, H * D, dtype=torch.float32, device=qkv.device)
+    vs = torch.empty(T, G * Dv, dtype=torch.float32, device=qkv.device) if save_v else None
+    p = _hip().ptr
+    _hip().call("lc_attn_prep", qkv.data_ptr(), max(qkv.stride(0), qkv.shape[1]), p(conv_w), taps,
+                p(conv_state) if taps > 1 else None, max(conv_state.stride(0), conv_state.shape[1]) if taps > 1 else 0,
+                ("", "whole", "head").index(norm), p(q_norm), p(k_norm), float(eps), p(inv_freq), int(rot_dims),
+                1 if pairs else 0, float(temperature[0]), float(temperature[1]), p(v_first),
+                max(v_first.stride(0), G * Dv) if v_first is not None else 0, float(v_mix), p(vs), p(lay.row_seq),
+                p(lay.cu_q), positions.data_ptr(), p(lay.state_slots), slot_mapping.data_ptr(), k_cache.data_ptr(),
+                v_cache.data_ptr(), _f32flag(k_cache.dtype), q.data_ptr(), T, H, G, D, Dv, k_cache.shape[2])
+    return q, vs
+
+
+def lightning_scan(proj: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, cu_q: torch.Tensor, positions: torch.Tensor,
+                   slots: torch.Tensor, H: int, D: int, Dv: int, max_len: int = 1) -> torch.Tensor:
+    """Linear attention with one constant decay per head (fp32 [H]) over the step's sequences: q, k, v are silu of
+    proj's first columns (fp32 [T, >= 2 H D + H Dv] = q | k | v), per head S <- decay S + k v^T, o = S^T q. state
+    fp32 [slots, H*D*Dv] (may be a column block of a wider plane), updated in place. Returns fp32 [T, H*Dv]."""
+    T = proj.shape[0]
+    if proj.dtype != torch.float32 or state.dtype != torch.float32 or proj.stride(1) != 1 or state.stride(1) != 1:
+        raise ValueError("lightning_scan: fp32 projections and state")
+    if state.shape[1] != H * D * Dv or decay.numel() != H or decay.dtype != torch.float32 or D > 256 or \
+            proj.shape[1] < 2 * H * D + H * Dv:
+        raise ValueError("lightning_scan: shapes do not fit the head sizes (key width at most 256)")
+    if not proj.is_cuda:
+        return ref.lightning_scan(proj, decay, state, cu_q, positions, slots, H, D, Dv)
+    out = torch.empty(T, H * Dv, dtype=torch.float32, device=proj.device)
+    B = slots.numel()
+    scratch = _scan_scratch(B, max_len, H * D * Dv, H * D, proj.device)
+    prep = torch.empty(T * H * D * 4, dtype=torch.float32, device=proj.device)     # (q, k, decay, -) per channel
+    _hip().call("lc_lightning_scan", proj.data_ptr(), max(proj.stride(0), proj.shape[1]), decay.data_ptr(), state.data_ptr(),
+                max(state.stride(0), state.shape[1]), cu_q.data_ptr(), positions.data_ptr(), slots.data_ptr(), out.data_ptr(),
+                T, B, H, D, Dv, int(max_len), _hip().ptr(scratch), prep.data_ptr())
+    return out
+
+
+def rownorm_gate(o: torch.Tensor, w: torch.Tensor, gate: torch.Tensor, eps: float, act_dtype: torch.dtype,
+                 out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """o / sqrt(mean(o^2) + eps) * w over whole rows (fp32 [T, n]), times sigmoid(gate) (fp32 logits, may be a column
+    slice), into ``out`` (a [T, n] block of a wider matrix) when given."""
+    T, n = o.shape
+    if gate.shape != o.shape or gate.stride(1) != 1 or o.dtype != torch.float32 or gate.dtype != torch.float32 or w.numel() != n:
+        raise ValueError("rownorm_gate: fp32 rows and gate logits of one shape, a weight per column")
+    if out is None:
+        out = torch.empty(T, n, dtype=act_dtype, device=o.device)
+    if out.shape != o.shape or out.dtype != act_dtype or out.stride(1) != 1:
+        raise ValueError("rownorm_gate: the output is a [T, n] block in the activation type")
+    if not o.is_cuda:
+        return out.copy_(ref.rownorm_gate(o, w, gate, eps, act_dtype))
+    o = o.contiguous()
+    _hip().call("lc_headnorm_gate", o.data_ptr(), w.data_ptr(), gate.data_ptr(), max(gate.stride(0), n), out.data_ptr(),
+                _f32flag(act_dtype), T, 1, n, float(eps), n, 0, 1, None, max(out.stride(0), n))
+    return out
+
+
+def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """cap * tanh(x / cap) in place (fp32, contiguous)."""
+    if not x.is_cuda:
+        return x.copy_(ref.capped(x, cap))
+    if x.dtype != torch.float32 or not x.is_contiguous() or not cap > 0:
+        raise ValueError("softcap_: a contiguous fp32 tensor and a positive cap")
+    _hip().call("lc_softcap", x.data_ptr(), x.numel(), float(cap))
+    return x

@@ -65,12 +65,12 @@ _SIGNATURES = {
     "lc_relu2": [_P, _P, _I, _I, _I, _I, _P],
     "lc_mingru_scan": [_P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P, _P],
     "lc_gla_scan": [_P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P],
-    "lc_headnorm_gate": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _I, _I, _I, _P, _P],
+    "lc_headnorm_gate": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _I, _I, _I, _P, _I, _P],
     "lc_qkv_prep": [_P, _I, _P, _P, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P],
     "lc_attn_masked": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I,
-                       _I, _I, _F, _I, _I, _I, _I, _I, _I, _P],
+                       _I, _I, _F, _I, _P, _P, _I, _P, _I, _F, _I, _I, _I, _I, _I, _I, _P],
     "lc_attn_tile": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I,
-                     _I, _I, _F, _I, _I, _I, _I, _I, _P],
+                     _I, _I, _F, _I, _P, _P, _I, _P, _I, _F, _I, _I, _I, _I, _I, _P],
     "lc_gemm_any": [_P, _I, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P],
     "lc_add_rmsnorm": [_P, _P, _P, _F, _P, _I, _I, _I, _P],
     "lc_latent_write": [_P, _I, _I, _I, _P, _F, _P, _P, _I, _I, _I, _P],
@@ -87,6 +87,13 @@ _SIGNATURES = {
     "lc_talk_mix": [_P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P],
     "lc_latent_rope_write": [_P, _I, _I, _P, _F, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "lc_xielu": [_P, _I, _P, _I, _I, _I, _F, _F, _P],
+    # gated residual steps, token shifts, attention pre-processing with convolutions and mixed values (hybrid_gated.hip)
+    "lc_gated_step": [_P, _P, _P, _I, _P, _P, _F, _P, _P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _P],
+    "lc_token_shift": [_P, _P, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _P],
+    "lc_attn_prep": [_P, _I, _P, _I, _P, _L, _I, _P, _P, _F, _P, _I, _I, _F, _F, _P, _I, _F, _P, _P, _P, _P, _P, _P, _P, _P,
+                     _I, _P, _I, _I, _I, _I, _I, _I, _P],
+    "lc_softcap": [_P, _L, _F, _P],
+    "lc_lightning_scan": [_P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _P],
     # routed feed-forwards of hybrid decoders (hybrid_moe.hip)
     "lc_route_grouped": [_P, _I, _P, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P],
     "lc_moe_sort": [_P, _I, _I, _I, _P, _P, _P, _P, _P, _P],

@@ -401,13 +401,15 @@ def qkv_prep(qkv: torch.Tensor, q_norm: torch.Tensor, k_norm: Optional[torch.Ten
 
 def attn_masked(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, positions, H: int, G: int, D: int, Dv: int,
                 scale: float, chunk: int, window: int, act_dtype, softcap: float = 0.0, sink: bool = False,
-                all_value_heads: bool = False) -> torch.Tensor:
+                all_value_heads: bool = False, sinks=None, slopes=None, keep: int = 0, gate=None,
+                out_scale: float = 1.0) -> torch.Tensor:
     """q fp32 [T, H*D]; paged keys [blocks, G, BS, D] and values [blocks, G, BS, Dv]. The row at
     position p sees keys j <= p with j >= floor(p / chunk) * chunk (``chunk`` > 0) and
     j > p - window (``window`` > 0). Scores, softmax and the weighted sum in fp32. ``softcap`` > 0: scores
     become softcap * tanh(score / softcap); ``sink``: the softmax's denominator carries an extra 1 (an entry of
-    score 0 without a value); ``all_value_heads``: every head's weights meet the values of all G value heads,
-    result [T, H * G * Dv]."""
+    score 0, or ``sinks`` [H], without a value); ``slopes`` [H]: slope * (p - j) off the scaled score before the
+    cap; ``keep``: the first keys stay visible; ``gate`` [T, H]: sigmoid factor per head; ``all_value_heads``: every
+    head's weights meet the values of all G value heads, result [T, H * G * Dv]."""
     T = q.shape[0]
     nv = G if all_value_heads else 1
     out = torch.zeros(T, H * nv * Dv, dtype=torch.float32, device=q.device)
@@ -425,25 +427,32 @@ def attn_masked(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, positions
         V = v_cache[blocks].permute(1, 0, 2, 3).reshape(G, nb * BS, Dv)[:, :n].float()
         Q = q[r0:r1].float().view(r1 - r0, G, rep, D)
         sc = torch.einsum("qgrd,gkd->grqk", Q, K) * scale
+        key = torch.arange(n, device=q.device)[None, :]
+        if slopes is not None:
+            sc = sc - slopes.float().view(G, rep)[:, :, None, None] * (pos[:, None] - key).float()[None, None]
         if softcap > 0:
             sc = softcap * torch.tanh(sc / softcap)
-        key = torch.arange(n, device=q.device)[None, :]
-        mask = key <= pos[:, None]
+        mask = torch.ones(r1 - r0, n, dtype=torch.bool, device=q.device)
         if chunk > 0:
             mask &= key >= (pos[:, None] // chunk) * chunk
         if window > 0:
             mask &= key > pos[:, None] - window
+        mask = (mask | (key < keep)) & (key <= pos[:, None])
         sc = sc.masked_fill(~mask[None, None], float("-inf"))
-        if sink:
-            m = sc.max(-1, keepdim=True).values.clamp_min(0.0)
+        if sink or sinks is not None:
+            s0 = sinks.float().view(G, rep)[:, :, None, None] if sinks is not None else torch.zeros(G, rep, 1, 1, device=q.device)
+            m = torch.maximum(sc.max(-1, keepdim=True).values, s0)
             e = torch.exp(sc - m)
-            w = e / (torch.exp(-m) + e.sum(-1, keepdim=True))
+            w = e / (torch.exp(s0 - m) + e.sum(-1, keepdim=True))
         else:
             w = torch.softmax(sc, dim=-1)
         if all_value_heads:
             out[r0:r1] = torch.einsum("grqk,ckv->qgrcv", w, V).reshape(r1 - r0, H * G * Dv)
         else:
             out[r0:r1] = torch.einsum("grqk,gkv->qgrv", w, V).reshape(r1 - r0, H * Dv)
+    out = out * out_scale
+    if gate is not None:
+        out = (out.view(T, H, -1) * torch.sigmoid(gate.float())[:, :, None]).view(T, -1)
     return out.to(act_dtype)
 
 
@@ -562,9 +571,12 @@ def route_grouped(z: torch.Tensor, correction: Optional[torch.Tensor], top: int,
     """Router over fp32 logits z [T, n]: s = softmax(z) (or sigmoid(z), each output on its own); choice = s + correction; the n outputs form
     ``groups`` equal runs of neighbours, a run's score is its largest choice, only the ``keep`` best runs
     stay eligible; the ``top`` largest eligible choices are taken (ties: the lower index) with weights
-    s * scale. Returns (ids int32 [T, top], weights fp32 [T, top])."""
+    s * scale. Score "softmax_top": s = z, and the weights are the softmax over the chosen logits times scale.
+    Returns (ids int32 [T, top], weights fp32 [T, top])."""
     T, n = z.shape
-    s = torch.softmax(z.float(), -1) if score == "softmax" else torch.sigmoid(z.float())
+    s = z.float()
+    if score != "softmax_top":
+        s = torch.softmax(s, -1) if score == "softmax" else torch.sigmoid(s)
     ch = s + correction.float() if correction is not None else s.clone()
     if groups > 1 and keep < groups:
         gs = ch.view(T, groups, n // groups).max(-1).values
@@ -572,7 +584,10 @@ def route_grouped(z: torch.Tensor, correction: Optional[torch.Tensor], top: int,
         allow = torch.zeros(T, groups, dtype=torch.bool, device=z.device).scatter_(1, order, True)
         ch = ch.masked_fill(~allow.repeat_interleave(n // groups, 1), float("-inf"))
     ids = torch.argsort(ch, dim=-1, descending=True, stable=True)[:, :top]
-    return ids.to(torch.int32), (s.gather(1, ids) * scale).float()
+    w = s.gather(1, ids)
+    if score == "softmax_top":
+        w = torch.softmax(w, -1)
+    return ids.to(torch.int32), (w * scale).float()
 
 
 def grouped_linear(x: torch.Tensor, row_index: Optional[torch.Tensor], offsets: torch.Tensor, W: torch.Tensor,
@@ -750,3 +765,110 @@ def latent_rope_write(proj: torch.Tensor, col_c: int, w, eps: float, inv_freq, p
 def xielu(y: torch.Tensor, ap: float, an: float, act_dtype) -> torch.Tensor:
     z = y.float()
     return torch.where(z > 0, ap * z * z + 0.5 * z, an * (torch.expm1(torch.clamp(z, max=0.0)) - z) + 0.5 * z).to(act_dtype)
+
+
+# ------------------------------------------------------------------ hybrid decoders: gated residual steps between two norms,
+# token shift, convolved / normed / mixed attention inputs, linear attention with one decay per head
+def gated_step(x: torch.Tensor, y, gate, w_out, w_in, eps: float, act_dtype, shift, lay, positions):
+    """x (fp32, in place) += rms_norm(y * sigmoid(gate)) * w_out; h = rms_norm(x) * w_in. Returns (h in ``act_dtype``,
+    h fp32, shifted h or None)."""
+    if y is not None:
+        v = y.float()
+        if gate is not None:
+            v = v * torch.sigmoid(gate.float())
+        if w_out is not None:
+            v = v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w_out.float()
+        x.add_(v)
+    if w_in is None:
+        return None, None, None
+    h = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * w_in.float()
+    return h.to(act_dtype), h, (token_shift(h, shift, lay, positions, act_dtype) if shift is not None else None)
+
+
+def token_shift(h: torch.Tensor, shift, lay, positions, act_dtype) -> torch.Tensor:
+    """Row t moves towards the row before it in its sequence by ``shift.mu``; a portion's first row towards the stored
+    row (zeros at position 0), which becomes the portion's last row."""
+    prev = torch.zeros_like(h)
+    prev[1:] = h[:-1]
+    for b in range(len(lay.state_slots)):
+        r0, r1, slot = int(lay.cu_q[b]), int(lay.cu_q[b + 1]), int(lay.state_slots[b])
+        if r1 <= r0:
+            continue
+        prev[r0] = shift.state[slot] if slot >= 0 and int(positions[r0]) != 0 else 0.0
+        if slot >= 0:
+            shift.state[slot] = h[r1 - 1]
+    return (h + (prev - h) * shift.mu.float()).to(act_dtype)
+
+
+def attn_prep(qkv: torch.Tensor, positions, slot_mapping, lay, k_cache, v_cache, H: int, G: int, D: int, Dv: int, conv_w,
+              conv_state, norm: str, q_norm, k_norm, eps: float, inv_freq, rot_dims: int, pairs: bool, temperature, v_first,
+              v_mix: float, save_v: bool):
+    """q | k | v of the step's rows: convolution over time, norms, rotation, query temperature, mixed values, paged
+    write. Returns (q fp32 [T, H*D], the values before the mix or None)."""
+    T = qkv.shape[0]
+    C = (H + G) * D + G * Dv
+    u = qkv[:, :C].float()
+    if conv_w is not None:
+        hist = conv_w.shape[0] - 1
+        y = torch.zeros_like(u)
+        for b in range(len(lay.cu_q) - 1):
+            r0, r1 = int(lay.cu_q[b]), int(lay.cu_q[b + 1])
+            if r1 <= r0:
+                continue
+            slot = int(lay.state_slots[b]) if lay.state_slots is not None else -1
+            before = torch.zeros(hist, C, dtype=torch.float32, device=u.device)
+            if hist and slot >= 0 and int(positions[r0]) != 0:
+                before = conv_state[slot].view(hist, C).clone()
+            ext = torch.cat([before, u[r0:r1]], 0)
+            y[r0:r1] = sum(conv_w[j].float() * ext[j:j + r1 - r0] for j in range(hist + 1))
+            if hist and slot >= 0:
+                conv_state[slot] = ext[-hist:].reshape(-1)
+        u = y
+    q, k, v = u[:, :H * D].view(T, H, D), u[:, H * D:(H + G) * D].view(T, G, D), u[:, (H + G) * D:]
+
+    def rms(z, w):
+        return z * torch.rsqrt(z.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+    if norm == "whole":
+        q, k = rms(q.reshape(T, -1), q_norm).view(T, H, D), rms(k.reshape(T, -1), k_norm).view(T, G, D)
+    elif norm == "head":
+        q, k = rms(q, q_norm), rms(k, k_norm)
+    q, k = rope_any(q, positions, rot_dims, inv_freq, pairs), rope_any(k, positions, rot_dims, inv_freq, pairs)
+    if temperature[0] != 0.0:
+        f = torch.floor((positions.double() + 1) / temperature[1]) + 1
+        q = q * (1 + temperature[0] * torch.log(f.float()))[:, None, None]
+    saved = v.clone() if save_v else None
+    if v_first is not None:
+        v = (1 - v_mix) * v + v_mix * v_first.float()
+    BS = k_cache.shape[2]
+    slots = slot_mapping.long()
+    ok = slots >= 0
+    blk, off = slots[ok] // BS, slots[ok] % BS
+    k_cache[blk, :, off, :] = k[ok].to(k_cache.dtype)
+    v_cache[blk, :, off, :] = v.reshape(T, G, Dv)[ok].to(v_cache.dtype)
+    return q.reshape(T, H * D).contiguous(), saved
+
+
+def lightning_scan(proj: torch.Tensor, decay, state, cu_q, positions, slots, H: int, D: int, Dv: int) -> torch.Tensor:
+    """q | k | v = silu of proj's first columns; per head S <- decay S + k v^T, o = S^T q (state [slots, H*D*Dv] fp32)."""
+    T = proj.shape[0]
+    u = torch.nn.functional.silu(proj[:, :2 * H * D + H * Dv].float())
+    q, k, v = u[:, :H * D].view(T, H, D), u[:, H * D:2 * H * D].view(T, H, D), u[:, 2 * H * D:].view(T, H, Dv)
+    out = torch.zeros(T, H, Dv, dtype=torch.float32, device=proj.device)
+    for b in range(len(slots)):
+        r0, r1, slot = int(cu_q[b]), int(cu_q[b + 1]), int(slots[b])
+        if slot < 0 or r1 <= r0:
+            continue
+        S = state[slot].reshape(H, D, Dv).clone()
+        if int(positions[r0]) == 0:
+            S.zero_()
+        for t in range(r0, r1):
+            S = decay.float()[:, None, None] * S + k[t][:, :, None] * v[t][:, None, :]
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[slot] = S.reshape(-1)
+    return out.view(T, H * Dv)
+
+
+def rownorm_gate(o: torch.Tensor, w, gate, eps: float, act_dtype) -> torch.Tensor:
+    """o / sqrt(mean(o^2) + eps) * w over whole rows, times sigmoid(gate)."""
+    v = o.float()
+    return (v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w.float() * torch.sigmoid(gate.float())).to(act_dtype)
