@@ -1,6 +1,6 @@
-"""Prefill and decode throughput of the hybrid decoders (Nidozen, Telurax, Surevik, Gizilorn) beside each other and a
+"""Prefill and decode throughput of the hybrid decoders (Nidozen, Telurax, Surevik, Gizilorn, Kulivik) beside each other and a
 Llama-shaped transformer of equal width, depth and head sizes (``bench.py --hybrid``,
-``--hybrid-models gizilorn,surevik,telurax,nidozen,llama``). Random weights, synthetic tokens.
+``--hybrid-models kulivik,gizilorn,surevik,telurax,nidozen,llama``). Random weights, synthetic tokens.
 
 Per size: one prompt of ``prompt`` tokens goes through each engine as a single step (prefill
 tokens/s), then ``batch`` requests decode ``new`` tokens each from recorded steps (decode tokens/s).
@@ -14,7 +14,9 @@ chosen, a gated shared expert of a quarter), its second and third layer run twic
 layer runs as the others have layers; the Gizilorn stack repeats (attention with mixed heads' weights, the same,
 latent attention with rows of its own, latent attention on those rows) over two residual streams, windows of the
 others' chunk, compressed rows of width 128 beside a turned key part of 64, a dense xIELU feed-forward in every
-layer; the transformer has full causal attention and a SwiGLU feed-forward. Prints one
+layer; the Kulivik stack repeats (window attention with kept first keys, attention beside linear attention, convolved
+attention over all earlier keys), a clamped gated dense feed-forward of half the others' width in the first layer, 32
+silu-gated experts of a sixteenth of the dense width (4 chosen) in the others; the transformer has full causal attention and a SwiGLU feed-forward. Prints one
 JSON line. Per-kernel times come from running this under ``rocprofv3 --kernel-trace --stats``.
 """
 from __future__ import annotations
@@ -118,6 +120,23 @@ def gizilorn_config(s: dict):
                              "streams": 2, "layers": layers}, name="gizilorn-bench")
 
 
+def kulivik_config(s: dict):
+    from .models.hybrid import config_from_dict
+
+    size = {"heads": s["heads"], "kv_heads": s["kv"], "dim": s["dim"], "vdim": s["dim"], "scale": s["dim"] ** -0.5}
+    lin = {"heads": s["heads"], "dim": s["dim"], "vdim": s["dim"],
+           "decay": [1.0 - 2.0 ** -(2 + 8.0 * i / s["heads"]) for i in range(s["heads"])]}
+    experts = {"kind": "moe", "expert": {"ff": s["ff"] // 16}, "router": {"experts": 32, "top": 4}}
+    mixers = [("attention_2", {**size, "softcap": 50.0, "mask": {"size": s["chunk"], "keep_first": 4},
+                               "rot": {"dims": s["dim"] // 2, "base": 10000.0}, "v_mix": True}),
+              ("parallel", {"left": {**size, "q_temp": {"coef": 0.1, "every": 1024}}, "right": lin, "left_scale": 0.7, "right_scale": 0.7}),
+              ("attention", {**size, "conv": 4, "v_mix": True})]
+    layers = [{"type": t, "mixer": m, "mlp": experts if i else {"kind": "dense", "ff": s["ff"] // 2, "limit": 7.0}}
+              for i, (t, m) in enumerate(mixers[i % 3] for i in range(s["layers"]))]
+    return config_from_dict({"architecture": "Kulivik", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6},
+                             "logit_scale": 1.0, "logit_softcap": 30.0, "layers": layers}, name="kulivik-bench")
+
+
 def transformer_config(s: dict):
     from .models.config import ModelConfig
 
@@ -191,6 +210,8 @@ def run(a) -> int:
                 model = HybridModel.random_init(surevik_config(s), dev, seed=1)
             elif kind == "gizilorn":
                 model = HybridModel.random_init(gizilorn_config(s), dev, seed=1)
+            elif kind == "kulivik":
+                model = HybridModel.random_init(kulivik_config(s), dev, seed=1)
             else:
                 model = TransformerModel.random_init(transformer_config(s), dev, seed=1)
             row[kind] = _measure(model, a.hybrid_prompt, a.hybrid_batch, a.hybrid_new, a.steps, a.warmup, phases)
@@ -202,7 +223,8 @@ def run(a) -> int:
             if all(k in row.get(m, {}) for m in ("nidozen", "llama")):
                 row[ph + "_ratio"] = row["nidozen"][k] / row["llama"][k]
             for mine, others in (("telurax", ("nidozen", "llama")), ("surevik", ("telurax", "nidozen", "llama")),
-                                 ("gizilorn", ("surevik", "telurax", "nidozen", "llama"))):
+                                 ("gizilorn", ("surevik", "telurax", "nidozen", "llama")),
+                                 ("kulivik", ("surevik", "gizilorn", "telurax", "nidozen", "llama"))):
                 for other in others:
                     if all(k in row.get(m, {}) for m in (mine, other)):
                         row[f"{ph}_{mine}_over_{other}"] = row[mine][k] / row[other][k]

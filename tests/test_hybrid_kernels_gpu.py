@@ -601,3 +601,179 @@ def test_xielu(dt):
         want = torch.where(z > 0, ap * z * z + z / 2, an * (torch.exp(z) - 1 - z) + z / 2)
         torch.testing.assert_close(got.float().cpu(), want.float().to(dt).float(), **_tol(dt))
         torch.testing.assert_close(ref.xielu(y[:, 3:40], ap, an, dt).float(), got.float().cpu(), **_tol(dt))
+
+
+# ---- gated residual steps, token shift, attention pre-processing, linear attention with one decay per head ----
+class _Layout:
+    def __init__(self, cu, rs, slots, dev="cpu"):
+        self.cu_q, self.row_seq, self.state_slots = cu.to(dev), rs.to(dev), slots.to(dev)
+
+
+@pytest.mark.parametrize("dt", ACTS)
+@pytest.mark.parametrize("d", [64, 40, 37, 1024, 4096, 5000])
+@pytest.mark.parametrize("gated,post", [(True, True), (False, True), (True, False)])
+def test_gated_step(dt, d, gated, post):
+    """Widths of the vector form, of the scalar one (no multiple of four) and of rows too wide for the registers."""
+    g = torch.Generator().manual_seed(d)
+    T = 7
+    x, y = torch.randn(T, d, generator=g), torch.randn(T, d, generator=g)
+    wide = torch.randn(T, d + 12, generator=g)
+    w_out, w_in, mu = torch.rand(d, generator=g) + 0.5, torch.rand(d, generator=g) + 0.5, torch.rand(d, generator=g)
+    xd = x.to(DEV)
+    gate, gate_d = (wide[:, 4:4 + d], wide.to(DEV)[:, 4:4 + d]) if gated else (None, None)
+    ha, h32, _ = ops.gated_step(xd, y.to(DEV), gate_d, w_out.to(DEV) if post else None, w_in.to(DEV), 1e-5, dt, want_f32=True)
+    xr = x.clone()
+    want_a, want32, _ = ref.gated_step(xr, y, gate, w_out if post else None, w_in, 1e-5, dt, None, None, None)
+    torch.testing.assert_close(xd.cpu(), xr, atol=2e-5, rtol=2e-5)
+    torch.testing.assert_close(ha.float().cpu(), want_a.float(), **_tol(dt))
+    torch.testing.assert_close(h32.cpu(), want32, atol=2e-5, rtol=2e-5)
+    # the sum alone, and the norm alone
+    assert ops.gated_step(xd, y.to(DEV), None, None, None, 1e-5, dt) == (None, None, None)
+    torch.testing.assert_close(xd.cpu(), xr + y, atol=2e-5, rtol=2e-5)
+    before = xd.cpu()
+    h, _, _ = ops.gated_step(xd, None, None, None, w_in.to(DEV), 1e-5, torch.float32)
+    torch.testing.assert_close(xd.cpu(), before)
+    torch.testing.assert_close(h.cpu(), before * torch.rsqrt(before.pow(2).mean(-1, keepdim=True) + 1e-5) * w_in, atol=2e-5, rtol=2e-5)
+    # steps of one row per sequence: the shift in the same launch; a fresh sequence, a row without a slot, a padding row
+    cu, pos, rs = _seqs([1] * T, [0, 5, 9, 0, 1, 70, 3])
+    rs[6] = -1
+    slots = torch.tensor([3, 1, 7, 0, -1, 5, 2], dtype=torch.int32)
+    plane = torch.randn(9, d + 8, generator=g)
+    pd, pr = plane.to(DEV), plane.clone()
+    _, _, hs = ops.gated_step(xd, y.to(DEV), gate_d, w_out.to(DEV), w_in.to(DEV), 1e-5, dt, shift=ops.ShiftState(mu.to(DEV), pd[:, 4:4 + d]),
+                              lay=_Layout(cu, rs, slots, DEV), positions=pos.to(DEV))
+    xr = before.clone()
+    slots_r = slots.clone()
+    slots_r[6] = -1
+    _, _, want = ref.gated_step(xr, y, gate, w_out, w_in, 1e-5, dt, ops.ShiftState(mu, pr[:, 4:4 + d]), _Layout(cu, rs, slots_r), pos)
+    torch.testing.assert_close(hs.float().cpu(), want.float(), **_tol(dt))
+    torch.testing.assert_close(pd.cpu(), pr, atol=2e-5, rtol=2e-5)
+
+
+@pytest.mark.parametrize("dt", ACTS)
+@pytest.mark.parametrize("d", [64, 37, 2048])
+def test_token_shift(dt, d):
+    g = torch.Generator().manual_seed(d)
+    cu, pos, rs = _seqs([6, 2, 70, 1, 1, 1], [0, 33, 5, 0, 8, 4])
+    slots = torch.tensor([4, 0, 2, 1, 5, -1], dtype=torch.int32)
+    h, mu, plane = torch.randn(81, d, generator=g), torch.rand(d, generator=g), torch.randn(6, d + 4, generator=g)
+    pr, pd = plane.clone(), plane.to(DEV)
+    got = ops.token_shift(h.to(DEV), ops.ShiftState(mu.to(DEV), pd[:, :d]), _Layout(cu, rs, slots, DEV), pos.to(DEV), dt)
+    want = ref.token_shift(h, ops.ShiftState(mu, pr[:, :d]), _Layout(cu, rs, slots), pos, dt)
+    torch.testing.assert_close(got.float().cpu(), want.float(), **_tol(dt))
+    torch.testing.assert_close(pd.cpu(), pr)
+
+
+@pytest.mark.parametrize("dt", ACTS)
+@pytest.mark.parametrize("H,G,D,Dv,taps,norm,rot,pairs,temp,mix", [
+    (4, 2, 12, 10, 3, "whole", 0, False, (0.0, 1.0), 0.3), (3, 3, 16, 8, 0, "head", 16, True, (0.0, 1.0), 0.0),
+    (4, 1, 7, 5, 1, "", 6, False, (0.7, 4.0), 1.0), (8, 2, 128, 128, 4, "whole", 64, True, (0.3, 16.0), 0.6),
+    (2, 1, 70, 66, 6, "head", 8, False, (0.0, 1.0), 0.2), (32, 8, 128, 128, 2, "", 0, False, (0.0, 1.0), 0.0),
+    (64, 16, 256, 128, 3, "head", 2, True, (0.0, 1.0), 0.5)])
+def test_attn_prep(dt, H, G, D, Dv, taps, norm, rot, pairs, temp, mix):
+    """Portions longer and shorter than the convolution's reach, fresh and continued, single tokens, a row without a
+    slot, a padding row; up to more channels than 64 KB hold."""
+    g = torch.Generator().manual_seed(H * 100 + D)
+    lens, starts = [37, 2, 3, 1, 1, 1, 1], [0, 30, 0, 55, 0, 9, 4]
+    BSZ, MB = 16, 5
+    cu, pos, rs = _seqs(lens, starts)
+    T, C = int(cu[-1]), (H + G) * D + G * Dv
+    tables = torch.randperm(7 * MB, generator=g).to(torch.int32).view(7, MB)
+    where = torch.tensor([int(tables[b, p // BSZ]) * BSZ + p % BSZ for b, p in zip(rs.tolist(), pos.tolist())], dtype=torch.int32)
+    where[-1] = -1
+    rs_d = rs.clone()
+    rs_d[-1] = -1
+    slots = torch.tensor([3, 0, 5, 1, 6, -1, 2], dtype=torch.int32)
+    slots_r = slots.clone()
+    slots_r[6] = -1
+    qkv = torch.randn(T, C + 3, generator=g)
+    kc, vc = torch.randn(7 * MB, G, BSZ, D, generator=g).to(dt), torch.randn(7 * MB, G, BSZ, Dv, generator=g).to(dt)
+    conv = torch.randn(taps, C, generator=g) * 0.6 if taps else None
+    hist = max(0, taps - 1)
+    plane = torch.randn(7, hist * C + 8, generator=g)
+    nq, nk = (torch.rand(n, generator=g) + 0.5 for n in ((H * D, G * D) if norm == "whole" else (D, D)))
+    inv = torch.tensor([1e3 ** (-2.0 * j / rot) for j in range(rot // 2)], dtype=torch.float64) if rot else None
+    first = torch.randn(T, G * Dv + 2, generator=g) if mix else None
+    res = []
+    for dev, r_s, sl in (("cpu", rs, slots_r), (DEV, rs_d, slots)):
+        to = lambda t: t.clone().to(dev) if t is not None else None   # noqa: E731
+        k, v, st = to(kc), to(vc), to(plane)
+        q, saved = ops.attn_prep(to(qkv), to(pos), to(where), _Layout(cu, r_s, sl, dev), k, v, H, G, D, Dv, conv_w=to(conv),
+                                 conv_state=st[:, 4:4 + hist * C] if taps > 1 else None, norm=norm, q_norm=to(nq), k_norm=to(nk), eps=1e-5,
+                                 inv_freq=to(inv), rot_dims=rot, pairs=pairs, temperature=temp,
+                                 v_first=to(first)[:, :G * Dv] if mix else None, v_mix=mix, save_v=True)
+        res.append([t.float().cpu() for t in (q, saved, k, v, st)])
+    for i, (want, got) in enumerate(zip(*res)):
+        torch.testing.assert_close(got, want, **(_tol(dt) if i in (2, 3) else dict(atol=5e-5, rtol=5e-5)), msg=lambda m, i=i: f"{i}: {m}")
+
+
+@pytest.mark.parametrize("dt", ACTS)
+@pytest.mark.parametrize("H,G,D,Dv,chunk,window,keep,cap", [(4, 2, 32, 32, 0, 7, 3, 0.0), (6, 3, 48, 16, 0, 40, 50, 5.0), (3, 1, 16, 48, 0, 0, 0, 0.0),
+                                                            (5, 1, 7, 6, 0, 9, 1, 1.5), (4, 4, 128, 128, 33, 0, 18, 0.0), (2, 1, 24, 300, 0, 30, 16, 2.0)])
+def test_attention_with_kept_keys_distances_sinks_and_gates(dt, H, G, D, Dv, chunk, window, keep, cap):
+    g = torch.Generator().manual_seed(H * 100 + D)
+    lens, starts = [37, 70, 1, 1, 1], [0, 130, 55, 3, 199]
+    BSZ, MB = 16, 14
+    cu, pos, rs = _seqs(lens, starts)
+    T = int(cu[-1])
+    tables = torch.randperm(5 * MB, generator=g).to(torch.int32).view(5, MB)
+    q = torch.randn(T, H * D, generator=g)
+    kc, vc = (torch.randn(5 * MB, G, BSZ, D, generator=g) * 0.5).to(dt), (torch.randn(5 * MB, G, BSZ, Dv, generator=g) * 0.5).to(dt)
+    sinks, slopes = torch.randn(H, generator=g) * 2, torch.rand(H, generator=g) * 0.2
+    gates = torch.randn(T, H + 5, generator=g)
+    c = lambda t: t.to(DEV)   # noqa: E731
+    for opt in (dict(sinks=sinks), dict(slopes=slopes, out_scale=0.6), dict(sinks=sinks, slopes=slopes, gate=gates[:, 2:2 + H]), {}):
+        want = ref.attn_masked(q, kc, vc, tables, cu, pos, H, G, D, Dv, 0.2, chunk, window, torch.float32, cap, False, False, keep=keep, **opt)
+        dopt = {k: (c(gates)[:, 2:2 + H] if k == "gate" else c(v) if torch.is_tensor(v) else v) for k, v in opt.items()}
+        for portions, rows in ((0, 0), (2, 107)):
+            wide = torch.zeros(T, 5 + H * Dv + 3, dtype=dt, device=DEV)
+            got = ops.attn_masked(c(q), c(kc), c(vc), c(tables), c(cu), c(rs), c(pos), H, G, D, Dv, 0.2, chunk, window, dt, n_portions=portions,
+                                  portion_rows=rows, max_len=70, softcap=cap, keep=keep, out=wide[:, 5:5 + H * Dv], **dopt)
+            torch.testing.assert_close(got.float().cpu(), want, **(_tol(dt) if dt == torch.bfloat16 else dict(atol=5e-5, rtol=5e-5)))
+            assert not wide[:, :5].any() and not wide[:, 5 + H * Dv:].any()
+
+
+@pytest.mark.parametrize("H,D,Dv", [(2, 32, 32), (3, 24, 70), (1, 100, 8), (4, 128, 128), (2, 200, 130)])
+@pytest.mark.parametrize("long", [False, True])
+def test_lightning_scan_and_rownorm(H, D, Dv, long):
+    """Whole-portion scans and segmented ones (a portion of 300 rows), fresh and continued sequences, decays of 0 and 1."""
+    g = torch.Generator().manual_seed(D)
+    lens, starts = ([300, 2, 1], [7, 0, 3]) if long else ([6, 1, 2, 1], [0, 5, 3, 0])
+    cu, pos, _ = _seqs(lens, starts)
+    slots = torch.tensor([1, 3, 0, -1][:len(lens)], dtype=torch.int32)
+    T = int(cu[-1])
+    n = T if long else T - 1                       # (the row without a slot is left alone)
+    proj = torch.randn(T, 2 * H * D + 2 * H * Dv + 5, generator=g)
+    decay = torch.tensor([0.97, 0.0, 1.0, 0.5])[:H].contiguous()
+    plane = torch.randn(4, H * D * Dv + 4, generator=g) * 0.3
+    pr, pd = plane.clone(), plane.to(DEV)
+    want = ref.lightning_scan(proj, decay, pr[:, 4:], cu, pos, slots, H, D, Dv)
+    got = ops.lightning_scan(proj.to(DEV), decay.to(DEV), pd[:, 4:], cu.to(DEV), pos.to(DEV), slots.to(DEV), H, D, Dv, max_len=max(lens))
+    tol = dict(atol=1e-3, rtol=2e-4)
+    torch.testing.assert_close(got.cpu()[:n], want[:n], **tol)
+    torch.testing.assert_close(pd.cpu(), pr, **tol)
+    w, a = torch.rand(H * Dv, generator=g) + 0.5, 2 * H * D + H * Dv
+    for dt in ACTS:
+        wide = torch.zeros(T, H * Dv + 7, dtype=dt, device=DEV)
+        y = ops.rownorm_gate(want.to(DEV), w.to(DEV), proj.to(DEV)[:, a:a + H * Dv], 1e-5, dt, out=wide[:, 7:])
+        torch.testing.assert_close(y.float().cpu(), ref.rownorm_gate(want, w, proj[:, a:a + H * Dv], 1e-5, dt).float(), **_tol(dt))
+        assert not wide[:, :7].any()
+
+
+@pytest.mark.parametrize("n,top", [(5, 2), (12, 12), (70, 4), (33, 1)])
+def test_routing_by_the_softmax_over_the_chosen_logits(n, top):
+    g = torch.Generator().manual_seed(n)
+    z = torch.randn(40, n + 3, generator=g) * 3
+    z[0, 2:2 + n] -= 200.0                          # (far below zero, far apart: nothing underflows in the choice)
+    z[1, 2:2 + n] = torch.linspace(0, 400, n)
+    ids, w = ops.route_grouped(z.to(DEV)[:, 2:2 + n], None, top, 1, 1, 1.0, score="softmax_top")
+    ids_r, w_r = ref.route_grouped(z[:, 2:2 + n], None, top, 1, 1, 1.0, score="softmax_top")
+    assert torch.equal(ids.cpu(), ids_r)
+    torch.testing.assert_close(w.cpu(), w_r, atol=1e-6, rtol=1e-5)
+    torch.testing.assert_close(w.cpu().sum(-1), torch.ones(40), atol=1e-5, rtol=1e-5)
+
+
+def test_softcap():
+    x = torch.randn(33, 71, generator=torch.Generator().manual_seed(1)) * 20
+    got = ops.softcap_(x.to(DEV), 7.5)
+    torch.testing.assert_close(got.cpu(), 7.5 * torch.tanh(x / 7.5), atol=1e-5, rtol=1e-5)
