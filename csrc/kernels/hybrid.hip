@@ -920,6 +920,12 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
   const int pw0 = p0 + 16 * wave;                           // position of this wave's first row
   const int wave_rows = max(0, min(16, nrows - 16 * wave));
   const int wave_lo = first_key(pw0), wave_hi = pw0 + wave_rows - 1;
+  int row_pos[4], row_lo[4];                                // of the four rows whose scores this lane holds
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    row_pos[r] = 4 * lk + r < wave_rows ? pw0 + 4 * lk + r : -1;     // (rows past the portion see nothing)
+    row_lo[r] = first_key(pw0 + 4 * lk + r);
+  }
   // staging: a tile is 16 keys x D (x Dv) elements = 2 D (2 Dv) units of 8; a thread owns up to two of each
   constexpr int NVU = kTileMaxVT / 8;                       // value units of 8 columns per thread (16 keys x ncols / 8 in all)
   const int ku = D / 8, vu = ncols / 8;
@@ -998,9 +1004,9 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int row = 4 * lk + r;
-      const int prow = pw0 + row;
-      const bool valid = row < wave_rows && j <= prow && (j >= first_key(prow) || j < keep);
-      const float sraw = sacc[0][r] + sacc[1][r] - slope * static_cast<float>(prow - j);
+      const bool valid = j <= row_pos[r] && (j >= row_lo[r] || j < keep);
+      float sraw = sacc[0][r] + sacc[1][r];
+      if (slope != 0.f) sraw -= slope * static_cast<float>(row_pos[r] - j);     // (the same for the whole block)
       const float sv = valid ? (softcap > 0.f ? softcap * tanhf(sraw / softcap) : sraw) : -INFINITY;
       float mt = sv;
 #pragma unroll
