@@ -830,17 +830,38 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
 // of 16 query rows of ONE sequence and ONE query head; key / value tiles of 16 positions are staged
 // in LDS as fp32 once per block (16-byte loads, the next tile's loads in flight during the current
 // tile's products) and serve all 64 rows. Per key tile and wave:
-//   S = Q K^T   D/4 MFMAs (A: q[row l&15][d + (l>>4)], B: k[key l&15][d + (l>>4)]; S[row 4(l>>4)+r][key l&15])
+//   S = Q K^T   D/4 MFMAs (A: q[row l&15][d + 4(l>>4) + i], B: the same of k[key l&15], i = 0..3 one MFMA each: which
+//               coordinates meet in an MFMA is free as long as both operands agree; S[row 4(l>>4)+r][key l&15])
 //   masking per element (rows of a tile may lie in different chunks), online softmax per row
-//   (the 16 lanes of a row's keys reduce by shuffles), P through LDS into the A layout,
+//   (the maximum over the 16 lanes of a row's keys by rotations inside the DPP row, the sums once at the end), P through LDS into the A layout,
 //   O += P V    4 MFMAs per 16 value columns (B: v[key 4j + (l>>4)][col l&15]).
 // Row strides in LDS are padded so that the 16 rows of an operand fall into different banks.
 // The options of the row kernel (row strides, score cap, sink, value heads side by side) apply here too; the value
 // tile then holds nvh * Dv columns.
-// A wave holds up to 16 accumulator tiles (256 value columns; with 32 tiles, 512 columns in one launch, the kernel ran
+// A wave holds 8 or 16 accumulator tiles (128 or 256 value columns; with 32 tiles, 512 columns in one launch, the kernel ran
 // slower than two launches of 256 that each form the scores again). A block may use more than 64 KB of LDS (wide queries).
 constexpr int kTileMaxVT = 16;
 constexpr int kTileMaxLds = 160 * 1024;
+
+// Maximum over the 16 lanes of a DPP row (lanes 16 k .. 16 k + 15), in every one of them: rotations inside the row,
+// on the vector ALU.
+template <int N>
+LC_DEVICE float row_rotate(float v) {
+  const int b = __builtin_bit_cast(int, v);
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(b, b, 0x120 + N, 0xf, 0xf, false));   // row_ror:N
+}
+LC_DEVICE float row16_max(float v) {
+  v = fmaxf(v, row_rotate<8>(v));
+  v = fmaxf(v, row_rotate<4>(v));
+  v = fmaxf(v, row_rotate<2>(v));
+  return fmaxf(v, row_rotate<1>(v));
+}
+LC_DEVICE float row16_sum(float v) {
+  v += row_rotate<8>(v);
+  v += row_rotate<4>(v);
+  v += row_rotate<2>(v);
+  return v + row_rotate<1>(v);
+}
 
 LC_DEVICE int lds_stride(int n, int want) { return n + ((want - n % 32 + 32) % 32); }
 
@@ -881,7 +902,10 @@ LC_DEVICE void store_raw8(const Raw8<CF32>& r, float* dst) {
   }
 }
 
-template <bool CF32, bool AF32>
+// VT: accumulator tiles a wave holds (8: up to 128 value columns). WIDE: which column a lane's tile t holds is
+// the group-of-64's column 4 lr + t % 4 (else t * 16 + lr), so that a lane reads the values of four tiles with one
+// 16-byte access; the columns then come in groups of 64.
+template <bool CF32, bool AF32, int VT, bool WIDE>
 __global__ __launch_bounds__(256) void attn_tile_kernel(
     const float* __restrict__ q, const void* __restrict__ kc, const void* __restrict__ vc,
     const int32_t* __restrict__ block_tables, int MB, const int32_t* __restrict__ cu_q,
@@ -927,7 +951,7 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
     row_lo[r] = first_key(pw0 + 4 * lk + r);
   }
   // staging: a tile is 16 keys x D (x Dv) elements = 2 D (2 Dv) units of 8; a thread owns up to two of each
-  constexpr int NVU = kTileMaxVT / 8;                       // value units of 8 columns per thread (16 keys x ncols / 8 in all)
+  constexpr int NVU = VT / 8;                       // value units of 8 columns per thread (16 keys x ncols / 8 in all)
   const int ku = D / 8, vu = ncols / 8;
   int kkey[2], kcol[2], vkey[NVU], vcol[NVU], vhead[NVU], vin[NVU];
 #pragma unroll
@@ -945,19 +969,27 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
     vin[i] = vcol[i] % Dv;
   }
   Raw8<CF32> kr[2], vr[NVU];
-  auto fetch = [&](int j0) {
+  // Blocks of whole tiles: a tile's keys lie in one block, whose table entry is read a tile ahead.
+  const bool whole = BS % 16 == 0;
+  auto block_of = [&](int j0) { return whole && j0 <= hi ? table[j0 / BS] : 0; };
+  auto fetch = [&](int j0, int block) {
+    const int in_block = whole ? j0 % BS : 0;
+    auto plane_row = [&](int j, int key, int head) {        // row of the key's (value's) plane
+      const int blk = whole ? block : table[j / BS];
+      return (static_cast<size_t>(blk) * G + head) * BS + (whole ? in_block + key : j % BS);
+    };
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
       const int jk = j0 + kkey[i];
       const bool kon = kkey[i] >= 0 && jk <= hi;
-      const size_t krow = kon ? (static_cast<size_t>(table[jk / BS]) * G + g) * BS + jk % BS : 0;
+      const size_t krow = kon ? plane_row(jk, kkey[i], g) : 0;
       kr[i] = load_raw8<CF32>(kc, krow * k_ld + kcol[i], kon);
     }
 #pragma unroll
     for (int i = 0; i < NVU; ++i) {
       const int jv = j0 + vkey[i];
       const bool von = vkey[i] >= 0 && jv <= hi;
-      const size_t vrow = von ? (static_cast<size_t>(table[jv / BS]) * G + vhead[i]) * BS + jv % BS : 0;
+      const size_t vrow = von ? plane_row(jv, vkey[i], vhead[i]) : 0;
       vr[i] = load_raw8<CF32>(vc, vrow * v_ld + vin[i], von);
     }
   };
@@ -966,21 +998,22 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
   const float softcap = opt.softcap;
   const int keep = opt.keep;
   float m[4], l[4];
-  f32x4 o[kTileMaxVT];
+  f32x4 o[VT];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     m[r] = opt.sink ? sink0 : -INFINITY;
-    l[r] = opt.sink ? 1.f : 0.f;
+    l[r] = opt.sink && lr == 0 ? 1.f : 0.f;
   }
 #pragma unroll
-  for (int t = 0; t < kTileMaxVT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int t = 0; t < VT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
   const float* Qw = Qs + wave * 16 * DS;
   // tiles of the kept first keys, then from the first row's first key on (the same for the whole block)
   const int lo_tile = (first_key(p0) / 16) * 16;
   auto next_tile = [&](int j) { return j + 16 >= keep && j + 16 < lo_tile ? lo_tile : j + 16; };
   int jn = 0;
   int j0 = keep > 0 ? 0 : lo_tile;
-  fetch(j0);
+  fetch(j0, block_of(j0));
+  int ahead = block_of(next_tile(j0));
   for (; j0 <= hi; j0 = jn) {
     jn = next_tile(j0);
     __syncthreads();                                        // the previous tile has been consumed
@@ -991,11 +1024,23 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
     for (int i = 0; i < NVU; ++i)
       if (vkey[i] >= 0) store_raw8<CF32>(vr[i], Vs + vkey[i] * VS + vcol[i]);
     __syncthreads();
-    if (jn <= hi) fetch(jn);                                // in flight while this tile is computed
+    if (jn <= hi) {                                         // in flight while this tile is computed
+      fetch(jn, ahead);
+      ahead = block_of(next_tile(jn));
+    }
     const bool mine = wave_rows > 0 && j0 <= wave_hi && (j0 + 15 >= wave_lo || j0 < keep);     // wave-uniform
     if (!mine) continue;
     f32x4 sacc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};      // two chains keep the matrix pipe busy
-    for (int d = 0; d < D; d += 8) {
+    int d = 0;
+    for (; d + 16 <= D; d += 16) {                          // 16-byte reads: a lane's four numbers feed four MFMAs
+      const float4 qv = *reinterpret_cast<const float4*>(Qw + lr * DS + d + 4 * lk);
+      const float4 kv = *reinterpret_cast<const float4*>(Ks + lr * DS + d + 4 * lk);
+      sacc[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv.x, kv.x, sacc[0], 0, 0, 0);
+      sacc[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv.y, kv.y, sacc[1], 0, 0, 0);
+      sacc[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv.z, kv.z, sacc[0], 0, 0, 0);
+      sacc[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(qv.w, kv.w, sacc[1], 0, 0, 0);
+    }
+    if (d < D) {                                            // (D is a multiple of 8)
       sacc[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(Qw[lr * DS + d + lk], Ks[lr * DS + d + lk], sacc[0], 0, 0, 0);
       sacc[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(Qw[lr * DS + d + 4 + lk], Ks[lr * DS + d + 4 + lk], sacc[1], 0, 0, 0);
     }
@@ -1008,17 +1053,11 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
       float sraw = sacc[0][r] + sacc[1][r];
       if (slope != 0.f) sraw -= slope * static_cast<float>(row_pos[r] - j);     // (the same for the whole block)
       const float sv = valid ? (softcap > 0.f ? softcap * tanhf(sraw / softcap) : sraw) : -INFINITY;
-      float mt = sv;
-#pragma unroll
-      for (int off = 8; off > 0; off >>= 1) mt = fmaxf(mt, __shfl_xor(mt, off, 64));
-      const float mn = fmaxf(m[r], mt);
+      const float mn = fmaxf(m[r], row16_max(sv));
       const float base = mn == -INFINITY ? 0.f : mn;        // nothing visible yet: weights 0, no NaN
       const float pv = valid ? expf(sv - base) : 0.f;
       corr[r] = expf(m[r] - base);
-      float ps = pv;
-#pragma unroll
-      for (int off = 8; off > 0; off >>= 1) ps += __shfl_xor(ps, off, 64);
-      l[r] = l[r] * corr[r] + ps;
+      l[r] = l[r] * corr[r] + pv;                             // this lane's keys only: summed over the row at the end
       m[r] = mn;
       Ps[row * 17 + lr] = pv;
     }
@@ -1030,16 +1069,38 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
     float pa[4];
 #pragma unroll
     for (int j4 = 0; j4 < 4; ++j4) pa[j4] = Ps[lr * 17 + 4 * j4 + lk];
+    if constexpr (WIDE) {
 #pragma unroll
-    for (int t = 0; t < kTileMaxVT; ++t) {
-      if (t < nt) {
-        f32x4 acc = o[t];
+      for (int t = 0; t < VT; t += 4) {
+        if (t < nt) {
+          float4 vv[4];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) acc[r] *= corr[r];
+          for (int j4 = 0; j4 < 4; ++j4) vv[j4] = *reinterpret_cast<const float4*>(Vs + (4 * j4 + lk) * VS + t * 16 + 4 * lr);
 #pragma unroll
-        for (int j4 = 0; j4 < 4; ++j4)
-          acc = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[j4], Vs[(4 * j4 + lk) * VS + t * 16 + lr], acc, 0, 0, 0);
-        o[t] = acc;
+          for (int i = 0; i < 4; ++i)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) o[t + i][r] *= corr[r];
+#pragma unroll
+          for (int j4 = 0; j4 < 4; ++j4) {                  // four independent chains
+            o[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[j4], vv[j4].x, o[t], 0, 0, 0);
+            o[t + 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[j4], vv[j4].y, o[t + 1], 0, 0, 0);
+            o[t + 2] = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[j4], vv[j4].z, o[t + 2], 0, 0, 0);
+            o[t + 3] = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[j4], vv[j4].w, o[t + 3], 0, 0, 0);
+          }
+        }
+      }
+    } else {
+#pragma unroll
+      for (int t = 0; t < VT; ++t) {
+        if (t < nt) {
+          f32x4 acc = o[t];
+#pragma unroll
+          for (int r = 0; r < 4; ++r) acc[r] *= corr[r];
+#pragma unroll
+          for (int j4 = 0; j4 < 4; ++j4)
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[j4], Vs[(4 * j4 + lk) * VS + t * 16 + lr], acc, 0, 0, 0);
+          o[t] = acc;
+        }
       }
     }
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");     // P is read before the next tile overwrites it
@@ -1049,12 +1110,13 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int row = 4 * lk + r;
+    const float sum = row16_sum(l[r]);
     if (row >= wave_rows) continue;
     const size_t tok = static_cast<size_t>(row0) + 16 * wave + row;
-    const float fin = opt.out_scale * (opt.gate != nullptr ? sigmoidf_(opt.gate[tok * opt.ld_gate + h]) : 1.f) / l[r];
+    const float fin = opt.out_scale * (opt.gate != nullptr ? sigmoidf_(opt.gate[tok * opt.ld_gate + h]) : 1.f) / sum;
 #pragma unroll
-    for (int t = 0; t < kTileMaxVT; ++t)
-      if (t < nt) Act<AF32>::store(dst, tok * opt.o_row + static_cast<size_t>(h) * o_ld + o_col0 + t * 16 + lr, o[t][r] * fin);
+    for (int t = 0; t < VT; ++t)
+      if (t < nt) Act<AF32>::store(dst, tok * opt.o_row + static_cast<size_t>(h) * o_ld + o_col0 + (WIDE ? (t & ~3) * 16 + 4 * lr + (t & 3) : t * 16 + lr), o[t][r] * fin);
   }
 }
 
@@ -1607,22 +1669,35 @@ LC_EXPORT int lc_attn_tile(const void* q, const void* kc, const void* vc, int ca
   const dim3 grid((max_len + 63) / 64, H, n_seq), block(256);
   static LcDeviceOnce attr_once;
   attr_once.run([&] {
-#define LC_TILE_ATTR(C32, A32)                                                             \
-  (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_tile_kernel<C32, A32>),     \
+#define LC_TILE_ATTR(C32, A32, VT, W)                                                             \
+  (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_tile_kernel<C32, A32, VT, W>),     \
                             hipFuncAttributeMaxDynamicSharedMemorySize, kTileMaxLds)
-    LC_TILE_ATTR(true, true); LC_TILE_ATTR(true, false); LC_TILE_ATTR(false, true); LC_TILE_ATTR(false, false);
+#define LC_TILE_ATTRS(C32, A32)                                       \
+  LC_TILE_ATTR(C32, A32, 8, false); LC_TILE_ATTR(C32, A32, 8, true);  \
+  LC_TILE_ATTR(C32, A32, kTileMaxVT, false); LC_TILE_ATTR(C32, A32, kTileMaxVT, true)
+    LC_TILE_ATTRS(true, true); LC_TILE_ATTRS(true, false); LC_TILE_ATTRS(false, true); LC_TILE_ATTRS(false, false);
+#undef LC_TILE_ATTRS
 #undef LC_TILE_ATTR
   });
-#define LC_TILE(C32, A32)                                                                                       \
-  attn_tile_kernel<C32, A32><<<grid, block, lds, st>>>(                                                         \
+  const bool wide = NC % 64 == 0, small = NC <= 128;
+#define LC_TILE_K(C32, A32, VT, W)                                                                              \
+  attn_tile_kernel<C32, A32, VT, W><<<grid, block, lds, st>>>(                                                  \
       static_cast<const float*>(q), kc, vc, static_cast<const int32_t*>(block_tables), MB,                      \
       static_cast<const int32_t*>(cu_q), static_cast<const int32_t*>(positions), out, H, G, D, Dv, BS, scale,   \
       chunk, window, k_ld, v_ld, opt, vh0, nvh, o_ld, o_col0)
+#define LC_TILE(C32, A32)                                     \
+  do {                                                        \
+    if (small && wide) LC_TILE_K(C32, A32, 8, true);          \
+    else if (small) LC_TILE_K(C32, A32, 8, false);            \
+    else if (wide) LC_TILE_K(C32, A32, kTileMaxVT, true);     \
+    else LC_TILE_K(C32, A32, kTileMaxVT, false);              \
+  } while (0)
   if (cache_f32 && act_f32) LC_TILE(true, true);
   else if (cache_f32) LC_TILE(true, false);
   else if (act_f32) LC_TILE(false, true);
   else LC_TILE(false, false);
 #undef LC_TILE
+#undef LC_TILE_K
   LC_RETURN_LAST_ERROR();
 }
 

@@ -708,12 +708,13 @@ def test_attn_prep(dt, H, G, D, Dv, taps, norm, rot, pairs, temp, mix):
 
 
 @pytest.mark.parametrize("dt", ACTS)
+@pytest.mark.parametrize("BSZ", [16, 24])         # pages of whole tiles, and pages whose borders cut tiles
 @pytest.mark.parametrize("H,G,D,Dv,chunk,window,keep,cap", [(4, 2, 32, 32, 0, 7, 3, 0.0), (6, 3, 48, 16, 0, 40, 50, 5.0), (3, 1, 16, 48, 0, 0, 0, 0.0),
                                                             (5, 1, 7, 6, 0, 9, 1, 1.5), (4, 4, 128, 128, 33, 0, 18, 0.0), (2, 1, 24, 300, 0, 30, 16, 2.0)])
-def test_attention_with_kept_keys_distances_sinks_and_gates(dt, H, G, D, Dv, chunk, window, keep, cap):
+def test_attention_with_kept_keys_distances_sinks_and_gates(dt, BSZ, H, G, D, Dv, chunk, window, keep, cap):
     g = torch.Generator().manual_seed(H * 100 + D)
     lens, starts = [37, 70, 1, 1, 1], [0, 130, 55, 3, 199]
-    BSZ, MB = 16, 14
+    MB = 14
     cu, pos, rs = _seqs(lens, starts)
     T = int(cu[-1])
     tables = torch.randperm(5 * MB, generator=g).to(torch.int32).view(5, MB)
