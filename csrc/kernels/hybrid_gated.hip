@@ -259,7 +259,38 @@ struct PrepArgs {
   void* vc;
   float* q_out;
   int H, G, D, Dv, BS;
+  int T, per_xcd;                 // rows, rows per chiplet (neighbouring rows share their inputs, so they share an L2)
+  int vec;                        // every row of qkv, of the state and of the weights starts on a 16-byte border
 };
+
+// u[c] = sum_j w[j][c] src_j[c] over TAPS input rows (null: zeros), 4 channels per thread and access.
+template <int TAPS>
+LC_DEVICE void conv_rows4(const PrepArgs& a, const RowSeq& s, const float* st, int r, int C, float* u) {
+  const float* src[TAPS];
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) {
+    const int k = r - (TAPS - 1) + j;                // input row inside the portion, < 0: before it
+    src[j] = k >= 0 ? a.qkv + static_cast<size_t>(s.first + k) * a.ld
+                    : (s.fresh ? nullptr : st + static_cast<size_t>(k + TAPS - 1) * C);
+  }
+  for (int c = threadIdx.x * 4; c < C; c += 1024) {
+    float4 x[TAPS], w[TAPS];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      w[j] = *reinterpret_cast<const float4*>(a.conv_w + static_cast<size_t>(j) * C + c);
+      x[j] = src[j] != nullptr ? *reinterpret_cast<const float4*>(src[j] + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+    }
+    float4 y = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      y.x += w[j].x * x[j].x;
+      y.y += w[j].y * x[j].y;
+      y.z += w[j].z * x[j].z;
+      y.w += w[j].w * x[j].w;
+    }
+    *reinterpret_cast<float4*>(u + c) = y;
+  }
+}
 
 template <bool CF32>
 __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs a) {
@@ -269,8 +300,8 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs a) {
   const int nq = H * D, nk = G * D, nv = G * Dv, C = nq + nk + nv;
   float* u = lds;                                    // [C] the token's channels
   float* cs = u + C;                                 // [rot_dims] cos | sin
-  float* hr = cs + a.rot_dims;                       // [H + G] reciprocal norms per head
-  const int t0 = blockIdx.x;
+  const int t0 = (blockIdx.x & 7) * a.per_xcd + (blockIdx.x >> 3);   // (workgroups go round robin over the 8 chiplets)
+  if (t0 >= a.T) return;
   const int hist = a.taps > 1 ? a.taps - 1 : 0;
   RowSeq s{t0, 1, -1, true};
   int count = 1;
@@ -288,7 +319,15 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs a) {
     const int r = t - s.first;                       // row inside the portion
     const int pos = a.positions[t];
     const float* row = a.qkv + static_cast<size_t>(t) * a.ld;
-    if (a.taps > 0) {
+    if (a.vec && a.taps == 2) {
+      conv_rows4<2>(a, s, st, r, C, u);
+    } else if (a.vec && a.taps == 3) {
+      conv_rows4<3>(a, s, st, r, C, u);
+    } else if (a.vec && a.taps == 4) {
+      conv_rows4<4>(a, s, st, r, C, u);
+    } else if (a.vec && a.taps == 0) {
+      for (int c = threadIdx.x * 4; c < C; c += 1024) *reinterpret_cast<float4*>(u + c) = *reinterpret_cast<const float4*>(row + c);
+    } else if (a.taps > 0) {
       for (int c = threadIdx.x; c < C; c += 256) {
         float y = 0.f;
         for (int j = 0; j < a.taps; ++j) {
@@ -325,50 +364,49 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs a) {
       for (int i = threadIdx.x; i < nk; i += 256) u[nq + i] *= rk * a.kn[i];
       __syncthreads();
     } else if (a.norm == 2) {
-      for (int g = wave; g < H + G; g += 4) {        // q heads, then key heads, side by side
+      for (int g = wave; g < H + G; g += 4) {        // q heads, then key heads: a wave owns a head
+        float* head = u + g * D;
+        const float* w = g < H ? a.qn : a.kn;
         float ss = 0.f;
-        for (int i = lane; i < D; i += 64) ss += u[g * D + i] * u[g * D + i];
-        ss = wave_sum(ss);
-        if (lane == 0) hr[g] = 1.f / sqrtf(ss / static_cast<float>(D) + a.eps);
+        for (int i = lane; i < D; i += 64) ss += head[i] * head[i];
+        const float rn = 1.f / sqrtf(wave_sum(ss) / static_cast<float>(D) + a.eps);
+        for (int i = lane; i < D; i += 64) head[i] *= rn * w[i];
       }
       __syncthreads();
-      for (int i = threadIdx.x; i < nq + nk; i += 256) u[i] *= hr[i / D] * (i < nq ? a.qn[i % D] : a.kn[i % D]);
-      __syncthreads();
     }
-    auto turned = [&](int at, int i) {               // coordinate i of the head at u[at]
-      const float v = u[at + i];
+    auto turned = [&](const float* head, int i) {    // coordinate i of a head
+      const float v = head[i];
       if (i >= a.rot_dims) return v;
       if (a.pairs) {
-        const float c = cs[i >> 1], sn = cs[half + (i >> 1)], o = u[at + (i ^ 1)];
+        const float c = cs[i >> 1], sn = cs[half + (i >> 1)], o = head[i ^ 1];
         return (i & 1) ? v * c + o * sn : v * c - o * sn;
       }
       const int j = i < half ? i : i - half;
       const float c = cs[j], sn = cs[half + j];
-      return i < half ? v * c - u[at + i + half] * sn : v * c + u[at + i - half] * sn;
+      return i < half ? v * c - head[i + half] * sn : v * c + head[i - half] * sn;
     };
-    for (int i = threadIdx.x; i < nq; i += 256) {
-      const int c = i % D;
-      a.q_out[static_cast<size_t>(t) * nq + i] = turned(i - c, c) * temp;
-    }
+    for (int g = wave; g < H; g += 4)
+      for (int i = lane; i < D; i += 64) a.q_out[static_cast<size_t>(t) * nq + g * D + i] = turned(u + g * D, i) * temp;
     const int slot = a.slot_mapping[t];
     const size_t blk = slot >= 0 ? slot / a.BS : 0, off = slot >= 0 ? slot % a.BS : 0;
     typedef typename Act<CF32>::type cache_t;
     if (slot >= 0)
-      for (int i = threadIdx.x; i < nk; i += 256) {
-        const int g = i / D, c = i - g * D;
-        Act<CF32>::store(static_cast<cache_t*>(a.kc), ((blk * G + g) * a.BS + off) * D + c, turned(nq + g * D, c));
+      for (int g = wave; g < G; g += 4)
+        for (int i = lane; i < D; i += 64)
+          Act<CF32>::store(static_cast<cache_t*>(a.kc), ((blk * G + g) * a.BS + off) * D + i, turned(u + nq + g * D, i));
+    for (int g = wave; g < G; g += 4)
+      for (int i = lane; i < Dv; i += 64) {
+        const int at = g * Dv + i;
+        float v = u[nq + nk + at];
+        if (a.v_save != nullptr) a.v_save[static_cast<size_t>(t) * nv + at] = v;
+        if (a.v_first != nullptr) v = (1.f - a.lambda) * v + a.lambda * a.v_first[static_cast<size_t>(t) * a.ld_vf + at];
+        if (slot >= 0) Act<CF32>::store(static_cast<cache_t*>(a.vc), ((blk * G + g) * a.BS + off) * Dv + i, v);
       }
-    for (int i = threadIdx.x; i < nv; i += 256) {
-      float v = u[nq + nk + i];
-      if (a.v_save != nullptr) a.v_save[static_cast<size_t>(t) * nv + i] = v;
-      if (a.v_first != nullptr) v = (1.f - a.lambda) * v + a.lambda * a.v_first[static_cast<size_t>(t) * a.ld_vf + i];
-      const int g = i / Dv, c = i - g * Dv;
-      if (slot >= 0) Act<CF32>::store(static_cast<cache_t*>(a.vc), ((blk * G + g) * a.BS + off) * Dv + c, v);
-    }
     if (rr + 1 < count) __syncthreads();             // the next row reuses the buffers
   }
   if (hist > 0 && st != nullptr && t0 == s.first) {
-    // a thread owns a channel: it has read the old inputs above, and row j + rows is read before row j + 1 is written
+    __syncthreads();                                 // every thread has read the old inputs
+    // a thread owns a channel: row j + rows is read before row j + 1 is written
     for (int c = threadIdx.x; c < C; c += 256)
       for (int j = 0; j < hist; ++j) {
         const int k = s.rows - hist + j;
@@ -455,7 +493,7 @@ LC_EXPORT int lc_attn_prep(const void* qkv, int ld, const void* conv_w, int taps
   if (rot_dims < 0 || rot_dims > D || (rot_dims & 1) || (rot_dims > 0 && inv_freq == nullptr)) return -1;
   if ((t_coef != 0.f && !(t_every > 0.f)) || (v_first != nullptr && ld_vf < G * Dv)) return -1;
   constexpr size_t kMaxLds = 159 * 1024;             // (the block sums' scratch is static)
-  const size_t lds = static_cast<size_t>(C + rot_dims + H + G) * sizeof(float);
+  const size_t lds = static_cast<size_t>(C + rot_dims) * sizeof(float);
   if (lds > kMaxLds) return -2;
   static LcDeviceOnce attr_once;
   attr_once.run([&] {
@@ -470,9 +508,10 @@ LC_EXPORT int lc_attn_prep(const void* qkv, int ld, const void* conv_w, int taps
                    static_cast<const float*>(v_first), ld_vf, lambda, static_cast<float*>(v_save),
                    static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(cu_q),
                    static_cast<const int32_t*>(positions), static_cast<const int32_t*>(slots),
-                   static_cast<const int32_t*>(slot_mapping), kc, vc, static_cast<float*>(q_out), H, G, D, Dv, BS};
-  if (cache_f32) attn_prep_kernel<true><<<dim3(T), dim3(256), lds, st>>>(a);
-  else attn_prep_kernel<false><<<dim3(T), dim3(256), lds, st>>>(a);
+                   static_cast<const int32_t*>(slot_mapping), kc, vc, static_cast<float*>(q_out), H, G, D, Dv, BS, T, (T + 7) / 8,
+                   C % 4 == 0 && ld % 4 == 0 && state_stride % 4 == 0 && aligned16(qkv) && aligned16(conv_w) && aligned16(state)};
+  if (cache_f32) attn_prep_kernel<true><<<dim3(8 * ((T + 7) / 8)), dim3(256), lds, st>>>(a);
+  else attn_prep_kernel<false><<<dim3(8 * ((T + 7) / 8)), dim3(256), lds, st>>>(a);
   LC_RETURN_LAST_ERROR();
 }
 

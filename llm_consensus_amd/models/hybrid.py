@@ -452,7 +452,7 @@ class HybridConfig:
                     raise ValueError(f"{self.name}: layer {i}: linear attention takes heads, dim <= 256, vdim and a decay per head")
             if l.prepped and (l.keep_first < 0 or l.window < 0 or l.softcap < 0 or l.conv < 0 or not l.q_temp[1] > 0):
                 raise ValueError(f"{self.name}: layer {i}: window, kept keys, cap and taps are not negative, q_temp.every is positive")
-            if l.prepped and (l.vdim > 512 or l.channels + l.rot_dims + l.heads + l.kv_heads > ops.ATTN_PREP_MAX_FLOATS):
+            if l.prepped and (l.vdim > 512 or l.channels + l.rot_dims > ops.ATTN_PREP_MAX_FLOATS):
                 raise ValueError(f"{self.name}: layer {i}: the kernels take vdim <= 512 and q | k | v of at most "
                                  f"{ops.ATTN_PREP_MAX_FLOATS} channels")
             if (l.attends or l.type == "gla") and (l.heads <= 0 or l.dim <= 0 or l.vdim <= 0):

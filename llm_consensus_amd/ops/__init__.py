@@ -1681,7 +1681,7 @@ def token_shift(h: torch.Tensor, shift: ShiftState, lay, positions: torch.Tensor
     return hs
 
 
-ATTN_PREP_MAX_FLOATS = 159 * 1024 // 4      # a token's channels, angles and head norms in one block's LDS
+ATTN_PREP_MAX_FLOATS = 159 * 1024 // 4      # a token's channels and angles in one block's LDS
 
 
 def attn_prep(qkv: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Tensor, lay, k_cache: torch.Tensor,
@@ -1717,7 +1717,7 @@ def attn_prep(qkv: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Te
         raise ValueError("attn_prep: rot_dims / 2 fp64 frequencies are needed")
     if v_first is not None and (v_first.shape != (T, G * Dv) or v_first.dtype != torch.float32 or v_first.stride(1) != 1):
         raise ValueError("attn_prep: the values to mix in are fp32 [T, G * Dv]")
-    if C + rot_dims + H + G > ATTN_PREP_MAX_FLOATS:
+    if C + rot_dims > ATTN_PREP_MAX_FLOATS:
         raise ValueError("attn_prep: a token's channels exceed one block's LDS")
     if not qkv.is_cuda:
         return ref.attn_prep(qkv, positions, slot_mapping, lay, k_cache, v_cache, H, G, D, Dv, conv_w, conv_state, norm, q_norm,
