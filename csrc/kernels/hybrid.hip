@@ -21,20 +21,54 @@
 namespace {
 
 // ---------------------------------------------------------------- embedding -> fp32 stream (+ activation copy)
+// With a pair table (``pair.table``, the type of E): row (previous token * mul_prev + token * mul_cur) mod buckets of it is
+// added, row ``buckets`` for a sequence's first token. The previous token is the row before in the step's portion; for a
+// portion's first row it comes from the sequence's state slot, which the same wave then replaces by the portion's last token
+// (one thread reads, then writes: rows of a launch run in any order, and no other row touches the slot).
+struct PairTable {
+  const void* table;             // [buckets + 1, d], null: none
+  long long buckets, mul_prev, mul_cur;
+  int32_t* last;                 // [slots, stride] last token of each sequence
+  long long stride;
+  const int32_t* row_seq;
+  const int32_t* cu_q;
+  const int32_t* positions;
+  const int32_t* slots;
+};
+
 template <bool EF32, bool AF32>
 __global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const void* __restrict__ E, float* __restrict__ x,
                                   void* __restrict__ xa, int T, int d, int vocab, const int32_t* __restrict__ feed_tok,
                                   const int32_t* __restrict__ feed_rows, float scale,
-                                  const int32_t* __restrict__ positions, const double* __restrict__ inv_freq) {
+                                  const int32_t* __restrict__ positions, const double* __restrict__ inv_freq,
+                                  PairTable pair) {
   const int row = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
   const int lane = threadIdx.x & 63;
   if (row >= T) return;
-  int id = ids[row];
-  if (feed_rows != nullptr) {
-    const int src = feed_rows[row];
-    if (src >= 0) id = feed_tok[src];
+  auto token = [&](int r) {
+    int v = ids[r];
+    if (feed_rows != nullptr) {
+      const int src = feed_rows[r];
+      if (src >= 0) v = feed_tok[src];
+    }
+    return v < 0 ? 0 : (v >= vocab ? vocab - 1 : v);
+  };
+  const int id = token(row);
+  const typename Act<EF32>::type* e2 = nullptr;
+  if (pair.table != nullptr) {
+    long long at = pair.buckets;
+    if (lane == 0) {
+      const RowSeq s = row_sequence(row, pair.row_seq, pair.cu_q, pair.positions, pair.slots);
+      long long prev = -1;                          // (no state: as at a sequence's start)
+      if (row > s.first) prev = token(row - 1);
+      else if (!s.fresh) prev = pair.last[static_cast<size_t>(s.slot) * pair.stride];
+      if (row == s.first && s.slot >= 0) pair.last[static_cast<size_t>(s.slot) * pair.stride] = token(s.first + s.rows - 1);
+      if (prev >= 0) at = static_cast<long long>((static_cast<unsigned long long>(prev) * pair.mul_prev +
+                                                  static_cast<unsigned long long>(id) * pair.mul_cur) % static_cast<unsigned long long>(pair.buckets));
+    }
+    at = __shfl(at, 0, 64);
+    e2 = static_cast<const typename Act<EF32>::type*>(pair.table) + static_cast<size_t>(at) * d;
   }
-  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
   const typename Act<EF32>::type* e = static_cast<const typename Act<EF32>::type*>(E) + static_cast<size_t>(id) * d;
   typename Act<AF32>::type* a = static_cast<typename Act<AF32>::type*>(xa);
   // optional sinusoidal position vector: entry 2i = sin(p f_i), entry 2i + 1 = cos(p f_i), f an fp64 table
@@ -57,7 +91,8 @@ __global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const void* _
     return;
   }
   for (int c = lane; c < d; c += 64) {
-    const float v = Act<EF32>::load(e, c) * scale;
+    float v = Act<EF32>::load(e, c) * scale;
+    if (e2 != nullptr) v += Act<EF32>::load(e2, c);
     x[static_cast<size_t>(row) * d + c] = v;
     if (a != nullptr) Act<AF32>::store(a, static_cast<size_t>(row) * d + c, v);
   }
@@ -487,15 +522,29 @@ __global__ __launch_bounds__(256) void add_rmsnorm_kernel(float* __restrict__ x,
   for (int c = lane; c < d; c += LANES) Act<AF32>::store(a, static_cast<size_t>(row) * d + c, xr[c] * r * w[c]);
 }
 
-// act(gate) * up of y [T, 2n] = (gate | up); act: relu (kind 0) or silu (1).
-template <bool AF32>
-__global__ void glu_kernel(const float* __restrict__ y, void* __restrict__ out, long long total, int n, int kind) {
-  const long long i = static_cast<long long>(blockIdx.x) * blockDim.x + threadIdx.x;
+// act(gate) * up of y [T, 2n] = (gate | up); act: relu (kind 0), silu (1) or the tanh form of gelu (2). ``ldo``: row stride of
+// the output (it may be a column block of a wider matrix). V neighbouring columns per thread (4: 16-byte reads).
+LC_DEVICE float glu_act(float g, int kind) {
+  if (kind == 0) return fmaxf(g, 0.f);
+  if (kind == 1) return siluf_(g);
+  // 0.5 g (1 + tanh(a)) = g sigmoid(2 a), a = sqrt(2 / pi) (g + 0.044715 g^3)
+  return g * sigmoidf_(1.5957691216057308f * (g + 0.044715f * g * g * g));
+}
+
+template <bool AF32, int V>
+__global__ void glu_kernel(const float* __restrict__ y, void* __restrict__ out, long long total, int n, int kind, int ldo) {
+  const long long i = (static_cast<long long>(blockIdx.x) * blockDim.x + threadIdx.x) * V;
   if (i >= total) return;
   const long long t = i / n;
   const int c = static_cast<int>(i - t * n);
-  const float g = y[t * 2 * n + c], u = y[t * 2 * n + n + c];
-  Act<AF32>::store(static_cast<typename Act<AF32>::type*>(out), i, (kind == 0 ? fmaxf(g, 0.f) : siluf_(g)) * u);
+  const float* g = y + t * 2 * n + c;
+  if constexpr (V == 4) {
+    const float4 a = *reinterpret_cast<const float4*>(g), u = *reinterpret_cast<const float4*>(g + n);
+    store_act4<AF32>(out, static_cast<size_t>(t) * ldo + c, make_float4(glu_act(a.x, kind) * u.x, glu_act(a.y, kind) * u.y,
+                                                                       glu_act(a.z, kind) * u.z, glu_act(a.w, kind) * u.w));
+  } else {
+    Act<AF32>::store(static_cast<typename Act<AF32>::type*>(out), static_cast<size_t>(t) * ldo + c, glu_act(g[0], kind) * g[n]);
+  }
 }
 
 // ---------------------------------------------------------------- residual step with a Dynamic Tanh norm
@@ -704,7 +753,7 @@ __global__ __launch_bounds__(256) void rope_pairs_write_kernel(
 // columns, written from column ``o_col0`` on.
 // Further options (AttnOpts): a bias per unit of distance (slope of the head times p - j, taken off the scaled score
 // before the cap), a learned sink score per head, the first ``keep`` keys visible whatever the window or chunk, a gate
-// logit per (row, head) and a scale on the result, and the row stride of the output.
+// logit per (row, head) and a scale on the result, the row stride of the output, and key heads that share value heads.
 constexpr int kMaxVCols = 8;   // value width up to 512
 
 struct AttnOpts {
@@ -717,6 +766,7 @@ struct AttnOpts {
   int ld_gate;
   float out_scale;
   int o_row;                   // elements between the output rows of two tokens
+  int v_share;                 // neighbouring key heads that share one value head (the value plane has G / v_share heads)
 };
 
 template <bool CF32, bool AF32>
@@ -737,6 +787,7 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
   const int p = positions[t];
   if (seq < 0 || p < 0) return;             // the same for every wave of the block
   const int g = h / (H / G);
+  const int gv = g / opt.v_share, GV = G / opt.v_share;
   for (int d = lane; d < D; d += 64) qs[d] = q[(static_cast<size_t>(t) * H + h) * D + d] * scale;
   int lo = 0;
   if (chunk > 0) lo = (p / chunk) * chunk;
@@ -763,7 +814,7 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
     const int c = lane + 64 * i;
     const int vh = c / Dv;
     vcol[i] = c - vh * Dv;
-    voff[i] = vh0 < 0 ? 0 : (vh0 + vh - g) * BS;
+    voff[i] = vh0 < 0 ? 0 : (vh0 + vh - gv) * BS;
   }
   __syncthreads();
   for (int j0 = 0; j0 < nkeys; j0 += 64) {
@@ -771,9 +822,11 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
     const int j = jx < kept ? jx : lo + jx - kept;
     const bool valid = jx < nkeys;
     float s = -INFINITY;
-    int crow = 0;
+    int vrow = 0;
     if (valid) {
-      crow = (table[j / BS] * G + g) * BS + (j % BS);
+      const int blk = table[j / BS], off = j % BS;
+      const int crow = (blk * G + g) * BS + off;
+      vrow = (blk * GV + gv) * BS + off;
       const typename Act<CF32>::type* kr = kbase + static_cast<size_t>(crow) * k_ld;
       float dot = 0.f;
       if (!CF32 && D % 8 == 0 && k_ld % 8 == 0) {
@@ -798,7 +851,7 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
     l = l * corr + wave_sum(pj);
     m = mt;
     ps[lane] = pj;
-    rows[lane] = crow;
+    rows[lane] = vrow;
     __syncthreads();
     const int n = min(64, nkeys - j0);
 #pragma unroll
@@ -965,7 +1018,7 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
     const int u = threadIdx.x + 256 * i;
     vkey[i] = u < 16 * vu ? u / vu : -1;
     vcol[i] = (u % vu) * 8;                                 // column in the tile; inside its head: vin
-    vhead[i] = vh0 < 0 ? g : vh0 + vcol[i] / Dv;
+    vhead[i] = vh0 < 0 ? g / opt.v_share : vh0 + vcol[i] / Dv;
     vin[i] = vcol[i] % Dv;
   }
   Raw8<CF32> kr[2], vr[NVU];
@@ -974,22 +1027,22 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
   auto block_of = [&](int j0) { return whole && j0 <= hi ? table[j0 / BS] : 0; };
   auto fetch = [&](int j0, int block) {
     const int in_block = whole ? j0 % BS : 0;
-    auto plane_row = [&](int j, int key, int head) {        // row of the key's (value's) plane
+    auto plane_row = [&](int j, int key, int head, int heads) {        // row of the key's (value's) plane
       const int blk = whole ? block : table[j / BS];
-      return (static_cast<size_t>(blk) * G + head) * BS + (whole ? in_block + key : j % BS);
+      return (static_cast<size_t>(blk) * heads + head) * BS + (whole ? in_block + key : j % BS);
     };
 #pragma unroll
     for (int i = 0; i < 2; ++i) {
       const int jk = j0 + kkey[i];
       const bool kon = kkey[i] >= 0 && jk <= hi;
-      const size_t krow = kon ? plane_row(jk, kkey[i], g) : 0;
+      const size_t krow = kon ? plane_row(jk, kkey[i], g, G) : 0;
       kr[i] = load_raw8<CF32>(kc, krow * k_ld + kcol[i], kon);
     }
 #pragma unroll
     for (int i = 0; i < NVU; ++i) {
       const int jv = j0 + vkey[i];
       const bool von = vkey[i] >= 0 && jv <= hi;
-      const size_t vrow = von ? plane_row(jv, vkey[i], vhead[i]) : 0;
+      const size_t vrow = von ? plane_row(jv, vkey[i], vhead[i], G / opt.v_share) : 0;
       vr[i] = load_raw8<CF32>(vc, vrow * v_ld + vin[i], von);
     }
   };
@@ -1268,16 +1321,23 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const void* __restrict
 // ================================================================= launchers
 LC_EXPORT int lc_embed_rows(const void* ids, const void* E, int e_f32, void* x, void* xa, int act_f32, int T, int d,
                             int vocab, const void* feed_tok, const void* feed_rows, float scale, const void* positions,
-                            const void* inv_freq, hipStream_t st) {
+                            const void* inv_freq, const void* pair, long long buckets, long long mul_prev, long long mul_cur,
+                            void* last, long long last_stride, const void* row_seq, const void* cu_q, const void* slots,
+                            hipStream_t st) {
   if (T <= 0) return 0;
   if (d <= 0 || vocab <= 0 || (inv_freq != nullptr && (positions == nullptr || (d & 1)))) return -1;
+  if (pair != nullptr && (buckets <= 0 || mul_prev < 0 || mul_cur < 0 || last == nullptr || last_stride <= 0 || row_seq == nullptr ||
+                          cu_q == nullptr || positions == nullptr || slots == nullptr || inv_freq != nullptr))
+    return -1;
+  const PairTable pt{pair, buckets, mul_prev, mul_cur, static_cast<int32_t*>(last), last_stride, static_cast<const int32_t*>(row_seq),
+                     static_cast<const int32_t*>(cu_q), static_cast<const int32_t*>(positions), static_cast<const int32_t*>(slots)};
   const dim3 grid((T + 3) / 4), block(256);
 #define LC_EMB(E32, A32)                                                                                      \
   embed_rows_kernel<E32, A32><<<grid, block, 0, st>>>(static_cast<const int32_t*>(ids), E, static_cast<float*>(x), \
                                                       xa, T, d, vocab, static_cast<const int32_t*>(feed_tok), \
                                                       static_cast<const int32_t*>(feed_rows), scale,          \
                                                       static_cast<const int32_t*>(positions),                 \
-                                                      static_cast<const double*>(inv_freq))
+                                                      static_cast<const double*>(inv_freq), pt)
   if (e_f32 && act_f32) LC_EMB(true, true);
   else if (e_f32) LC_EMB(true, false);
   else if (act_f32) LC_EMB(false, true);
@@ -1463,12 +1523,18 @@ LC_EXPORT int lc_add_rmsnorm(void* x, const void* y, const void* w, float eps, v
   LC_RETURN_LAST_ERROR();
 }
 
-LC_EXPORT int lc_glu(const void* y, void* out, int act_f32, int T, int n, int kind, hipStream_t st) {
+LC_EXPORT int lc_glu(const void* y, void* out, int act_f32, int T, int n, int kind, int ldo, hipStream_t st) {
   if (T <= 0 || n <= 0) return 0;
+  if (kind < 0 || kind > 2 || ldo < n) return -1;
   const long long total = static_cast<long long>(T) * n;
-  const dim3 grid(static_cast<unsigned>((total + 255) / 256)), block(256);
-  if (act_f32) glu_kernel<true><<<grid, block, 0, st>>>(static_cast<const float*>(y), out, total, n, kind);
-  else glu_kernel<false><<<grid, block, 0, st>>>(static_cast<const float*>(y), out, total, n, kind);
+  const int v = n % 4 == 0 && ldo % 4 == 0 && aligned16(y) && aligned16(out) ? 4 : 1;
+  const dim3 grid(static_cast<unsigned>((total / v + 255) / 256)), block(256);
+#define LC_GLU(A32, V) glu_kernel<A32, V><<<grid, block, 0, st>>>(static_cast<const float*>(y), out, total, n, kind, ldo)
+  if (act_f32 && v == 4) LC_GLU(true, 4);
+  else if (act_f32) LC_GLU(true, 1);
+  else if (v == 4) LC_GLU(false, 4);
+  else LC_GLU(false, 1);
+#undef LC_GLU
   LC_RETURN_LAST_ERROR();
 }
 
@@ -1619,16 +1685,17 @@ LC_EXPORT int lc_attn_masked(const void* q, const void* kc, const void* vc, int 
                              int MB, const void* row_seq, const void* positions, void* out, int act_f32, int T, int H,
                              int G, int D, int Dv, int BS, float scale, int chunk, int window, int k_ld, int v_ld,
                              float softcap, int sink, const void* sinks, const void* slopes, int keep, const void* gate,
-                             int ld_gate, float out_scale, int o_row, int vh0, int nvh, int o_ld, int o_col0, int vz,
+                             int ld_gate, float out_scale, int o_row, int v_share, int vh0, int nvh, int o_ld, int o_col0, int vz,
                              hipStream_t st) {
   if (T <= 0) return 0;
   if (H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || BS <= 0 || MB <= 0 || vz <= 0 || vz > 65535) return -1;
   // ``vz`` groups of nvh value heads each, one per block along z (vz = 1 unless value heads are named)
   if (nvh <= 0 || nvh * Dv > 64 * kMaxVCols || (vh0 < 0 && (nvh != 1 || vz != 1)) || (vh0 >= 0 && vh0 + vz * nvh > G)) return -1;
   if (k_ld < D || v_ld < Dv || o_col0 < 0 || o_ld < o_col0 + vz * nvh * Dv || softcap < 0.f) return -1;
+  if (v_share <= 0 || G % v_share || (v_share > 1 && vh0 >= 0)) return -1;
   if (keep < 0 || (gate != nullptr && ld_gate < H) || o_row < H * o_ld || (sinks != nullptr && !sink)) return -1;
   const AttnOpts opt{softcap, sink, static_cast<const float*>(sinks), static_cast<const float*>(slopes), keep,
-                     static_cast<const float*>(gate), ld_gate, out_scale, o_row};
+                     static_cast<const float*>(gate), ld_gate, out_scale, o_row, v_share};
   const size_t lds = 4 * static_cast<size_t>(D + 128) * sizeof(float);
   if (lds > 64 * 1024) return -1;
   const dim3 grid(T, (H + 3) / 4, vz), block(256);
@@ -1651,15 +1718,16 @@ LC_EXPORT int lc_attn_tile(const void* q, const void* kc, const void* vc, int ca
                            int MB, const void* cu_q, const void* positions, void* out, int act_f32, int n_seq,
                            int max_len, int H, int G, int D, int Dv, int BS, float scale, int chunk, int window,
                            int k_ld, int v_ld, float softcap, int sink, const void* sinks, const void* slopes, int keep,
-                           const void* gate, int ld_gate, float out_scale, int o_row, int vh0, int nvh, int o_ld,
+                           const void* gate, int ld_gate, float out_scale, int o_row, int v_share, int vh0, int nvh, int o_ld,
                            int o_col0, hipStream_t st) {
   if (n_seq <= 0 || max_len <= 0) return 0;
   if (H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || BS <= 0 || MB <= 0) return -1;
   if (nvh <= 0 || (vh0 < 0 && nvh != 1) || (vh0 >= 0 && vh0 + nvh > G)) return -1;
   if (k_ld < D || v_ld < Dv || o_col0 < 0 || o_ld < o_col0 + nvh * Dv || softcap < 0.f) return -1;
+  if (v_share <= 0 || G % v_share || (v_share > 1 && vh0 >= 0)) return -1;
   if (keep < 0 || (gate != nullptr && ld_gate < H) || o_row < H * o_ld || (sinks != nullptr && !sink)) return -1;
   const AttnOpts opt{softcap, sink, static_cast<const float*>(sinks), static_cast<const float*>(slopes), keep,
-                     static_cast<const float*>(gate), ld_gate, out_scale, o_row};
+                     static_cast<const float*>(gate), ld_gate, out_scale, o_row, v_share};
   const int NC = nvh * Dv;
   // (16-byte loads of the staged tiles: rows and column blocks start on 16-byte borders)
   if (D % 8 || Dv % 8 || NC % 16 || NC > 16 * kTileMaxVT || D > 256 || k_ld % 8 || v_ld % 8) return -2;

@@ -12,42 +12,15 @@
 
 namespace {
 
-// Where a row's sequence starts and which state it owns.
-struct RowSeq {
-  int first, rows;               // row range of the step
-  int slot;                      // < 0: none
-  bool fresh;                    // starts at position 0 (or has no state): zeros before it
-};
-
-LC_DEVICE RowSeq row_sequence(int t, const int32_t* __restrict__ row_seq, const int32_t* __restrict__ cu_q,
-                              const int32_t* __restrict__ positions, const int32_t* __restrict__ slots) {
-  RowSeq r{t, 1, -1, true};
-  const int b = row_seq[t];
-  if (b < 0) return r;
-  r.first = cu_q[b];
-  r.rows = cu_q[b + 1] - r.first;
-  r.slot = slots[b];
-  r.fresh = r.slot < 0 || positions[r.first] == 0;
-  return r;
-}
-
 // ---------------------------------------------------------------- residual step with a gate and two norms
 // With y [T, d]: v = y * sigmoid(gate) (gate given: logits, row stride ld_gate), then rms-normed times w_out (w_out
 // given), x += v. With w_in: h = x / sqrt(mean(x^2) + eps) * w_in, written to ``ha`` in the activation type and, when
 // given, to ``h32``. With ``mu`` (steps whose sequences all have ONE row): ``hs`` = h + (h' - h) * mu in the
-// activation type, h' the sequence's stored row (zeros at position 0), and h becomes the stored row.
+// activation type, h' the sequence's stored row (zeros at position 0), and h becomes the stored row. With ``w_in2``: ``ha2`` =
+// x / sqrt(mean(x^2) + eps) * w_in2 beside it (two sublayers that read the same stream through norms of their own).
 // A block per row. Rows of up to 4 * 256 * kStepVec coordinates whose pieces are 16-byte aligned (VEC) stay in registers
 // between the sums; others are read again.
 constexpr int kStepVec = 4;
-
-template <bool AF32>
-LC_DEVICE void store_act4(void* p, size_t i, const float4& v) {
-  if (AF32) {
-    *reinterpret_cast<float4*>(static_cast<float*>(p) + i) = v;
-  } else {
-    *reinterpret_cast<uint2*>(static_cast<bf16_t*>(p) + i) = make_uint2(pack_bf16x2(v.x, v.y), pack_bf16x2(v.z, v.w));
-  }
-}
 
 LC_DEVICE float4 shift4(const float4& h, const float4& p, const float4& m) {
   return make_float4(h.x + (p.x - h.x) * m.x, h.y + (p.y - h.y) * m.y, h.z + (p.z - h.z) * m.z, h.w + (p.w - h.w) * m.w);
@@ -63,6 +36,8 @@ struct StepArgs {
   float eps;
   void* ha;
   float* h32;
+  const float* w_in2;            // a second norm of the same row (null: none)
+  void* ha2;
   // the shift of single-row sequences
   const float* mu;
   float* state;
@@ -139,6 +114,10 @@ __global__ __launch_bounds__(256) void gated_step_kernel(StepArgs a) {
         const float4 w = reinterpret_cast<const float4*>(a.w_in)[c];
         const float4 h = make_float4(xv[i].x * r2 * w.x, xv[i].y * r2 * w.y, xv[i].z * r2 * w.z, xv[i].w * r2 * w.w);
         store_act4<AF32>(a.ha, row + 4 * c, h);
+        if (a.w_in2 != nullptr) {
+          const float4 w2 = reinterpret_cast<const float4*>(a.w_in2)[c];
+          store_act4<AF32>(a.ha2, row + 4 * c, make_float4(xv[i].x * r2 * w2.x, xv[i].y * r2 * w2.y, xv[i].z * r2 * w2.z, xv[i].w * r2 * w2.w));
+        }
         if (a.h32 != nullptr) reinterpret_cast<float4*>(a.h32 + row)[c] = h;
         if (a.mu != nullptr) {
           float4 p = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -174,6 +153,7 @@ __global__ __launch_bounds__(256) void gated_step_kernel(StepArgs a) {
     for (int c = threadIdx.x; c < d; c += 256) {      // (a thread reads what it wrote itself)
       const float h = a.x[row + c] * r2 * a.w_in[c];
       Act<AF32>::store(static_cast<act_t*>(a.ha), row + c, h);
+      if (a.w_in2 != nullptr) Act<AF32>::store(static_cast<act_t*>(a.ha2), row + c, a.x[row + c] * r2 * a.w_in2[c]);
       if (a.h32 != nullptr) a.h32[row + c] = h;
       if (a.mu != nullptr) {
         const float p = fresh ? 0.f : prev[c];
@@ -230,20 +210,18 @@ __global__ __launch_bounds__(256) void token_shift_kernel(const float* __restric
 //     i + rot_dims / 2) by position * inv_freq[i] (angles fp64);
 //   temperature: q *= 1 + coef * ln(floor((p + 1) / every) + 1);
 //   value mix: v <- (1 - lambda) v + lambda v_first[t]; before it v is written to v_save when given.
-// q goes to q_out [T, H*D] fp32, k and v to the paged planes [blocks, G, BS, D] / [blocks, G, BS, Dv].
+// q goes to q_out [T, H*D] fp32, k and v to the paged planes [blocks, G, BS, D] / [blocks, G, BS, Dv]. With ``maps`` > 1 a head
+// has several query / key maps over the same values: H and G count the maps of all heads (head by head), GV = G / maps value
+// heads; the queries leave in the order (key/value head, map, head of the group), so that those of one key head are neighbours.
 struct PrepArgs {
-  const float* qkv;
-  int ld;
-  const float* conv_w;
-  int taps;                       // 0: no convolution
-  float* state;
-  long long state_stride;
+  ConvIn in;                      // q | k | v and their convolution over time
   int norm;
   const float* qn;
   const float* kn;
   float eps;
   const double* inv_freq;
   int rot_dims, pairs;
+  float rot_mag;                  // factor on cosine and sine
   float t_coef;                   // 0: no temperature
   double t_every;
   const float* v_first;
@@ -258,98 +236,44 @@ struct PrepArgs {
   void* kc;
   void* vc;
   float* q_out;
-  int H, G, D, Dv, BS;
+  int H, G, GV, D, Dv, BS;
+  int maps;                       // G / GV key heads per value head
   int T, per_xcd;                 // rows, rows per chiplet (neighbouring rows share their inputs, so they share an L2)
-  int vec;                        // every row of qkv, of the state and of the weights starts on a 16-byte border
 };
-
-// u[c] = sum_j w[j][c] src_j[c] over TAPS input rows (null: zeros), 4 channels per thread and access.
-template <int TAPS>
-LC_DEVICE void conv_rows4(const PrepArgs& a, const RowSeq& s, const float* st, int r, int C, float* u) {
-  const float* src[TAPS];
-#pragma unroll
-  for (int j = 0; j < TAPS; ++j) {
-    const int k = r - (TAPS - 1) + j;                // input row inside the portion, < 0: before it
-    src[j] = k >= 0 ? a.qkv + static_cast<size_t>(s.first + k) * a.ld
-                    : (s.fresh ? nullptr : st + static_cast<size_t>(k + TAPS - 1) * C);
-  }
-  for (int c = threadIdx.x * 4; c < C; c += 1024) {
-    float4 x[TAPS], w[TAPS];
-#pragma unroll
-    for (int j = 0; j < TAPS; ++j) {
-      w[j] = *reinterpret_cast<const float4*>(a.conv_w + static_cast<size_t>(j) * C + c);
-      x[j] = src[j] != nullptr ? *reinterpret_cast<const float4*>(src[j] + c) : make_float4(0.f, 0.f, 0.f, 0.f);
-    }
-    float4 y = make_float4(0.f, 0.f, 0.f, 0.f);
-#pragma unroll
-    for (int j = 0; j < TAPS; ++j) {
-      y.x += w[j].x * x[j].x;
-      y.y += w[j].y * x[j].y;
-      y.z += w[j].z * x[j].z;
-      y.w += w[j].w * x[j].w;
-    }
-    *reinterpret_cast<float4*>(u + c) = y;
-  }
-}
 
 template <bool CF32>
 __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs a) {
   extern __shared__ float lds[];
   __shared__ float red[16];
-  const int H = a.H, G = a.G, D = a.D, Dv = a.Dv;
-  const int nq = H * D, nk = G * D, nv = G * Dv, C = nq + nk + nv;
+  const int H = a.H, G = a.G, GV = a.GV, D = a.D, Dv = a.Dv;
+  const int nq = H * D, nk = G * D, nv = GV * Dv, C = nq + nk + nv;
   float* u = lds;                                    // [C] the token's channels
   float* cs = u + C;                                 // [rot_dims] cos | sin
   const int t0 = (blockIdx.x & 7) * a.per_xcd + (blockIdx.x >> 3);   // (workgroups go round robin over the 8 chiplets)
   if (t0 >= a.T) return;
-  const int hist = a.taps > 1 ? a.taps - 1 : 0;
+  const int hist = a.in.taps > 1 ? a.in.taps - 1 : 0;
   RowSeq s{t0, 1, -1, true};
   int count = 1;
   if (hist > 0) {
     s = row_sequence(t0, a.row_seq, a.cu_q, a.positions, a.slots);
-    const int r = t0 - s.first;
-    if (r > 0 && r < hist) return;                   // served by the portion's first row
-    if (r == 0) count = min(s.rows, hist);
+    count = conv_rows_of_block(t0, s, hist);
+    if (count == 0) return;                          // served by the portion's first row
   }
-  float* st = s.slot >= 0 ? a.state + static_cast<size_t>(s.slot) * a.state_stride : nullptr;
+  float* st = s.slot >= 0 ? a.in.state + static_cast<size_t>(s.slot) * a.in.state_stride : nullptr;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int half = a.rot_dims >> 1;
   for (int rr = 0; rr < count; ++rr) {
     const int t = t0 + rr;
-    const int r = t - s.first;                       // row inside the portion
     const int pos = a.positions[t];
-    const float* row = a.qkv + static_cast<size_t>(t) * a.ld;
-    if (a.vec && a.taps == 2) {
-      conv_rows4<2>(a, s, st, r, C, u);
-    } else if (a.vec && a.taps == 3) {
-      conv_rows4<3>(a, s, st, r, C, u);
-    } else if (a.vec && a.taps == 4) {
-      conv_rows4<4>(a, s, st, r, C, u);
-    } else if (a.vec && a.taps == 0) {
-      for (int c = threadIdx.x * 4; c < C; c += 1024) *reinterpret_cast<float4*>(u + c) = *reinterpret_cast<const float4*>(row + c);
-    } else if (a.taps > 0) {
-      for (int c = threadIdx.x; c < C; c += 256) {
-        float y = 0.f;
-        for (int j = 0; j < a.taps; ++j) {
-          const int k = r - hist + j;                // input row inside the portion, < 0: before it
-          float in = 0.f;
-          if (k >= 0) in = a.qkv[static_cast<size_t>(s.first + k) * a.ld + c];
-          else if (!s.fresh) in = st[static_cast<size_t>(k + hist) * C + c];
-          y += a.conv_w[static_cast<size_t>(j) * C + c] * in;
-        }
-        u[c] = y;
-      }
-    } else {
-      for (int c = threadIdx.x; c < C; c += 256) u[c] = row[c];
-    }
+    conv_token<false>(a.in, s, st, t - s.first, u);
     for (int j = threadIdx.x; j < half; j += 256) {
       constexpr double kTwoPi = 6.283185307179586476925286766559;
       double ang = static_cast<double>(pos) * a.inv_freq[j];
       ang -= kTwoPi * rint(ang / kTwoPi);
       float sn, cn;
       sincosf(static_cast<float>(ang), &sn, &cn);
-      cs[j] = cn;
-      cs[half + j] = sn;
+      cs[j] = cn * a.rot_mag;
+      cs[half + j] = sn * a.rot_mag;
     }
     __syncthreads();
     float temp = 1.f;
@@ -385,8 +309,13 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs a) {
       const float c = cs[j], sn = cs[half + j];
       return i < half ? v * c - head[i + half] * sn : v * c + head[i - half] * sn;
     };
-    for (int g = wave; g < H; g += 4)
-      for (int i = lane; i < D; i += 64) a.q_out[static_cast<size_t>(t) * nq + g * D + i] = turned(u + g * D, i) * temp;
+    const int rep = H / G;
+    for (int g = wave; g < H; g += 4) {
+      // (several maps per head: the queries of one key head lie side by side)
+      const int m = g % a.maps, qh = g / a.maps;
+      const int at = ((qh / rep) * a.maps + m) * rep + qh % rep;
+      for (int i = lane; i < D; i += 64) a.q_out[static_cast<size_t>(t) * nq + at * D + i] = turned(u + g * D, i) * temp;
+    }
     const int slot = a.slot_mapping[t];
     const size_t blk = slot >= 0 ? slot / a.BS : 0, off = slot >= 0 ? slot % a.BS : 0;
     typedef typename Act<CF32>::type cache_t;
@@ -394,27 +323,19 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs a) {
       for (int g = wave; g < G; g += 4)
         for (int i = lane; i < D; i += 64)
           Act<CF32>::store(static_cast<cache_t*>(a.kc), ((blk * G + g) * a.BS + off) * D + i, turned(u + nq + g * D, i));
-    for (int g = wave; g < G; g += 4)
+    for (int g = wave; g < GV; g += 4)
       for (int i = lane; i < Dv; i += 64) {
         const int at = g * Dv + i;
         float v = u[nq + nk + at];
         if (a.v_save != nullptr) a.v_save[static_cast<size_t>(t) * nv + at] = v;
         if (a.v_first != nullptr) v = (1.f - a.lambda) * v + a.lambda * a.v_first[static_cast<size_t>(t) * a.ld_vf + at];
-        if (slot >= 0) Act<CF32>::store(static_cast<cache_t*>(a.vc), ((blk * G + g) * a.BS + off) * Dv + i, v);
+        if (slot >= 0) Act<CF32>::store(static_cast<cache_t*>(a.vc), ((blk * GV + g) * a.BS + off) * Dv + i, v);
       }
     if (rr + 1 < count) __syncthreads();             // the next row reuses the buffers
   }
   if (hist > 0 && st != nullptr && t0 == s.first) {
     __syncthreads();                                 // every thread has read the old inputs
-    // a thread owns a channel: row j + rows is read before row j + 1 is written
-    for (int c = threadIdx.x; c < C; c += 256)
-      for (int j = 0; j < hist; ++j) {
-        const int k = s.rows - hist + j;
-        float in = 0.f;
-        if (k >= 0) in = a.qkv[static_cast<size_t>(s.first + k) * a.ld + c];
-        else if (!s.fresh) in = st[static_cast<size_t>(k + hist) * C + c];
-        st[static_cast<size_t>(j) * C + c] = in;
-      }
+    conv_keep(a.in, s, st);
   }
 }
 
@@ -425,29 +346,29 @@ __global__ void softcap_kernel(float* __restrict__ x, long long n, float cap) {
   if (i < n) x[i] = cap * tanhf(x[i] / cap);
 }
 
-bool aligned16(const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; }
-
 }  // namespace
 
 // ================================================================= launchers
 LC_EXPORT int lc_gated_step(void* x, const void* y, const void* gate, int ld_gate, const void* w_out, const void* w_in,
-                            float eps, void* ha, void* h32, int act_f32, const void* mu, void* state,
+                            float eps, void* ha, void* h32, const void* w_in2, void* ha2, int act_f32, const void* mu, void* state,
                             long long state_stride, const void* row_seq, const void* positions, const void* slots, void* hs,
                             int T, int d, hipStream_t st) {
   if (T <= 0) return 0;
   if (d <= 0 || (y == nullptr && w_in == nullptr) || (w_in != nullptr && ha == nullptr)) return -1;
   if (gate != nullptr && (y == nullptr || ld_gate < d)) return -1;
+  if (w_in2 != nullptr && (w_in == nullptr || ha2 == nullptr)) return -1;
   if (mu != nullptr && (w_in == nullptr || hs == nullptr || state == nullptr || row_seq == nullptr || positions == nullptr ||
                         slots == nullptr || state_stride < d))
     return -1;
   const StepArgs a{static_cast<float*>(x), static_cast<const float*>(y), static_cast<const float*>(gate), ld_gate,
                    static_cast<const float*>(w_out), static_cast<const float*>(w_in), eps, ha, static_cast<float*>(h32),
+                   static_cast<const float*>(w_in2), ha2,
                    static_cast<const float*>(mu), static_cast<float*>(state), state_stride,
                    static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(positions),
                    static_cast<const int32_t*>(slots), hs, d};
   const bool vec = d % 4 == 0 && d <= 4 * 256 * kStepVec && ld_gate % 4 == 0 && state_stride % 4 == 0 && aligned16(x) &&
                    aligned16(y) && aligned16(gate) && aligned16(w_out) && aligned16(w_in) && aligned16(ha) &&
-                   aligned16(h32) && aligned16(mu) && aligned16(state) && aligned16(hs);
+                   aligned16(h32) && aligned16(w_in2) && aligned16(ha2) && aligned16(mu) && aligned16(state) && aligned16(hs);
 #define LC_GS(A32, V) gated_step_kernel<A32, V><<<dim3(T), dim3(256), 0, st>>>(a)
   if (act_f32 && vec) LC_GS(true, true);
   else if (act_f32) LC_GS(true, false);
@@ -478,20 +399,21 @@ LC_EXPORT int lc_token_shift(const void* h, const void* mu, void* state, long lo
 
 LC_EXPORT int lc_attn_prep(const void* qkv, int ld, const void* conv_w, int taps, void* state, long long state_stride,
                            int norm, const void* qn, const void* kn, float eps, const void* inv_freq, int rot_dims, int pairs,
-                           float t_coef, float t_every, const void* v_first, int ld_vf, float lambda, void* v_save,
+                           float rot_mag, int maps, float t_coef, float t_every, const void* v_first, int ld_vf, float lambda, void* v_save,
                            const void* row_seq, const void* cu_q, const void* positions, const void* slots,
                            const void* slot_mapping, void* kc, void* vc, int cache_f32, void* q_out, int T, int H, int G,
                            int D, int Dv, int BS, hipStream_t st) {
   if (T <= 0) return 0;
   if (H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || BS <= 0 || kc == nullptr || vc == nullptr || q_out == nullptr) return -1;
-  const int C = (H + G) * D + G * Dv;
+  if (maps <= 0 || G % maps) return -1;
+  const int GV = G / maps, C = (H + G) * D + GV * Dv;
   if (ld < C || taps < 0 || norm < 0 || norm > 2 || (norm != 0 && (qn == nullptr || kn == nullptr))) return -1;
   if (taps > 0 && conv_w == nullptr) return -1;
   if (taps > 1 && (state == nullptr || state_stride < static_cast<long long>(taps - 1) * C || row_seq == nullptr ||
                    cu_q == nullptr || slots == nullptr))
     return -1;
   if (rot_dims < 0 || rot_dims > D || (rot_dims & 1) || (rot_dims > 0 && inv_freq == nullptr)) return -1;
-  if ((t_coef != 0.f && !(t_every > 0.f)) || (v_first != nullptr && ld_vf < G * Dv)) return -1;
+  if ((t_coef != 0.f && !(t_every > 0.f)) || (v_first != nullptr && ld_vf < GV * Dv)) return -1;
   constexpr size_t kMaxLds = 159 * 1024;             // (the block sums' scratch is static)
   const size_t lds = static_cast<size_t>(C + rot_dims) * sizeof(float);
   if (lds > kMaxLds) return -2;
@@ -502,14 +424,15 @@ LC_EXPORT int lc_attn_prep(const void* qkv, int ld, const void* conv_w, int taps
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_prep_kernel<false>),
                               hipFuncAttributeMaxDynamicSharedMemorySize, static_cast<int>(kMaxLds));
   });
-  const PrepArgs a{static_cast<const float*>(qkv), ld, static_cast<const float*>(conv_w), taps, static_cast<float*>(state),
-                   state_stride, norm, static_cast<const float*>(qn), static_cast<const float*>(kn), eps,
-                   static_cast<const double*>(inv_freq), rot_dims, pairs, t_coef, static_cast<double>(t_every),
+  const ConvIn in{static_cast<const float*>(qkv), ld, static_cast<const float*>(conv_w), taps, static_cast<float*>(state),
+                  state_stride, C, conv_vec(qkv, ld, conv_w, state, state_stride, C)};
+  const PrepArgs a{in, norm, static_cast<const float*>(qn), static_cast<const float*>(kn), eps,
+                   static_cast<const double*>(inv_freq), rot_dims, pairs, rot_mag, t_coef, static_cast<double>(t_every),
                    static_cast<const float*>(v_first), ld_vf, lambda, static_cast<float*>(v_save),
                    static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(cu_q),
                    static_cast<const int32_t*>(positions), static_cast<const int32_t*>(slots),
-                   static_cast<const int32_t*>(slot_mapping), kc, vc, static_cast<float*>(q_out), H, G, D, Dv, BS, T, (T + 7) / 8,
-                   C % 4 == 0 && ld % 4 == 0 && state_stride % 4 == 0 && aligned16(qkv) && aligned16(conv_w) && aligned16(state)};
+                   static_cast<const int32_t*>(slot_mapping), kc, vc, static_cast<float*>(q_out), H, G, GV, D, Dv, BS, maps, T,
+                   (T + 7) / 8};
   if (cache_f32) attn_prep_kernel<true><<<dim3(8 * ((T + 7) / 8)), dim3(256), lds, st>>>(a);
   else attn_prep_kernel<false><<<dim3(8 * ((T + 7) / 8)), dim3(256), lds, st>>>(a);
   LC_RETURN_LAST_ERROR();

@@ -1,10 +1,28 @@
 """Hybrid decoders: a stack whose layers each pick one mixer -- chunk-masked attention over the
 paged cache, latent attention over a cache of compressed rows, minGRU, gated linear attention,
-mLSTM, or attention beside linear attention -- around an fp32 residual stream.
+mLSTM, attention beside linear attention, differential attention, or a gated delta rule -- around an
+fp32 residual stream.
 
-Five designs are served, told apart by ``architecture`` in ``config.json`` (``DESIGNS``); the file lists
+Six designs are served, told apart by ``architecture`` in ``config.json`` (``DESIGNS``); the file lists
 the layers (``layers[i].type``, ``.mixer`` sizes, ``.mlp``), and every size and constant comes from
 there or from a tensor's shape.
+
+Rizurax (mixer and feed-forward side by side):
+
+* ``x = embed[token] + bigram[row]``, the row a hash of the previous and the current token (the last row for a sequence's
+  first token; the previous token is per-sequence state); a layer computes ``x += mixer(n1(x)) + ff(n2(x))`` with
+  ``n(x) = x / sqrt(mean(x^2) + eps) * (1 + w)``; ``loop`` as for Surevik, with nothing between the passes; logits
+  ``head . n_final(x)``;
+* ``delta``: q, k, v go through a short causal convolution over time per channel and silu (its last inputs are state); q and
+  k are unit vectors per head, ``q`` times ``dim^-1/2``; per head ``S <- g S``, ``u = beta (v - S^T k)``, ``S <- S + k u^T``,
+  ``o = S^T q`` with ``beta = sigmoid(W_b h)`` and ``g = exp(-exp(A) softplus(W_a h + dt))``, one each per head; an RMS norm
+  per head, a weight, a gate ``silu(W_g h)``, ``W_o``;
+* ``attention``: two maps (query / key pairs) per head over the same values. Neighbouring pairs of the first ``rot.dims``
+  coordinates of every map turn (``rot.scaling``: the long wavelengths of the frequencies interpolated, cosine and
+  sine scaled); all earlier keys; ``o = a_1 - lambda a_2``, ``lambda`` one number per layer from four vectors and ``diff``;
+  an RMS norm per head without a weight, times ``1 - diff``; ``W_o``;
+* feed-forward: ``down(gelu(gate h) * up h)`` (the tanh form). The mixer's and the feed-forward's last products are one
+  product over both results side by side.
 
 Kulivik (every sublayer between two norms, gated, reading the previous token beside the current one):
 
@@ -130,7 +148,8 @@ class Design:
     norm_offset: float = 0.0        # stored norm weights are offsets from this value
     pos_base: float = 0.0           # > 0: a sinusoidal position vector of this base is added to the embedding
     dense_ff: str = "relu2"         # dense feed-forward: down(relu(up x)^2) | "glu_relu": down(relu(gate x) * up x) |
-                                    # "xielu": down(xielu(up x + b)) + b with the activation's two numbers in ``mlp.act`` | "": none
+                                    # "xielu": down(xielu(up x + b)) + b with the activation's two numbers in ``mlp.act`` |
+                                    # "glu_gelu_tanh": down(gelu(gate x) * up x) | "": none
     norm: str = "rms"               # "dyt": Dynamic Tanh, tanh(alpha x) * w + b (tensors <name>, <name>.b, <name>.alpha)
     tied_head: bool = False         # logits from the embedding table (no ``head`` tensor)
     attention: str = "normed"       # what the ``attention`` mixer is: "normed" (biases, whole-projection q / k norms,
@@ -139,7 +158,8 @@ class Design:
                                     # | "talking" (biased q / k / v, rotate-half pairs on q and k, values turned by their own
                                     # position, capped scores, ``mask.size`` = window, a sink in the softmax, the heads'
                                     # weights mixed by a matrix) | "convolved" (a convolution over time on q / k / v,
-                                    # whole-projection norms, no positions, a learned sink and a gate per head)
+                                    # whole-projection norms, no positions, a learned sink and a gate per head) |
+                                    # "differential" (two maps per head, the second taken off the first)
     latent: str = "plain"           # latent attention: "plain" (no positions, all earlier rows, a gate per head) | "rotary" (a
                                     # turned key part shared by all heads beside the compressed row, a window, a gate per
                                     # output coordinate, ``kv_from``)
@@ -147,6 +167,9 @@ class Design:
     hyper: bool = False             # the residual is ``streams`` parallel streams (tensors ``<layer>.hc<q>.{in,out,mix}``)
     routed_ff: str = "grouped_relu2"    # "sigmoid_clamped": sigmoid scores, weight on the expert's input, clamped gated experts |
                                     # "top_silu": biased logits, softmax over the chosen ones, silu-gated experts | "": none
+    parallel_ff: bool = False       # mixer and feed-forward read the same stream through norms of their own; both results are added
+    loop_inject: bool = True        # every pass of a loop begins with x <- W_in [x; x0] (tensor ``loop.in``); else nothing between passes
+    pair_embed: bool = False        # a second embedding table indexed by (previous, current) token (tensor ``bigram``)
     sandwich: bool = False          # norms on the sublayers' inputs AND results, results gated from the input, the mixer's input
                                     # shifted towards the previous token's (tensors norm<q>, norm<q>b, rg<q>, rg<q>.b, shift)
     # constants of the clamped gated unit g * sigmoid(slope g) * (u + shift)
@@ -162,6 +185,8 @@ DESIGNS: Dict[str, Design] = {
                       attention="keys_as_values", routed_ff="sigmoid_clamped"),
     "Kulivik": Design("Kulivik", ("parallel", "attention", "attention_2"), pre_norm=True, norm_offset=1.0, sandwich=True,
                       dense_ff="clamped_glu", tied_head=True, attention="convolved", routed_ff="top_silu"),
+    "Rizurax": Design("Rizurax", ("delta", "attention"), pre_norm=True, norm_offset=1.0, parallel_ff=True, loop_inject=False,
+                      pair_embed=True, dense_ff="glu_gelu_tanh", attention="differential", routed_ff=""),
     "Gizilorn": Design("Gizilorn", ("attention", "latent_attention"), pre_norm=True, dense_ff="xielu", attention="talking",
                        latent="rotary", embed_norm=True, hyper=True, routed_ff=""),
 }
@@ -257,6 +282,11 @@ class LayerSpec:
     head_gate: bool = False
     distance_bias: bool = False
     out_scale: float = 1.0
+    # differential attention: maps per head over one value, the share of the second that is always taken off; frequency
+    # scaling of the rotation (factor, original length, fast and slow turn counts; None: none)
+    maps: int = 1
+    diff: float = 0.0
+    rot_scaling: Optional[Tuple[float, float, float, float]] = None
     right: Optional["LayerSpec"] = None
     # linear attention with one constant decay per head
     decay: Tuple[float, ...] = ()
@@ -279,6 +309,10 @@ class LayerSpec:
     @property
     def channels(self) -> int:
         """Width of q | k | v."""
+        if self.type == "delta":
+            return 2 * self.kv_heads * self.dim + self.heads * self.vdim
+        if self.maps > 1:
+            return (self.heads + self.kv_heads) * self.maps * self.dim + self.kv_heads * self.vdim
         return (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
 
     @property
@@ -291,9 +325,11 @@ class LayerSpec:
 
     def state_parts(self) -> Dict[str, Tuple[int, int]]:
         """(first column, numbers) of what a layer with several kinds of state keeps: the previous input row, the
-        convolution's last inputs, the linear attention's memory. Every part starts on a 16-byte border."""
-        sizes = {"shift": self.shift, "conv": max(0, self.conv - 1) * self.channels,
-                 "memory": self.right.state_size() if self.right is not None else 0}
+        convolution's last inputs, the linear attention's or the delta rule's memory. Every part starts on a 16-byte border."""
+        memory = self.right.state_size() if self.right is not None else 0
+        if self.type == "delta":
+            memory = self.heads * self.dim * self.vdim
+        sizes = {"shift": self.shift, "conv": max(0, self.conv - 1) * self.channels, "memory": memory}
         out, at = {}, 0
         for name, n in sizes.items():
             if n:
@@ -303,7 +339,7 @@ class LayerSpec:
 
     def state_size(self) -> int:
         """fp32 numbers of recurrent state per sequence."""
-        if self.prepped:
+        if self.prepped or self.type == "delta":
             parts = list(self.state_parts().values())
             return (parts[-1][0] + parts[-1][1] + 3) // 4 * 4 if parts else 0
         if self.type == "lightning":
@@ -321,7 +357,7 @@ class LayerSpec:
         if self.owns_kv and self.values_are_keys:     # rotated keys, and the un-rotated ones unless nothing rotates
             return self.kv_heads * self.dim * (2 if self.rot_dims else 1)
         if self.owns_kv:
-            return self.kv_heads * (self.dim + self.vdim)
+            return self.kv_heads * (self.maps * self.dim + self.vdim)
         return self.kv_rank + self.rot_dim if self.owns_latent else 0
 
 
@@ -341,6 +377,7 @@ class HybridConfig:
     loop: Tuple[int, int, int] = (0, 0, 1)      # layers [start, stop) run ``times`` times in a row (times 1: no loop)
     streams: int = 0                # parallel residual streams (designs with hyper-connections)
     logit_softcap: float = 0.0      # > 0: logits become cap * tanh(logits / cap)
+    pair: Optional[Tuple[int, int, int]] = None     # pair embedding: (buckets, mul_prev, mul_cur)
 
     @property
     def design(self) -> Design:
@@ -359,7 +396,7 @@ class HybridConfig:
             return tuple((i, False) for i in range(len(self.layers)))
         out = [(i, False) for i in range(start)]
         for _ in range(times):
-            out += [(i, i == start) for i in range(start, stop)]
+            out += [(i, i == start and self.design.loop_inject) for i in range(start, stop)]
         return tuple(out + [(i, False) for i in range(stop, len(self.layers))])
 
     @property
@@ -368,7 +405,7 @@ class HybridConfig:
 
     @property
     def has_state(self) -> bool:
-        return any(l.state_size() for l in self.layers)
+        return self.pair is not None or any(l.state_size() for l in self.layers)
 
     @property
     def num_heads(self) -> int:
@@ -385,7 +422,7 @@ class HybridConfig:
         return self.kv_elems_per_token() * bytes_per_elem
 
     def state_floats(self) -> int:
-        return sum(self.layers[i].state_size() for i, _ in self.runs)
+        return sum(self.layers[i].state_size() for i, _ in self.runs) + (1 if self.pair is not None else 0)
 
     def param_count(self) -> int:
         return sum(_numel(s) for s in param_shapes(self).values())
@@ -411,6 +448,8 @@ class HybridConfig:
             raise ValueError(f"{self.name}: 1..{ops.MAX_STREAMS} residual streams are needed, and no loop")
         if self.logit_softcap < 0:
             raise ValueError(f"{self.name}: the logits' cap is positive, or 0 for none")
+        if self.pair is not None and (not self.design.pair_embed or not 0 < self.pair[0] < 1 << 31):
+            raise ValueError(f"{self.name}: a pair embedding has 1..2^31 - 1 buckets, in a design that has one")
         mixing = [l for l in self.layers if l.v_mix]
         if any(l.kv_heads * l.vdim != mixing[0].kv_heads * mixing[0].vdim for l in mixing):
             raise ValueError(f"{self.name}: layers that mix values have one value width (kv_heads * vdim)")
@@ -446,6 +485,18 @@ class HybridConfig:
                     raise ValueError(f"{self.name}: layer {i}: the kept groups must hold `top` (at most 32) router outputs")
             if l.type == "mingru" and l.width <= 0:
                 raise ValueError(f"{self.name}: layer {i}: minGRU needs a width")
+            if l.type == "delta":
+                if l.heads <= 0 or l.kv_heads <= 0 or l.heads % l.kv_heads or l.dim <= 0 or l.dim > 256 or l.vdim <= 0 or l.conv < 1:
+                    raise ValueError(f"{self.name}: layer {i}: the delta rule takes heads in whole groups of kv_heads, dim <= 256, "
+                                     f"vdim and at least one convolution tap")
+                if l.channels > ops.ATTN_PREP_MAX_FLOATS:
+                    raise ValueError(f"{self.name}: layer {i}: the kernels take q | k | v of at most {ops.ATTN_PREP_MAX_FLOATS} channels")
+            if l.maps > 1 and (l.maps != 2 or l.conv or l.qk_norm or l.v_mix or l.window or l.chunk or not l.prepped):
+                raise ValueError(f"{self.name}: layer {i}: differential attention has two maps over all earlier keys")
+            if l.rot_scaling is not None:
+                f, o, fast, slow = l.rot_scaling
+                if not (f > 0 and o > 0 and fast > 0 and slow > 0 and l.rot_base > 1):
+                    raise ValueError(f"{self.name}: layer {i}: rot.scaling takes positive numbers and a base above one")
             if l.right is not None:
                 g = l.right
                 if g.heads <= 0 or g.dim <= 0 or g.dim > 256 or g.vdim <= 0 or len(g.decay) != g.heads:
@@ -485,6 +536,46 @@ def _numel(shape) -> int:
     for s in shape:
         n *= s
     return n
+
+
+def _parallel_of(t: str, m: dict, ff: int) -> LayerSpec:
+    """A Rizurax layer."""
+    heads, dim = int(m["heads"]), int(m["dim"])
+    kw = dict(heads=heads, kv_heads=int(m.get("kv_heads", heads)), dim=dim, vdim=int(m.get("vdim", dim)), ff=ff)
+    if t == "delta":
+        return LayerSpec(t, conv=int(m.get("conv", 1)), **kw)
+    rot = m.get("rot") or {}
+    s = rot.get("scaling")
+    return LayerSpec(t, scale=float(m.get("scale", dim ** -0.5)), rot_dims=int(rot.get("dims", 0)), rot_pairs=True,
+                     rot_base=float(rot.get("base", 10000.0)), prepped=True, maps=2, diff=float(m["diff"]),
+                     rot_scaling=tuple(float(s[k]) for k in ("factor", "original", "fast", "slow")) if s else None, **kw)
+
+
+def _parallel_to_dict(l: LayerSpec) -> dict:
+    m = {"heads": l.heads, "kv_heads": l.kv_heads, "dim": l.dim, "vdim": l.vdim}
+    if l.type == "delta":
+        return {**m, "conv": l.conv}
+    rot = {"dims": l.rot_dims, "base": l.rot_base}
+    if l.rot_scaling is not None:
+        rot["scaling"] = dict(zip(("factor", "original", "fast", "slow"), l.rot_scaling))
+    return {**m, "scale": l.scale, "diff": l.diff, "rot": rot}
+
+
+def rotary_frequencies(dims: int, base: float, scaling: Optional[Tuple[float, float, float, float]] = None):
+    """(angle per position of pair i in fp64, factor on cosine and sine): base^(-2i / dims), and with ``scaling`` = (factor,
+    original length, fast, slow) those pairs that turn fewer than ``slow`` times over the original length are slowed down by
+    the factor, those that turn more than ``fast`` times are not, and the pairs between go from one to the other linearly."""
+    f = [base ** (-2.0 * i / dims) for i in range(dims // 2)]
+    if scaling is None:
+        return f, 1.0
+    factor, original, fast, slow = scaling
+
+    def pair_at(turns: float) -> float:               # (fractional) dimension whose pair turns that often
+        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+    lo, hi = max(math.floor(pair_at(fast)), 0), min(math.ceil(pair_at(slow)), dims - 1)
+    width = max(hi - lo, 0.001)
+    ramp = [min(1.0, max(0.0, (i - lo) / width)) for i in range(dims // 2)]
+    return [x / factor * r + x * (1.0 - r) for x, r in zip(f, ramp)], 0.1 * math.log(factor) + 1.0
 
 
 def _prepped_of(name: str, i: int, t: str, m: dict, width: int, ff: int, limit: float, moe: Optional[MoESpec]) -> LayerSpec:
@@ -570,6 +661,8 @@ def config_from_dict(c: dict, name: str = "hybrid", tensor_shapes: Optional[Dict
         if design.sandwich:
             limit = float((L.get("mlp") or {}).get("limit", math.inf)) if ff else 0.0
             layers.append(_prepped_of(name, i, t, m, int(c["width"]), ff, limit, moe))
+        elif design.parallel_ff:
+            layers.append(_parallel_of(t, m, ff))
         elif t == "attention" and design.attention == "keys_as_values":
             mask, rot = m.get("mask") or {}, m.get("rot") or {}
             layers.append(LayerSpec(t, heads=int(m["heads"]), kv_heads=int(m.get("kv_heads", m["heads"])),
@@ -616,13 +709,15 @@ def config_from_dict(c: dict, name: str = "hybrid", tensor_shapes: Optional[Dict
         else:
             layers.append(LayerSpec(t, heads=int(m["heads"]), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])),
                                     gate_cap=float(m.get("gate_cap", 0.0)), ff=ff, moe=moe))
+    pair = (c.get("embedding") or {}).get("bigram")
     cfg = HybridConfig(name=name, vocab_size=int(c["vocab"]), hidden_size=int(c["width"]),
                        rms_eps=float(c["norm"]["eps"]), layers=tuple(layers),
                        max_position=int(c.get("max_position", 1 << 20)), model_type=arch.lower(), architecture=arch,
                        embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)),
                        logit_scale=float(c.get("logit_scale", 1.0)), residual_mult=float(c.get("residual_mult", 1.0)),
                        loop=_loop_of(c.get("loop")), streams=int(c.get("streams", 1)) if design.hyper else 0,
-                       logit_softcap=float(c.get("logit_softcap") or 0.0))
+                       logit_softcap=float(c.get("logit_softcap") or 0.0),
+                       pair=tuple(int(pair[k]) for k in ("buckets", "mul_prev", "mul_cur")) if pair else None)
     cfg.validate()
     return cfg
 
@@ -630,7 +725,9 @@ def config_from_dict(c: dict, name: str = "hybrid", tensor_shapes: Optional[Dict
 def config_to_dict(cfg: HybridConfig) -> dict:
     layers = []
     for l in cfg.layers:
-        if l.prepped:
+        if cfg.design.parallel_ff:
+            m = _parallel_to_dict(l)
+        elif l.prepped:
             m = _prepped_to_dict(l)
         elif l.type == "attention" and l.values_are_keys:
             m = {"heads": l.heads, "kv_heads": l.kv_heads, "dim": l.dim, "vdim": l.vdim, "scale": l.scale,
@@ -684,6 +781,12 @@ def config_to_dict(cfg: HybridConfig) -> dict:
         if cfg.logit_softcap:
             out["logit_softcap"] = cfg.logit_softcap
         return out
+    if cfg.design.parallel_ff:
+        if cfg.pair is not None:
+            out["embedding"] = {"bigram": dict(zip(("buckets", "mul_prev", "mul_cur"), cfg.pair))}
+        if cfg.looped:
+            out["loop"] = {"start": cfg.loop[0], "stop": cfg.loop[1], "times": cfg.loop[2]}
+        return out
     if cfg.design.pre_norm:
         out["embedding"] = {"scale": cfg.embed_scale}
     if cfg.design.pre_norm and not cfg.design.tied_head:
@@ -720,8 +823,10 @@ def param_shapes(cfg: HybridConfig) -> Dict[str, tuple]:
         out[name] = norm
         if dyt:
             out[name + ".b"], out[name + ".alpha"] = (d,), ()
-    if cfg.looped:
+    if cfg.looped and cfg.design.loop_inject:
         out["loop.in"] = (d, 2 * d)
+    if cfg.pair is not None:
+        out["bigram"] = (cfg.pair[0] + 1, d)
     if cfg.design.embed_norm:
         out["embed.norm"] = (d,)
     for i, l in enumerate(cfg.layers):
@@ -738,7 +843,18 @@ def param_shapes(cfg: HybridConfig) -> Dict[str, tuple]:
             for q in ("hc1.", "hc2.") if l.has_ff else ("hc1.",):
                 out[p + q + "in"], out[p + q + "out"], out[p + q + "mix"] = (cfg.streams,), (cfg.streams,), (cfg.streams, cfg.streams)
         m = p + "mix."
-        if l.prepped:
+        if l.type == "delta":
+            for n, k in (("q", l.kv_heads * l.dim), ("k", l.kv_heads * l.dim), ("v", l.heads * l.vdim)):
+                out[m + n], out[m + n + ".conv"] = (k, d), (k, l.conv)
+            out[m + "b"], out[m + "a"], out[m + "g"] = (l.heads, d), (l.heads, d), (l.heads * l.vdim, d)
+            out[m + "A_log"], out[m + "dt_bias"], out[m + "norm"] = (l.heads,), (l.heads,), (l.vdim,)
+            out[m + "o"] = (d, l.heads * l.vdim)
+        elif l.maps > 1:
+            out[m + "q"], out[m + "k"] = (l.heads * l.maps * l.dim, d), (l.kv_heads * l.maps * l.dim, d)
+            out[m + "v"], out[m + "o"] = (l.kv_heads * l.vdim, d), (d, l.heads * l.vdim)
+            for n in ("lq1", "lk1", "lq2", "lk2"):
+                out[m + n] = (l.dim,)
+        elif l.prepped:
             x = m + "left." if l.right is not None else m
             rows = {"q": l.heads * l.dim, "k": l.kv_heads * l.dim, "v": l.kv_heads * l.vdim}
             for n, k in rows.items():
@@ -824,7 +940,7 @@ def param_shapes(cfg: HybridConfig) -> Dict[str, tuple]:
                     out[f + "shared.gate"], out[f + "shared.sg"] = (e.shared_ff, d), (1, d)
                 out[f + "shared.up"], out[f + "shared.down"] = (e.shared_ff, d), (d, e.shared_ff)
         elif l.ff:
-            if cfg.design.dense_ff in ("glu_relu", "clamped_glu"):
+            if cfg.design.dense_ff in ("glu_relu", "glu_gelu_tanh", "clamped_glu"):
                 out[f + "gate"] = (l.ff, d)
             out[f + "up"], out[f + "down"] = (l.ff, d), (d, l.ff)
             if cfg.design.dense_ff == "xielu":
@@ -849,8 +965,8 @@ class StepLayout:
 class HybridCache:
     """Paged keys / values of the attention layers that own any, the paged compressed rows of the
     latent-attention layers that own any, and the fp32 state slots of the layers that keep state (recurrences, the
-    previous input row of a token shift, a convolution's last inputs), in ONE pool. Key
-    planes are [blocks, G, BS, dim], value planes [blocks, G, BS, vdim], latent planes
+    previous input row of a token shift, a convolution's last inputs) and of the model (the sequences' last tokens, for a
+    pair embedding), in ONE pool. Key planes are [blocks, G, BS, dim] (G * maps heads when a head has several maps), value planes [blocks, G, BS, vdim], latent planes
     [blocks, 1, BS, kv_rank + rot_dim] (keys; their first kv_rank columns are the values) in the model's activation type; a state
     plane is [slots, size] fp32. Planes belong to layer RUNS (``HybridConfig.runs``): a layer that a
     loop runs several times has a set per pass; without a loop run r is layer r."""
@@ -866,10 +982,11 @@ class HybridCache:
             at = off
             off = (off + nbytes + 255) // 256 * 256
             return at
+        last_at = take(max(1, num_slots) * 16) if cfg.pair is not None else -1      # (a 16-byte row per slot)
         for i, (li, _) in enumerate(cfg.runs):
             l = cfg.layers[li]
             if l.owns_kv:
-                plan.append(("k", i, take(num_blocks * l.kv_heads * block_size * l.dim * es)))
+                plan.append(("k", i, take(num_blocks * l.kv_heads * l.maps * block_size * l.dim * es)))
                 if not (l.values_are_keys and l.rot_dims == 0):      # (un-rotated keys that are the values: one plane)
                     plan.append(("v", i, take(num_blocks * l.kv_heads * block_size * l.vdim * es)))
             elif l.owns_latent:
@@ -886,11 +1003,15 @@ class HybridCache:
         self._k: Dict[int, torch.Tensor] = {}
         self._v: Dict[int, torch.Tensor] = {}
         self._s: Dict[int, torch.Tensor] = {}
+        self.last_tokens: Optional[torch.Tensor] = None          # int32 [slots, 1]
+        if last_at >= 0:
+            n = max(1, num_slots) * 16
+            self.last_tokens = raw[last_at:last_at + n].view(torch.int32).view(max(1, num_slots), 4)[:, :1]
         for kind, i, at in plan:
             l = cfg.layers[cfg.runs[i][0]]
             if kind == "k":
-                n = num_blocks * l.kv_heads * block_size * l.dim * es
-                self._k[i] = raw[at:at + n].view(dtype).view(num_blocks, l.kv_heads, block_size, l.dim)
+                n = num_blocks * l.kv_heads * l.maps * block_size * l.dim * es
+                self._k[i] = raw[at:at + n].view(dtype).view(num_blocks, l.kv_heads * l.maps, block_size, l.dim)
                 if l.values_are_keys and l.rot_dims == 0:
                     self._v[i] = self._k[i]
             elif kind == "v":
@@ -978,6 +1099,11 @@ class HybridLayer:
     slopes: Optional[torch.Tensor] = None           # fp32 [H]: score taken off per unit of distance
     v_lambda: float = 0.0                           # share of the first mixing layer's values
     decay: Optional[torch.Tensor] = None            # fp32 [heads]: linear attention's constant decays
+    # mixer and feed-forward side by side (``out`` then reads both results)
+    neg_rate: Optional[torch.Tensor] = None         # fp32 [heads]: delta rule, -exp(A)
+    dt_bias: Optional[torch.Tensor] = None          # fp32 [heads]
+    rot_mag: float = 1.0                            # factor on cosine and sine
+    lam: float = 0.0                                # differential attention: weight of the second map
 
 
 @dataclass
@@ -1008,6 +1134,7 @@ class HybridModel:
         self.final_norm: Optional[torch.Tensor] = None
         self.lm_head: Optional[ops.LinearWeight] = None
         self.loop_in: Optional[ops.LinearWeight] = None     # [d, 2 d]: the stream's re-injection before every pass of a loop
+        self.pair_table: Optional[torch.Tensor] = None      # [buckets + 1, d]: embedding of (previous, current) token
         self.embed_norm: Optional[torch.Tensor] = None      # fp32 [d]: norm weight on the embedding rows
         self.stream_sum: Optional[torch.Tensor] = None      # fp32 [S] of ones: the model's output reads every stream once
         self.layers: List[HybridLayer] = []
@@ -1058,7 +1185,8 @@ class HybridModel:
         self.final_norm = norm_w("final.norm", c.logit_scale) if c.design.pre_norm else f32(load("final.norm"))
         # (a tied head is the embedding table once more, in the layout of the matrix products)
         self.lm_head = lin(load("embed" if c.design.tied_head else "head"))
-        self.loop_in = lin(load("loop.in")) if c.looped else None
+        self.loop_in = lin(load("loop.in")) if c.looped and c.design.loop_inject else None
+        self.pair_table = load("bigram").to(dt).contiguous() if c.pair is not None else None
         self.embed_norm = f32(load("embed.norm")) if c.design.embed_norm else None
         self.stream_sum = torch.ones(c.streams, dtype=torch.float32, device=dev) if c.design.hyper else None
 
@@ -1071,7 +1199,9 @@ class HybridModel:
             if c.design.hyper:
                 for q in ("hc1", "hc2") if l.has_ff else ("hc1",):
                     kw[q] = StreamWeights(f32(load(p + q + ".in")), f32(load(p + q + ".out")), f32(load(p + q + ".mix")))
-            if l.prepped:
+            if c.design.parallel_ff:
+                proj, out = self._load_parallel(p, l, load, lin, f32, kw)
+            elif l.prepped:
                 proj, out = self._load_prepped(p, l, load, lin, f32, inv_freqs, kw)
             elif l.type == "attention" and l.talk:
                 if l.rot_dims:
@@ -1183,6 +1313,8 @@ class HybridModel:
                     kw["experts_down"] = ops.ExpertWeights.from_dense(downs, dev)
                 else:
                     kw["experts_up"], kw["experts_down"] = ups.to(dt).contiguous(), downs.to(dt).contiguous()
+            elif l.ff and c.design.parallel_ff:
+                kw["gate_up"] = lin(torch.cat([load(f + "gate"), load(f + "up")], 0))
             elif l.ff and c.design.sandwich:
                 kw["down"] = lin(load(f + "down"))
             elif l.ff and c.design.dense_ff == "xielu":
@@ -1237,6 +1369,27 @@ class HybridModel:
             kw["head_norm"] = (f32(load(x + "norm")) * g.out_scale).contiguous()
         return lin(torch.cat(Ws, 0), bias, pad=True), lin(Wo, bo)
 
+    def _load_parallel(self, p: str, l: LayerSpec, load, lin, f32, kw: dict):
+        """A layer whose mixer and feed-forward stand side by side: (input product of the mixer, ONE output product over the
+        mixer's and the feed-forward's results side by side)."""
+        dev, m = self.device, p + "mix."
+        Wo = load(m + "o")
+        if l.ff:
+            Wo = torch.cat([Wo, load(p + "mlp.down")], 1)
+        if l.type == "delta":
+            # q | k | v | result gate | step-size logits | decay logits
+            proj = lin(torch.cat([load(m + n) for n in ("q", "k", "v", "g", "b", "a")], 0), pad=True)
+            kw["conv_w"] = torch.cat([load(m + n + ".conv") for n in ("q", "k", "v")], 0).t().contiguous()
+            kw["neg_rate"] = (-torch.exp(f32(load(m + "A_log")).double())).float()
+            kw["dt_bias"], kw["head_norm"] = f32(load(m + "dt_bias")), f32(load(m + "norm"))
+            return proj, lin(Wo)
+        if l.rot_dims:
+            f, kw["rot_mag"] = rotary_frequencies(l.rot_dims, l.rot_base, l.rot_scaling)
+            kw["inv_freq"] = torch.tensor(f, dtype=torch.float64).to(dev)
+        v = {n: f32(load(m + n)).double().cpu() for n in ("lq1", "lk1", "lq2", "lk2")}
+        kw["lam"] = float(torch.exp((v["lq1"] * v["lk1"]).sum()) - torch.exp((v["lq2"] * v["lk2"]).sum())) + l.diff
+        return lin(torch.cat([load(m + n) for n in ("q", "k", "v")], 0), pad=True), lin(Wo)
+
     @classmethod
     def random_init(cls, cfg: HybridConfig, device, seed: int = 0, dtype: torch.dtype = torch.bfloat16,
                     **_ignored) -> "HybridModel":
@@ -1268,6 +1421,8 @@ class HybridModel:
                 t = 0.1 * torch.randn(shape, generator=gen)
             elif name.endswith("norm") or name.endswith("norm1") or name.endswith("norm2"):
                 t = 1.0 + 0.1 * torch.randn(shape, generator=gen)
+            elif name.endswith("mix.dt_bias"):
+                t = -3.0 + torch.randn(shape, generator=gen)
             elif name.endswith("a2.b") or name.endswith("mix.f.b"):
                 t = 2.0 + torch.randn(shape, generator=gen)
             elif name.endswith("correction"):
@@ -1281,6 +1436,7 @@ class HybridModel:
     def weight_bytes(self) -> int:
         n = self.embed.numel() * self.embed.element_size() + self.lm_head.nbytes()
         n += self.loop_in.nbytes() if self.loop_in is not None else 0
+        n += self.pair_table.numel() * self.pair_table.element_size() if self.pair_table is not None else 0
         for L in self.layers:
             for w in (L.proj, L.out, L.up, L.down, L.decay_up, L.gate_up, L.router, L.shared_up, L.shared_down, L.gate1, L.ff_in):
                 n += w.nbytes() if w is not None else 0
@@ -1328,6 +1484,8 @@ class HybridModel:
             if meta.is_prefill else (0, 0)
         if c.design.sandwich:
             return self._forward_sandwich(token_ids, positions, slot_mapping, meta, lay, cache, taps)
+        if c.design.parallel_ff:
+            return self._forward_parallel(token_ids, positions, slot_mapping, meta, lay, cache, taps)
         if c.design.hyper:
             return self._forward_streams(token_ids, positions, slot_mapping, meta, lay, cache, taps)
         if c.design.pre_norm:
@@ -1473,6 +1631,65 @@ class HybridModel:
             if taps is not None:
                 taps.append(x.clone())
         return x
+
+    def _forward_parallel(self, token_ids, positions, slot_mapping, meta, lay: StepLayout, cache: HybridCache,
+                          taps: Optional[list]) -> torch.Tensor:
+        """Layers whose mixer and feed-forward read the same stream through norms of their own. Both write their results
+        side by side into one matrix, one product brings them back to the stream's width (their sum), and one launch
+        adds it to the stream and forms the next layer's two inputs."""
+        c, dt, eps = self.cfg, self.dtype, self.cfg.rms_eps
+        pair = None
+        if c.pair is not None:
+            n, mp, mc = c.pair
+            pair = ops.PairEmbedding(self.pair_table, n, mp % n, mc % n, cache.last_tokens)
+        x, _ = ops.embed_rows(token_ids, self.embed, None, meta.token_feed, positions=positions if pair is not None else None,
+                              pair=pair, lay=lay)
+        runs = c.runs
+        first = self.layers[runs[0][0]]
+        h1, h2 = ops.dual_norm_step(x, None, first.norm1, first.norm2, eps, dt)
+        for r, (i, _) in enumerate(runs):
+            L = self.layers[i]
+            l = L.spec
+            n = l.heads * l.vdim
+            both = torch.empty(x.shape[0], n + l.ff, dtype=dt, device=x.device)
+            if l.type == "delta":
+                self._delta(r, L, h1, positions, lay, cache, both[:, :n])
+            else:
+                self._attention_diff(r, L, h1, positions, slot_mapping, lay, cache, both[:, :n])
+            if l.ff:
+                ops.glu(ops.linear(h2, L.gate_up, out_f32=True), dt, "gelu_tanh", out=both[:, n:])
+            y = ops.linear(both, L.out, out_f32=True)
+            nxt = self.layers[runs[r + 1][0]] if r + 1 < len(runs) else None
+            h1, h2 = ops.dual_norm_step(x, y, nxt.norm1 if nxt else None, nxt.norm2 if nxt else None, eps, dt)
+            if taps is not None:
+                taps.append(x.clone())
+        return x
+
+    def _delta(self, r: int, L: HybridLayer, xa, positions, lay: StepLayout, cache: HybridCache, out: torch.Tensor) -> None:
+        """Gated delta rule: operands, recurrence, per-head norm and gate into ``out`` [T, H * Dv]."""
+        l = L.spec
+        H, G, D, Dv, C = l.heads, l.kv_heads, l.dim, l.vdim, l.channels
+        proj = ops.linear(xa, L.proj, out_f32=True)                 # q | k | v | result gate | step sizes | decays
+        g0, b0 = C, C + H * Dv
+        x = ops.delta_prep(proj, L.conv_w, cache.state_part(r, "conv") if l.conv > 1 else None, b0, b0 + H, L.neg_rate, L.dt_bias,
+                           positions, lay, H, G, D, Dv)
+        o = ops.delta_scan(x, cache.state_part(r, "memory"), lay.cu_q, positions, lay.state_slots, H, G, D, Dv, self._max_len)
+        ops.headnorm_gate(o, L.head_norm, proj[:, g0:g0 + H * Dv], Dv, self.cfg.rms_eps, self.dtype, out=out)
+
+    def _attention_diff(self, r: int, L: HybridLayer, xa, positions, slot_mapping, lay: StepLayout, cache: HybridCache,
+                        out: torch.Tensor) -> None:
+        """Differential attention into ``out`` [T, H * Dv]. The maps of all heads are query heads of their own over key
+        heads of their own; neighbouring key heads share a value head."""
+        l = L.spec
+        M, D, Dv = l.maps, l.dim, l.vdim
+        kc, vc = cache.k(r), cache.v(r)
+        qkv = ops.linear(xa, L.proj, out_f32=True)
+        q, _ = ops.attn_prep(qkv, positions, slot_mapping, lay, kc, vc, l.heads * M, l.kv_heads * M, D, Dv, inv_freq=L.inv_freq,
+                             rot_dims=l.rot_dims, pairs=True, rot_mag=L.rot_mag, maps=M)
+        a = ops.attn_masked(q, kc, vc, lay.block_tables, lay.cu_q, lay.row_seq, positions, l.heads * M, l.kv_heads * M, D, Dv,
+                            l.scale, 0, 0, torch.float32, n_portions=self._portions[0], portion_rows=self._portions[1],
+                            max_len=self._max_len, value_share=M)
+        ops.diff_norm(a, L.lam, self.cfg.rms_eps, 1.0 - l.diff, l.heads, l.kv_heads, Dv, self.dtype, out=out)
 
     def _clamped_dense(self, L: HybridLayer, fi: torch.Tensor) -> torch.Tensor:
         d, n, des = self.cfg.hidden_size, L.spec.ff, self.cfg.design

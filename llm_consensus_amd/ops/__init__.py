@@ -902,14 +902,41 @@ def linear_any(x: torch.Tensor, w: LinearWeight, out_f32: bool = True, epi_relu2
     return y
 
 
+@dataclass
+class PairEmbedding:
+    """A second embedding table indexed by a token and the one before it: row (previous * mul_prev + current * mul_cur) mod
+    buckets of ``table`` [buckets + 1, d], the last row for a sequence's first token. ``last`` (int32 [slots, 1], may be a
+    column of a wider plane) holds the sequences' last tokens and is updated in place."""
+
+    table: torch.Tensor
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+    last: torch.Tensor
+
+    def check(self, E: torch.Tensor) -> None:
+        if self.table.shape != (self.buckets + 1, E.shape[1]) or self.table.dtype != E.dtype or not self.table.is_contiguous():
+            raise ValueError("embed_rows: the pair table is [buckets + 1, d] in the embedding's type")
+        if self.last.dtype != torch.int32 or self.last.dim() != 2 or self.last.shape[1] != 1:
+            raise ValueError("embed_rows: the last tokens are int32 [slots, 1]")
+        if self.buckets <= 0 or not (0 <= self.mul_prev < 1 << 31 and 0 <= self.mul_cur < 1 << 31):
+            raise ValueError("embed_rows: buckets are positive, the multipliers within 31 bits")
+
+
 def embed_rows(ids: torch.Tensor, E: torch.Tensor, act_dtype: Optional[torch.dtype],
                feed: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, scale: float = 1.0,
-               positions: Optional[torch.Tensor] = None, inv_freq: Optional[torch.Tensor] = None):
+               positions: Optional[torch.Tensor] = None, inv_freq: Optional[torch.Tensor] = None,
+               pair: Optional["PairEmbedding"] = None, lay=None):
     """Rows E[ids] * scale as (fp32 [T, d], copy in ``act_dtype`` or None). E is bf16 or fp32; with
     ``act_dtype`` fp32 the copy IS the fp32 tensor. ``feed`` as in ``embed``. With ``positions`` and
     ``inv_freq`` (fp64 [d/2]) a sinusoidal position vector is added: entry 2i is sin(p f_i), entry
-    2i + 1 cos(p f_i), the angle and its reduction in fp64. Also the row gather of an fp32 matrix."""
+    2i + 1 cos(p f_i), the angle and its reduction in fp64. With ``pair`` a second row, indexed by the previous and the current token, is added
+    (``positions`` and ``lay``, the step's layout, say where sequences start). Also the row gather of an fp32 matrix."""
     T, d = ids.numel(), E.shape[1]
+    if pair is not None:
+        pair.check(E)
+        if positions is None or lay is None or lay.state_slots is None or inv_freq is not None:
+            raise ValueError("embed_rows: a pair table needs positions and the step's layout (and no position vector)")
     if inv_freq is not None and (positions is None or 2 * inv_freq.numel() != d or inv_freq.dtype != torch.float64):
         raise ValueError("embed_rows: the position table needs positions and d / 2 fp64 frequencies")
     if not ids.is_cuda:
@@ -921,13 +948,18 @@ def embed_rows(ids: torch.Tensor, E: torch.Tensor, act_dtype: Optional[torch.dty
             x = x * scale
         if inv_freq is not None:
             x = x + ref.sinusoid_rows(positions, inv_freq)
+        if pair is not None:
+            x = x + ref.embed(ref.pair_rows(ids, positions, lay, pair, E.shape[0]), pair.table).float()
         return x, (x if act_dtype in (None, torch.float32) else x.to(act_dtype))
     x = torch.empty(T, d, dtype=torch.float32, device=E.device)
     xa = torch.empty(T, d, dtype=act_dtype, device=E.device) if act_dtype == torch.bfloat16 else None
     _hip().call("lc_embed_rows", ids.data_ptr(), E.data_ptr(), _f32flag(E.dtype), x.data_ptr(), _hip().ptr(xa), 0, T, d,
                 E.shape[0], feed[0].data_ptr() if feed is not None else None,
                 feed[1].data_ptr() if feed is not None else None, float(scale),
-                positions.data_ptr() if inv_freq is not None else None, _hip().ptr(inv_freq))
+                positions.data_ptr() if (inv_freq is not None or pair is not None) else None, _hip().ptr(inv_freq),
+                *((pair.table.data_ptr(), pair.buckets, pair.mul_prev, pair.mul_cur, pair.last.data_ptr(),
+                   max(pair.last.stride(0), 1), lay.row_seq.data_ptr(), lay.cu_q.data_ptr(), lay.state_slots.data_ptr())
+                  if pair is not None else (None, 0, 0, 0, None, 0, None, None, None)))
     return x, (xa if xa is not None else (x if act_dtype is not None else None))
 
 
@@ -1014,19 +1046,29 @@ def gla_scan(proj: torch.Tensor, decay_logits: torch.Tensor, state: torch.Tensor
     return out
 
 
+def _out_block(out: Optional[torch.Tensor], T: int, n: int, act_dtype: torch.dtype, device, what: str) -> torch.Tensor:
+    """``out`` checked as a [T, n] block in the activation type (of a wider matrix), or a new matrix."""
+    if out is None:
+        return torch.empty(T, n, dtype=act_dtype, device=device)
+    if out.shape != (T, n) or out.dtype != act_dtype or (n > 1 and out.stride(1) != 1):
+        raise ValueError(f"{what}: the output is a [T, {n}] block in the activation type")
+    return out
+
+
 def headnorm_gate(o: torch.Tensor, w: torch.Tensor, gate: torch.Tensor, Dv: int, eps: float,
-                  act_dtype: torch.dtype) -> torch.Tensor:
+                  act_dtype: torch.dtype, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Per head of width Dv: o / sqrt(mean(o^2) + eps) * w, times silu(gate). ``gate`` may be a
-    column slice of a wider fp32 matrix."""
+    column slice of a wider fp32 matrix. ``out``: write into this [T, heads * Dv] block (of a wider matrix)."""
     if not o.is_cuda:
-        return ref.headnorm_gate(o, w, gate, Dv, eps, act_dtype)
+        y = ref.headnorm_gate(o, w, gate, Dv, eps, act_dtype)
+        return y if out is None else out.copy_(y)
     T, n = o.shape
     if gate.shape != o.shape or gate.stride(1) != 1 or o.dtype != torch.float32 or gate.dtype != torch.float32:
         raise ValueError("headnorm_gate: fp32 read-out and gate of one shape")
     o = o.contiguous()
-    out = torch.empty(T, n, dtype=act_dtype, device=o.device)
-    _hip().call("lc_headnorm_gate", o.data_ptr(), w.data_ptr(), gate.data_ptr(), gate.stride(0), out.data_ptr(),
-                _f32flag(act_dtype), T, n // Dv, Dv, float(eps), Dv, 0, 0, None, n)
+    out = _out_block(out, T, n, act_dtype, o.device, "headnorm_gate")
+    _hip().call("lc_headnorm_gate", o.data_ptr(), w.data_ptr(), gate.data_ptr(), max(gate.stride(0), n), out.data_ptr(),
+                _f32flag(act_dtype), T, n // Dv, Dv, float(eps), Dv, 0, 0, None, max(out.stride(0), n))
     return out
 
 
@@ -1084,7 +1126,7 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
                 portion_rows: int = 0, max_len: int = 0, softcap: float = 0.0, sink: bool = False,
                 all_value_heads: bool = False, sinks: Optional[torch.Tensor] = None, slopes: Optional[torch.Tensor] = None,
                 keep: int = 0, gate: Optional[torch.Tensor] = None, out_scale: float = 1.0,
-                out: Optional[torch.Tensor] = None) -> torch.Tensor:
+                out: Optional[torch.Tensor] = None, value_share: int = 1) -> torch.Tensor:
     """Attention of fp32 queries [T, H*D] over paged keys / values of widths D / Dv. The row at
     position p sees keys j <= p with j >= floor(p / chunk) * chunk (``chunk`` > 0) and
     j > p - window (``window`` > 0), counted from the start of its sequence. ``row_seq`` [T]
@@ -1098,12 +1140,15 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
     the scaled score (before the cap). ``keep``: the first ``keep`` keys of the sequence stay visible outside the
     window / chunk. ``gate`` (fp32 logits [T, H], may be a column slice): head h's result is multiplied by its
     sigmoid; ``out_scale`` multiplies every result. ``out``: write into this [T, H * Dv] block (of a wider matrix).
+    ``value_share``: that many neighbouring key heads share a value head (value planes of G / value_share heads).
 
     Two kernels: the first ``n_portions`` sequences (rows [0, portion_rows), the longest of
     ``max_len`` rows) are prompt portions and go, 64 rows of a head per block, through fp32 MFMA
     tiles; the rows behind them (single decoded tokens) and shapes the tiles do not take go
     through the row kernel, one wave per (row, head)."""
     T = q.shape[0]
+    if value_share < 1 or G % value_share or (value_share > 1 and all_value_heads):
+        raise ValueError("attn_masked: the key heads that share a value head divide the key heads")
     for c in (sinks, slopes):
         if c is not None and (c.numel() != H or c.dtype != torch.float32 or not c.is_contiguous()):
             raise ValueError("attn_masked: sinks and slopes are fp32, one per head")
@@ -1113,11 +1158,11 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
         raise ValueError("attn_masked: the output block is [T, H * Dv] in the activation type")
     if not q.is_cuda:
         y = ref.attn_masked(q, k_cache, v_cache, block_tables, cu_q, positions, H, G, D, Dv, scale, chunk, window,
-                            act_dtype, softcap, sink, all_value_heads, sinks, slopes, keep, gate, out_scale)
+                            act_dtype, softcap, sink, all_value_heads, sinks, slopes, keep, gate, out_scale, value_share)
         return y if out is None else out.copy_(y)
     if q.dtype != torch.float32 or not q.is_contiguous() or k_cache.dtype != v_cache.dtype:
         raise ValueError("attn_masked: contiguous fp32 queries, caches of one type")
-    k_ld, v_ld = _cache_ld(k_cache, G, D, "key"), _cache_ld(v_cache, G, Dv, "value")
+    k_ld, v_ld = _cache_ld(k_cache, G, D, "key"), _cache_ld(v_cache, G // value_share, Dv, "value")
     if k_cache.shape[2] != v_cache.shape[2]:
         raise ValueError("attn_masked: key and value planes of one block size")
     if not 0 <= portion_rows <= T or n_portions > block_tables.shape[0]:
@@ -1138,7 +1183,7 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
     def opts(first: int):
         g = gate[first:] if gate is not None else None
         return (float(softcap), 1 if (sink or sinks is not None) else 0, _hip().ptr(sinks), _hip().ptr(slopes), int(keep),
-                _hip().ptr(g), max(gate.stride(0), H) if gate is not None else 0, float(out_scale), o_row)
+                _hip().ptr(g), max(gate.stride(0), H) if gate is not None else 0, float(out_scale), o_row, int(value_share))
     first = 0
     # value heads side by side in one tile: equal groups whose width the tiles take (whole MFMA steps of 16 columns)
     tile_cols = max([n * Dv for n in range(1, nv + 1) if nv % n == 0 and Dv % 8 == 0 and attn_tile_ok(D, n * Dv)] or [0])
@@ -1268,14 +1313,21 @@ def mlstm_out(o: torch.Tensor, m: torch.Tensor, w: torch.Tensor, gate: torch.Ten
     return out
 
 
-def glu(y: torch.Tensor, act_dtype: torch.dtype, kind: str = "relu") -> torch.Tensor:
-    """fp32 y [T, 2n] = (gate | up) -> act(gate) * up [T, n] in ``act_dtype`` (act: relu or silu)."""
-    if not y.is_cuda:
-        return ref.glu(y, act_dtype, kind)
+GLU_KINDS = ("relu", "silu", "gelu_tanh")
+
+
+def glu(y: torch.Tensor, act_dtype: torch.dtype, kind: str = "relu", out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """fp32 y [T, 2n] = (gate | up) -> act(gate) * up [T, n] in ``act_dtype`` (act: relu, silu or the tanh form of gelu).
+    ``out``: write into this [T, n] block (of a wider matrix)."""
+    if kind not in GLU_KINDS:
+        raise ValueError(f"glu: activation {kind!r}: {', '.join(GLU_KINDS)}")
     T, n = y.shape[0], y.shape[1] // 2
+    if not y.is_cuda:
+        r = ref.glu(y, act_dtype, kind)
+        return r if out is None else out.copy_(r)
     y = y.contiguous()
-    out = torch.empty(T, n, dtype=act_dtype, device=y.device)
-    _hip().call("lc_glu", y.data_ptr(), out.data_ptr(), _f32flag(act_dtype), T, n, {"relu": 0, "silu": 1}[kind])
+    out = _out_block(out, T, n, act_dtype, y.device, "glu")
+    _hip().call("lc_glu", y.data_ptr(), out.data_ptr(), _f32flag(act_dtype), T, n, GLU_KINDS.index(kind), max(out.stride(0), n))
     return out
 
 
@@ -1659,10 +1711,34 @@ def gated_step(x: torch.Tensor, y: Optional[torch.Tensor], gate: Optional[torch.
     p = _hip().ptr
     _hip().call("lc_gated_step", x.data_ptr(), p(y.contiguous() if y is not None else None), p(gate),
                 max(gate.stride(0), d) if gate is not None else 0, p(w_out), p(w_in), float(eps), p(ha), p(h32),
-                _f32flag(act_dtype), p(shift.mu) if shift else None, p(shift.state) if shift else None,
+                None, None, _f32flag(act_dtype), p(shift.mu) if shift else None, p(shift.state) if shift else None,
                 max(shift.state.stride(0), d) if shift else 0, p(lay.row_seq) if shift else None,
                 p(positions) if shift else None, p(lay.state_slots) if shift else None, p(hs), T, d)
     return ha, (ha if f32 else h32), hs
+
+
+def dual_norm_step(x: torch.Tensor, y: Optional[torch.Tensor], w1: Optional[torch.Tensor], w2: Optional[torch.Tensor], eps: float,
+                   act_dtype: torch.dtype):
+    """The residual step of a layer whose mixer and feed-forward read the same stream through norms of their own, one
+    launch: x (fp32, in place) += y (when given); returns (rms_norm(x) * w1, rms_norm(x) * w2) in ``act_dtype`` (``w2``, or
+    both, may be None)."""
+    T, d = x.shape
+    if x.dtype != torch.float32 or not x.is_contiguous():
+        raise ValueError("dual_norm_step: the residual stream is a contiguous fp32 tensor")
+    if y is not None and (y.shape != x.shape or y.dtype != torch.float32):
+        raise ValueError("dual_norm_step: the sublayers' output must be fp32 of the stream's shape")
+    if w1 is None and w2 is not None:
+        raise ValueError("dual_norm_step: the second norm stands beside the first")
+    if not x.is_cuda:
+        return ref.dual_norm_step(x, y, w1, w2, eps, act_dtype)
+    if y is None and w1 is None:
+        return None, None
+    h1 = torch.empty(T, d, dtype=act_dtype, device=x.device) if w1 is not None else None
+    h2 = torch.empty(T, d, dtype=act_dtype, device=x.device) if w2 is not None else None
+    p = _hip().ptr
+    _hip().call("lc_gated_step", x.data_ptr(), p(y.contiguous() if y is not None else None), None, 0, None, p(w1), float(eps),
+                p(h1), None, p(w2), p(h2), _f32flag(act_dtype), None, None, 0, None, None, None, None, T, d)
+    return h1, h2
 
 
 def token_shift(h: torch.Tensor, shift: ShiftState, lay, positions: torch.Tensor, act_dtype: torch.dtype) -> torch.Tensor:
@@ -1689,20 +1765,27 @@ def attn_prep(qkv: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Te
               conv_state: Optional[torch.Tensor] = None, norm: str = "", q_norm: Optional[torch.Tensor] = None,
               k_norm: Optional[torch.Tensor] = None, eps: float = 0.0, inv_freq: Optional[torch.Tensor] = None,
               rot_dims: int = 0, pairs: bool = False, temperature: Tuple[float, float] = (0.0, 1.0),
-              v_first: Optional[torch.Tensor] = None, v_mix: float = 0.0, save_v: bool = False):
+              v_first: Optional[torch.Tensor] = None, v_mix: float = 0.0, save_v: bool = False, rot_mag: float = 1.0,
+              maps: int = 1):
     """Attention pre-processing and cache write in one launch. qkv fp32 [T, >= (H + G) D + G Dv] = q | k | v. In this
     order, each optional: a causal convolution per channel (``conv_w`` fp32 [taps, C], the newest tap last;
     ``conv_state`` fp32 [slots, (taps - 1) * C], the sequences' last inputs, oldest first, updated in place); RMS
     norms over the ``"whole"`` projection (weights [H D] / [G D]) or per ``"head"`` ([D]); a turn of the first ``rot_dims``
-    coordinates of q and k heads (``inv_freq`` fp64; ``pairs``: neighbours); q times
+    coordinates of q and k heads (``inv_freq`` fp64; ``pairs``: neighbours; ``rot_mag``: factor on cosine and sine); q times
     1 + coef * ln(floor((p + 1) / every) + 1) for ``temperature`` = (coef, every); values mixed with ``v_first`` (fp32
-    [T, G Dv]) by ``v_mix``. Returns (q fp32 [T, H D], the values before the mix when ``save_v``)."""
+    [T, G Dv]) by ``v_mix``. Returns (q fp32 [T, H D], the values before the mix when ``save_v``).
+    ``maps`` > 1: every head has that many query and key maps over one value: q and k are laid out head by head, map by
+    map, H and G count the maps of all heads, the value heads are G / maps, and the queries are returned in the order
+    (key/value head, map, head of the group): the H / G queries of a key map side by side."""
     T = qkv.shape[0]
-    C = (H + G) * D + G * Dv
+    if maps < 1 or G % maps:
+        raise ValueError("attn_prep: every head has the same number of maps")
+    GV = G // maps
+    C = (H + G) * D + GV * Dv
     taps = conv_w.shape[0] if conv_w is not None else 0
     if qkv.dtype != torch.float32 or qkv.stride(1) != 1 or qkv.shape[1] < C:
         raise ValueError("attn_prep: fp32 projections q | k | v")
-    if k_cache.shape[1:] != (G, k_cache.shape[2], D) or v_cache.shape[1:] != (G, k_cache.shape[2], Dv) or \
+    if k_cache.shape[1:] != (G, k_cache.shape[2], D) or v_cache.shape[1:] != (GV, k_cache.shape[2], Dv) or \
             not k_cache.is_contiguous() or not v_cache.is_contiguous() or k_cache.dtype != v_cache.dtype:
         raise ValueError("attn_prep: cache planes do not fit the head sizes")
     if conv_w is not None and (conv_w.shape != (taps, C) or conv_w.dtype != torch.float32 or not conv_w.is_contiguous()):
@@ -1715,21 +1798,21 @@ def attn_prep(qkv: torch.Tensor, positions: torch.Tensor, slot_mapping: torch.Te
         raise ValueError("attn_prep: norms over the whole projection or per head, with weights of that size")
     if rot_dims and (inv_freq is None or inv_freq.dtype != torch.float64 or inv_freq.numel() != rot_dims // 2):
         raise ValueError("attn_prep: rot_dims / 2 fp64 frequencies are needed")
-    if v_first is not None and (v_first.shape != (T, G * Dv) or v_first.dtype != torch.float32 or v_first.stride(1) != 1):
+    if v_first is not None and (v_first.shape != (T, GV * Dv) or v_first.dtype != torch.float32 or v_first.stride(1) != 1):
         raise ValueError("attn_prep: the values to mix in are fp32 [T, G * Dv]")
     if C + rot_dims > ATTN_PREP_MAX_FLOATS:
         raise ValueError("attn_prep: a token's channels exceed one block's LDS")
     if not qkv.is_cuda:
         return ref.attn_prep(qkv, positions, slot_mapping, lay, k_cache, v_cache, H, G, D, Dv, conv_w, conv_state, norm, q_norm,
-                             k_norm, eps, inv_freq, rot_dims, pairs, temperature, v_first, v_mix, save_v)
+                             k_norm, eps, inv_freq, rot_dims, pairs, temperature, v_first, v_mix, save_v, rot_mag, maps)
     q = torch.empty(T, H * D, dtype=torch.float32, device=qkv.device)
-    vs = torch.empty(T, G * Dv, dtype=torch.float32, device=qkv.device) if save_v else None
+    vs = torch.empty(T, GV * Dv, dtype=torch.float32, device=qkv.device) if save_v else None
     p = _hip().ptr
     _hip().call("lc_attn_prep", qkv.data_ptr(), max(qkv.stride(0), qkv.shape[1]), p(conv_w), taps,
                 p(conv_state) if taps > 1 else None, max(conv_state.stride(0), conv_state.shape[1]) if taps > 1 else 0,
                 ("", "whole", "head").index(norm), p(q_norm), p(k_norm), float(eps), p(inv_freq), int(rot_dims),
-                1 if pairs else 0, float(temperature[0]), float(temperature[1]), p(v_first),
-                max(v_first.stride(0), G * Dv) if v_first is not None else 0, float(v_mix), p(vs), p(lay.row_seq),
+                1 if pairs else 0, float(rot_mag), int(maps), float(temperature[0]), float(temperature[1]), p(v_first),
+                max(v_first.stride(0), GV * Dv) if v_first is not None else 0, float(v_mix), p(vs), p(lay.row_seq),
                 p(lay.cu_q), positions.data_ptr(), p(lay.state_slots), slot_mapping.data_ptr(), k_cache.data_ptr(),
                 v_cache.data_ptr(), _f32flag(k_cache.dtype), q.data_ptr(), T, H, G, D, Dv, k_cache.shape[2])
     return q, vs
@@ -1774,6 +1857,96 @@ def rownorm_gate(o: torch.Tensor, w: torch.Tensor, gate: torch.Tensor, eps: floa
     o = o.contiguous()
     _hip().call("lc_headnorm_gate", o.data_ptr(), w.data_ptr(), gate.data_ptr(), max(gate.stride(0), n), out.data_ptr(),
                 _f32flag(act_dtype), T, 1, n, float(eps), n, 0, 1, None, max(out.stride(0), n))
+    return out
+
+
+# ---- gated delta rule, differential attention (hybrid_delta.hip) ----
+@dataclass
+class DeltaOperands:
+    """What a gated delta rule reads per row, fp32: unit queries (times D^-1/2) and unit keys ``qk`` [T, 2, G, Dp], values
+    ``v`` [T, H, Dvp] (widths padded to multiples of 16 with zeros on the GPU), ``gates`` [T, H, 2] = (step size, log
+    decay), ``kq`` [T, G] = q . k."""
+
+    qk: torch.Tensor
+    v: torch.Tensor
+    gates: torch.Tensor
+    kq: Optional[torch.Tensor]
+
+
+def delta_prep(proj: torch.Tensor, conv_w: torch.Tensor, conv_state: Optional[torch.Tensor], col_b: int, col_a: int,
+               neg_rate: torch.Tensor, dt_bias: torch.Tensor, positions: torch.Tensor, lay, H: int, G: int, D: int,
+               Dv: int) -> DeltaOperands:
+    """Operands of a gated delta rule, one launch. proj fp32 [T, >= 2 G D + H Dv] = q | k | v | ...: a causal convolution
+    over time per channel (``conv_w`` fp32 [taps, channels], the newest tap last; ``conv_state`` fp32 [slots, (taps - 1) *
+    channels], the sequences' last inputs, oldest first, updated in place), silu, q and k as unit vectors per head
+    (x / sqrt(sum x^2 + 1e-6)), q times D^-1/2. Step size sigmoid of column ``col_b`` + h, log decay
+    neg_rate[h] * softplus(column ``col_a`` + h, plus dt_bias[h])."""
+    T, C = proj.shape[0], 2 * G * D + H * Dv
+    taps = conv_w.shape[0]
+    if proj.dtype != torch.float32 or proj.stride(1) != 1 or proj.shape[1] < max(C, col_b + H, col_a + H) or H % G:
+        raise ValueError("delta_prep: fp32 projections q | k | v | gates of whole groups of heads")
+    if conv_w.shape[1] != C or conv_w.dtype != torch.float32 or not conv_w.is_contiguous():
+        raise ValueError("delta_prep: convolution weights are fp32 [taps, channels]")
+    if lay.state_slots is None or (taps > 1 and (conv_state is None or conv_state.shape[1] != (taps - 1) * C
+                                                 or conv_state.dtype != torch.float32 or conv_state.stride(1) != 1)):
+        raise ValueError("delta_prep: the convolution's inputs before the step are fp32 [slots, (taps - 1) * channels]")
+    for c in (neg_rate, dt_bias):
+        if c.numel() != H or c.dtype != torch.float32 or not c.is_contiguous():
+            raise ValueError("delta_prep: decay rates and biases are fp32, one per head")
+    if C > ATTN_PREP_MAX_FLOATS:
+        raise ValueError("delta_prep: a token's channels exceed one block's LDS")
+    if not proj.is_cuda:
+        return DeltaOperands(*ref.delta_prep(proj, conv_w, conv_state, col_b, col_a, neg_rate, dt_bias, positions, lay, H, G, D, Dv), None)
+    Dp, Dvp = (D + 15) // 16 * 16, (Dv + 15) // 16 * 16
+    dev = proj.device
+    x = DeltaOperands(torch.empty(T, 2, G, Dp, dtype=torch.float32, device=dev), torch.empty(T, H, Dvp, dtype=torch.float32, device=dev),
+                      torch.empty(T, H, 2, dtype=torch.float32, device=dev), torch.empty(T, G, dtype=torch.float32, device=dev))
+    p = _hip().ptr
+    _hip().call("lc_delta_prep", proj.data_ptr(), max(proj.stride(0), proj.shape[1]), conv_w.data_ptr(), taps,
+                p(conv_state) if taps > 1 else None, max(conv_state.stride(0), conv_state.shape[1]) if taps > 1 else 0,
+                int(col_b), int(col_a), neg_rate.data_ptr(), dt_bias.data_ptr(), lay.row_seq.data_ptr(), lay.cu_q.data_ptr(),
+                positions.data_ptr(), lay.state_slots.data_ptr(), x.qk.data_ptr(), x.v.data_ptr(), x.gates.data_ptr(),
+                x.kq.data_ptr(), T, H, G, D, Dv, float(D) ** -0.5)
+    return x
+
+
+def delta_scan(x: DeltaOperands, state: torch.Tensor, cu_q: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, H: int,
+               G: int, D: int, Dv: int, max_len: int = 1) -> torch.Tensor:
+    """Gated delta rule over the step's sequences: per head S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q (head h
+    reads the q / k head h / (H / G)). state fp32 [slots, H*D*Dv] (may be a column block of a wider plane), updated in
+    place. Portions of a few rows run row by row, longer ones in chunks of 64 rows whose products are matrix products.
+    ``max_len``: the longest portion of the step (host-known). Returns the read-out fp32 [T, H*Dv]."""
+    if state.dtype != torch.float32 or state.stride(1) != 1 or state.shape[1] != H * D * Dv or D > 256 or H % G:
+        raise ValueError("delta_scan: fp32 state of the heads' sizes (key width at most 256)")
+    if not x.qk.is_cuda:
+        return ref.delta_scan(x.qk, x.v, x.gates, state, cu_q, positions, slots, H, G, D, Dv)
+    T, B = x.qk.shape[0], slots.numel()
+    if x.qk.shape != (T, 2, G, (D + 15) // 16 * 16) or x.v.shape != (T, H, (Dv + 15) // 16 * 16) or x.gates.shape != (T, H, 2):
+        raise ValueError("delta_scan: the operands do not fit the head sizes")
+    out = torch.empty(T, H * Dv, dtype=torch.float32, device=x.qk.device)
+    n = int(_hip().lib().lc_delta_scratch_floats(T, B, int(max_len), H, D, Dv))
+    scratch = torch.empty(n, dtype=torch.float32, device=x.qk.device) if n else None
+    _hip().call("lc_delta_scan", x.qk.data_ptr(), x.v.data_ptr(), x.gates.data_ptr(), x.kq.data_ptr(), state.data_ptr(),
+                max(state.stride(0), state.shape[1]), cu_q.data_ptr(), positions.data_ptr(), slots.data_ptr(), out.data_ptr(), T, B,
+                H, G, D, Dv, int(max_len), _hip().ptr(scratch))
+    return out
+
+
+def diff_norm(o: torch.Tensor, lam: float, eps: float, scale: float, H: int, G: int, Dv: int, act_dtype: torch.dtype,
+              out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Two attention maps per head, o fp32 [T, G * 2 * (H / G) * Dv] in the order (key/value head, map, head of the group):
+    y = o_1 - lam * o_2, y / sqrt(mean(y^2) + eps) * scale per head, [T, H * Dv] in ``act_dtype`` (into ``out``, a block of a
+    wider matrix, when given)."""
+    T = o.shape[0]
+    if o.shape[1] != 2 * H * Dv or o.dtype != torch.float32 or H % G or Dv > 512:
+        raise ValueError("diff_norm: fp32 results of two maps per head (value width at most 512)")
+    if not o.is_cuda:
+        y = ref.diff_norm(o, lam, eps, scale, H, G, Dv, act_dtype)
+        return y if out is None else out.copy_(y)
+    o = o.contiguous()
+    out = _out_block(out, T, H * Dv, act_dtype, o.device, "diff_norm")
+    _hip().call("lc_diff_norm", o.data_ptr(), float(lam), float(eps), float(scale), out.data_ptr(), _f32flag(act_dtype),
+                max(out.stride(0), H * Dv), T, H, G, Dv)
     return out
 
 

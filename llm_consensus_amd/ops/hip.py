@@ -60,7 +60,7 @@ _SIGNATURES = {
     "lc_ep_recv_index": [_P, _I, _I, _I, _P, _P, _P],
     "lc_scatter_rows": [_P, _P, _P, _I, _I, _P, _P],
     # hybrid decoders (hybrid.hip)
-    "lc_embed_rows": [_P, _P, _I, _P, _P, _I, _I, _I, _I, _P, _P, _F, _P, _P, _P],
+    "lc_embed_rows": [_P, _P, _I, _P, _P, _I, _I, _I, _I, _P, _P, _F, _P, _P, _P, _L, _L, _L, _P, _L, _P, _P, _P, _P],
     "lc_scalar_norm_add": [_P, _P, _P, _F, _P, _I, _I, _I, _P],
     "lc_relu2": [_P, _P, _I, _I, _I, _I, _P],
     "lc_mingru_scan": [_P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _P, _P],
@@ -68,15 +68,15 @@ _SIGNATURES = {
     "lc_headnorm_gate": [_P, _P, _P, _I, _P, _I, _I, _I, _I, _F, _I, _I, _I, _P, _I, _P],
     "lc_qkv_prep": [_P, _I, _P, _P, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _P],
     "lc_attn_masked": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I,
-                       _I, _I, _F, _I, _P, _P, _I, _P, _I, _F, _I, _I, _I, _I, _I, _I, _P],
+                       _I, _I, _F, _I, _P, _P, _I, _P, _I, _F, _I, _I, _I, _I, _I, _I, _I, _P],
     "lc_attn_tile": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I,
-                     _I, _I, _F, _I, _P, _P, _I, _P, _I, _F, _I, _I, _I, _I, _I, _P],
+                     _I, _I, _F, _I, _P, _P, _I, _P, _I, _F, _I, _I, _I, _I, _I, _I, _P],
     "lc_gemm_any": [_P, _I, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P],
     "lc_add_rmsnorm": [_P, _P, _P, _F, _P, _I, _I, _I, _P],
     "lc_latent_write": [_P, _I, _I, _I, _P, _F, _P, _P, _I, _I, _I, _P],
     "lc_head_linear": [_P, _I, _I, _P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
     "lc_mlstm_scan": [_P, _I, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P],
-    "lc_glu": [_P, _P, _I, _I, _I, _I, _P],
+    "lc_glu": [_P, _P, _I, _I, _I, _I, _I, _P],
     "lc_add_dyt": [_P, _P, _F, _F, _P, _P, _P, _I, _I, _I, _I, _P],
     "lc_glu_clamped": [_P, _I, _I, _I, _I, _F, _F, _F, _P, _P, _P, _I, _I, _P],
     "lc_rope_pairs_write": [_P, _I, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P],
@@ -88,19 +88,24 @@ _SIGNATURES = {
     "lc_latent_rope_write": [_P, _I, _I, _P, _F, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "lc_xielu": [_P, _I, _P, _I, _I, _I, _F, _F, _P],
     # gated residual steps, token shifts, attention pre-processing with convolutions and mixed values (hybrid_gated.hip)
-    "lc_gated_step": [_P, _P, _P, _I, _P, _P, _F, _P, _P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _P],
+    "lc_gated_step": [_P, _P, _P, _I, _P, _P, _F, _P, _P, _P, _P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _P],
     "lc_token_shift": [_P, _P, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _P],
-    "lc_attn_prep": [_P, _I, _P, _I, _P, _L, _I, _P, _P, _F, _P, _I, _I, _F, _F, _P, _I, _F, _P, _P, _P, _P, _P, _P, _P, _P,
+    "lc_attn_prep": [_P, _I, _P, _I, _P, _L, _I, _P, _P, _F, _P, _I, _I, _F, _I, _F, _F, _P, _I, _F, _P, _P, _P, _P, _P, _P, _P, _P,
                      _I, _P, _I, _I, _I, _I, _I, _I, _P],
     "lc_softcap": [_P, _L, _F, _P],
     "lc_lightning_scan": [_P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _P],
+    # gated delta rule, differential attention (hybrid_delta.hip)
+    "lc_delta_prep": [_P, _I, _P, _I, _P, _L, _I, _I, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _P],
+    "lc_delta_scan": [_P, _P, _P, _P, _P, _L, _P, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _P, _P],
+    "lc_diff_norm": [_P, _F, _F, _F, _P, _I, _I, _I, _I, _I, _I, _P],
     # routed feed-forwards of hybrid decoders (hybrid_moe.hip)
     "lc_route_grouped": [_P, _I, _P, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P],
     "lc_moe_sort": [_P, _I, _I, _I, _P, _P, _P, _P, _P, _P],
     "lc_gemm_any_grouped": [_P, _I, _I, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P],
     "lc_moe_mix": [_P, _P, _P, _P, _P, _I, _P, _P, _I, _P, _I, _I, _I, _I, _P],
 }
-_RESTYPES = {"lc_scan_scratch_floats": ([_I, _I, _L, _L], c_longlong)}      # helpers that return no status
+_RESTYPES = {"lc_scan_scratch_floats": ([_I, _I, _L, _L], c_longlong),
+             "lc_delta_scratch_floats": ([_I, _I, _I, _I, _I, _I], c_longlong)}      # helpers that return no status
 
 _lib = None
 

@@ -402,14 +402,15 @@ def qkv_prep(qkv: torch.Tensor, q_norm: torch.Tensor, k_norm: Optional[torch.Ten
 def attn_masked(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, positions, H: int, G: int, D: int, Dv: int,
                 scale: float, chunk: int, window: int, act_dtype, softcap: float = 0.0, sink: bool = False,
                 all_value_heads: bool = False, sinks=None, slopes=None, keep: int = 0, gate=None,
-                out_scale: float = 1.0) -> torch.Tensor:
+                out_scale: float = 1.0, value_share: int = 1) -> torch.Tensor:
     """q fp32 [T, H*D]; paged keys [blocks, G, BS, D] and values [blocks, G, BS, Dv]. The row at
     position p sees keys j <= p with j >= floor(p / chunk) * chunk (``chunk`` > 0) and
     j > p - window (``window`` > 0). Scores, softmax and the weighted sum in fp32. ``softcap`` > 0: scores
     become softcap * tanh(score / softcap); ``sink``: the softmax's denominator carries an extra 1 (an entry of
     score 0, or ``sinks`` [H], without a value); ``slopes`` [H]: slope * (p - j) off the scaled score before the
     cap; ``keep``: the first keys stay visible; ``gate`` [T, H]: sigmoid factor per head; ``all_value_heads``: every
-    head's weights meet the values of all G value heads, result [T, H * G * Dv]."""
+    head's weights meet the values of all G value heads, result [T, H * G * Dv]; ``value_share``: that many neighbouring
+    key heads share a value head (planes of G / value_share heads)."""
     T = q.shape[0]
     nv = G if all_value_heads else 1
     out = torch.zeros(T, H * nv * Dv, dtype=torch.float32, device=q.device)
@@ -424,7 +425,8 @@ def attn_masked(q: torch.Tensor, k_cache, v_cache, block_tables, cu_q, positions
         nb = (n + BS - 1) // BS
         blocks = block_tables[b, :nb].long()
         K = k_cache[blocks].permute(1, 0, 2, 3).reshape(G, nb * BS, D)[:, :n].float()
-        V = v_cache[blocks].permute(1, 0, 2, 3).reshape(G, nb * BS, Dv)[:, :n].float()
+        V = v_cache[blocks].permute(1, 0, 2, 3).reshape(G // value_share, nb * BS, Dv)[:, :n].float()
+        V = V.repeat_interleave(value_share, 0)
         Q = q[r0:r1].float().view(r1 - r0, G, rep, D)
         sc = torch.einsum("qgrd,gkd->grqk", Q, K) * scale
         key = torch.arange(n, device=q.device)[None, :]
@@ -562,7 +564,7 @@ def glu(y: torch.Tensor, act_dtype, kind: str = "relu") -> torch.Tensor:
     """y [T, 2n] = (gate | up) -> act(gate) * up."""
     n = y.shape[1] // 2
     g, u = y[:, :n].float(), y[:, n:].float()
-    g = torch.relu(g) if kind == "relu" else g * torch.sigmoid(g)
+    g = {"relu": torch.relu, "silu": torch.nn.functional.silu, "gelu_tanh": lambda z: torch.nn.functional.gelu(z, approximate="tanh")}[kind](g)
     return (g * u).to(act_dtype)
 
 
@@ -785,6 +787,14 @@ def gated_step(x: torch.Tensor, y, gate, w_out, w_in, eps: float, act_dtype, shi
     return h.to(act_dtype), h, (token_shift(h, shift, lay, positions, act_dtype) if shift is not None else None)
 
 
+def dual_norm_step(x: torch.Tensor, y, w1, w2, eps: float, act_dtype):
+    """x (fp32, in place) += y; (rms_norm(x) * w1, rms_norm(x) * w2)."""
+    if y is not None:
+        x.add_(y.float())
+    u = x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps)
+    return tuple((u * w.float()).to(act_dtype) if w is not None else None for w in (w1, w2))
+
+
 def token_shift(h: torch.Tensor, shift, lay, positions, act_dtype) -> torch.Tensor:
     """Row t moves towards the row before it in its sequence by ``shift.mu``; a portion's first row towards the stored
     row (zeros at position 0), which becomes the portion's last row."""
@@ -800,30 +810,38 @@ def token_shift(h: torch.Tensor, shift, lay, positions, act_dtype) -> torch.Tens
     return (h + (prev - h) * shift.mu.float()).to(act_dtype)
 
 
+def causal_conv(u: torch.Tensor, conv_w: torch.Tensor, conv_state, positions, lay) -> torch.Tensor:
+    """u fp32 [T, C], conv_w [taps, C]: per channel sum_j w[j] u_(t - taps + 1 + j) inside each sequence; inputs before the
+    step from ``conv_state`` [slots, (taps - 1) * C] (oldest first, updated), zeros before position 0."""
+    C = u.shape[1]
+    hist = conv_w.shape[0] - 1
+    y = torch.zeros_like(u)
+    for b in range(len(lay.cu_q) - 1):
+        r0, r1 = int(lay.cu_q[b]), int(lay.cu_q[b + 1])
+        if r1 <= r0:
+            continue
+        slot = int(lay.state_slots[b]) if lay.state_slots is not None else -1
+        before = torch.zeros(hist, C, dtype=torch.float32, device=u.device)
+        if hist and slot >= 0 and int(positions[r0]) != 0:
+            before = conv_state[slot].view(hist, C).clone()
+        ext = torch.cat([before, u[r0:r1]], 0)
+        y[r0:r1] = sum(conv_w[j].float() * ext[j:j + r1 - r0] for j in range(hist + 1))
+        if hist and slot >= 0:
+            conv_state[slot] = ext[-hist:].reshape(-1)
+    return y
+
+
 def attn_prep(qkv: torch.Tensor, positions, slot_mapping, lay, k_cache, v_cache, H: int, G: int, D: int, Dv: int, conv_w,
               conv_state, norm: str, q_norm, k_norm, eps: float, inv_freq, rot_dims: int, pairs: bool, temperature, v_first,
-              v_mix: float, save_v: bool):
+              v_mix: float, save_v: bool, rot_mag: float = 1.0, maps: int = 1):
     """q | k | v of the step's rows: convolution over time, norms, rotation, query temperature, mixed values, paged
     write. Returns (q fp32 [T, H*D], the values before the mix or None)."""
     T = qkv.shape[0]
-    C = (H + G) * D + G * Dv
+    GV = G // maps
+    C = (H + G) * D + GV * Dv
     u = qkv[:, :C].float()
     if conv_w is not None:
-        hist = conv_w.shape[0] - 1
-        y = torch.zeros_like(u)
-        for b in range(len(lay.cu_q) - 1):
-            r0, r1 = int(lay.cu_q[b]), int(lay.cu_q[b + 1])
-            if r1 <= r0:
-                continue
-            slot = int(lay.state_slots[b]) if lay.state_slots is not None else -1
-            before = torch.zeros(hist, C, dtype=torch.float32, device=u.device)
-            if hist and slot >= 0 and int(positions[r0]) != 0:
-                before = conv_state[slot].view(hist, C).clone()
-            ext = torch.cat([before, u[r0:r1]], 0)
-            y[r0:r1] = sum(conv_w[j].float() * ext[j:j + r1 - r0] for j in range(hist + 1))
-            if hist and slot >= 0:
-                conv_state[slot] = ext[-hist:].reshape(-1)
-        u = y
+        u = causal_conv(u, conv_w, conv_state, positions, lay)
     q, k, v = u[:, :H * D].view(T, H, D), u[:, H * D:(H + G) * D].view(T, G, D), u[:, (H + G) * D:]
 
     def rms(z, w):
@@ -833,9 +851,15 @@ def attn_prep(qkv: torch.Tensor, positions, slot_mapping, lay, k_cache, v_cache,
     elif norm == "head":
         q, k = rms(q, q_norm), rms(k, k_norm)
     q, k = rope_any(q, positions, rot_dims, inv_freq, pairs), rope_any(k, positions, rot_dims, inv_freq, pairs)
+    if rot_mag != 1.0 and rot_dims:
+        q, k = q.clone(), k.clone()
+        q[..., :rot_dims] *= rot_mag
+        k[..., :rot_dims] *= rot_mag
+    if maps > 1:                                # (key/value head, head of the group, map) -> (key/value head, map, head)
+        q = q.view(T, GV, H // G, maps, D).transpose(2, 3)
     if temperature[0] != 0.0:
         f = torch.floor((positions.double() + 1) / temperature[1]) + 1
-        q = q * (1 + temperature[0] * torch.log(f.float()))[:, None, None]
+        q = q.reshape(T, H, D) * (1 + temperature[0] * torch.log(f.float()))[:, None, None]
     saved = v.clone() if save_v else None
     if v_first is not None:
         v = (1 - v_mix) * v + v_mix * v_first.float()
@@ -844,7 +868,7 @@ def attn_prep(qkv: torch.Tensor, positions, slot_mapping, lay, k_cache, v_cache,
     ok = slots >= 0
     blk, off = slots[ok] // BS, slots[ok] % BS
     k_cache[blk, :, off, :] = k[ok].to(k_cache.dtype)
-    v_cache[blk, :, off, :] = v.reshape(T, G, Dv)[ok].to(v_cache.dtype)
+    v_cache[blk, :, off, :] = v.reshape(T, GV, Dv)[ok].to(v_cache.dtype)
     return q.reshape(T, H * D).contiguous(), saved
 
 
@@ -872,3 +896,68 @@ def rownorm_gate(o: torch.Tensor, w, gate, eps: float, act_dtype) -> torch.Tenso
     """o / sqrt(mean(o^2) + eps) * w over whole rows, times sigmoid(gate)."""
     v = o.float()
     return (v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * w.float() * torch.sigmoid(gate.float())).to(act_dtype)
+
+
+# ------------------------------------------------------------------ hybrid decoders: a second embedding table indexed by token
+# pairs, gated delta rule, differential attention
+def pair_rows(ids: torch.Tensor, positions, lay, pair, vocab: int) -> torch.Tensor:
+    """Row of the pair table per token: (previous * mul_prev + current * mul_cur) mod buckets, row ``buckets`` at a
+    sequence's start. ``pair.last`` [slots, 1] holds the sequences' last tokens (updated)."""
+    tok = ids.long().clamp(0, vocab - 1)
+    rows = torch.full_like(tok, pair.buckets)
+    for b in range(len(lay.cu_q) - 1):
+        r0, r1, slot = int(lay.cu_q[b]), int(lay.cu_q[b + 1]), int(lay.state_slots[b])
+        if r1 <= r0:
+            continue
+        for t in range(r0, r1):
+            prev = int(tok[t - 1]) if t > r0 else (int(pair.last[slot, 0]) if slot >= 0 and int(positions[r0]) != 0 else -1)
+            if prev >= 0:
+                rows[t] = (prev * pair.mul_prev + int(tok[t]) * pair.mul_cur) % pair.buckets
+        if slot >= 0:
+            pair.last[slot, 0] = tok[r1 - 1].to(pair.last.dtype)
+    return rows
+
+
+def delta_prep(proj: torch.Tensor, conv_w, conv_state, col_b: int, col_a: int, neg_rate, dt_bias, positions, lay, H: int, G: int,
+               D: int, Dv: int):
+    """(qk [T, 2, G, D], v [T, H, Dv], gates [T, H, 2]) of a gated delta rule (see ops.delta_prep)."""
+    T, C = proj.shape[0], 2 * G * D + H * Dv
+    u = torch.nn.functional.silu(causal_conv(proj[:, :C].float(), conv_w, conv_state, positions, lay))
+    qk = u[:, :2 * G * D].view(T, 2, G, D)
+    qk = qk / torch.sqrt(qk.pow(2).sum(-1, keepdim=True) + 1e-6)
+    qk[:, 0] *= D ** -0.5
+    beta = torch.sigmoid(proj[:, col_b:col_b + H].float())
+    log_g = neg_rate.float() * torch.nn.functional.softplus(proj[:, col_a:col_a + H].float() + dt_bias.float())
+    return qk, u[:, 2 * G * D:].view(T, H, Dv), torch.stack([beta, log_g], -1)
+
+
+def delta_scan(qk: torch.Tensor, v: torch.Tensor, gates: torch.Tensor, state, cu_q, positions, slots, H: int, G: int, D: int,
+               Dv: int) -> torch.Tensor:
+    """Per head S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q (state [slots, H*D*Dv] fp32). fp32 [T, H*Dv]."""
+    T = qk.shape[0]
+    q, k = qk[:, 0, :, :D].repeat_interleave(H // G, 1), qk[:, 1, :, :D].repeat_interleave(H // G, 1)
+    v = v[..., :Dv]
+    beta, g = gates[..., 0], torch.exp(gates[..., 1])
+    out = torch.zeros(T, H, Dv, dtype=torch.float32, device=qk.device)
+    for b in range(len(slots)):
+        r0, r1, slot = int(cu_q[b]), int(cu_q[b + 1]), int(slots[b])
+        if slot < 0 or r1 <= r0:
+            continue
+        S = state[slot].reshape(H, D, Dv).clone()
+        if int(positions[r0]) == 0:
+            S.zero_()
+        for t in range(r0, r1):
+            S = S * g[t][:, None, None]
+            u = beta[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
+            S = S + k[t][:, :, None] * u[:, None, :]
+            out[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        state[slot] = S.reshape(-1)
+    return out.view(T, H * Dv)
+
+
+def diff_norm(o: torch.Tensor, lam: float, eps: float, scale: float, H: int, G: int, Dv: int, act_dtype) -> torch.Tensor:
+    """o [T, G, 2, H / G, Dv]: y = o_1 - lam o_2 per head, rms-normed over Dv, times ``scale`` -> [T, H * Dv]."""
+    T = o.shape[0]
+    o5 = o.float().view(T, G, 2, H // G, Dv)
+    y = (o5[:, :, 0] - lam * o5[:, :, 1]).reshape(T, H, Dv)
+    return (y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps) * scale).reshape(T, H * Dv).to(act_dtype)

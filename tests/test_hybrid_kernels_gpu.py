@@ -778,3 +778,168 @@ def test_softcap():
     x = torch.randn(33, 71, generator=torch.Generator().manual_seed(1)) * 20
     got = ops.softcap_(x.to(DEV), 7.5)
     torch.testing.assert_close(got.cpu(), 7.5 * torch.tanh(x / 7.5), atol=1e-5, rtol=1e-5)
+
+
+# ---------------------------------------------------------------- token pairs, gated delta rule, differential attention
+@pytest.mark.parametrize("dt", ACTS)
+def test_embedding_of_token_pairs(dt):
+    """Portions fresh and continued, single tokens, a row without a slot, a padding row; tokens fed on the device; products
+    of token and multiplier past 32 bits."""
+    g = torch.Generator().manual_seed(3)
+    lens, starts = [9, 2, 1, 1, 1, 1], [0, 30, 0, 55, 9, 4]
+    cu, pos, rs = _seqs(lens, starts)
+    T, V, d, n = int(cu[-1]), 60000, 72, 1999
+    rs_d = rs.clone()
+    rs_d[-1] = -1
+    slots = torch.tensor([3, 0, 5, 1, -1, 2], dtype=torch.int32)
+    slots_r = slots.clone()
+    slots_r[5] = -1
+    ids = torch.randint(0, V, (T,), generator=g, dtype=torch.int32)
+    E, P = torch.randn(V, d, generator=g).to(dt), torch.randn(n + 1, d, generator=g).to(dt)
+    plane = torch.randint(0, V, (6, 4), generator=g, dtype=torch.int32)
+    fed, rows = torch.randint(0, V, (3,), generator=g, dtype=torch.int32), torch.full((T,), -1, dtype=torch.int32)
+    rows[11], rows[12] = 2, 0
+    mp, mc = (1 << 31) - 19, (1 << 31) - 61
+    for feed in (None, (fed, rows)):
+        res = []
+        for dev, r_s, sl in (("cpu", rs, slots_r), (DEV, rs_d, slots)):
+            to = lambda t: t.clone().to(dev)   # noqa: E731
+            last = to(plane)
+            x, _ = ops.embed_rows(to(ids), to(E), None, tuple(to(f) for f in feed) if feed else None, positions=to(pos),
+                                  pair=ops.PairEmbedding(to(P), n, mp, mc, last[:, 2:3]), lay=_Layout(cu, r_s, sl, dev))
+            res.append((x.cpu(), last.cpu()))
+        torch.testing.assert_close(res[1][0][:-1], res[0][0][:-1], atol=1e-6, rtol=1e-6)
+        assert torch.equal(res[0][1], res[1][1])
+        assert int(res[1][1][3, 2]) == int(ids[8]) and torch.equal(res[1][1][:, [0, 1, 3]], plane[:, [0, 1, 3]])
+
+
+@pytest.mark.parametrize("dt", ACTS)
+@pytest.mark.parametrize("T,d", [(5, 40), (3, 37), (600, 192), (2, 5000)])
+def test_residual_step_with_two_norms(dt, T, d):
+    g = torch.Generator().manual_seed(T + d)
+    x, y = torch.randn(T, d, generator=g), torch.randn(T, d, generator=g)
+    w1, w2 = torch.rand(d, generator=g) + 0.5, torch.rand(d, generator=g) - 2.0
+    for yy in (None, y):
+        for ww in ((w1, w2), (w1, None), (None, None)):
+            if yy is None and ww[0] is None:
+                continue
+            xc, xd = x.clone(), x.to(DEV)
+            want = ops.dual_norm_step(xc, yy, *ww, 1e-5, dt)
+            got = ops.dual_norm_step(xd, yy.to(DEV) if yy is not None else None, *(w.to(DEV) if w is not None else None for w in ww), 1e-5, dt)
+            torch.testing.assert_close(xd.cpu(), xc, atol=1e-5, rtol=1e-5)
+            for a, b in zip(got, want):
+                assert (a is None) == (b is None)
+                if a is not None:
+                    torch.testing.assert_close(a.float().cpu(), b.float(), **_tol(dt))
+
+
+@pytest.mark.parametrize("dt", ACTS)
+@pytest.mark.parametrize("n", [64, 45])
+def test_gelu_gated_unit_into_a_column_block(dt, n):
+    g = torch.Generator().manual_seed(n)
+    y = torch.randn(7, 2 * n, generator=g) * 4
+    y[0, 0], y[0, 1] = -60.0, 60.0
+    for kind in ("relu", "silu", "gelu_tanh"):
+        want = ref.glu(y, torch.float32, kind)
+        wide = torch.zeros(7, n + 12, dtype=dt, device=DEV)
+        got = ops.glu(y.to(DEV), dt, kind, out=wide[:, 8:8 + n])
+        torch.testing.assert_close(got.float().cpu(), want, **_tol(dt))
+        torch.testing.assert_close(ops.glu(y.to(DEV), dt, kind).float().cpu(), want, **_tol(dt))
+        assert not wide[:, :8].any() and not wide[:, 8 + n:].any()
+
+
+@pytest.mark.parametrize("H,G,D,Dv,taps", [(4, 2, 32, 32, 4), (3, 3, 24, 70, 3), (6, 1, 20, 8, 1), (4, 4, 128, 128, 2), (2, 1, 200, 130, 6),
+                                           (4, 2, 48, 16, 4)])
+@pytest.mark.parametrize("longest", [7, 64, 65, 300])
+def test_delta_rule_operands_and_scan(H, G, D, Dv, taps, longest):
+    """Portions row by row and in chunks of 64 rows side by side (whole chunks, one row past a chunk, a few rows), fresh and
+    continued, single tokens, a sequence without a slot, a padding row; memories that fade within a row, last, and never fade."""
+    g = torch.Generator().manual_seed(H * 100 + D + longest)
+    lens, starts = [longest, 2, 1, 1, min(longest, 20), 1, 1], [0, 30, 0, 55, 7, 9, 4]
+    cu, pos, rs = _seqs(lens, starts)
+    T, C = int(cu[-1]), 2 * G * D + H * Dv
+    rs_d = rs.clone()
+    rs_d[-1] = -1
+    slots = torch.tensor([3, 0, 5, 1, 6, -1, -1], dtype=torch.int32)
+    proj = torch.randn(T, C + 2 * H + 5, generator=g)
+    conv = torch.randn(taps, C, generator=g) * 0.6
+    hist = taps - 1
+    plane = torch.randn(7, hist * C + 8 + H * D * Dv, generator=g)
+    rate, dt_bias = -torch.logspace(-3, 1.5, H), torch.linspace(-4, 1, H)
+    rate[0] = 0.0
+    res = []
+    for dev, r_s, sl in (("cpu", rs, slots), (DEV, rs_d, slots)):
+        to = lambda t: t.clone().to(dev)   # noqa: E731
+        st, lay, p = to(plane), _Layout(cu, r_s, sl, dev), to(pos)
+        x = ops.delta_prep(to(proj), to(conv), st[:, 4:4 + hist * C] if taps > 1 else None, C + 2, C + 2 + H, to(rate), to(dt_bias), p,
+                           lay, H, G, D, Dv)
+        o = ops.delta_scan(x, st[:, hist * C + 8:], lay.cu_q, p, lay.state_slots, H, G, D, Dv, max(lens))
+        if dev != "cpu":
+            assert not x.qk[..., D:].any() and not x.v[..., Dv:].any()
+            torch.testing.assert_close(x.kq, (x.qk[:, 0] * x.qk[:, 1]).sum(-1), atol=1e-5, rtol=1e-5)
+        res.append([t.cpu() for t in (x.qk[..., :D], x.v[..., :Dv], x.gates, st)] + [o.cpu()])
+    live = torch.ones(T, dtype=torch.bool)
+    live[-2:] = False
+    for i, (want, got) in enumerate(zip(*res)):
+        if i == 4:
+            want, got = want[live], got[live]
+        torch.testing.assert_close(got, want, atol=5e-5, rtol=5e-5, msg=lambda m, i=i: f"{i}: {m}")
+
+
+@pytest.mark.parametrize("beta,rate", [(20.0, 0.0), (20.0, -60.0), (-3.0, -0.01)])
+def test_delta_rule_with_repeated_keys_full_steps_and_steep_decays(beta, rate):
+    """One key over and over with step sizes of one (every write erases the one before), decays that fall to nothing
+    within a row beside rows that do not decay, and slow learning: the chunks' triangular systems at their stiffest."""
+    g = torch.Generator().manual_seed(5)
+    H, G, D, Dv, T = 2, 1, 16, 32, 200
+    C = 2 * G * D + H * Dv
+    cu, pos, rs = _seqs([T], [0])
+    proj = torch.randn(T, C + 2 * H, generator=g)
+    proj[:, G * D:2 * G * D] = proj[:1, G * D:2 * G * D]
+    proj[:, C:C + H] = beta
+    proj[:, C + H:] = torch.where(torch.rand(T, 1, generator=g) < 0.3, 3.0, -30.0)
+    res = []
+    for dev in ("cpu", DEV):
+        lay = _Layout(cu, rs, torch.zeros(1, dtype=torch.int32), dev)
+        st = torch.ones(1, H * D * Dv, device=dev)
+        x = ops.delta_prep(proj.to(dev), torch.ones(1, C, device=dev), None, C, C + H, torch.full((H,), rate, device=dev),
+                           torch.zeros(H, device=dev), pos.to(dev), lay, H, G, D, Dv)
+        res.append((ops.delta_scan(x, st, lay.cu_q, pos.to(dev), lay.state_slots, H, G, D, Dv, T).cpu(), st.cpu()))
+    for want, got in zip(*res):
+        torch.testing.assert_close(got, want, atol=5e-5, rtol=5e-5)
+
+
+@pytest.mark.parametrize("dt", ACTS)
+@pytest.mark.parametrize("BSZ", [16, 24])
+@pytest.mark.parametrize("H,G,D,Dv,rot", [(4, 2, 32, 64, 16), (6, 2, 40, 80, 20), (3, 1, 16, 20, 0), (5, 5, 7, 6, 2), (4, 2, 128, 256, 128)])
+def test_two_maps_per_head_over_shared_values(dt, BSZ, H, G, D, Dv, rot):
+    g = torch.Generator().manual_seed(H * 100 + D)
+    lens, starts = [37, 70, 1, 1, 1], [0, 130, 55, 3, 199]
+    MB = 14
+    cu, pos, rs = _seqs(lens, starts)
+    T, C = int(cu[-1]), (H + G) * 2 * D + G * Dv
+    tables = torch.randperm(5 * MB, generator=g).to(torch.int32).view(5, MB)
+    where = torch.tensor([int(tables[b, p // BSZ]) * BSZ + p % BSZ for b, p in zip(rs.tolist(), pos.tolist())], dtype=torch.int32)
+    qkv = torch.randn(T, C + 3, generator=g)
+    kc, vc = (torch.randn(5 * MB, 2 * G, BSZ, D, generator=g) * 0.5).to(dt), (torch.randn(5 * MB, G, BSZ, Dv, generator=g) * 0.5).to(dt)
+    inv = torch.tensor([1e3 ** (-2.0 * j / rot) for j in range(rot // 2)], dtype=torch.float64) if rot else None
+    for portions, rows in ((0, 0), (2, 107)):
+        res = []
+        for dev in ("cpu", DEV):
+            to = lambda t: t.clone().to(dev) if t is not None else None   # noqa: E731
+            k, v = to(kc), to(vc)
+            q, _ = ops.attn_prep(to(qkv), to(pos), to(where), _Layout(cu, rs, rs[:5], dev), k, v, 2 * H, 2 * G, D, Dv, inv_freq=to(inv),
+                                 rot_dims=rot, pairs=True, rot_mag=1.3, maps=2)
+            a = ops.attn_masked(q, k, v, to(tables), to(cu), to(rs), to(pos), 2 * H, 2 * G, D, Dv, 0.2, 0, 0, torch.float32,
+                                n_portions=portions, portion_rows=rows, max_len=70, value_share=2)
+            wide = torch.zeros(T, H * Dv + 9, dtype=dt, device=dev)
+            y = ops.diff_norm(a, 0.4, 1e-5, 0.7, H, G, Dv, dt, out=wide[:, 4:4 + H * Dv])
+            assert not wide[:, :4].any() and not wide[:, 4 + H * Dv:].any()
+            res.append([t.float().cpu() for t in (q, k, v, a, y)])
+        for i, (want, got) in enumerate(zip(*res)):
+            tol = _tol(dt) if i in (1, 2, 4) else dict(atol=2e-2, rtol=2e-2) if dt == torch.bfloat16 and i == 3 else dict(atol=5e-5, rtol=5e-5)
+            torch.testing.assert_close(got, want, **tol, msg=lambda m, i=i: f"{i}: {m}")
+        # the maps' order: key/value head, map, head of the group
+        plain = qkv[:, :2 * H * D].view(T, G, H // G, 2, D).transpose(2, 3).reshape(T, 2 * H, D)
+        if rot == 0:
+            torch.testing.assert_close(res[1][0].view(T, 2 * H, D), plain)
