@@ -1,6 +1,6 @@
-"""Prefill and decode throughput of the hybrid decoders (Nidozen, Telurax, Surevik, Gizilorn, Kulivik) beside each other and a
+"""Prefill and decode throughput of the hybrid decoders (Nidozen, Telurax, Surevik, Gizilorn, Kulivik, Rizurax) beside each other and a
 Llama-shaped transformer of equal width, depth and head sizes (``bench.py --hybrid``,
-``--hybrid-models kulivik,gizilorn,surevik,telurax,nidozen,llama``). Random weights, synthetic tokens.
+``--hybrid-models rizurax,kulivik,gizilorn,surevik,telurax,nidozen,llama``). Random weights, synthetic tokens.
 
 Per size: one prompt of ``prompt`` tokens goes through each engine as a single step (prefill
 tokens/s), then ``batch`` requests decode ``new`` tokens each from recorded steps (decode tokens/s).
@@ -16,7 +16,9 @@ latent attention with rows of its own, latent attention on those rows) over two 
 others' chunk, compressed rows of width 128 beside a turned key part of 64, a dense xIELU feed-forward in every
 layer; the Kulivik stack repeats (window attention with kept first keys, attention beside linear attention, convolved
 attention over all earlier keys), a clamped gated dense feed-forward of half the others' width in the first layer, 32
-silu-gated experts of a sixteenth of the dense width (4 chosen) in the others; the transformer has full causal attention and a SwiGLU feed-forward. Prints one
+silu-gated experts of a sixteenth of the dense width (4 chosen) in the others; the Rizurax stack alternates a gated delta rule and differential attention over all earlier keys
+(half as many heads of two maps each, values twice as wide), a gated dense feed-forward of the others' width beside the
+mixer in every layer, its second and third layer run twice, a pair embedding of 65521 rows; the transformer has full causal attention and a SwiGLU feed-forward. Prints one
 JSON line. Per-kernel times come from running this under ``rocprofv3 --kernel-trace --stats``.
 """
 from __future__ import annotations
@@ -137,6 +139,20 @@ def kulivik_config(s: dict):
                              "logit_scale": 1.0, "logit_softcap": 30.0, "layers": layers}, name="kulivik-bench")
 
 
+def rizurax_config(s: dict):
+    from .models.hybrid import config_from_dict
+
+    ff = {"kind": "dense", "ff": s["ff"]}
+    delta = {"type": "delta", "mixer": {"heads": s["heads"], "kv_heads": s["kv"], "dim": s["dim"], "vdim": s["dim"], "conv": 4}, "mlp": ff}
+    rot = {"dims": s["dim"] // 2, "base": 10000.0, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}
+    attn = {"type": "attention", "mixer": {"heads": s["heads"] // 2, "kv_heads": max(1, s["kv"] // 2), "dim": s["dim"], "vdim": 2 * s["dim"],
+                                           "scale": s["dim"] ** -0.5, "diff": 0.6, "rot": rot}, "mlp": ff}
+    return config_from_dict({"architecture": "Rizurax", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6},
+                             "embedding": {"bigram": {"buckets": 65521, "mul_prev": 31, "mul_cur": 7}},
+                             "layers": [delta if i % 2 == 0 else attn for i in range(s["layers"] - 2)],
+                             "loop": {"start": 1, "stop": 3, "times": 2}}, name="rizurax-bench")
+
+
 def transformer_config(s: dict):
     from .models.config import ModelConfig
 
@@ -212,6 +228,8 @@ def run(a) -> int:
                 model = HybridModel.random_init(gizilorn_config(s), dev, seed=1)
             elif kind == "kulivik":
                 model = HybridModel.random_init(kulivik_config(s), dev, seed=1)
+            elif kind == "rizurax":
+                model = HybridModel.random_init(rizurax_config(s), dev, seed=1)
             else:
                 model = TransformerModel.random_init(transformer_config(s), dev, seed=1)
             row[kind] = _measure(model, a.hybrid_prompt, a.hybrid_batch, a.hybrid_new, a.steps, a.warmup, phases)
@@ -224,7 +242,8 @@ def run(a) -> int:
                 row[ph + "_ratio"] = row["nidozen"][k] / row["llama"][k]
             for mine, others in (("telurax", ("nidozen", "llama")), ("surevik", ("telurax", "nidozen", "llama")),
                                  ("gizilorn", ("surevik", "telurax", "nidozen", "llama")),
-                                 ("kulivik", ("surevik", "gizilorn", "telurax", "nidozen", "llama"))):
+                                 ("kulivik", ("surevik", "gizilorn", "telurax", "nidozen", "llama")),
+                                 ("rizurax", ("kulivik", "surevik", "gizilorn", "telurax", "nidozen", "llama"))):
                 for other in others:
                     if all(k in row.get(m, {}) for m in (mine, other)):
                         row[f"{ph}_{mine}_over_{other}"] = row[mine][k] / row[other][k]
