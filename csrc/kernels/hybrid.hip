@@ -23,7 +23,7 @@ namespace {
 // ---------------------------------------------------------------- embedding -> fp32 stream (+ activation copy)
 // With a pair table (``pair.table``, the type of E): row (previous token * mul_prev + token * mul_cur) mod buckets of it is
 // added, row ``buckets`` for a sequence's first token. The previous token is the row before in the step's portion; for a
-// portion's first row it comes from the sequence's state slot, which the same wave then replaces by the portion's last token
+// portion's first row it comes from the sequence's state slot, which is then replaced by the portion's last token
 // (one thread reads, then writes: rows of a launch run in any order, and no other row touches the slot).
 struct PairTable {
   const void* table;             // [buckets + 1, d], null: none
@@ -37,14 +37,13 @@ struct PairTable {
 };
 
 template <bool EF32, bool AF32>
-__global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const void* __restrict__ E, float* __restrict__ x,
+__global__ __launch_bounds__(256) void embed_rows_kernel(const int32_t* __restrict__ ids, const void* __restrict__ E, float* __restrict__ x,
                                   void* __restrict__ xa, int T, int d, int vocab, const int32_t* __restrict__ feed_tok,
                                   const int32_t* __restrict__ feed_rows, float scale,
                                   const int32_t* __restrict__ positions, const double* __restrict__ inv_freq,
                                   PairTable pair) {
-  const int row = blockIdx.x * (blockDim.x >> 6) + (threadIdx.x >> 6);
-  const int lane = threadIdx.x & 63;
-  if (row >= T) return;
+  __shared__ long long pair_row;
+  const int row = blockIdx.x;
   auto token = [&](int r) {
     int v = ids[r];
     if (feed_rows != nullptr) {
@@ -56,8 +55,8 @@ __global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const void* _
   const int id = token(row);
   const typename Act<EF32>::type* e2 = nullptr;
   if (pair.table != nullptr) {
-    long long at = pair.buckets;
-    if (lane == 0) {
+    if (threadIdx.x == 0) {
+      long long at = pair.buckets;
       const RowSeq s = row_sequence(row, pair.row_seq, pair.cu_q, pair.positions, pair.slots);
       long long prev = -1;                          // (no state: as at a sequence's start)
       if (row > s.first) prev = token(row - 1);
@@ -65,9 +64,10 @@ __global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const void* _
       if (row == s.first && s.slot >= 0) pair.last[static_cast<size_t>(s.slot) * pair.stride] = token(s.first + s.rows - 1);
       if (prev >= 0) at = static_cast<long long>((static_cast<unsigned long long>(prev) * pair.mul_prev +
                                                   static_cast<unsigned long long>(id) * pair.mul_cur) % static_cast<unsigned long long>(pair.buckets));
+      pair_row = at;
     }
-    at = __shfl(at, 0, 64);
-    e2 = static_cast<const typename Act<EF32>::type*>(pair.table) + static_cast<size_t>(at) * d;
+    __syncthreads();
+    e2 = static_cast<const typename Act<EF32>::type*>(pair.table) + static_cast<size_t>(pair_row) * d;
   }
   const typename Act<EF32>::type* e = static_cast<const typename Act<EF32>::type*>(E) + static_cast<size_t>(id) * d;
   typename Act<AF32>::type* a = static_cast<typename Act<AF32>::type*>(xa);
@@ -76,7 +76,7 @@ __global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const void* _
     // the angle p * f and its reduction to [-pi, pi] in fp64 (thousands of radians would cost an fp32
     // angle four digits), sine and cosine of the reduced angle in fp32
     const double pos = static_cast<double>(positions[row]);
-    for (int i = lane; 2 * i < d; i += 64) {
+    for (int i = threadIdx.x; 2 * i < d; i += 256) {
       const double ang = pos * inv_freq[i];
       const double red = ang - 6.283185307179586476925 * rint(ang * 0.159154943091895335769);
       float sn, cs;
@@ -90,7 +90,20 @@ __global__ void embed_rows_kernel(const int32_t* __restrict__ ids, const void* _
     }
     return;
   }
-  for (int c = lane; c < d; c += 64) {
+  if (d % 4 == 0) {                                 // (tables and stream start on 16-byte borders)
+    for (int c = 4 * threadIdx.x; c < d; c += 1024) {
+      float4 v = load_act4<EF32>(e + c);
+      v = make_float4(v.x * scale, v.y * scale, v.z * scale, v.w * scale);
+      if (e2 != nullptr) {
+        const float4 w = load_act4<EF32>(e2 + c);
+        v = make_float4(v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w);
+      }
+      *reinterpret_cast<float4*>(x + static_cast<size_t>(row) * d + c) = v;
+      if (a != nullptr) store_act4<AF32>(a, static_cast<size_t>(row) * d + c, v);
+    }
+    return;
+  }
+  for (int c = threadIdx.x; c < d; c += 256) {
     float v = Act<EF32>::load(e, c) * scale;
     if (e2 != nullptr) v += Act<EF32>::load(e2, c);
     x[static_cast<size_t>(row) * d + c] = v;
@@ -769,7 +782,30 @@ struct AttnOpts {
   int v_share;                 // neighbouring key heads that share one value head (the value plane has G / v_share heads)
 };
 
-template <bool CF32, bool AF32>
+// VW > 0: value heads of exactly 64 VW columns under one head's weights; a lane owns VW neighbouring columns and reads them
+// in one access. VW = 0: any width, columns 64 apart.
+template <bool CF32, int VW>
+LC_DEVICE void load_values(const typename Act<CF32>::type* p, float* v) {
+  if constexpr (CF32) {
+#pragma unroll
+    for (int i = 0; i < VW; i += 2) {
+      const float2 x = *reinterpret_cast<const float2*>(p + i);
+      v[i] = x.x;
+      v[i + 1] = x.y;
+    }
+  } else {
+    uint32_t w[VW / 2];
+    if constexpr (VW == 2) w[0] = *reinterpret_cast<const uint32_t*>(p);
+    else __builtin_memcpy(w, __builtin_assume_aligned(p, 8), 2 * VW);
+#pragma unroll
+    for (int i = 0; i < VW / 2; ++i) {
+      v[2 * i] = __uint_as_float(w[i] << 16);
+      v[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
+    }
+  }
+}
+
+template <bool CF32, bool AF32, int VW>
 __global__ __launch_bounds__(256) void attn_masked_kernel(
     const float* __restrict__ q, const void* __restrict__ kc, const void* __restrict__ vc,
     const int32_t* __restrict__ block_tables, int MB, const int32_t* __restrict__ row_seq,
@@ -854,8 +890,20 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
     rows[lane] = vrow;
     __syncthreads();
     const int n = min(64, nkeys - j0);
+    if constexpr (VW > 0) {
 #pragma unroll
-    for (int i = 0; i < kMaxVCols; ++i) {
+      for (int i = 0; i < VW; ++i) acc[i] *= corr;
+#pragma unroll 8
+      for (int jj = 0; jj < n; ++jj) {
+        float v[VW];
+        load_values<CF32, VW>(vbase + static_cast<size_t>(rows[jj]) * v_ld + lane * VW, v);
+        const float pj = ps[jj];
+#pragma unroll
+        for (int i = 0; i < VW; ++i) acc[i] += pj * v[i];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < kMaxVCols && VW == 0; ++i) {
       const int c = lane + 64 * i;
       if (c < ncols) {
         float a = acc[i] * corr;
@@ -870,8 +918,8 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
   typename Act<AF32>::type* o = static_cast<typename Act<AF32>::type*>(out);
   const float fin = opt.out_scale * (opt.gate != nullptr ? sigmoidf_(opt.gate[static_cast<size_t>(t) * opt.ld_gate + h]) : 1.f);
 #pragma unroll
-  for (int i = 0; i < kMaxVCols; ++i) {
-    const int c = lane + 64 * i;
+  for (int i = 0; i < (VW > 0 ? VW : kMaxVCols); ++i) {
+    const int c = VW > 0 ? lane * VW + i : lane + 64 * i;
     if (live && c < ncols)
       Act<AF32>::store(o, static_cast<size_t>(t) * opt.o_row + static_cast<size_t>(h) * o_ld + o_col0 + c, acc[i] / l * fin);
   }
@@ -967,7 +1015,10 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
   extern __shared__ float lds[];
   const int b = blockIdx.z, h = blockIdx.y;
   const int q0 = cu_q[b], q1 = cu_q[b + 1];
-  const int row0 = q0 + blockIdx.x * 64;
+  // A portion's later rows see more keys. Workgroups i and i + 256 share a CU, so every other 256 walk the row tiles
+  // backwards: a long tile and a short one meet on a CU instead of two long ones.
+  const bool forward = (((b * static_cast<int>(gridDim.y) + h) * static_cast<int>(gridDim.x)) >> 8) & 1;
+  const int row0 = q0 + (forward ? blockIdx.x : gridDim.x - 1 - blockIdx.x) * 64;
   if (row0 >= q1) return;                                   // the same for the whole block
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int lr = lane & 15, lk = lane >> 4;
@@ -1331,7 +1382,8 @@ LC_EXPORT int lc_embed_rows(const void* ids, const void* E, int e_f32, void* x, 
     return -1;
   const PairTable pt{pair, buckets, mul_prev, mul_cur, static_cast<int32_t*>(last), last_stride, static_cast<const int32_t*>(row_seq),
                      static_cast<const int32_t*>(cu_q), static_cast<const int32_t*>(positions), static_cast<const int32_t*>(slots)};
-  const dim3 grid((T + 3) / 4), block(256);
+  if (d % 4 == 0 && !(aligned16(E) && aligned16(x) && aligned16(xa) && aligned16(pair))) return -1;
+  const dim3 grid(T), block(256);
 #define LC_EMB(E32, A32)                                                                                      \
   embed_rows_kernel<E32, A32><<<grid, block, 0, st>>>(static_cast<const int32_t*>(ids), E, static_cast<float*>(x), \
                                                       xa, T, d, vocab, static_cast<const int32_t*>(feed_tok), \
@@ -1699,8 +1751,16 @@ LC_EXPORT int lc_attn_masked(const void* q, const void* kc, const void* vc, int 
   const size_t lds = 4 * static_cast<size_t>(D + 128) * sizeof(float);
   if (lds > 64 * 1024) return -1;
   const dim3 grid(T, (H + 3) / 4, vz), block(256);
-#define LC_ATT(C32, A32)                                                                                        \
-  attn_masked_kernel<C32, A32><<<grid, block, lds, st>>>(                                                       \
+  // (neighbouring columns in one access: 8- or 4-byte borders in bf16 planes, 8-byte ones in fp32 planes)
+  const bool vec = vh0 < 0 && v_ld % 4 == 0 && reinterpret_cast<uintptr_t>(vc) % 8 == 0;
+#define LC_ATT(C32, A32)                                  \
+  do {                                                    \
+    if (vec && Dv == 256) LC_ATT_K(C32, A32, 4);          \
+    else if (vec && Dv == 128) LC_ATT_K(C32, A32, 2);     \
+    else LC_ATT_K(C32, A32, 0);                           \
+  } while (0)
+#define LC_ATT_K(C32, A32, VW)                                                                                  \
+  attn_masked_kernel<C32, A32, VW><<<grid, block, lds, st>>>(                                                       \
       static_cast<const float*>(q), kc, vc, static_cast<const int32_t*>(block_tables), MB,                      \
       static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(positions), out, H, G, D, Dv, BS, scale, \
       chunk, window, k_ld, v_ld, opt, vh0, nvh, o_ld, o_col0)
@@ -1708,6 +1768,7 @@ LC_EXPORT int lc_attn_masked(const void* q, const void* kc, const void* vc, int 
   else if (cache_f32) LC_ATT(true, false);
   else if (act_f32) LC_ATT(false, true);
   else LC_ATT(false, false);
+#undef LC_ATT_K
 #undef LC_ATT
   LC_RETURN_LAST_ERROR();
 }

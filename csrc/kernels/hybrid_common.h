@@ -29,6 +29,18 @@ LC_DEVICE void store_act4(void* p, size_t i, const float4& v) {
   }
 }
 
+// Four neighbouring elements of a table of that type as floats (8- / 16-byte border).
+template <bool F32>
+LC_DEVICE float4 load_act4(const typename Act<F32>::type* p) {
+  if constexpr (F32) {
+    return *reinterpret_cast<const float4*>(p);
+  } else {
+    const uint2 w = *reinterpret_cast<const uint2*>(p);
+    return make_float4(__uint_as_float(w.x << 16), __uint_as_float(w.x & 0xffff0000u), __uint_as_float(w.y << 16),
+                       __uint_as_float(w.y & 0xffff0000u));
+  }
+}
+
 LC_DEVICE float sigmoidf_(float x) { return 1.f / (1.f + expf(-x)); }
 LC_DEVICE float siluf_(float x) { return x / (1.f + expf(-x)); }
 // log sigmoid(z) = min(z, 0) - log1p(exp(-|z|))

@@ -112,7 +112,8 @@ struct DeltaArgs {
   float* w;                      // [chunks, H, 64, Dp]
   float* ut;                     // [chunks, H, Dvp, 64]
   float* s0;                     // [chunks, H, Dvp, Dp]  state at the chunk's start, transposed
-  double* cum;                   // [chunks, H, 64]       cumulative log decays
+  double* cum;                   // [chunks, H, 64]       cumulative log decays L
+  float* dec;                    // [chunks, H, 68]       e^(L_last - L_t), then e^(L_last)
 };
 
 // ---------------------------------------------------------------- row by row
@@ -187,6 +188,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaArgs a) {
 // i = 0..3 (which indices meet is free as long as both operands agree), so operands that are contiguous in the depth are read
 // 16 bytes at a time. Rows past the portion's end have beta 0 and log decay 0: they change nothing.
 constexpr int kChunk = 64;
+constexpr int kDec = kChunk + 4;
 constexpr int kTS = kChunk + 4;                      // row stride of 64 x 64 matrices in LDS
 
 LC_DEVICE f32x4 mfma4(const float4& x, const float4& y, f32x4 acc) {
@@ -240,6 +242,10 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a) {
     beta[lane] = gate.x;
     bdec[lane] = gate.x * expf(static_cast<float>(L));
     a.cum[(ck.index * a.H + h) * kChunk + lane] = L;
+    const double end = __shfl(L, 63, 64);
+    float* dec = a.dec + (ck.index * a.H + h) * kDec;
+    dec[lane] = expf(static_cast<float>(end - L));
+    if (lane == 0) dec[kChunk] = expf(static_cast<float>(end));
   }
   __syncthreads();
   for (int ct = 0; ct <= wave; ++ct) {               // wave w: rows 16 w .. 16 w + 15 of A
@@ -354,9 +360,9 @@ __global__ __launch_bounds__(256) void delta_state_kernel(DeltaArgs a) {
   constexpr int NT = (DT + 3) / 4;
   __shared__ __attribute__((aligned(16))) float Ss[16][16 * DT + 4];
   __shared__ __attribute__((aligned(16))) float Us[16][kTS];
-  const int h = blockIdx.y, b = blockIdx.z, g = h / (a.H / a.G);
+  const int h = blockIdx.x, b = blockIdx.z, g = h / (a.H / a.G);      // (a head's blocks on one chiplet: they read the same W and K)
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lr = lane & 15, lk = lane >> 4;
-  const int col = blockIdx.x * 16 + lr;
+  const int col = blockIdx.y * 16 + lr;
   const int q0 = a.cu_q[b], q1 = a.cu_q[b + 1];
   const int slot = a.slots[b];
   if (slot < 0 || q1 - q0 <= a.short_rows) return;
@@ -375,28 +381,32 @@ __global__ __launch_bounds__(256) void delta_state_kernel(DeltaArgs a) {
   auto fetch = [&](int c, DeltaChunkRegs<DT>& r) {
     const Chunk ck = chunk_of(a, b, c);
     const size_t ch = ck.index * a.H + h;
-    const int last = ck.row0 + ck.rows - 1;
     const float* w = a.w + (ch * kChunk + 16 * wave + lr) * Dp + 4 * lk;
 #pragma unroll
     for (int kk = 0; kk < DT; ++kk)
       if (kk < nd) r.w[kk] = *reinterpret_cast<const float4*>(w + 16 * kk);
+    const float* k = a.qk + ((static_cast<size_t>(ck.row0) * 2 + 1) * a.G + g) * Dp;     // the chunk's first key
+    const int step = 2 * a.G * Dp;                   // to the next row's
+    if (ck.rows == kChunk) {                         // (uniform bases, one lane offset)
 #pragma unroll
-    for (int n = 0; n < NT; ++n)
-      if (wave + 4 * n < nd) {
-        const int d = 16 * (wave + 4 * n) + lr;
+      for (int n = 0; n < NT; ++n)
+        if (wave + 4 * n < nd) {
+          const int at = 4 * lk * step + 16 * (wave + 4 * n) + lr;
 #pragma unroll
-        for (int i = 0; i < 16; ++i) {
-          const size_t row = min(ck.row0 + 16 * (i >> 2) + 4 * lk + (i & 3), last);
-          r.k[n][i] = a.qk[((row * 2 + 1) * a.G + g) * Dp + d];
+          for (int i = 0; i < 16; ++i) r.k[n][i] = (k + (16 * (i >> 2) + (i & 3)) * step)[at];
         }
-      }
+    } else {
+#pragma unroll
+      for (int n = 0; n < NT; ++n)
+        if (wave + 4 * n < nd) {
+          const int d = 16 * (wave + 4 * n) + lr;
+#pragma unroll
+          for (int i = 0; i < 16; ++i) r.k[n][i] = k[min(16 * (i >> 2) + 4 * lk + (i & 3), ck.rows - 1) * step + d];
+        }
+    }
     r.uv = *reinterpret_cast<const float4*>(a.ut + (ch * a.Dvp + col) * kChunk + 16 * wave + 4 * lk);
-    const double* cum = a.cum + ch * kChunk;
-    const double end = cum[kChunk - 1];
-    r.all = expf(static_cast<float>(end));
-    const int t = 16 * wave + 4 * lk;
-    r.dec = make_float4(expf(static_cast<float>(end - cum[t])), expf(static_cast<float>(end - cum[t + 1])),
-                        expf(static_cast<float>(end - cum[t + 2])), expf(static_cast<float>(end - cum[t + 3])));
+    r.all = a.dec[ch * kDec + kChunk];
+    r.dec = *reinterpret_cast<const float4*>(a.dec + ch * kDec + 16 * wave + 4 * lk);
   };
   DeltaChunkRegs<DT> cur, nxt;
   fetch(0, nxt);
@@ -616,7 +626,7 @@ LC_EXPORT int lc_delta_prep(const void* proj, int ld, const void* conv_w, int ta
 LC_EXPORT long long lc_delta_scratch_floats(int T, int B, int max_len, int H, int D, int Dv) {
   if (max_len <= kShortRows) return 0;
   const long long Dp = round16(D), Dvp = round16(Dv);
-  return static_cast<long long>(chunk_slots(T, B)) * H * (kChunk * Dp + Dvp * kChunk + Dvp * Dp + 2 * kChunk);
+  return static_cast<long long>(chunk_slots(T, B)) * H * (kChunk * Dp + Dvp * kChunk + Dvp * Dp + 2 * kChunk + kDec);
 }
 
 LC_EXPORT int lc_delta_scan(const void* qk, const void* v, const void* gates, const void* kq, void* state,
@@ -630,11 +640,12 @@ LC_EXPORT int lc_delta_scan(const void* qk, const void* v, const void* gates, co
   DeltaArgs a{static_cast<const float*>(qk), static_cast<const float*>(v), static_cast<const float2*>(gates),
               static_cast<const float*>(kq), static_cast<float*>(state), state_stride, static_cast<const int32_t*>(cu_q),
               static_cast<const int32_t*>(positions), static_cast<const int32_t*>(slots), static_cast<float*>(out), H, G, D, Dp,
-              Dv, Dvp, kShortRows, nullptr, nullptr, nullptr, nullptr};
+              Dv, Dvp, kShortRows, nullptr, nullptr, nullptr, nullptr, nullptr};
   if (chunked) {
     const size_t n = chunk_slots(T, B) * H;
     a.cum = static_cast<double*>(scratch);           // (the widest type first)
-    a.w = reinterpret_cast<float*>(a.cum + n * kChunk);
+    a.dec = reinterpret_cast<float*>(a.cum + n * kChunk);
+    a.w = a.dec + n * kDec;
     a.ut = a.w + n * kChunk * Dp;
     a.s0 = a.ut + n * Dvp * kChunk;
     const int nc = (max_len + kChunk - 1) / kChunk;
@@ -647,7 +658,7 @@ LC_EXPORT int lc_delta_scan(const void* qk, const void* v, const void* gates, co
       (void)hipFuncSetAttribute(reinterpret_cast<const void*>(delta_out_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, most);
     });
     delta_chunk_kernel<<<dim3(nc, H, B), dim3(256), lds, st>>>(a);
-    const dim3 sgrid(Dvp / 16, H, B);
+    const dim3 sgrid(H, Dvp / 16, B);
     if (Dp <= 64) delta_state_kernel<4><<<sgrid, dim3(256), 0, st>>>(a);
     else if (Dp <= 128) delta_state_kernel<8><<<sgrid, dim3(256), 0, st>>>(a);
     else delta_state_kernel<16><<<sgrid, dim3(256), 0, st>>>(a);
