@@ -158,11 +158,30 @@ LC_DEVICE void conv_token(const ConvIn& a, const RowSeq& s, const float* st, int
 }
 
 // The state becomes the portion's last taps - 1 inputs (by the block of its first row, after every thread of the block
-// has read the old ones). A thread owns a channel: row j + rows is read before row j + 1 is written.
+// has read the old ones). A thread owns a channel (four of them): all its inputs are read before one is written.
+template <int HIST>
+LC_DEVICE void conv_keep4(const ConvIn& a, const RowSeq& s, float* st) {
+  for (int c = threadIdx.x * 4; c < a.C; c += 1024) {
+    float4 in[HIST];
+#pragma unroll
+    for (int j = 0; j < HIST; ++j) {
+      const int k = s.rows - HIST + j;
+      in[j] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (k >= 0) in[j] = *reinterpret_cast<const float4*>(a.x + static_cast<size_t>(s.first + k) * a.ld + c);
+      else if (!s.fresh) in[j] = *reinterpret_cast<const float4*>(st + static_cast<size_t>(k + HIST) * a.C + c);
+    }
+#pragma unroll
+    for (int j = 0; j < HIST; ++j) *reinterpret_cast<float4*>(st + static_cast<size_t>(j) * a.C + c) = in[j];
+  }
+}
+
 LC_DEVICE void conv_keep(const ConvIn& a, const RowSeq& s, float* st) {
   const int hist = a.taps - 1;
+  if (a.vec && hist == 1) return conv_keep4<1>(a, s, st);
+  if (a.vec && hist == 2) return conv_keep4<2>(a, s, st);
+  if (a.vec && hist == 3) return conv_keep4<3>(a, s, st);
   for (int c = threadIdx.x; c < a.C; c += 256)
-    for (int j = 0; j < hist; ++j) {
+    for (int j = 0; j < hist; ++j) {                 // (row j + rows is read before row j + 1 is written)
       const int k = s.rows - hist + j;
       float in = 0.f;
       if (k >= 0) in = a.x[static_cast<size_t>(s.first + k) * a.ld + c];

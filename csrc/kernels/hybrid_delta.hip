@@ -110,10 +110,12 @@ struct DeltaArgs {
   int short_rows;                // portions of up to this many rows run row by row, longer ones in chunks
   // chunks of all portions, compactly: chunk c of sequence b has index cu_q[b] / 64 + b + c
   float* w;                      // [chunks, H, 64, Dp]
-  float* ut;                     // [chunks, H, Dvp, 64]
+  float* kt;                     // [chunks, H, Dp, 64]   (e^(L_last - L_t) k_t)^T, zero past the portion's end
+  float* ut;                     // [chunks, H, Dvp, 64]  (T diag(beta) V)^T
+  float* u;                      // [chunks, H, Dvp, 64]  U^T
   float* s0;                     // [chunks, H, Dvp, Dp]  state at the chunk's start, transposed
   double* cum;                   // [chunks, H, 64]       cumulative log decays L
-  float* dec;                    // [chunks, H, 68]       e^(L_last - L_t), then e^(L_last)
+  float* decay;                  // [chunks, H]           e^(L_last)
 };
 
 // ---------------------------------------------------------------- row by row
@@ -188,7 +190,6 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(DeltaArgs a) {
 // i = 0..3 (which indices meet is free as long as both operands agree), so operands that are contiguous in the depth are read
 // 16 bytes at a time. Rows past the portion's end have beta 0 and log decay 0: they change nothing.
 constexpr int kChunk = 64;
-constexpr int kDec = kChunk + 4;
 constexpr int kTS = kChunk + 4;                      // row stride of 64 x 64 matrices in LDS
 
 LC_DEVICE f32x4 mfma4(const float4& x, const float4& y, f32x4 acc) {
@@ -216,6 +217,7 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a) {
   extern __shared__ float lds[];
   __shared__ double cum[kChunk];
   __shared__ float beta[kChunk], bdec[kChunk];       // beta, beta e^L
+  __shared__ float rest[kChunk];                     // e^(L_last - L), zero past the portion's end
   const int h = blockIdx.y, g = h / (a.H / a.G);
   const Chunk ck = chunk_of(a, blockIdx.z, blockIdx.x);
   if (ck.rows == 0) return;                          // the same for the whole block
@@ -243,11 +245,16 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a) {
     bdec[lane] = gate.x * expf(static_cast<float>(L));
     a.cum[(ck.index * a.H + h) * kChunk + lane] = L;
     const double end = __shfl(L, 63, 64);
-    float* dec = a.dec + (ck.index * a.H + h) * kDec;
-    dec[lane] = expf(static_cast<float>(end - L));
-    if (lane == 0) dec[kChunk] = expf(static_cast<float>(end));
+    rest[lane] = in ? expf(static_cast<float>(end - L)) : 0.f;
+    if (lane == 0) a.decay[ck.index * a.H + h] = expf(static_cast<float>(end));
   }
   __syncthreads();
+  float* kt = a.kt + (ck.index * a.H + h) * Dp * kChunk;
+  for (int i = threadIdx.x; i < Dp * (kChunk / 4); i += 256) {       // neighbouring lanes: neighbouring keys' coordinates
+    const int d = i % Dp, t = 4 * (i / Dp);
+    const float* k = Ks + t * DS + d;
+    *reinterpret_cast<float4*>(kt + d * kChunk + t) = make_float4(k[0] * rest[t], k[DS] * rest[t + 1], k[2 * DS] * rest[t + 2], k[3 * DS] * rest[t + 3]);
+  }
   for (int ct = 0; ct <= wave; ++ct) {               // wave w: rows 16 w .. 16 w + 15 of A
     f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
     for (int kk = 0; kk < Dp; kk += 16) {
@@ -344,32 +351,32 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaArgs a) {
 }
 
 // Pass 2. A block keeps 16 columns of the state: in accumulators (wave w: its 16-row tiles w, w + 4, ...) and, as the right
-// operand of U, transposed in LDS. The operands of the next chunk are loaded while the current one is computed.
-// DT: 16-row tiles of the widest key (Dp <= 16 DT).
+// operand of U, transposed in LDS. The loop over chunks is one dependent chain, so its body has no branches and the next
+// chunk's operands are loaded (ahead of the stores, which then need not be waited for) while the current one is computed.
+// DT: 16-row tiles of the key width (Dp = 16 DT).
 template <int DT>
 struct DeltaChunkRegs {
   float4 w[DT];                                      // rows 16 wave + lr of W
-  float k[(DT + 3) / 4][16];                         // columns of K^T
+  float4 k[(DT + 3) / 4][4];                         // rows of (e^(L_last - L_t) k_t)^T
   float4 uv;
-  float4 dec;                                        // e^(L_last - L_t) of the wave's rows
   float all;                                         // e^(L_last)
 };
 
 template <int DT>
 __global__ __launch_bounds__(256) void delta_state_kernel(DeltaArgs a) {
-  constexpr int NT = (DT + 3) / 4;
-  __shared__ __attribute__((aligned(16))) float Ss[16][16 * DT + 4];
+  constexpr int NT = (DT + 3) / 4, Dp = 16 * DT;
+  __shared__ __attribute__((aligned(16))) float Ss[16][Dp + 4];
   __shared__ __attribute__((aligned(16))) float Us[16][kTS];
-  const int h = blockIdx.x, b = blockIdx.z, g = h / (a.H / a.G);      // (a head's blocks on one chiplet: they read the same W and K)
+  const int h = blockIdx.x, b = blockIdx.z;          // (a head's blocks on one chiplet: they read the same W and K)
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lr = lane & 15, lk = lane >> 4;
   const int col = blockIdx.y * 16 + lr;
   const int q0 = a.cu_q[b], q1 = a.cu_q[b + 1];
   const int slot = a.slots[b];
   if (slot < 0 || q1 - q0 <= a.short_rows) return;
-  const int Dp = a.Dp, nd = Dp / 16;
   const int chunks = (q1 - q0 + kChunk - 1) / kChunk;
   float* st = a.state + static_cast<size_t>(slot) * a.state_stride + static_cast<size_t>(h) * a.D * a.Dv;
   const bool fresh = a.positions[q0] == 0;
+  auto mine = [&](int n) { return DT % 4 == 0 || wave + 4 * n < DT; };       // whether the wave has an n-th tile
   f32x4 S[NT];
 #pragma unroll
   for (int n = 0; n < NT; ++n)
@@ -378,78 +385,66 @@ __global__ __launch_bounds__(256) void delta_state_kernel(DeltaArgs a) {
       const int d = 16 * (wave + 4 * n) + 4 * lk + e;
       S[n][e] = !fresh && d < a.D && col < a.Dv ? st[static_cast<size_t>(d) * a.Dv + col] : 0.f;
     }
+  const size_t first = chunk_of(a, b, 0).index;
+  const int w_at = (16 * wave + lr) * Dp + 4 * lk, u_at = col * kChunk + 16 * wave + 4 * lk;
   auto fetch = [&](int c, DeltaChunkRegs<DT>& r) {
-    const Chunk ck = chunk_of(a, b, c);
-    const size_t ch = ck.index * a.H + h;
-    const float* w = a.w + (ch * kChunk + 16 * wave + lr) * Dp + 4 * lk;
+    const size_t ch = (first + c) * a.H + h;
+    const float* w = a.w + ch * kChunk * Dp + w_at;
+    const float* k = a.kt + ch * Dp * kChunk + (16 * wave + lr) * kChunk + 4 * lk;
 #pragma unroll
-    for (int kk = 0; kk < DT; ++kk)
-      if (kk < nd) r.w[kk] = *reinterpret_cast<const float4*>(w + 16 * kk);
-    const float* k = a.qk + ((static_cast<size_t>(ck.row0) * 2 + 1) * a.G + g) * Dp;     // the chunk's first key
-    const int step = 2 * a.G * Dp;                   // to the next row's
-    if (ck.rows == kChunk) {                         // (uniform bases, one lane offset)
-#pragma unroll
-      for (int n = 0; n < NT; ++n)
-        if (wave + 4 * n < nd) {
-          const int at = 4 * lk * step + 16 * (wave + 4 * n) + lr;
-#pragma unroll
-          for (int i = 0; i < 16; ++i) r.k[n][i] = (k + (16 * (i >> 2) + (i & 3)) * step)[at];
-        }
-    } else {
-#pragma unroll
-      for (int n = 0; n < NT; ++n)
-        if (wave + 4 * n < nd) {
-          const int d = 16 * (wave + 4 * n) + lr;
-#pragma unroll
-          for (int i = 0; i < 16; ++i) r.k[n][i] = k[min(16 * (i >> 2) + 4 * lk + (i & 3), ck.rows - 1) * step + d];
-        }
-    }
-    r.uv = *reinterpret_cast<const float4*>(a.ut + (ch * a.Dvp + col) * kChunk + 16 * wave + 4 * lk);
-    r.all = a.dec[ch * kDec + kChunk];
-    r.dec = *reinterpret_cast<const float4*>(a.dec + ch * kDec + 16 * wave + 4 * lk);
-  };
-  DeltaChunkRegs<DT> cur, nxt;
-  fetch(0, nxt);
-  for (int c = 0; c < chunks; ++c) {
-    cur = nxt;
-    const size_t ch = chunk_of(a, b, c).index * a.H + h;
-    float* s0 = a.s0 + (ch * a.Dvp + col) * Dp;
+    for (int kk = 0; kk < DT; ++kk) r.w[kk] = lds4(w + 16 * kk);
+    r.uv = lds4(a.ut + ch * a.Dvp * kChunk + u_at);
 #pragma unroll
     for (int n = 0; n < NT; ++n)
-      if (wave + 4 * n < nd) {
-        const int d = 16 * (wave + 4 * n) + 4 * lk;
-        const float4 v = make_float4(S[n][0], S[n][1], S[n][2], S[n][3]);
-        *reinterpret_cast<float4*>(&Ss[lr][d]) = v;
-        *reinterpret_cast<float4*>(s0 + d) = v;
+      if (mine(n)) {
+#pragma unroll
+        for (int kk = 0; kk < 4; ++kk) r.k[n][kk] = lds4(k + 4 * n * 16 * kChunk + 16 * kk);
       }
+    r.all = a.decay[ch];
+  };
+  auto step = [&](int c, const DeltaChunkRegs<DT>& cur, DeltaChunkRegs<DT>& nxt) {
+    const size_t ch = (first + c) * a.H + h;
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+      if (mine(n)) *reinterpret_cast<float4*>(&Ss[lr][16 * (wave + 4 * n) + 4 * lk]) = make_float4(S[n][0], S[n][1], S[n][2], S[n][3]);
     __syncthreads();
-    if (c + 1 < chunks) fetch(c + 1, nxt);
+    fetch(min(c + 1, chunks - 1), nxt);
+    __builtin_amdgcn_sched_barrier(0);               // (the loads are issued here, not where their first use is near)
+    float* s0 = a.s0 + (ch * a.Dvp + col) * Dp + 4 * lk;
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+      if (mine(n)) *reinterpret_cast<float4*>(s0 + 16 * (wave + 4 * n)) = make_float4(S[n][0], S[n][1], S[n][2], S[n][3]);
     f32x4 u0 = {0.f, 0.f, 0.f, 0.f}, u1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int kk = 0; kk < DT; ++kk)
-      if (kk < nd) {
-        const float4 y = lds4(&Ss[lr][16 * kk + 4 * lk]);
-        u0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.w[kk].x, y.x, u0, 0, 0, 0);
-        u1 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.w[kk].y, y.y, u1, 0, 0, 0);
-        u0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.w[kk].z, y.z, u0, 0, 0, 0);
-        u1 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.w[kk].w, y.w, u1, 0, 0, 0);
-      }
+    for (int kk = 0; kk < DT; ++kk) {
+      const float4 y = lds4(&Ss[lr][16 * kk + 4 * lk]);
+      u0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.w[kk].x, y.x, u0, 0, 0, 0);
+      u1 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.w[kk].y, y.y, u1, 0, 0, 0);
+      u0 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.w[kk].z, y.z, u0, 0, 0, 0);
+      u1 = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.w[kk].w, y.w, u1, 0, 0, 0);
+    }
     const float4 u = make_float4(cur.uv.x - u0[0] - u1[0], cur.uv.y - u0[1] - u1[1], cur.uv.z - u0[2] - u1[2], cur.uv.w - u0[3] - u1[3]);
-    *reinterpret_cast<float4*>(a.ut + (ch * a.Dvp + col) * kChunk + 16 * wave + 4 * lk) = u;
-    *reinterpret_cast<float4*>(&Us[lr][16 * wave + 4 * lk]) = make_float4(u.x * cur.dec.x, u.y * cur.dec.y, u.z * cur.dec.z, u.w * cur.dec.w);
+    *reinterpret_cast<float4*>(&Us[lr][16 * wave + 4 * lk]) = u;
+    *reinterpret_cast<float4*>(a.u + ch * a.Dvp * kChunk + u_at) = u;
     __syncthreads();
     float4 y[4];
 #pragma unroll
     for (int kk = 0; kk < 4; ++kk) y[kk] = lds4(&Us[lr][16 * kk + 4 * lk]);
 #pragma unroll
     for (int n = 0; n < NT; ++n)
-      if (wave + 4 * n < nd) {
 #pragma unroll
-        for (int e = 0; e < 4; ++e) S[n][e] *= cur.all;
+      for (int e = 0; e < 4; ++e) S[n][e] *= cur.all;
 #pragma unroll
-        for (int kk = 0; kk < 4; ++kk)
-          S[n] = mfma4(make_float4(cur.k[n][4 * kk], cur.k[n][4 * kk + 1], cur.k[n][4 * kk + 2], cur.k[n][4 * kk + 3]), y[kk], S[n]);
-      }
+    for (int kk = 0; kk < 4; ++kk)
+#pragma unroll
+      for (int n = 0; n < NT; ++n)
+        if (mine(n)) S[n] = mfma4(cur.k[n][kk], y[kk], S[n]);
+  };
+  DeltaChunkRegs<DT> even, odd;                      // two sets in turn: nothing is moved between them
+  fetch(0, even);
+  for (int c = 0; c < chunks; c += 2) {
+    step(c, even, odd);
+    if (c + 1 < chunks) step(c + 1, odd, even);
   }
 #pragma unroll
   for (int n = 0; n < NT; ++n)
@@ -530,8 +525,8 @@ __global__ __launch_bounds__(256) void delta_out_kernel(DeltaArgs a) {
       acc[0][i][e] *= dec;
       acc[1][i][e] *= dec;
     }
-  const float* u0 = a.ut + (ch * a.Dvp + c0) * kChunk + 4 * lk;
-  const float* u1 = a.ut + (ch * a.Dvp + c1) * kChunk + 4 * lk;
+  const float* u0 = a.u + (ch * a.Dvp + c0) * kChunk + 4 * lk;
+  const float* u1 = a.u + (ch * a.Dvp + c1) * kChunk + 4 * lk;
 #pragma unroll
   for (int k = 0; k < 4; ++k) {
     const float4 x0 = *reinterpret_cast<const float4*>(u0 + 16 * k), x1 = *reinterpret_cast<const float4*>(u1 + 16 * k);
@@ -586,6 +581,13 @@ __global__ __launch_bounds__(256) void diff_norm_kernel(const float* __restrict_
 
 int round16(int n) { return (n + 15) / 16 * 16; }
 
+// Padded key width: the state pass is compiled for these numbers of 16-coordinate tiles.
+int pad_keys(int d) {
+  for (int t : {1, 2, 3, 4, 6, 8, 12, 16})
+    if (d <= 16 * t) return 16 * t;
+  return round16(d);
+}
+
 constexpr int kShortRows = 16;                       // portions of up to this many rows run row by row
 
 size_t chunk_slots(int T, int B) { return static_cast<size_t>(T) / kChunk + B + 1; }
@@ -616,17 +618,20 @@ LC_EXPORT int lc_delta_prep(const void* proj, int ld, const void* conv_w, int ta
   const DeltaPrepArgs a{in, col_b, col_a, static_cast<const float*>(neg_rate), static_cast<const float*>(dt_bias),
                         static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(cu_q),
                         static_cast<const int32_t*>(positions), static_cast<const int32_t*>(slots), static_cast<float*>(qk),
-                        static_cast<float*>(v), static_cast<float2*>(gates), static_cast<float*>(kq), H, G, D, round16(D), Dv,
+                        static_cast<float*>(v), static_cast<float2*>(gates), static_cast<float*>(kq), H, G, D, pad_keys(D), Dv,
                         round16(Dv), qscale, T, (T + 7) / 8};
   delta_prep_kernel<<<dim3(8 * ((T + 7) / 8)), dim3(256), lds, st>>>(a);
   LC_RETURN_LAST_ERROR();
 }
 
+// Width of the keys and queries that lc_delta_prep writes for heads of D coordinates.
+LC_EXPORT long long lc_delta_key_width(int D) { return pad_keys(D); }
+
 // fp32 numbers of scratch for a step of T rows in B sequences, the longest of max_len rows (0: none needed).
 LC_EXPORT long long lc_delta_scratch_floats(int T, int B, int max_len, int H, int D, int Dv) {
   if (max_len <= kShortRows) return 0;
-  const long long Dp = round16(D), Dvp = round16(Dv);
-  return static_cast<long long>(chunk_slots(T, B)) * H * (kChunk * Dp + Dvp * kChunk + Dvp * Dp + 2 * kChunk + kDec);
+  const long long Dp = pad_keys(D), Dvp = round16(Dv);
+  return static_cast<long long>(chunk_slots(T, B)) * H * (2 * kChunk * Dp + 2 * Dvp * kChunk + Dvp * Dp + 2 * kChunk + 1);
 }
 
 LC_EXPORT int lc_delta_scan(const void* qk, const void* v, const void* gates, const void* kq, void* state,
@@ -634,20 +639,22 @@ LC_EXPORT int lc_delta_scan(const void* qk, const void* v, const void* gates, co
                             int T, int B, int H, int G, int D, int Dv, int max_len, void* scratch, hipStream_t st) {
   if (B <= 0 || T <= 0) return 0;
   if (H <= 0 || G <= 0 || H % G || D <= 0 || Dv <= 0 || D > 256 || state_stride < static_cast<long long>(H) * D * Dv) return -1;
-  const int Dp = round16(D), Dvp = round16(Dv);
+  const int Dp = pad_keys(D), Dvp = round16(Dv);
   const bool chunked = max_len > kShortRows;
   if (chunked && scratch == nullptr) return -1;
   DeltaArgs a{static_cast<const float*>(qk), static_cast<const float*>(v), static_cast<const float2*>(gates),
               static_cast<const float*>(kq), static_cast<float*>(state), state_stride, static_cast<const int32_t*>(cu_q),
               static_cast<const int32_t*>(positions), static_cast<const int32_t*>(slots), static_cast<float*>(out), H, G, D, Dp,
-              Dv, Dvp, kShortRows, nullptr, nullptr, nullptr, nullptr, nullptr};
+              Dv, Dvp, kShortRows, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, nullptr};
   if (chunked) {
     const size_t n = chunk_slots(T, B) * H;
     a.cum = static_cast<double*>(scratch);           // (the widest type first)
-    a.dec = reinterpret_cast<float*>(a.cum + n * kChunk);
-    a.w = a.dec + n * kDec;
-    a.ut = a.w + n * kChunk * Dp;
-    a.s0 = a.ut + n * Dvp * kChunk;
+    a.w = reinterpret_cast<float*>(a.cum + n * kChunk);
+    a.kt = a.w + n * kChunk * Dp;
+    a.ut = a.kt + n * kChunk * Dp;
+    a.u = a.ut + n * Dvp * kChunk;
+    a.s0 = a.u + n * Dvp * kChunk;
+    a.decay = a.s0 + n * Dvp * Dp;
     const int nc = (max_len + kChunk - 1) / kChunk;
     const int groups = (Dvp + kOutCols - 1) / kOutCols;
     const size_t lds = static_cast<size_t>(kChunk) * (Dp + 4 + kTS) * sizeof(float);
@@ -659,9 +666,12 @@ LC_EXPORT int lc_delta_scan(const void* qk, const void* v, const void* gates, co
     });
     delta_chunk_kernel<<<dim3(nc, H, B), dim3(256), lds, st>>>(a);
     const dim3 sgrid(H, Dvp / 16, B);
-    if (Dp <= 64) delta_state_kernel<4><<<sgrid, dim3(256), 0, st>>>(a);
-    else if (Dp <= 128) delta_state_kernel<8><<<sgrid, dim3(256), 0, st>>>(a);
-    else delta_state_kernel<16><<<sgrid, dim3(256), 0, st>>>(a);
+    switch (Dp / 16) {
+#define LC_DS(DT) case DT: delta_state_kernel<DT><<<sgrid, dim3(256), 0, st>>>(a); break
+      LC_DS(1); LC_DS(2); LC_DS(3); LC_DS(4); LC_DS(6); LC_DS(8); LC_DS(12); LC_DS(16);
+#undef LC_DS
+      default: return -1;
+    }
     delta_out_kernel<<<dim3(nc, H * groups, B), dim3(256), lds, st>>>(a);
   }
   if (!chunked || B > 1) {                           // (a lone portion is of one kind)

@@ -1864,7 +1864,7 @@ def rownorm_gate(o: torch.Tensor, w: torch.Tensor, gate: torch.Tensor, eps: floa
 @dataclass
 class DeltaOperands:
     """What a gated delta rule reads per row, fp32: unit queries (times D^-1/2) and unit keys ``qk`` [T, 2, G, Dp], values
-    ``v`` [T, H, Dvp] (widths padded to multiples of 16 with zeros on the GPU), ``gates`` [T, H, 2] = (step size, log
+    ``v`` [T, H, Dvp] (widths padded with zeros to whole matrix tiles on the GPU), ``gates`` [T, H, 2] = (step size, log
     decay), ``kq`` [T, G] = q . k."""
 
     qk: torch.Tensor
@@ -1897,7 +1897,7 @@ def delta_prep(proj: torch.Tensor, conv_w: torch.Tensor, conv_state: Optional[to
         raise ValueError("delta_prep: a token's channels exceed one block's LDS")
     if not proj.is_cuda:
         return DeltaOperands(*ref.delta_prep(proj, conv_w, conv_state, col_b, col_a, neg_rate, dt_bias, positions, lay, H, G, D, Dv), None)
-    Dp, Dvp = (D + 15) // 16 * 16, (Dv + 15) // 16 * 16
+    Dp, Dvp = int(_hip().lib().lc_delta_key_width(D)), (Dv + 15) // 16 * 16
     dev = proj.device
     x = DeltaOperands(torch.empty(T, 2, G, Dp, dtype=torch.float32, device=dev), torch.empty(T, H, Dvp, dtype=torch.float32, device=dev),
                       torch.empty(T, H, 2, dtype=torch.float32, device=dev), torch.empty(T, G, dtype=torch.float32, device=dev))
@@ -1921,7 +1921,7 @@ def delta_scan(x: DeltaOperands, state: torch.Tensor, cu_q: torch.Tensor, positi
     if not x.qk.is_cuda:
         return ref.delta_scan(x.qk, x.v, x.gates, state, cu_q, positions, slots, H, G, D, Dv)
     T, B = x.qk.shape[0], slots.numel()
-    if x.qk.shape != (T, 2, G, (D + 15) // 16 * 16) or x.v.shape != (T, H, (Dv + 15) // 16 * 16) or x.gates.shape != (T, H, 2):
+    if x.qk.shape != (T, 2, G, int(_hip().lib().lc_delta_key_width(D))) or x.v.shape != (T, H, (Dv + 15) // 16 * 16) or x.gates.shape != (T, H, 2):
         raise ValueError("delta_scan: the operands do not fit the head sizes")
     out = torch.empty(T, H * Dv, dtype=torch.float32, device=x.qk.device)
     n = int(_hip().lib().lc_delta_scratch_floats(T, B, int(max_len), H, D, Dv))

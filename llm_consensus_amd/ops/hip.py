@@ -105,7 +105,8 @@ _SIGNATURES = {
     "lc_moe_mix": [_P, _P, _P, _P, _P, _I, _P, _P, _I, _P, _I, _I, _I, _I, _P],
 }
 _RESTYPES = {"lc_scan_scratch_floats": ([_I, _I, _L, _L], c_longlong),
-             "lc_delta_scratch_floats": ([_I, _I, _I, _I, _I, _I], c_longlong)}      # helpers that return no status
+             "lc_delta_scratch_floats": ([_I, _I, _I, _I, _I, _I], c_longlong),
+             "lc_delta_key_width": ([_I], c_longlong)}      # helpers that return no status
 
 _lib = None
 
