@@ -350,7 +350,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const bf16_t* __restrict__
       // Staged rows are 128 bytes: a wave's 64 columns, or with SwiGLU the 32 + 32 output
       // columns of two waves that are neighbours in n (they share a region and split its rows).
       constexpr int ROWB = 128, CH = 8;
-      char* mine = smem + (EPI == EPI_SWIGLU ? (wm * 2 + (wn >> 1)) : wave) * (128 * ROWB);
+      char* mine = smem + (epi_gated(EPI) ? (wm * 2 + (wn >> 1)) : wave) * (128 * ROWB);
       const int g = lane >> 4, r16 = lane & 15;
 #pragma unroll
       for (int j = 0; j < 8; ++j) {
@@ -359,7 +359,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const bf16_t* __restrict__
         for (int i = 0; i < 4; ++i) {
           u32x2 o;
           int chunk;
-          if constexpr (EPI == EPI_SWIGLU) {
+          if constexpr (epi_gated(EPI)) {
             if (i & 1) continue;
             const int nb = nbase + i * 16 + 4 * g;
             float gt[4], up[4];
@@ -368,8 +368,8 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const bf16_t* __restrict__
               gt[r] = acc[i][j][r] + (bias ? bf16_to_f32(bias[nb + r]) : 0.f);
               up[r] = acc[i + 1][j][r] + (bias ? bf16_to_f32(bias[nb + 16 + r]) : 0.f);
             }
-            o[0] = pack_bf16x2(silu(gt[0]) * up[0], silu(gt[1]) * up[1]);
-            o[1] = pack_bf16x2(silu(gt[2]) * up[2], silu(gt[3]) * up[3]);
+            o[0] = pack_bf16x2(gate_act<EPI>(gt[0]) * up[0], gate_act<EPI>(gt[1]) * up[1]);
+            o[1] = pack_bf16x2(gate_act<EPI>(gt[2]) * up[2], gate_act<EPI>(gt[3]) * up[3]);
             chunk = (wn & 1) * 4 + (i >> 1) * 2 + (g >> 1);
           } else {
             const int nb = nbase + i * 16 + 4 * g;
@@ -386,10 +386,10 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const bf16_t* __restrict__
       }
       constexpr int RPI = 64 / CH;                         // rows per store instruction
       const int c16 = lane & (CH - 1), rsub = lane / CH;
-      const int ncol = (EPI == EPI_SWIGLU ? tn * (G2_BN / 2) + (wn >> 1) * 64 : nbase) + c16 * 8;
-      constexpr int PASSES = EPI == EPI_SWIGLU ? 8 : 16;
-      const int p0 = EPI == EPI_SWIGLU ? (wn & 1) * 8 : 0;
-      if constexpr (EPI == EPI_SWIGLU) G2_BARRIER();       // the partner wave's half rows are in place
+      const int ncol = (epi_gated(EPI) ? tn * (G2_BN / 2) + (wn >> 1) * 64 : nbase) + c16 * 8;
+      constexpr int PASSES = epi_gated(EPI) ? 8 : 16;
+      const int p0 = epi_gated(EPI) ? (wn & 1) * 8 : 0;
+      if constexpr (epi_gated(EPI)) G2_BARRIER();       // the partner wave's half rows are in place
 #pragma unroll
       for (int pp = 0; pp < PASSES; ++pp) {
         const int p = p0 + pp;
@@ -405,7 +405,7 @@ __global__ __launch_bounds__(512) void gemm256_kernel(const bf16_t* __restrict__
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
-      if constexpr (EPI == EPI_SWIGLU) {
+      if constexpr (epi_gated(EPI)) {
         if (i & 1) continue;
         store_tile<EPI>(acc[i][j], &acc[i + 1][j], Y, bias, mbase + j * 16, nbase + i * 16, M, N, ldy, lane, 0);
       } else {
@@ -456,6 +456,8 @@ LC_EXPORT int lc_gemm256(const void* Wp, const void* X, void* Y, const void* bia
                           hipFuncAttributeMaxDynamicSharedMemorySize, G2B_LDS);
       (void)hipFuncSetAttribute(reinterpret_cast<const void*>(gemm256_kernel<EPI_F32, false, 2>),
                           hipFuncAttributeMaxDynamicSharedMemorySize, G2B_LDS);
+      (void)hipFuncSetAttribute(reinterpret_cast<const void*>(gemm256_kernel<EPI_GEGLU, false, 2>),
+                                hipFuncAttributeMaxDynamicSharedMemorySize, G2B_LDS);
       (void)hipFuncSetAttribute(reinterpret_cast<const void*>(gemm256_kernel<EPI_SWIGLU, false, 2>),
                           hipFuncAttributeMaxDynamicSharedMemorySize, G2B_LDS);
     });
@@ -465,6 +467,8 @@ LC_EXPORT int lc_gemm256(const void* Wp, const void* X, void* Y, const void* bia
       gemm256_kernel<EPI_F32, false, 2><<<grid, block, G2B_LDS, stream>>>(w, x, Y, b, M, N, K, ldy, tiles_m, tiles_n);
     else if (epi == EPI_SWIGLU)
       gemm256_kernel<EPI_SWIGLU, false, 2><<<grid, block, G2B_LDS, stream>>>(w, x, Y, b, M, N, K, ldy, tiles_m, tiles_n);
+    else if (epi == EPI_GEGLU)
+      gemm256_kernel<EPI_GEGLU, false, 2><<<grid, block, G2B_LDS, stream>>>(w, x, Y, b, M, N, K, ldy, tiles_m, tiles_n);
     else
       return -2;
     LC_RETURN_LAST_ERROR();

@@ -11,7 +11,11 @@ enum Epilogue : int {
   EPI_SWIGLU = 2,  // n-tiles alternate gate/up; Y bf16 [M, N/2] = silu(gate)*up (+bias before act)
   EPI_RELU2 = 3,   // Y bf16 [M, ldy] = relu(. + bias)^2 (the grouped kernels)
   EPI_GLU_CLAMPED = 4,  // n-tiles alternate gate/up; Y bf16 [M, N/2] = clamped gated unit with a scale per row (the grouped kernels)
+  EPI_GEGLU = 5,   // as EPI_SWIGLU with the tanh form of gelu instead of silu (gemm256)
 };
+
+// Epilogues that store act(gate) * up.
+constexpr bool epi_gated(int epi) { return epi == EPI_SWIGLU || epi == EPI_GEGLU; }
 
 // Constants of the clamped gated unit: with s = row_scale[row] (1 without the array), g = min(s * gate, limit),
 // u = clamp(s * up, -limit, limit), the output is g * sigmoid(slope * g) * (u + shift).
@@ -21,6 +25,12 @@ struct GluClamp {
 };
 
 LC_DEVICE float silu(float x) { return x / (1.f + __expf(-x)); }
+
+// 0.5 x (1 + tanh(a)) = x sigmoid(2 a), a = sqrt(2 / pi) (x + 0.044715 x^3)
+LC_DEVICE float gelu_tanh(float x) { return x / (1.f + __expf(-1.5957691216057308f * (x + 0.044715f * x * x * x))); }
+
+template <int EPI>
+LC_DEVICE float gate_act(float x) { return EPI == EPI_GEGLU ? gelu_tanh(x) : silu(x); }
 
 // The clamped gated unit over a gate tile and the up tile next to it (same layout as the SwiGLU store below).
 // ``row_scale`` is indexed like the output rows.
@@ -52,7 +62,7 @@ LC_DEVICE void store_tile(const f32x4& acc, const f32x4* acc_up, void* __restric
   const int m = m0 + (lane & 15);
   const int nb = n0 + 4 * (lane >> 4);
   if (m >= M) return;
-  if constexpr (EPI == EPI_SWIGLU) {
+  if constexpr (epi_gated(EPI)) {
     // n0 is the gate tile's origin in the interleaved space; output column = n0/2 + ...
     if (nb >= N) return;
     const int ob = (n0 >> 1) + 4 * (lane >> 4);
@@ -67,8 +77,8 @@ LC_DEVICE void store_tile(const f32x4& acc, const f32x4* acc_up, void* __restric
       }
     }
     u32x2 o;
-    o[0] = pack_bf16x2(silu(g[0]) * u[0], silu(g[1]) * u[1]);
-    o[1] = pack_bf16x2(silu(g[2]) * u[2], silu(g[3]) * u[3]);
+    o[0] = pack_bf16x2(gate_act<EPI>(g[0]) * u[0], gate_act<EPI>(g[1]) * u[1]);
+    o[1] = pack_bf16x2(gate_act<EPI>(g[2]) * u[2], gate_act<EPI>(g[3]) * u[3]);
     *reinterpret_cast<u32x2*>(static_cast<bf16_t*>(Y) + static_cast<size_t>(m) * ldy + ob) = o;
   } else {
     if (nb >= N) return;

@@ -544,19 +544,33 @@ LC_DEVICE float glu_act(float g, int kind) {
   return g * sigmoidf_(1.5957691216057308f * (g + 0.044715f * g * g * g));
 }
 
+// ``parts`` slabs of [T, 2n], ``slab`` elements apart, are summed first (a product whose depth was split). ``tiled``: gate and up
+// alternate in tiles of 16 columns instead of standing one behind the other.
 template <bool AF32, int V>
-__global__ void glu_kernel(const float* __restrict__ y, void* __restrict__ out, long long total, int n, int kind, int ldo) {
+__global__ void glu_kernel(const float* __restrict__ y, int parts, long long slab, int tiled, void* __restrict__ out, long long total,
+                           int n, int kind, int ldo) {
   const long long i = (static_cast<long long>(blockIdx.x) * blockDim.x + threadIdx.x) * V;
   if (i >= total) return;
   const long long t = i / n;
   const int c = static_cast<int>(i - t * n);
-  const float* g = y + t * 2 * n + c;
+  const int gc = tiled ? (c & ~15) * 2 + (c & 15) : c, du = tiled ? 16 : n;
+  const float* g = y + t * 2 * n + gc;
   if constexpr (V == 4) {
-    const float4 a = *reinterpret_cast<const float4*>(g), u = *reinterpret_cast<const float4*>(g + n);
+    float4 a = *reinterpret_cast<const float4*>(g), u = *reinterpret_cast<const float4*>(g + du);
+    for (int s = 1; s < parts; ++s) {
+      const float4 p = *reinterpret_cast<const float4*>(g + s * slab), q = *reinterpret_cast<const float4*>(g + s * slab + du);
+      a = make_float4(a.x + p.x, a.y + p.y, a.z + p.z, a.w + p.w);
+      u = make_float4(u.x + q.x, u.y + q.y, u.z + q.z, u.w + q.w);
+    }
     store_act4<AF32>(out, static_cast<size_t>(t) * ldo + c, make_float4(glu_act(a.x, kind) * u.x, glu_act(a.y, kind) * u.y,
                                                                        glu_act(a.z, kind) * u.z, glu_act(a.w, kind) * u.w));
   } else {
-    Act<AF32>::store(static_cast<typename Act<AF32>::type*>(out), static_cast<size_t>(t) * ldo + c, glu_act(g[0], kind) * g[n]);
+    float a = g[0], u = g[du];
+    for (int s = 1; s < parts; ++s) {
+      a += g[s * slab];
+      u += g[s * slab + du];
+    }
+    Act<AF32>::store(static_cast<typename Act<AF32>::type*>(out), static_cast<size_t>(t) * ldo + c, glu_act(a, kind) * u);
   }
 }
 
@@ -1575,13 +1589,13 @@ LC_EXPORT int lc_add_rmsnorm(void* x, const void* y, const void* w, float eps, v
   LC_RETURN_LAST_ERROR();
 }
 
-LC_EXPORT int lc_glu(const void* y, void* out, int act_f32, int T, int n, int kind, int ldo, hipStream_t st) {
+LC_EXPORT int lc_glu(const void* y, int parts, int tiled, void* out, int act_f32, int T, int n, int kind, int ldo, hipStream_t st) {
   if (T <= 0 || n <= 0) return 0;
-  if (kind < 0 || kind > 2 || ldo < n) return -1;
+  if (kind < 0 || kind > 2 || ldo < n || parts < 1 || (tiled && n % 16)) return -1;
   const long long total = static_cast<long long>(T) * n;
   const int v = n % 4 == 0 && ldo % 4 == 0 && aligned16(y) && aligned16(out) ? 4 : 1;
   const dim3 grid(static_cast<unsigned>((total / v + 255) / 256)), block(256);
-#define LC_GLU(A32, V) glu_kernel<A32, V><<<grid, block, 0, st>>>(static_cast<const float*>(y), out, total, n, kind, ldo)
+#define LC_GLU(A32, V) glu_kernel<A32, V><<<grid, block, 0, st>>>(static_cast<const float*>(y), parts, 2 * total, tiled, out, total, n, kind, ldo)
   if (act_f32 && v == 4) LC_GLU(true, 4);
   else if (act_f32) LC_GLU(true, 1);
   else if (v == 4) LC_GLU(false, 4);

@@ -13,7 +13,7 @@
 namespace {
 
 // ---------------------------------------------------------------- residual step with a gate and two norms
-// With y [T, d]: v = y * sigmoid(gate) (gate given: logits, row stride ld_gate), then rms-normed times w_out (w_out
+// With y [T, d] (a product whose depth was split comes as the slabs of its partial sums): v = y * sigmoid(gate) (gate given: logits, row stride ld_gate), then rms-normed times w_out (w_out
 // given), x += v. With w_in: h = x / sqrt(mean(x^2) + eps) * w_in, written to ``ha`` in the activation type and, when
 // given, to ``h32``. With ``mu`` (steps whose sequences all have ONE row): ``hs`` = h + (h' - h) * mu in the
 // activation type, h' the sequence's stored row (zeros at position 0), and h becomes the stored row. With ``w_in2``: ``ha2`` =
@@ -28,7 +28,9 @@ LC_DEVICE float4 shift4(const float4& h, const float4& p, const float4& m) {
 
 struct StepArgs {
   float* x;
-  const float* y;
+  const float* y;                // ``parts`` slabs of [T, d], ``slab`` elements apart, whose sum is the sublayer's result
+  int parts;
+  size_t slab;
   const float* gate;
   int ld_gate;
   const float* w_out;
@@ -77,6 +79,10 @@ __global__ __launch_bounds__(256) void gated_step_kernel(StepArgs a) {
         xv[i] = reinterpret_cast<const float4*>(a.x + row)[c];
         if (a.y != nullptr) {
           float4 v = reinterpret_cast<const float4*>(a.y + row)[c];
+          for (int s = 1; s < a.parts; ++s) {
+            const float4 w = reinterpret_cast<const float4*>(a.y + s * a.slab + row)[c];
+            v = make_float4(v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w);
+          }
           if (grow != nullptr) {
             const float4 g = reinterpret_cast<const float4*>(grow)[c];
             v = make_float4(v.x * sigmoidf_(g.x), v.y * sigmoidf_(g.y), v.z * sigmoidf_(g.z), v.w * sigmoidf_(g.w));
@@ -130,7 +136,11 @@ __global__ __launch_bounds__(256) void gated_step_kernel(StepArgs a) {
   } else {
     typedef typename Act<AF32>::type act_t;
     float r = 1.f;
-    auto result = [&](int c) { return grow != nullptr ? a.y[row + c] * sigmoidf_(grow[c]) : a.y[row + c]; };
+    auto result = [&](int c) {
+      float v = a.y[row + c];
+      for (int s = 1; s < a.parts; ++s) v += a.y[s * a.slab + row + c];
+      return grow != nullptr ? v * sigmoidf_(grow[c]) : v;
+    };
     if (a.y != nullptr && a.w_out != nullptr) {
       float ss = 0.f;
       for (int c = threadIdx.x; c < d; c += 256) {
@@ -349,19 +359,19 @@ __global__ void softcap_kernel(float* __restrict__ x, long long n, float cap) {
 }  // namespace
 
 // ================================================================= launchers
-LC_EXPORT int lc_gated_step(void* x, const void* y, const void* gate, int ld_gate, const void* w_out, const void* w_in,
+LC_EXPORT int lc_gated_step(void* x, const void* y, int parts, const void* gate, int ld_gate, const void* w_out, const void* w_in,
                             float eps, void* ha, void* h32, const void* w_in2, void* ha2, int act_f32, const void* mu, void* state,
                             long long state_stride, const void* row_seq, const void* positions, const void* slots, void* hs,
                             int T, int d, hipStream_t st) {
   if (T <= 0) return 0;
-  if (d <= 0 || (y == nullptr && w_in == nullptr) || (w_in != nullptr && ha == nullptr)) return -1;
+  if (d <= 0 || parts < 1 || (y == nullptr && w_in == nullptr) || (w_in != nullptr && ha == nullptr)) return -1;
   if (gate != nullptr && (y == nullptr || ld_gate < d)) return -1;
   if (w_in2 != nullptr && (w_in == nullptr || ha2 == nullptr)) return -1;
   if (mu != nullptr && (w_in == nullptr || hs == nullptr || state == nullptr || row_seq == nullptr || positions == nullptr ||
                         slots == nullptr || state_stride < d))
     return -1;
-  const StepArgs a{static_cast<float*>(x), static_cast<const float*>(y), static_cast<const float*>(gate), ld_gate,
-                   static_cast<const float*>(w_out), static_cast<const float*>(w_in), eps, ha, static_cast<float*>(h32),
+  const StepArgs a{static_cast<float*>(x), static_cast<const float*>(y), parts, static_cast<size_t>(T) * d,
+                   static_cast<const float*>(gate), ld_gate, static_cast<const float*>(w_out), static_cast<const float*>(w_in), eps, ha, static_cast<float*>(h32),
                    static_cast<const float*>(w_in2), ha2,
                    static_cast<const float*>(mu), static_cast<float*>(state), state_stride,
                    static_cast<const int32_t*>(row_seq), static_cast<const int32_t*>(positions),

@@ -1314,7 +1314,11 @@ class HybridModel:
                 else:
                     kw["experts_up"], kw["experts_down"] = ups.to(dt).contiguous(), downs.to(dt).contiguous()
             elif l.ff and c.design.parallel_ff:
-                kw["gate_up"] = lin(torch.cat([load(f + "gate"), load(f + "up")], 0))
+                if l.ff % 16 == 0:                  # (tiles of gate and up: the gated unit can be the product's epilogue)
+                    kw["gate_up"] = lin(ops.interleave_gate_up(load(f + "gate"), load(f + "up")))
+                    kw["gate_up"].tiled = True
+                else:
+                    kw["gate_up"] = lin(torch.cat([load(f + "gate"), load(f + "up")], 0))
             elif l.ff and c.design.sandwich:
                 kw["down"] = lin(load(f + "down"))
             elif l.ff and c.design.dense_ff == "xielu":
@@ -1657,8 +1661,8 @@ class HybridModel:
             else:
                 self._attention_diff(r, L, h1, positions, slot_mapping, lay, cache, both[:, :n])
             if l.ff:
-                ops.glu(ops.linear(h2, L.gate_up, out_f32=True), dt, "gelu_tanh", out=both[:, n:])
-            y = ops.linear(both, L.out, out_f32=True)
+                ops.glu_linear(h2, L.gate_up, "gelu_tanh", dt, out=both[:, n:])
+            y = ops.linear(both, L.out, out_f32=True, defer_reduce=True)
             nxt = self.layers[runs[r + 1][0]] if r + 1 < len(runs) else None
             h1, h2 = ops.dual_norm_step(x, y, nxt.norm1 if nxt else None, nxt.norm2 if nxt else None, eps, dt)
             if taps is not None:

@@ -15,7 +15,7 @@ import torch
 
 from . import reference as ref
 
-EPI_BF16, EPI_F32, EPI_SWIGLU = 0, 1, 2
+EPI_BF16, EPI_F32, EPI_SWIGLU, EPI_GEGLU = 0, 1, 2, 5
 
 # M at or below which the decode kernels (one activation panel) are used instead of the tile kernels.
 WS_MAX_M = int(os.environ.get("LC_WS_MAX_M", "256"))
@@ -102,13 +102,15 @@ def interleave_gate_up(Wg: torch.Tensor, Wu: torch.Tensor) -> torch.Tensor:
 @dataclass
 class LinearWeight:
     """A linear layer's weights in device layout. ``data`` is packed on GPU and row-major
-    [N, K] on CPU. ``swiglu`` marks gate/up interleaving (output width N/2)."""
+    [N, K] on CPU. ``swiglu`` marks gate/up interleaving (output width N/2). ``tiled``: the rows are gate and up in alternate
+    tiles of 16, but the product is an ordinary one unless ``glu_linear`` runs it."""
 
     data: torch.Tensor
     n: int
     k: int
     bias: Optional[torch.Tensor] = None
     swiglu: bool = False
+    tiled: bool = False
 
     @property
     def n_pad(self) -> int:
@@ -262,7 +264,7 @@ def linear(x: torch.Tensor, w: LinearWeight, out_f32: bool = False, defer_reduce
             part = torch.empty(splits, M, w.n, dtype=torch.float32, device=x.device)
             h.call("lc_gemm256_splitk", w.data.data_ptr(), x.data_ptr(), part.data_ptr(), M, w.n, w.k, w.n_pad, w.n,
                    splits)
-            if defer_reduce and not out_f32:
+            if defer_reduce:
                 return PartialSum(part, w.bias)
             h.call("lc_splitk_reduce", part.data_ptr(), h.ptr(w.bias), y.data_ptr(), splits, M, w.n, out_n,
                    1 if out_f32 else 0)
@@ -302,7 +304,7 @@ def linear(x: torch.Tensor, w: LinearWeight, out_f32: bool = False, defer_reduce
     part = torch.empty(splits, M, w.n, dtype=torch.float32, device=x.device)
     h.call(kernel, w.data.data_ptr(), x.data_ptr(), part.data_ptr(), None, M, w.n, w.k, w.n_pad, w.n, EPI_F32, splits,
            *extra)
-    if defer_reduce and not w.swiglu and not out_f32:
+    if defer_reduce and not w.swiglu:
         return PartialSum(part, w.bias)
     mode = 2 if w.swiglu else (1 if out_f32 else 0)
     h.call("lc_splitk_reduce", part.data_ptr(), h.ptr(w.bias), y.data_ptr(), splits, M, w.n, out_n, mode)
@@ -1313,21 +1315,50 @@ def mlstm_out(o: torch.Tensor, m: torch.Tensor, w: torch.Tensor, gate: torch.Ten
     return out
 
 
+def _slabs(y, what: str) -> Tuple[torch.Tensor, int]:
+    """(storage, number of fp32 slabs whose sum is y) of a matrix or of a ``PartialSum``."""
+    if isinstance(y, PartialSum):
+        if y.bias is not None:
+            raise ValueError(f"{what}: partial sums of a product without a bias")
+        return y.part, y.part.shape[0]
+    return y.contiguous(), 1
+
+
+def glu_linear(x: torch.Tensor, w: LinearWeight, kind: str, act_dtype: torch.dtype, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """act(gate) * up of x's product with ``w`` (rows gate | up, or in alternate tiles of 16 when ``w.tiled``), [T, n] in
+    ``act_dtype``, into ``out`` (a block of a wider matrix) when given. Large bf16 products of tiled weights store the gated unit
+    from their accumulators (gelu_tanh); otherwise the fp32 product is gated in a launch of its own, which also sums the slabs
+    of a split one."""
+    M, n = x.shape[0], w.n // 2
+    if x.is_cuda and w.is_packed and w.tiled and w.bias is None and kind == "gelu_tanh" and act_dtype == torch.bfloat16 \
+            and M > WS_MAX_M and w.n_pad % 256 == 0 and GEMM256_MIN_TILES >= 0:
+        tiles = ((M + 255) // 256) * (w.n_pad // 256)
+        y = _out_block(out, M, n, act_dtype, x.device, "glu_linear")
+        ldy = max(y.stride(0), n)
+        if tiles >= max(GEMM256_MIN_TILES, 1) and _choose_gemm256_splits(tiles, w.k) == 1 and ldy % 8 == 0 and y.data_ptr() % 16 == 0:
+            _hip().call("lc_gemm256", w.data.data_ptr(), x.contiguous().data_ptr(), y.data_ptr(), None, M, w.n, w.k, w.n_pad, ldy, EPI_GEGLU)
+            return y
+    return glu(linear(x, w, out_f32=True, defer_reduce=True), act_dtype, kind, out=out, tiled=w.tiled)
+
+
 GLU_KINDS = ("relu", "silu", "gelu_tanh")
 
 
-def glu(y: torch.Tensor, act_dtype: torch.dtype, kind: str = "relu", out: Optional[torch.Tensor] = None) -> torch.Tensor:
+def glu(y, act_dtype: torch.dtype, kind: str = "relu", out: Optional[torch.Tensor] = None, tiled: bool = False) -> torch.Tensor:
     """fp32 y [T, 2n] = (gate | up) -> act(gate) * up [T, n] in ``act_dtype`` (act: relu, silu or the tanh form of gelu).
-    ``out``: write into this [T, n] block (of a wider matrix)."""
+    ``out``: write into this [T, n] block (of a wider matrix). ``tiled``: gate and up alternate in tiles of 16 columns.
+    y may be a ``PartialSum`` (without a bias)."""
     if kind not in GLU_KINDS:
         raise ValueError(f"glu: activation {kind!r}: {', '.join(GLU_KINDS)}")
     T, n = y.shape[0], y.shape[1] // 2
+    if tiled and n % 16:
+        raise ValueError("glu: tiles of 16 columns")
+    y, parts = _slabs(y, "glu")
     if not y.is_cuda:
-        r = ref.glu(y, act_dtype, kind)
+        r = ref.glu(y.view(T, n // 16, 2, 16).transpose(1, 2).reshape(T, 2 * n) if tiled else y, act_dtype, kind)
         return r if out is None else out.copy_(r)
-    y = y.contiguous()
     out = _out_block(out, T, n, act_dtype, y.device, "glu")
-    _hip().call("lc_glu", y.data_ptr(), out.data_ptr(), _f32flag(act_dtype), T, n, GLU_KINDS.index(kind), max(out.stride(0), n))
+    _hip().call("lc_glu", y.data_ptr(), parts, 1 if tiled else 0, out.data_ptr(), _f32flag(act_dtype), T, n, GLU_KINDS.index(kind), max(out.stride(0), n))
     return out
 
 
@@ -1709,7 +1740,7 @@ def gated_step(x: torch.Tensor, y: Optional[torch.Tensor], gate: Optional[torch.
     h32 = torch.empty(T, d, dtype=torch.float32, device=dev) if (w_in is not None and want_f32 and not f32) else None
     hs = torch.empty(T, d, dtype=act_dtype, device=dev) if shift is not None else None
     p = _hip().ptr
-    _hip().call("lc_gated_step", x.data_ptr(), p(y.contiguous() if y is not None else None), p(gate),
+    _hip().call("lc_gated_step", x.data_ptr(), p(y.contiguous() if y is not None else None), 1, p(gate),
                 max(gate.stride(0), d) if gate is not None else 0, p(w_out), p(w_in), float(eps), p(ha), p(h32),
                 None, None, _f32flag(act_dtype), p(shift.mu) if shift else None, p(shift.state) if shift else None,
                 max(shift.state.stride(0), d) if shift else 0, p(lay.row_seq) if shift else None,
@@ -1717,15 +1748,15 @@ def gated_step(x: torch.Tensor, y: Optional[torch.Tensor], gate: Optional[torch.
     return ha, (ha if f32 else h32), hs
 
 
-def dual_norm_step(x: torch.Tensor, y: Optional[torch.Tensor], w1: Optional[torch.Tensor], w2: Optional[torch.Tensor], eps: float,
+def dual_norm_step(x: torch.Tensor, y, w1: Optional[torch.Tensor], w2: Optional[torch.Tensor], eps: float,
                    act_dtype: torch.dtype):
     """The residual step of a layer whose mixer and feed-forward read the same stream through norms of their own, one
-    launch: x (fp32, in place) += y (when given); returns (rms_norm(x) * w1, rms_norm(x) * w2) in ``act_dtype`` (``w2``, or
+    launch: x (fp32, in place) += y (when given; it may be a ``PartialSum``); returns (rms_norm(x) * w1, rms_norm(x) * w2) in ``act_dtype`` (``w2``, or
     both, may be None)."""
     T, d = x.shape
     if x.dtype != torch.float32 or not x.is_contiguous():
         raise ValueError("dual_norm_step: the residual stream is a contiguous fp32 tensor")
-    if y is not None and (y.shape != x.shape or y.dtype != torch.float32):
+    if y is not None and (y.shape != x.shape or (torch.is_tensor(y) and y.dtype != torch.float32)):
         raise ValueError("dual_norm_step: the sublayers' output must be fp32 of the stream's shape")
     if w1 is None and w2 is not None:
         raise ValueError("dual_norm_step: the second norm stands beside the first")
@@ -1736,7 +1767,8 @@ def dual_norm_step(x: torch.Tensor, y: Optional[torch.Tensor], w1: Optional[torc
     h1 = torch.empty(T, d, dtype=act_dtype, device=x.device) if w1 is not None else None
     h2 = torch.empty(T, d, dtype=act_dtype, device=x.device) if w2 is not None else None
     p = _hip().ptr
-    _hip().call("lc_gated_step", x.data_ptr(), p(y.contiguous() if y is not None else None), None, 0, None, p(w1), float(eps),
+    part, parts = _slabs(y, "dual_norm_step") if y is not None else (None, 1)
+    _hip().call("lc_gated_step", x.data_ptr(), p(part), parts, None, 0, None, p(w1), float(eps),
                 p(h1), None, p(w2), p(h2), _f32flag(act_dtype), None, None, 0, None, None, None, None, T, d)
     return h1, h2
 

@@ -76,7 +76,7 @@ _SIGNATURES = {
     "lc_latent_write": [_P, _I, _I, _I, _P, _F, _P, _P, _I, _I, _I, _P],
     "lc_head_linear": [_P, _I, _I, _P, _I, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _I, _I, _P],
     "lc_mlstm_scan": [_P, _I, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _I, _I, _F, _I, _P, _P, _P],
-    "lc_glu": [_P, _P, _I, _I, _I, _I, _I, _P],
+    "lc_glu": [_P, _I, _I, _P, _I, _I, _I, _I, _I, _P],
     "lc_add_dyt": [_P, _P, _F, _F, _P, _P, _P, _I, _I, _I, _I, _P],
     "lc_glu_clamped": [_P, _I, _I, _I, _I, _F, _F, _F, _P, _P, _P, _I, _I, _P],
     "lc_rope_pairs_write": [_P, _I, _P, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _P],
@@ -88,7 +88,7 @@ _SIGNATURES = {
     "lc_latent_rope_write": [_P, _I, _I, _P, _F, _P, _P, _P, _P, _I, _P, _I, _I, _I, _I, _I, _I, _I, _P],
     "lc_xielu": [_P, _I, _P, _I, _I, _I, _F, _F, _P],
     # gated residual steps, token shifts, attention pre-processing with convolutions and mixed values (hybrid_gated.hip)
-    "lc_gated_step": [_P, _P, _P, _I, _P, _P, _F, _P, _P, _P, _P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _P],
+    "lc_gated_step": [_P, _P, _I, _P, _I, _P, _P, _F, _P, _P, _P, _P, _I, _P, _P, _L, _P, _P, _P, _P, _I, _I, _P],
     "lc_token_shift": [_P, _P, _P, _L, _P, _P, _P, _P, _P, _I, _I, _I, _P],
     "lc_attn_prep": [_P, _I, _P, _I, _P, _L, _I, _P, _P, _F, _P, _I, _I, _F, _I, _F, _F, _P, _I, _F, _P, _P, _P, _P, _P, _P, _P, _P,
                      _I, _P, _I, _I, _I, _I, _I, _I, _P],

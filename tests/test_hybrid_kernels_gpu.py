@@ -943,3 +943,37 @@ def test_two_maps_per_head_over_shared_values(dt, BSZ, H, G, D, Dv, rot):
         plain = qkv[:, :2 * H * D].view(T, G, H // G, 2, D).transpose(2, 3).reshape(T, 2 * H, D)
         if rot == 0:
             torch.testing.assert_close(res[1][0].view(T, 2 * H, D), plain)
+
+
+@pytest.mark.parametrize("M,N,K", [(9, 512, 2048), (40, 256, 1024), (300, 512, 2048), (2048, 4096, 256), (2100, 2048, 64), (5, 96, 64)])
+def test_gated_unit_of_a_product_with_tiled_weights(M, N, K):
+    """Decode shapes (depth split over workgroups: the gated unit sums the slabs), portions whose product stores the gated
+    unit itself, portions too small for that; into a column block whose rows start on 16-byte borders and one whose do not."""
+    g = torch.Generator().manual_seed(M)
+    n = N // 2
+    x, Wg, Wu = torch.randn(M, K, generator=g).bfloat16(), *(torch.randn(n, K, generator=g) * 2 / K ** 0.5 for _ in range(2))
+    w = ops.LinearWeight.from_dense(ops.interleave_gate_up(Wg, Wu), None, DEV)
+    w.tiled = True
+    want = ref.glu(torch.cat([x.float() @ Wg.bfloat16().float().T, x.float() @ Wu.bfloat16().float().T], 1), torch.float32, "gelu_tanh")
+    for left, right in ((0, 0), (16, 8), (4, 3)):
+        wide = torch.zeros(M, left + n + right, dtype=torch.bfloat16, device=DEV)
+        got = ops.glu_linear(x.to(DEV), w, "gelu_tanh", torch.bfloat16, out=wide[:, left:left + n])
+        torch.testing.assert_close(got.float().cpu(), want, **_tol(torch.bfloat16))
+        assert not wide[:, :left].any() and not wide[:, left + n:].any()
+    wc = ops.LinearWeight.from_dense(ops.interleave_gate_up(Wg, Wu), None, "cpu")
+    wc.tiled = True
+    torch.testing.assert_close(ops.glu_linear(x, wc, "gelu_tanh", torch.bfloat16).float(), want, **_tol(torch.bfloat16))
+
+
+@pytest.mark.parametrize("d", [64, 37, 2048])
+def test_slabs_of_a_split_product_join_the_residual_step_and_the_gated_unit(d):
+    g = torch.Generator().manual_seed(d)
+    x, part, w = torch.randn(6, d, generator=g), torch.randn(3, 6, d, generator=g), torch.rand(d, generator=g)
+    xc, xd = x.clone(), x.to(DEV)
+    want = ref.dual_norm_step(xc, part.sum(0), w, 2 * w, 1e-5, torch.float32)
+    got = ops.dual_norm_step(xd, ops.PartialSum(part.to(DEV)), w.to(DEV), (2 * w).to(DEV), 1e-5, torch.float32)
+    torch.testing.assert_close(xd.cpu(), xc, atol=1e-5, rtol=1e-5)
+    for a, b in zip(got, want):
+        torch.testing.assert_close(a.cpu(), b, atol=2e-5, rtol=2e-5)
+    if d % 2 == 0:
+        torch.testing.assert_close(ops.glu(ops.PartialSum(part.to(DEV)), torch.float32, "gelu_tanh").cpu(), ref.glu(part.sum(0), torch.float32, "gelu_tanh"), atol=2e-5, rtol=2e-5)
