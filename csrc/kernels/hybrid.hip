@@ -957,6 +957,7 @@ __global__ __launch_bounds__(256) void attn_masked_kernel(
 // slower than two launches of 256 that each form the scores again). A block may use more than 64 KB of LDS (wide queries).
 constexpr int kTileMaxVT = 16;
 constexpr int kTileMaxLds = 160 * 1024;
+constexpr float kLog2e = 1.4426950408889634f;
 
 // Maximum over the 16 lanes of a DPP row (lanes 16 k .. 16 k + 15), in every one of them: rotations inside the row,
 // on the vector ALU.
@@ -1173,12 +1174,14 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
       const float sv = valid ? (softcap > 0.f ? softcap * tanhf(sraw / softcap) : sraw) : -INFINITY;
       const float mn = fmaxf(m[r], row16_max(sv));
       const float base = mn == -INFINITY ? 0.f : mn;        // nothing visible yet: weights 0, no NaN
-      const float pv = valid ? expf(sv - base) : 0.f;
-      corr[r] = expf(m[r] - base);
+      const float pv = valid ? fast_exp2((sv - base) * kLog2e) : 0.f;
+      corr[r] = fast_exp2((m[r] - base) * kLog2e);
       l[r] = l[r] * corr[r] + pv;                             // this lane's keys only: summed over the row at the end
       m[r] = mn;
       Ps[row * 17 + lr] = pv;
     }
+    // (the running maxima settle after a few tiles: the sums then need no rescaling, exactly as if by factors of one)
+    const bool rescale = __any(corr[0] != 1.f || corr[1] != 1.f || corr[2] != 1.f || corr[3] != 1.f);
     // P goes from the score layout to the operand layout through this wave's own LDS patch: the
     // wave's LDS accesses execute in order, the fences keep the compiler from moving them
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
@@ -1194,10 +1197,12 @@ __global__ __launch_bounds__(256) void attn_tile_kernel(
           float4 vv[4];
 #pragma unroll
           for (int j4 = 0; j4 < 4; ++j4) vv[j4] = *reinterpret_cast<const float4*>(Vs + (4 * j4 + lk) * VS + t * 16 + 4 * lr);
+          if (rescale) {
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
+            for (int i = 0; i < 4; ++i)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) o[t + i][r] *= corr[r];
+              for (int r = 0; r < 4; ++r) o[t + i][r] *= corr[r];
+          }
 #pragma unroll
           for (int j4 = 0; j4 < 4; ++j4) {                  // four independent chains
             o[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(pa[j4], vv[j4].x, o[t], 0, 0, 0);

@@ -79,7 +79,8 @@ __global__ __launch_bounds__(256) void gated_step_kernel(StepArgs a) {
         xv[i] = reinterpret_cast<const float4*>(a.x + row)[c];
         if (a.y != nullptr) {
           float4 v = reinterpret_cast<const float4*>(a.y + row)[c];
-          for (int s = 1; s < a.parts; ++s) {
+#pragma unroll 8
+          for (int s = 1; s < a.parts; ++s) {       // (several slabs in flight)
             const float4 w = reinterpret_cast<const float4*>(a.y + s * a.slab + row)[c];
             v = make_float4(v.x + w.x, v.y + w.y, v.z + w.z, v.w + w.w);
           }

@@ -1144,9 +1144,9 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
     sigmoid; ``out_scale`` multiplies every result. ``out``: write into this [T, H * Dv] block (of a wider matrix).
     ``value_share``: that many neighbouring key heads share a value head (value planes of G / value_share heads).
 
-    Two kernels: the first ``n_portions`` sequences (rows [0, portion_rows), the longest of
+    The first ``n_portions`` sequences (rows [0, portion_rows), the longest of
     ``max_len`` rows) are prompt portions and go, 64 rows of a head per block, through fp32 MFMA
-    tiles; the rows behind them (single decoded tokens) and shapes the tiles do not take go
+    tiles (of 32 keys for common widths and plain masks over bf16 planes, of 16 otherwise); the rows behind them (single decoded tokens) and shapes the tiles do not take go
     through the row kernel, one wave per (row, head)."""
     T = q.shape[0]
     if value_share < 1 or G % value_share or (value_share > 1 and all_value_heads):
@@ -1189,8 +1189,18 @@ def attn_masked(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, b
     first = 0
     # value heads side by side in one tile: equal groups whose width the tiles take (whole MFMA steps of 16 columns)
     tile_cols = max([n * Dv for n in range(1, nv + 1) if nv % n == 0 and Dv % 8 == 0 and attn_tile_ok(D, n * Dv)] or [0])
+    portions = n_portions > 0 and portion_rows > 0 and max_len >= ATTN_TILE_MIN_ROWS
+    if portions and not cf and nv == 1 and softcap == 0 and slopes is None and keep == 0 and not (sink and sinks is None) and \
+            k_ld % 8 == 0 and v_ld % 8 == 0 and o_row % 4 == 0 and Dv % 4 == 0 and \
+            all(t.data_ptr() % 16 == 0 for t in (q, k_cache, v_cache, out)) and _hip().lib().lc_attn_keys32_ok(D, Dv, BS):
+        # (masks that are an interval per row over bf16 planes, at widths in whole groups of MFMA steps)
+        _hip().call("lc_attn_keys32", q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr(), MB,
+                    cu_q.data_ptr(), positions.data_ptr(), out.data_ptr(), af, int(n_portions), int(max_len), H, G, D, Dv, BS,
+                    float(scale), int(chunk), int(window), k_ld, v_ld, _hip().ptr(sinks), _hip().ptr(gate),
+                    max(gate.stride(0), H) if gate is not None else 0, float(out_scale), o_row, int(value_share), o_ld)
+        first, portions = portion_rows, False
     aligned = k_ld % 8 == 0 and v_ld % 8 == 0 and k_cache.data_ptr() % 16 == 0 and v_cache.data_ptr() % 16 == 0
-    if n_portions > 0 and portion_rows > 0 and max_len >= ATTN_TILE_MIN_ROWS and tile_cols and aligned:
+    if portions and tile_cols and aligned:
         for vh0, nvh, col0 in value_groups(tile_cols):
             _hip().call("lc_attn_tile", q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), cf, block_tables.data_ptr(),
                         MB, cu_q.data_ptr(), positions.data_ptr(), out.data_ptr(), af, int(n_portions), int(max_len), H, G,

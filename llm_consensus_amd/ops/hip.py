@@ -71,6 +71,8 @@ _SIGNATURES = {
                        _I, _I, _F, _I, _P, _P, _I, _P, _I, _F, _I, _I, _I, _I, _I, _I, _I, _P],
     "lc_attn_tile": [_P, _P, _P, _I, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I,
                      _I, _I, _F, _I, _P, _P, _I, _P, _I, _F, _I, _I, _I, _I, _I, _I, _P],
+    "lc_attn_keys32_ok": [_I, _I, _I],
+    "lc_attn_keys32": [_P, _P, _P, _P, _I, _P, _P, _P, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _I, _P, _P, _I, _F, _I, _I, _I, _P],
     "lc_gemm_any": [_P, _I, _I, _P, _I, _P, _P, _I, _I, _I, _I, _I, _P],
     "lc_add_rmsnorm": [_P, _P, _P, _F, _P, _I, _I, _I, _P],
     "lc_latent_write": [_P, _I, _I, _I, _P, _F, _P, _P, _I, _I, _I, _P],

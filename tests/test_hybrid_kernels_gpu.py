@@ -977,3 +977,40 @@ def test_slabs_of_a_split_product_join_the_residual_step_and_the_gated_unit(d):
         torch.testing.assert_close(a.cpu(), b, atol=2e-5, rtol=2e-5)
     if d % 2 == 0:
         torch.testing.assert_close(ops.glu(ops.PartialSum(part.to(DEV)), torch.float32, "gelu_tanh").cpu(), ref.glu(part.sum(0), torch.float32, "gelu_tanh"), atol=2e-5, rtol=2e-5)
+
+
+@pytest.mark.parametrize("D,Dv", [(64, 64), (64, 128), (128, 128), (128, 256)])
+@pytest.mark.parametrize("BSZ", [32, 64, 96])
+@pytest.mark.parametrize("chunk,window", [(0, 0), (0, 7), (0, 90), (33, 0), (150, 40)])
+def test_portions_in_tiles_of_32_keys(D, Dv, BSZ, chunk, window):
+    """Portions that start at position 0, inside a tile and far in, of fewer rows than a tile, one more than a block and
+    several blocks; shared values, sinks, gates, a column block as output; planes that are column blocks of wider rows; cells
+    behind a sequence's last key hold no numbers. fp32 results, so that only the kernel's own rounding shows."""
+    g = torch.Generator().manual_seed(D + Dv + window)
+    H, G = 4, 2
+    lens, starts = [65, 20, 150, 1], [0, 301, 77, 40]
+    MB = (330 + BSZ - 1) // BSZ
+    cu, pos, rs = _seqs(lens, starts)
+    T = int(cu[-1])
+    tables = torch.randperm(4 * MB, generator=g).to(torch.int32).view(4, MB)
+    q = torch.randn(T, H * D, generator=g)
+    c = lambda t: t.to(DEV)   # noqa: E731
+    for share in (1, 2):
+        kc = torch.randn(4 * MB, G, BSZ, D + 8, generator=g).bfloat16()
+        vc = torch.randn(4 * MB, G // share, BSZ, Dv + 16, generator=g).bfloat16()
+        for b, (n, s) in enumerate(zip(lens, starts)):
+            for j in range(s + n, MB * BSZ):
+                kc[tables[b, j // BSZ], :, j % BSZ] = float("nan")
+                vc[tables[b, j // BSZ], :, j % BSZ] = float("nan")
+        kd, vd = c(kc), c(vc)
+        sinks, gates = torch.randn(H, generator=g) * 2, torch.randn(T, H + 5, generator=g)
+        for opt in ({}, dict(sinks=sinks, gate=gates[:, 2:2 + H], out_scale=0.6)):
+            want = ref.attn_masked(q, kc[..., :D], vc[..., :Dv], tables, cu, pos, H, G, D, Dv, 0.15, chunk, window, torch.float32,
+                                   value_share=share, **opt)
+            dopt = {k: (c(gates)[:, 2:2 + H] if k == "gate" else c(v) if torch.is_tensor(v) else v) for k, v in opt.items()}
+            for dt in ACTS:
+                wide = torch.zeros(T, 8 + H * Dv + 4, dtype=dt, device=DEV)
+                got = ops.attn_masked(c(q), kd[..., :D], vd[..., :Dv], c(tables), c(cu), c(rs), c(pos), H, G, D, Dv, 0.15, chunk, window, dt,
+                                      n_portions=3, portion_rows=235, max_len=150, out=wide[:, 8:8 + H * Dv], value_share=share, **dopt)
+                torch.testing.assert_close(got.float().cpu(), want, **(_tol(dt) if dt == torch.bfloat16 else dict(atol=3e-5, rtol=3e-5)))
+                assert not wide[:, :8].any() and not wide[:, 8 + H * Dv:].any()
