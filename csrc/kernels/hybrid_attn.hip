@@ -11,6 +11,9 @@
 //     i = 0..3, so that an operand's four numbers come in one access. A lane's four neighbouring value columns belong to four
 //     accumulator tiles for the same reason.
 //   - Tiles that every row of the wave sees whole need no mask; accumulators are rescaled only when a maximum moved.
+//   - GROUPS = 2: eight waves, of which the second four take every other tile of keys for the same rows; the two results are
+//     joined at the end. One wave alone leaves a SIMD idle more than half of the time, and the last rows' block, which has
+//     twice the mean number of keys, decides how long a small launch takes: two groups halve its chain.
 #include "hybrid_common.h"
 
 namespace {
@@ -61,24 +64,38 @@ struct TileArgs {
 
 constexpr int kKeys = 32;
 
-template <bool AF32, int DT, int VT>
-__global__ __launch_bounds__(256, 2) void attn_keys32_kernel(TileArgs a) {
+// LDS of one group of four waves: two buffers of keys and values, the weights of four waves.
+template <int DT, int VT>
+constexpr int group_lds() {
+  return 2 * kKeys * (16 * DT + 8 + 16 * VT + 16) * 2 + 4 * 16 * (kKeys + 4) * 4;
+}
+
+template <bool AF32, int DT, int VT, int GROUPS>
+__global__ __launch_bounds__(256 * GROUPS, 2) void attn_keys32_kernel(TileArgs a) {
   constexpr int D = 16 * DT, NC = 16 * VT;
   constexpr int KS = D + 8, VS = NC + 16;            // row strides (bf16): 16 operand rows in different banks
   constexpr int PS = kKeys + 4;
   constexpr int KU = kKeys * D / 8 / 256, VU = kKeys * NC / 8 / 256;      // 16-byte units of a tile per thread
   static_assert(KU >= 1 && VU >= 1 && VT % 4 == 0, "tiles of at least one unit per thread");
-  __shared__ __attribute__((aligned(16))) bf16_t Ks[2][kKeys * KS];
-  __shared__ __attribute__((aligned(16))) bf16_t Vs[2][kKeys * VS];
-  __shared__ __attribute__((aligned(16))) float Ps[4][16 * PS];
-  const int b = blockIdx.z, h = blockIdx.y;
+  extern __shared__ __attribute__((aligned(16))) char lds[];
+  const int tid = threadIdx.x & 255, group = threadIdx.x >> 8;
+  bf16_t* Ks = reinterpret_cast<bf16_t*>(lds + group * group_lds<DT, VT>());      // [2][kKeys * KS]
+  bf16_t* Vs = Ks + 2 * kKeys * KS;                  // [2][kKeys * VS]
+  float* Ps = reinterpret_cast<float*>(Vs + 2 * kKeys * VS);                      // [4][16 * PS]
+  const int b = blockIdx.z, h = GROUPS == 1 ? blockIdx.y : blockIdx.x;
   const int q0 = a.cu_q[b], q1 = a.cu_q[b + 1];
-  // A portion's later rows see more keys. Workgroups i and i + 256 share a CU, so every other 256 walk the row tiles
-  // backwards: a long tile and a short one meet on a CU instead of two long ones.
-  const bool forward = (((b * static_cast<int>(gridDim.y) + h) * static_cast<int>(gridDim.x)) >> 8) & 1;
-  const int row0 = q0 + (forward ? blockIdx.x : gridDim.x - 1 - blockIdx.x) * 64;
+  int tile;
+  if (GROUPS == 1) {
+    // A portion's later rows see more keys. Workgroups i and i + 256 share a CU, so every other 256 walk the row tiles
+    // backwards: a long tile and a short one meet on a CU instead of two long ones.
+    const bool forward = (((b * static_cast<int>(gridDim.y) + h) * static_cast<int>(gridDim.x)) >> 8) & 1;
+    tile = forward ? blockIdx.x : gridDim.x - 1 - blockIdx.x;
+  } else {
+    tile = gridDim.y - 1 - blockIdx.y;               // a block has a CU to itself: the long tiles of all heads first
+  }
+  const int row0 = q0 + tile * 64;
   if (row0 >= q1) return;                            // the same for the whole block
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, lr = lane & 15, lk = lane >> 4;
+  const int wave = tid >> 6, lane = threadIdx.x & 63, lr = lane & 15, lk = lane >> 4;
   const int g = h / (a.H / a.G), gv = g / a.v_share, GV = a.G / a.v_share;
   const int32_t* table = a.block_tables + static_cast<size_t>(b) * a.MB;
   const int p0 = a.positions[row0];                  // rows of a portion are consecutive positions
@@ -116,49 +133,56 @@ __global__ __launch_bounds__(256, 2) void attn_keys32_kernel(TileArgs a) {
     const bf16_t* v = a.vc + ((static_cast<size_t>(block) * GV + gv) * a.BS + j0 % a.BS) * a.v_ld;
 #pragma unroll
     for (int i = 0; i < KU; ++i) {
-      const int u = threadIdx.x + 256 * i;           // (keys past hi are cells of the same block: read, never seen)
+      const int u = tid + 256 * i;                   // (keys past hi are cells of the same block: read, never seen)
       kr[i] = *reinterpret_cast<const u32x4*>(k + (u / (D / 8)) * a.k_ld + (u % (D / 8)) * 8);
     }
 #pragma unroll
     for (int i = 0; i < VU; ++i) {
-      const int u = threadIdx.x + 256 * i;
-      const int key = u / (NC / 8);
-      vr[i] = *reinterpret_cast<const u32x4*>(v + key * a.v_ld + (u % (NC / 8)) * 8);
-      if (j0 + key > hi) vr[i] = u32x4{0u, 0u, 0u, 0u};       // (what nobody wrote may be no number; its weight is zero)
+      const int u = tid + 256 * i;
+      vr[i] = *reinterpret_cast<const u32x4*>(v + (u / (NC / 8)) * a.v_ld + (u % (NC / 8)) * 8);
     }
   };
-  auto stage = [&](int buf) {
+  auto stage = [&](int buf, int j0) {                // (the first use of what fetch loaded)
+    if (j0 + kKeys - 1 > hi) {
+#pragma unroll
+      for (int i = 0; i < VU; ++i)                   // what nobody wrote may be no number, and its weight of zero times it
+        if (j0 + (tid + 256 * i) / (NC / 8) > hi) vr[i] = u32x4{0u, 0u, 0u, 0u};
+    }
 #pragma unroll
     for (int i = 0; i < KU; ++i) {
-      const int u = threadIdx.x + 256 * i;
-      *reinterpret_cast<u32x4*>(&Ks[buf][(u / (D / 8)) * KS + (u % (D / 8)) * 8]) = kr[i];
+      const int u = tid + 256 * i;
+      *reinterpret_cast<u32x4*>(&Ks[buf * kKeys * KS + (u / (D / 8)) * KS + (u % (D / 8)) * 8]) = kr[i];
     }
 #pragma unroll
     for (int i = 0; i < VU; ++i) {
-      const int u = threadIdx.x + 256 * i;
-      *reinterpret_cast<u32x4*>(&Vs[buf][(u / (NC / 8)) * VS + (u % (NC / 8)) * 8]) = vr[i];
+      const int u = tid + 256 * i;
+      *reinterpret_cast<u32x4*>(&Vs[buf * kKeys * VS + (u / (NC / 8)) * VS + (u % (NC / 8)) * 8]) = vr[i];
     }
   };
   float m[4], l[4];
   f32x4 o[VT];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
-    m[r] = a.sinks != nullptr ? a.sinks[h] * kLog2e : -INFINITY;
-    l[r] = a.sinks != nullptr && lr == 0 ? 1.f : 0.f;
+    m[r] = a.sinks != nullptr && group == 0 ? a.sinks[h] * kLog2e : -INFINITY;
+    l[r] = a.sinks != nullptr && group == 0 && lr == 0 ? 1.f : 0.f;
   }
 #pragma unroll
   for (int t = 0; t < VT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float* Pw = Ps[wave];
+  float* Pw = Ps + wave * 16 * PS;
+  constexpr int STEP = kKeys * GROUPS;
   const int lo_tile = (first_key(p0) / kKeys) * kKeys;
-  fetch(lo_tile, block_of(lo_tile));
-  stage(0);
-  int ahead = block_of(lo_tile + kKeys), buf = 0;
-  for (int j0 = lo_tile; j0 <= hi; j0 += kKeys, buf ^= 1) {
+  int j0 = lo_tile + group * kKeys;                  // this group's first tile
+  if (j0 <= hi) {
+    fetch(j0, block_of(j0));
+    stage(0, j0);
+  }
+  int ahead = block_of(j0 + STEP), buf = 0;
+  for (int jb = lo_tile; jb <= hi; jb += STEP, j0 += STEP, buf ^= 1) {      // (all groups take the same number of turns)
     __syncthreads();                                 // this tile is in place, and nobody reads the other buffer any more
-    const bool more = j0 + kKeys <= hi;
+    const bool more = j0 + STEP <= hi;
     if (more) {
-      fetch(j0 + kKeys, ahead);
-      ahead = block_of(j0 + 2 * kKeys);
+      fetch(j0 + STEP, ahead);
+      ahead = block_of(j0 + 2 * STEP);
     }
     if (wave_rows > 0 && j0 <= wave_hi && j0 + kKeys - 1 >= wave_lo) {      // wave-uniform
       f32x4 s[2][2];
@@ -168,7 +192,7 @@ __global__ __launch_bounds__(256, 2) void attn_keys32_kernel(TileArgs a) {
       for (int kk = 0; kk < DT; ++kk)
 #pragma unroll
         for (int e = 0; e < 2; ++e) {
-          const float4 k = widen4(*reinterpret_cast<const uint2*>(&Ks[buf][(16 * e + lr) * KS + 16 * kk + 4 * lk]));
+          const float4 k = widen4(*reinterpret_cast<const uint2*>(&Ks[buf * kKeys * KS + (16 * e + lr) * KS + 16 * kk + 4 * lk]));
           s[e][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[kk].x, k.x, s[e][0], 0, 0, 0);
           s[e][1] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[kk].y, k.y, s[e][1], 0, 0, 0);
           s[e][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[kk].z, k.z, s[e][0], 0, 0, 0);
@@ -219,7 +243,7 @@ __global__ __launch_bounds__(256, 2) void attn_keys32_kernel(TileArgs a) {
           float4 v[4];
 #pragma unroll
           for (int i = 0; i < 4; ++i)
-            v[i] = widen4(*reinterpret_cast<const uint2*>(&Vs[buf][(16 * e + 4 * lk + i) * VS + t * 16 + 4 * lr]));
+            v[i] = widen4(*reinterpret_cast<const uint2*>(&Vs[buf * kKeys * VS + (16 * e + 4 * lk + i) * VS + t * 16 + 4 * lr]));
           const float pi[4] = {p.x, p.y, p.z, p.w};
 #pragma unroll
           for (int i = 0; i < 4; ++i) {              // four independent chains
@@ -233,7 +257,35 @@ __global__ __launch_bounds__(256, 2) void attn_keys32_kernel(TileArgs a) {
       __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");     // P is read before the next tile overwrites it
       __builtin_amdgcn_wave_barrier();
     }
-    if (more) stage(buf ^ 1);
+    if (more) stage(buf ^ 1, j0 + STEP);
+  }
+  if constexpr (GROUPS == 2) {
+    // the second group's sums go through LDS (the tiles are done with), register after register, to the first one's lanes
+    static_assert((4 * VT + 8) * 256 * 4 <= 2 * group_lds<DT, VT>(), "the sums fit where the tiles were");
+    float* xs = reinterpret_cast<float*>(lds);
+    __syncthreads();
+    if (group == 1) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        xs[r * 256 + tid] = m[r];
+        xs[(4 + r) * 256 + tid] = l[r];
+      }
+#pragma unroll
+      for (int t = 0; t < VT; ++t)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) xs[(8 + 4 * t + r) * 256 + tid] = o[t][r];
+    }
+    __syncthreads();
+    if (group == 1) return;                          // (no barrier follows)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float m1 = xs[r * 256 + tid], mn = fmaxf(m[r], m1);
+      const float base = mn == -INFINITY ? 0.f : mn;
+      const float f0 = fast_exp2(m[r] - base), f1 = fast_exp2(m1 - base);
+      l[r] = l[r] * f0 + xs[(4 + r) * 256 + tid] * f1;
+#pragma unroll
+      for (int t = 0; t < VT; ++t) o[t][r] = o[t][r] * f0 + xs[(8 + 4 * t + r) * 256 + tid] * f1;
+    }
   }
   typedef typename Act<AF32>::type act_t;
 #pragma unroll
@@ -251,6 +303,9 @@ __global__ __launch_bounds__(256, 2) void attn_keys32_kernel(TileArgs a) {
 }
 
 }  // namespace
+
+// Launches of up to this many row tiles run two groups of waves per tile.
+constexpr long long kTwoGroupBlocks = 1024;
 
 // Whether lc_attn_keys32 takes the shape (1) or not (0).
 LC_EXPORT int lc_attn_keys32_ok(int D, int Dv, int BS) {
@@ -271,16 +326,31 @@ LC_EXPORT int lc_attn_keys32(const void* q, const void* kc, const void* vc, cons
                    static_cast<const int32_t*>(block_tables), MB, static_cast<const int32_t*>(cu_q),
                    static_cast<const int32_t*>(positions), out, H, G, BS, scale, chunk, window, k_ld, v_ld, v_share,
                    static_cast<const float*>(sinks), static_cast<const float*>(gate), ld_gate, out_scale, o_row, o_ld};
-  const dim3 grid((max_len + 63) / 64, H, n_seq), block(256);
-#define LC_K32(DT, VT)                                                            \
-  do {                                                                            \
-    if (act_f32) attn_keys32_kernel<true, DT, VT><<<grid, block, 0, st>>>(a);     \
-    else attn_keys32_kernel<false, DT, VT><<<grid, block, 0, st>>>(a);            \
+  const int tiles = (max_len + 63) / 64;
+  const bool two = static_cast<long long>(tiles) * H * n_seq <= kTwoGroupBlocks;
+#define LC_K32_G(A32, DT, VT)                                                                                             \
+  do {                                                                                                                    \
+    constexpr int one_lds = group_lds<DT, VT>();                                                                          \
+    static LcDeviceOnce attr_once;                                                                                        \
+    attr_once.run([&] {                                                                                                   \
+      (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_keys32_kernel<A32, DT, VT, 1>),                        \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, one_lds);                                     \
+      (void)hipFuncSetAttribute(reinterpret_cast<const void*>(attn_keys32_kernel<A32, DT, VT, 2>),                        \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, 2 * one_lds);                                 \
+    });                                                                                                                   \
+    if (two) attn_keys32_kernel<A32, DT, VT, 2><<<dim3(H, tiles, n_seq), dim3(512), 2 * one_lds, st>>>(a);                \
+    else attn_keys32_kernel<A32, DT, VT, 1><<<dim3(tiles, H, n_seq), dim3(256), one_lds, st>>>(a);                        \
+  } while (0)
+#define LC_K32(DT, VT)                        \
+  do {                                        \
+    if (act_f32) LC_K32_G(true, DT, VT);      \
+    else LC_K32_G(false, DT, VT);             \
   } while (0)
   if (D == 64 && Dv == 64) LC_K32(4, 4);
   else if (D == 64) LC_K32(4, 8);
   else if (Dv == 128) LC_K32(8, 8);
   else LC_K32(8, 16);
 #undef LC_K32
+#undef LC_K32_G
   LC_RETURN_LAST_ERROR();
 }
